@@ -27,6 +27,9 @@ HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 # ablation builds: extra device-compile flags (e.g. "-DMP_RW_WAVES=8") go to their own object
 # directory and library name (``--out``), never over the default library
 EXTRA = os.environ.get("MPAMD_HIPCC_EXTRA", "").split()
+# device code keeps to scalar fp32 instructions: the packed fp32 forms the optimizer would otherwise
+# pick from ordinary float code are switched off for every kernel
+DEVICE_FLAGS = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 
 def _torch_paths():
@@ -67,7 +70,7 @@ def build(force: bool = False, jobs: int = 0, verbose: bool = False, out: str = 
         raise SystemExit("MPAMD_HIPCC_EXTRA builds need --out (the default library stays the default build)")
     LIB_PATH = os.path.abspath(out) if out else globals()["LIB_PATH"]
     BUILD = globals()["BUILD"] + ("_" + hashlib.sha256(xtag.encode()).hexdigest()[:8] if xtag else "")
-    tag = _digest(hips + [binding] + headers, extra=ARCH + HIPCC + xtag)
+    tag = _digest(hips + [binding] + headers, extra=ARCH + HIPCC + xtag + " ".join(DEVICE_FLAGS))
     stamp = os.path.join(BUILD, "stamp")
     if not force and os.path.exists(LIB_PATH) and os.path.exists(stamp):
         with open(stamp) as f:
@@ -75,10 +78,10 @@ def build(force: bool = False, jobs: int = 0, verbose: bool = False, out: str = 
                 return LIB_PATH
     os.makedirs(BUILD, exist_ok=True)
     inc, libdir = _torch_paths()
-    common = ["-O3", "-fPIC", "-std=c++17", f"--offload-arch={ARCH}", "-I" + CSRC] + EXTRA
+    common = ["-O3", "-fPIC", "-std=c++17", f"--offload-arch={ARCH}", "-I" + CSRC] + DEVICE_FLAGS + EXTRA
     objs = []
     cmds = []
-    hdr_tag = _digest(headers, extra=ARCH + HIPCC + xtag)
+    hdr_tag = _digest(headers, extra=ARCH + HIPCC + xtag + " ".join(DEVICE_FLAGS))
 
     def stale(src, obj):
         # per-object stamp: the source + every csrc header (a kernel edit rebuilds one object)
