@@ -17,9 +17,71 @@ from __future__ import annotations
 import dataclasses
 import json
 import os
-from typing import Optional
+from typing import Callable, Dict, Optional, Tuple
 
-SUPPORTED_TYPES = ("llama", "mistral", "mixtral", "gpt2")
+SUPPORTED_TYPES = ("llama", "mistral", "mixtral", "gpt2", "kafunex")
+MIXERS = ("attention", "hgrn2")
+
+
+@dataclasses.dataclass(frozen=True)
+class LayerSpec:
+    """One layer of a hybrid decoder (``ModelConfig.layers``): its token mixer with that mixer's sizes and
+    the width of its feed-forward (0 = none).  Layers of one model may differ in every field.
+
+    ``attention``: chunked talking-heads attention whose values are the projected keys; ``hgrn2``: the
+    gated linear recurrence (no kv heads, no mask, no scale)."""
+    mixer: str
+    heads: int
+    dim: int
+    vdim: int
+    ff: int = 0
+    kv_heads: int = 0
+    chunk: int = 0
+    scale: float = 1.0
+
+    @property
+    def recurrent(self) -> bool:
+        return self.mixer == "hgrn2"
+
+    @property
+    def in_rows(self) -> int:
+        """Rows of the fused input projection: [q | f | v] or [q | k | gate]."""
+        if self.recurrent:
+            return self.heads * (2 * self.dim + self.vdim)
+        return (2 * self.heads + self.kv_heads) * self.dim
+
+    @property
+    def out_cols(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def kv_elems(self) -> int:
+        """Cached elements per token (one shared key/value row)."""
+        return 0 if self.recurrent else self.kv_heads * self.dim
+
+    @property
+    def state_elems(self) -> int:
+        """fp32 state elements per session."""
+        return self.heads * self.dim * self.vdim if self.recurrent else 0
+
+    def param_count(self, width: int) -> int:
+        n = width * (self.in_rows + self.out_cols + 2 * self.ff) + 2 * width
+        if self.recurrent:
+            return n + 2 * self.heads * self.dim + self.vdim
+        return n + (self.heads + self.kv_heads) * self.dim + self.heads * self.heads
+
+    def validate(self) -> None:
+        if self.mixer not in MIXERS:
+            raise ValueError(f"unsupported mixer {self.mixer!r}; supported: {MIXERS}")
+        if min(self.heads, self.dim, self.vdim) < 1 or self.ff < 0:
+            raise ValueError(f"bad layer sizes: {self}")
+        if self.mixer == "attention":
+            if self.kv_heads < 1 or self.heads % self.kv_heads:
+                raise ValueError("attention heads must be a multiple of kv_heads")
+            if self.dim != self.vdim:
+                raise ValueError("the values are the keys: vdim must equal dim")
+            if self.chunk < 1:
+                raise ValueError("attention needs a mask size >= 1")
 
 
 @dataclasses.dataclass
@@ -46,6 +108,12 @@ class ModelConfig:
     num_experts_per_tok: int = 2
     # Mistral / Mixtral sliding-window attention (None = full causal attention)
     sliding_window: Optional[int] = None
+    # hybrid decoders: one LayerSpec per layer (None = the uniform families above)
+    layers: Optional[Tuple[LayerSpec, ...]] = None
+
+    @property
+    def hybrid(self) -> bool:
+        return self.layers is not None
 
     @property
     def is_moe(self) -> bool:
@@ -66,7 +134,9 @@ class ModelConfig:
     def layer_param_bytes(self, bytes_per_param: float = 2.0) -> int:
         """Weights of one decoder block (survey V11 `get_block_size`)."""
         H, F = self.hidden_size, self.intermediate_size
-        if self.model_type == "gpt2":
+        if self.hybrid:  # layers differ: the mean
+            n = sum(sp.param_count(H) for sp in self.layers) / max(len(self.layers), 1)
+        elif self.model_type == "gpt2":
             n = 4 * H * H + 2 * H * F + 9 * H + F
         else:
             mlp = self.num_local_experts * (3 * H * F + H) if self.is_moe else 3 * H * F
@@ -74,11 +144,20 @@ class ModelConfig:
         return int(n * bytes_per_param)
 
     def kv_bytes_per_token_per_layer(self, bytes_per_elt: int = 2) -> int:
+        if self.hybrid:  # shared key/value rows + one fp32 per attention layer, averaged over the layers
+            n = sum(sp.kv_elems * bytes_per_elt + 4 for sp in self.layers if not sp.recurrent)
+            return -(-n // max(len(self.layers), 1))
         return 2 * self.kv_dim * bytes_per_elt
 
     def validate(self) -> None:
         if self.model_type not in SUPPORTED_TYPES:
             raise ValueError(f"unsupported model_type {self.model_type!r}; supported: {SUPPORTED_TYPES}")
+        if self.hybrid:
+            if len(self.layers) != self.num_hidden_layers:
+                raise ValueError("layers must list every layer")
+            for sp in self.layers:
+                sp.validate()
+            return
         if self.num_attention_heads % self.num_key_value_heads:
             raise ValueError("num_attention_heads must be a multiple of num_key_value_heads")
         if self.head_dim % 8:
@@ -91,6 +170,11 @@ class ModelConfig:
 
     @classmethod
     def from_hf_dict(cls, d: dict, name: str = "custom") -> "ModelConfig":
+        arch = d.get("architecture")
+        if arch is not None:
+            if arch not in ARCHITECTURES:
+                raise ValueError(f"unknown architecture {arch!r}; known: {sorted(ARCHITECTURES)}")
+            return ARCHITECTURES[arch](d, name)
         mt = d.get("model_type", "llama")
         if mt == "gpt2":
             H = d.get("n_embd", d.get("hidden_size", 768))
@@ -124,7 +208,50 @@ class ModelConfig:
                    sliding_window=d.get("sliding_window"))
 
 
+def hybrid_config(model_type: str, vocab: int, width: int, eps: float, layers, name: str,
+                  max_positions: int = 32768) -> ModelConfig:
+    """A hybrid decoder's ModelConfig.  The uniform fields (heads, kv heads, head size, ff) describe its
+    first attention layer, else its first layer: estimates and announcements read them, kernels do not."""
+    layers = tuple(layers)
+    ref = next((sp for sp in layers if not sp.recurrent), layers[0])
+    return ModelConfig(model_type=model_type, vocab_size=vocab, hidden_size=width, intermediate_size=ref.ff,
+                       num_hidden_layers=len(layers), num_attention_heads=ref.heads,
+                       num_key_value_heads=ref.kv_heads or ref.heads, head_dim=ref.dim, rms_norm_eps=eps,
+                       max_position_embeddings=max_positions, name=name, layers=layers)
+
+
+def _kafunex_config(d: dict, name: str) -> ModelConfig:
+    layers = []
+    for i, e in enumerate(d["layers"]):
+        m, mlp = e["mixer"], e.get("mlp")
+        if mlp is not None and mlp.get("kind", "dense") != "dense":
+            raise ValueError(f"layer {i}: unsupported feed-forward kind {mlp['kind']!r}")
+        ff = int(mlp["ff"]) if mlp is not None else 0
+        if e["type"] == "hgrn2":
+            layers.append(LayerSpec("hgrn2", int(m["heads"]), int(m["dim"]), int(m["vdim"]), ff))
+        elif e["type"] == "attention":
+            layers.append(LayerSpec("attention", int(m["heads"]), int(m["dim"]), int(m.get("vdim", m["dim"])), ff,
+                                    int(m["kv_heads"]), int(m["mask"]["size"]), float(m["scale"])))
+        else:
+            raise ValueError(f"layer {i}: unsupported mixer {e['type']!r}; supported: {MIXERS}")
+    return hybrid_config("kafunex", int(d["vocab"]), int(d["width"]), float(d["norm"]["eps"]), layers, name)
+
+
+# config.json "architecture" -> reader (the other families are told apart by Hugging Face's "model_type")
+ARCHITECTURES: Dict[str, Callable[[dict, str], ModelConfig]] = {"Kafunex": _kafunex_config}
+
+
+def _kafunex_preset(name, vocab, width, ff, groups, rec, att) -> ModelConfig:
+    """``groups`` x [three recurrent layers, one attention layer]."""
+    return hybrid_config("kafunex", vocab, width, 1e-6, ((rec,) * 3 + (att,)) * groups, name)
+
+
 PRESETS = {
+    # hybrid decoders: a small one for tests, and one with a 7B-class model's layer sizes
+    "tiny-kafunex": _kafunex_preset("tiny-kafunex", 640, 128, 256, 1, LayerSpec("hgrn2", 2, 32, 48, 256),
+                                    LayerSpec("attention", 4, 32, 32, 256, 2, 40, 32 ** -0.5)),
+    "kafunex-7b": _kafunex_preset("kafunex-7b", 32000, 4096, 16384, 8, LayerSpec("hgrn2", 32, 128, 128, 16384),
+                                  LayerSpec("attention", 32, 128, 128, 16384, 8, 1024, 128 ** -0.5)),
     "llama2-7b": ModelConfig(name="llama2-7b"),
     "llama3-8b": ModelConfig(vocab_size=128256, intermediate_size=14336, num_key_value_heads=8,
                              rope_theta=500000.0, max_position_embeddings=8192, bos_token_id=128000,

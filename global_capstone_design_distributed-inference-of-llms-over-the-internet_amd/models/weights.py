@@ -26,7 +26,7 @@ from typing import Dict, List, Optional
 
 import torch
 
-from .config import ModelConfig
+from .config import LayerSpec, ModelConfig
 from ..ops.reference import GU_BLOCK
 
 INIT_STD = 0.02
@@ -126,6 +126,31 @@ class GPT2Layer:
 
 
 @dataclasses.dataclass
+class HybridLayer:
+    """A layer of a hybrid decoder.  GEMM weights have the stage's dtype; norms, gates and mixing matrices
+    are fp32.  ``w_in`` fuses the mixer's input projections ([q | f | v] or [q | k | gate]); ``*_p`` are the
+    fragment-native copies for the decode GEMM where the shape allows one."""
+    spec: LayerSpec
+    w_in: torch.Tensor                       # [in_rows, W]
+    w_o: torch.Tensor                        # [W, heads * vdim]
+    n1: torch.Tensor                         # [W] mixer output norm gain x layer scale
+    w_up: Optional[torch.Tensor] = None      # [ff, W]
+    w_down: Optional[torch.Tensor] = None    # [W, ff]
+    n2: Optional[torch.Tensor] = None        # [W]
+    f_bias: Optional[torch.Tensor] = None    # hgrn2 [heads * dim]
+    f_lower: Optional[torch.Tensor] = None   # hgrn2 [heads * dim]
+    o_norm: Optional[torch.Tensor] = None    # hgrn2 [vdim]
+    w_qk: Optional[torch.Tensor] = None      # attention [heads * dim]: query norm x its kv head's key norm
+    talk: Optional[torch.Tensor] = None      # attention [heads, heads]
+    w_in_p: Optional[torch.Tensor] = None
+    w_o_p: Optional[torch.Tensor] = None
+    w_up_p: Optional[torch.Tensor] = None
+    w_down_p: Optional[torch.Tensor] = None
+
+    GEMMS = ("w_in", "w_o", "w_up", "w_down")
+
+
+@dataclasses.dataclass
 class StageWeights:
     cfg: ModelConfig
     start: int
@@ -166,6 +191,12 @@ class StageWeights:
         from .. import ops
 
         for lay in self.layers:
+            if isinstance(lay, HybridLayer):
+                for name in HybridLayer.GEMMS:
+                    w = getattr(lay, name)
+                    if w is not None and w.dtype == torch.bfloat16 and w.shape[0] % 16 == 0 and w.shape[1] % 128 == 0 \
+                            and getattr(lay, name + "_p") is None:
+                        setattr(lay, name + "_p", ops.pack_weight(w))
             if isinstance(lay, LlamaLayer) and lay.qkv_p is None and lay.qkv is not None:
                 if fold_norms and not lay.moe:
                     lay.qkv_p = ops.pack_weight((lay.qkv.float() * lay.input_norm.float()[None, :])
@@ -188,7 +219,7 @@ class StageWeights:
                     lay.down_p = ops.pack_weight(lay.down)
         if self.lm_head is not None and self.lm_head_p is None and self.cfg.model_type != "gpt2":
             V, H = self.lm_head.shape
-            if H % 32 == 0:
+            if H % 32 == 0 and self.lm_head.dtype == torch.bfloat16:
                 pad = (-V) % 16
                 w = self.lm_head if pad == 0 else torch.cat([self.lm_head, self.lm_head.new_zeros(pad, H)])
                 # fused-norm decode: the final RMSNorm weight folded in as for qkv / gate_up, so a
@@ -258,7 +289,7 @@ class StageWeights:
         for lay in self.layers:
             for f in dataclasses.fields(lay):
                 t = getattr(lay, f.name)
-                if t is not None and id(t) not in seen:
+                if isinstance(t, torch.Tensor) and id(t) not in seen:
                     seen.add(id(t))
                     yield t
         for t in (self.embed, self.pos_embed, self.final_norm, self.final_norm_b, self.lm_head, self.lm_head_p):
@@ -309,12 +340,86 @@ def _random_gpt2_layer(cfg: ModelConfig, idx: int, device, dtype, seed: int) -> 
                      z(H), o(H), z(H), _randn((F, H), g, device, dtype), z(F), _randn((H, F), g, device, dtype), z(H))
 
 
+# ------------------------------------------------------------------ hybrid decoders
+def _hybrid_names(spec: LayerSpec, width: int) -> Dict[str, tuple]:
+    """Checkpoint tensors of one layer (after its 'l<i>.' prefix) -> shape."""
+    n: Dict[str, tuple] = {"norm1": (), "ls1": (width,)}
+    H, D, V = spec.heads, spec.dim, spec.vdim
+    if spec.recurrent:
+        n.update({"mix.q": (H * D, width), "mix.f": (H * D, width), "mix.f.b": (H * D,), "mix.lower": (H * D,),
+                  "mix.v": (H * V, width), "mix.norm": (V,), "mix.o": (width, H * V)})
+    else:
+        KD = spec.kv_heads * D
+        n.update({"mix.q": (H * D, width), "mix.k": (KD, width), "mix.q.norm": (H * D,), "mix.k.norm": (KD,),
+                  "mix.talk": (H, H), "mix.g": (H * D, width), "mix.o": (width, H * D)})
+    if spec.ff:
+        n.update({"mlp.up": (spec.ff, width), "mlp.down": (width, spec.ff), "norm2": (), "ls2": (width,)})
+    return n
+
+
+def _hybrid_layer(spec: LayerSpec, width: int, get, device, dtype) -> HybridLayer:
+    """``get(name)``: checkpoint tensor of this layer (any device / dtype)."""
+    raw = {}
+    for name, shape in _hybrid_names(spec, width).items():
+        t = get(name)
+        if tuple(t.shape) != shape:
+            raise ValueError(f"{name}: shape {tuple(t.shape)}, expected {shape}")
+        raw[name] = t.to(device)
+    f32 = lambda n: raw[n].float().contiguous()  # noqa: E731
+    g = lambda n: raw[n].to(dtype).contiguous()  # noqa: E731
+    parts = ("mix.q", "mix.f", "mix.v") if spec.recurrent else ("mix.q", "mix.k", "mix.g")
+    lay = HybridLayer(spec, torch.cat([raw[p].to(dtype) for p in parts], 0).contiguous(), g("mix.o"),
+                      f32("norm1") * f32("ls1"))
+    if spec.ff:
+        lay.w_up, lay.w_down, lay.n2 = g("mlp.up"), g("mlp.down"), f32("norm2") * f32("ls2")
+    if spec.recurrent:
+        lay.f_bias, lay.f_lower, lay.o_norm = f32("mix.f.b"), f32("mix.lower"), f32("mix.norm")
+    else:
+        kn = f32("mix.k.norm").view(spec.kv_heads, 1, spec.dim)
+        kn = kn.expand(spec.kv_heads, spec.heads // spec.kv_heads, spec.dim).reshape(-1)
+        lay.w_qk, lay.talk = (f32("mix.q.norm") * kn).contiguous(), f32("mix.talk")
+    return lay
+
+
+def random_hybrid_tensors(cfg: ModelConfig, idx: int, device="cpu", dtype=torch.bfloat16,
+                          seed: int = 0) -> Dict[str, torch.Tensor]:
+    """Synthetic checkpoint tensors of layer ``idx`` (names without the layer prefix)."""
+    g = _gen(device, seed * 100003 + idx + 1)
+    spec, W = cfg.layers[idx], cfg.hidden_size
+    out = {}
+    for name, shape in _hybrid_names(spec, W).items():
+        if name.endswith("norm") or name in ("norm1", "norm2", "ls1", "ls2"):
+            t = torch.ones(shape, device=device)
+        elif name == "mix.talk":
+            t = torch.eye(shape[0], device=device) + _randn(shape, g, device, torch.float32, 0.3 / shape[0] ** 0.5)
+        elif name == "mix.f.b":  # forget gates near 1: the state remembers
+            t = 2.0 + _randn(shape, g, device, torch.float32, 1.0)
+        elif name == "mix.lower":
+            t = torch.empty(shape, device=device).uniform_(0.0, 0.9, generator=g)
+        else:
+            t = _randn(shape, g, device, torch.float32, shape[-1] ** -0.5)
+        out[name] = t.to(dtype)
+    return out
+
+
+def _random_hybrid_layer(cfg: ModelConfig, idx: int, device, dtype, seed: int) -> HybridLayer:
+    raw = random_hybrid_tensors(cfg, idx, device, dtype, seed)
+    return _hybrid_layer(cfg.layers[idx], cfg.hidden_size, raw.__getitem__, device, dtype)
+
+
+def _pad_rows(w: torch.Tensor, m: int) -> torch.Tensor:
+    """``w`` with zero rows up to a multiple of ``m`` (an lm_head whose logits rows stay 16-B aligned)."""
+    pad = (-w.shape[0]) % m
+    return w if pad == 0 else torch.cat([w, w.new_zeros(pad, w.shape[1])])
+
+
 def random_stage_weights(cfg: ModelConfig, start: int, end: int, *, has_embed: bool, has_head: bool, device,
                          dtype=torch.bfloat16, seed: int = 0, fp8: bool = False) -> StageWeights:
     """``fp8``: quantize each block as soon as it is generated (bf16 copies dropped), so a
     70B stage never holds its full bf16 weights."""
     device = torch.device(device)
-    mk = _random_gpt2_layer if cfg.model_type == "gpt2" else _random_llama_layer
+    mk = _random_hybrid_layer if cfg.hybrid else \
+        _random_gpt2_layer if cfg.model_type == "gpt2" else _random_llama_layer
     layers = []
     for i in range(start, end):
         lay = mk(cfg, i, device, dtype, seed)
@@ -335,11 +440,13 @@ def random_stage_weights(cfg: ModelConfig, start: int, end: int, *, has_embed: b
         if has_head and cfg.tie_word_embeddings:
             sw.lm_head = emb
     if has_head:
-        sw.final_norm = torch.ones(H, dtype=dtype, device=device)
+        sw.final_norm = torch.ones(H, dtype=torch.float32 if cfg.hybrid else dtype, device=device)
         if cfg.model_type == "gpt2":
             sw.final_norm_b = torch.zeros(H, dtype=dtype, device=device)
         if sw.lm_head is None:
             sw.lm_head = _randn((V, H), _gen(device, seed * 100003 + 7937), device, dtype)
+        if cfg.hybrid:
+            sw.lm_head = _pad_rows(sw.lm_head, 16)
     return sw
 
 
@@ -423,6 +530,17 @@ def load_stage_weights(cfg: ModelConfig, path: str, start: int, end: int, *, has
         return ck.get(key).to(device=dev, dtype=dtype)
 
     layers: List = []
+    if cfg.hybrid:
+        W = cfg.hidden_size
+        for i in range(start, end):
+            layers.append(_hybrid_layer(cfg.layers[i], W, lambda n, p=f"l{i}.": ck.get(p + n), dev, dtype))
+        sw = StageWeights(cfg, start, end, layers)
+        if has_embed:
+            sw.embed = t("embed").contiguous()
+        if has_head:
+            sw.final_norm = ck.get("final.norm").to(dev).float().reshape(1).repeat(W)
+            sw.lm_head = _pad_rows(t("head"), 16).contiguous()
+        return sw
     if cfg.model_type == "gpt2":
         pre = "transformer." if ck.has("transformer.wte.weight") else ""
         for i in range(start, end):

@@ -1447,3 +1447,7 @@ def autotune_w8(shapes, device, ms=(4, 16, 32, 48, 64), iters: int = 12, rounds:
     finally:
         _W8_MODE = saved
     return dict(_W8_CHOICE)
+
+
+# the hybrid decoders' ops (imported last: they dispatch through this module)
+from . import hybrid  # noqa: E402,F401

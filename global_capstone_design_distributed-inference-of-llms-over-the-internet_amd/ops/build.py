@@ -1,7 +1,7 @@
 """In-tree build of the gfx950 HIP kernels into one torch custom-op library.
 
 No hipify, no torch JIT cache: every ``csrc/*.hip`` file is compiled by ``hipcc
---offload-arch=gfx950`` and linked with ``csrc/bindings.cpp`` (TORCH_LIBRARY
+--offload-arch=gfx950`` and linked with ``csrc/bindings*.cpp`` (TORCH_LIBRARY
 registrations) into ``ops/_mpamd_kernels.so`` next to this file, so the built
 library travels with the repository snapshot to the GPU box.
 
@@ -43,7 +43,8 @@ def _torch_paths():
 
 def _sources():
     hip = sorted(f for f in os.listdir(CSRC) if f.endswith(".hip"))
-    return [os.path.join(CSRC, f) for f in hip], os.path.join(CSRC, "bindings.cpp")
+    cpp = sorted(f for f in os.listdir(CSRC) if f.startswith("bindings") and f.endswith(".cpp"))
+    return [os.path.join(CSRC, f) for f in hip], [os.path.join(CSRC, f) for f in cpp]
 
 
 def _digest(paths, extra=""):
@@ -63,14 +64,14 @@ def _run(cmd):
 
 def build(force: bool = False, jobs: int = 0, verbose: bool = False, out: str = None) -> str:
     """Compile (if stale) and return the path of the kernel library."""
-    hips, binding = _sources()
+    hips, bindings = _sources()
     headers = [os.path.join(CSRC, f) for f in sorted(os.listdir(CSRC)) if f.endswith(".h")]
     xtag = " ".join(EXTRA)
     if xtag and not out:
         raise SystemExit("MPAMD_HIPCC_EXTRA builds need --out (the default library stays the default build)")
     LIB_PATH = os.path.abspath(out) if out else globals()["LIB_PATH"]
     BUILD = globals()["BUILD"] + ("_" + hashlib.sha256(xtag.encode()).hexdigest()[:8] if xtag else "")
-    tag = _digest(hips + [binding] + headers, extra=ARCH + HIPCC + xtag + " ".join(DEVICE_FLAGS))
+    tag = _digest(hips + bindings + headers, extra=ARCH + HIPCC + xtag + " ".join(DEVICE_FLAGS))
     stamp = os.path.join(BUILD, "stamp")
     if not force and os.path.exists(LIB_PATH) and os.path.exists(stamp):
         with open(stamp) as f:
@@ -97,13 +98,14 @@ def build(force: bool = False, jobs: int = 0, verbose: bool = False, out: str = 
         t = stale(src, obj)
         if t is not None:
             cmds.append(([HIPCC] + common + ["-c", src, "-o", obj], obj, t))
-    bobj = os.path.join(BUILD, "bindings.o")
-    objs.append(bobj)
-    t = stale(binding, bobj)
-    if t is not None:
-        # host-only translation unit (torch headers): plain C++, no device pass
-        cmds.append(([HIPCC, "-x", "c++", "-O2", "-fPIC", "-std=c++17", "-DUSE_ROCM=1", "-D__HIP_PLATFORM_AMD__=1",
-                      "-I/opt/rocm/include"] + [f"-I{p}" for p in inc] + ["-c", binding, "-o", bobj], bobj, t))
+    for binding in bindings:
+        bobj = os.path.join(BUILD, os.path.basename(binding)[:-4] + ".o")
+        objs.append(bobj)
+        t = stale(binding, bobj)
+        if t is not None:
+            # host-only translation unit (torch headers): plain C++, no device pass
+            cmds.append(([HIPCC, "-x", "c++", "-O2", "-fPIC", "-std=c++17", "-DUSE_ROCM=1", "-D__HIP_PLATFORM_AMD__=1",
+                          "-I/opt/rocm/include"] + [f"-I{p}" for p in inc] + ["-c", binding, "-o", bobj], bobj, t))
 
     def run_one(job):
         cmd, obj, t = job

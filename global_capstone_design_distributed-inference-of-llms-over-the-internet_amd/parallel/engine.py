@@ -434,7 +434,7 @@ class PipelineServingEngine:
         self._exchange_capacity()
         # stage-local recovery (opt-in): park KV on failure, keep a replay cache of the outputs
         self.park_on_fail = bool(replay_cache)
-        self.replay = (ReplayCache(self.max_handles, self.max_len, self.H, executor.dtype, self.dev)
+        self.replay = (ReplayCache(self.max_handles, self.max_len, self.H, executor.hidden_dtype, self.dev)
                        if replay_cache and not self.is_tail else None)
         self.resume = dict(resume or {})  # {"prefix": failed channel's engine name, "cache": its ReplayCache}
         self.failed_sessions: Dict[str, Tuple[int, Request]] = {}  # head: rid -> (handle, request) at failure
@@ -793,7 +793,7 @@ class PipelineServingEngine:
             # (posting the receive stays outside the lock too: a first RCCL receive can block on its
             # peer's connection set-up; decode graphs are captured in thread-local mode, so this
             # thread's stream calls never invalidate another thread's capture)
-            t, waiter = self.ch.recv(self.rank - 1, (rows, self.H), self.ex.dtype, into=into)
+            t, waiter = self.ch.recv(self.rank - 1, (rows, self.H), self.ex.hidden_dtype, into=into)
             self.recvs += 1
             self.recvs_into += int(into is not None and t is into[0])
             hw = getattr(waiter, "host_wait", None)
@@ -984,7 +984,7 @@ class PipelineServingEngine:
             if self.rank == target - 1:
                 self._replay_send(torch.cat([self.replay.rows(int(h), int(L)) for h, L, _ in recs]))
             elif self.rank == target:
-                _, waiter = self.ch.recv(self.rank - 1, (T, self.H), self.ex.dtype)
+                _, waiter = self.ch.recv(self.rank - 1, (T, self.H), self.ex.hidden_dtype)
                 x = waiter()
                 out = self.ex.forward([(self._key(int(h)), int(L)) for h, L, _ in recs], x, reset=[True] * n,
                                       max_length=self.max_len)

@@ -521,7 +521,7 @@ class StageConnectionHandler:
         if ex.is_first:
             x = torch.cat([r.x.reshape(-1).to(torch.long) for r in batch]).to(ex.device)
         else:
-            x = torch.cat([r.x for r in batch]).to(ex.device, ex.dtype)
+            x = torch.cat([r.x for r in batch]).to(ex.device, ex.hidden_dtype)
         ml = max((int(r.max_length) for r in batch if r.max_length), default=None)
         phase = "handler.prefill" if any(r.x.shape[0] > 1 for r in batch) else "handler.decode"
         prompts = [r.prompts for r in batch] if any(r.prompts is not None for r in batch) else None

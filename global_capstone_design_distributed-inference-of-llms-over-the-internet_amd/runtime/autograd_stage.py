@@ -41,6 +41,8 @@ class AutogradStage:
     """Differentiable view of a stage's blocks (LLaMA-family and GPT-2)."""
 
     def __init__(self, cfg, weights, device, dtype=None):
+        if cfg.hybrid:
+            raise ValueError("training RPCs cover the uniform decoder families, not hybrid decoders")
         self.cfg = cfg
         self.w = weights
         self.device = torch.device(device)

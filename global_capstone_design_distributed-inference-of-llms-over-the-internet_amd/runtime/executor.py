@@ -34,8 +34,10 @@ from .. import native, ops
 from ..ops import moe
 from ..models.config import ModelConfig
 from ..models.weights import StageWeights
-from .kv_cache import PagedKVCache
+from .hybrid import HybridStage
+from .kv_cache import PagedKVCache, SharedKVCache
 from .session import SessionManager, SessionState
+from .state_cache import RecurrentState
 
 logger = logging.getLogger(__name__)
 
@@ -66,6 +68,8 @@ class Plan:
     superblocks: Optional[torch.Tensor] = None  # [2, NSB] runs of <= 4 blocks (grouped prefill kernel)
     fablocks: Optional[torch.Tensor] = None  # [2, NBF] FA2 prefill workgroup blocks (csrc/attention_fa.hip)
     fa_waves: int = 4                   # waves per FA2 workgroup (ops.fa_plan)
+    hybrid: Optional[dict] = None       # hybrid decoders: the step's plan (HybridStage.plan)
+    logit_rows: Optional[torch.Tensor] = None  # flat rows whose logits are asked for (None: each last row)
     _dev: Optional[Tuple[torch.Tensor, torch.Tensor]] = None
     _upload: Optional[object] = None    # callable making the device copies
 
@@ -100,6 +104,8 @@ class Plan:
 
     @property
     def last_rows(self):
+        if self.logit_rows is not None:
+            return self.logit_rows
         return self.meta_i32[2 * self.T:]
 
 
@@ -133,8 +139,10 @@ class StageExecutor:
                  page_size: int = 64, max_sessions: int = 256, max_seq_len: Optional[int] = None,
                  kv_cache_bytes: Optional[int] = None, kv_fraction: float = 0.9, use_graphs: Optional[bool] = None,
                  graph_max_batch: int = 256, max_tokens_per_step: int = 8192, offload: bool = False,
-                 keep_layers_on_gpu: int = 0, tp=None, warmup: Optional[bool] = None):
-        """``tp``: a ``parallel.tensor_parallel.TPGroup`` when ``weights`` is a tensor-parallel
+                 keep_layers_on_gpu: int = 0, tp=None, warmup: Optional[bool] = None,
+                 num_pages: Optional[int] = None):
+        """``num_pages``: cache pages of a hybrid decoder's stage (default: from ``kv_cache_bytes``).
+        ``tp``: a ``parallel.tensor_parallel.TPGroup`` when ``weights`` is a tensor-parallel
         shard (``cfg`` is then the shard config); partial sums are all-reduced after the
         o and down projections."""
         cfg.validate()
@@ -143,6 +151,8 @@ class StageExecutor:
             # also reads the router and per-expert row-major weights.  Mixtral-8x7B (93 GB bf16)
             # fits one MI355X resident, so offload is rejected rather than half-supported.
             raise ValueError("CPU offload is not supported for MoE (Mixtral) models: serve them resident")
+        if cfg.hybrid and (offload or (tp is not None and tp.size > 1)):
+            raise ValueError("hybrid decoders are served resident on one GPU per stage (no offload, no tensor split)")
         self._tp = tp if (tp is not None and getattr(tp, "active", tp.size > 1)) else None
         self.cfg = cfg
         self.w = weights
@@ -161,16 +171,20 @@ class StageExecutor:
             logger.info(f"max_seq_len capped at sliding_window={cfg.sliding_window}")
             self.max_seq_len = int(cfg.sliding_window)
         self.max_tokens = max_tokens_per_step
-        if cfg.model_type != "gpt2":
+        if cfg.model_type != "gpt2" and not cfg.hybrid:
             self.cos, self.sin = ops.rope_cos_sin(self.D, self.max_seq_len, cfg.rope_theta, self.device,
                                                   cfg.rope_scaling)
         if kv_cache_bytes is None:
             kv_cache_bytes = PagedKVCache.auto_budget_bytes(self.device, fraction=kv_fraction)
-        num_pages = PagedKVCache.pages_for_bytes(kv_cache_bytes, self.n_layers, self.nkv, self.D, page_size)
         max_useful = max_sessions * math.ceil(self.max_seq_len / page_size)
-        num_pages = max(1, min(num_pages, max_useful))
-        self.cache = PagedKVCache(self.n_layers, num_pages, self.nkv, self.D, page_size, dtype, self.device)
-        self.sessions = SessionManager(self.cache, max_sessions, self.max_seq_len)
+        self.state = None
+        if cfg.hybrid:
+            num_pages = self._init_hybrid_memory(kv_cache_bytes, page_size, max_sessions, max_useful, num_pages)
+        else:
+            num_pages = PagedKVCache.pages_for_bytes(kv_cache_bytes, self.n_layers, self.nkv, self.D, page_size)
+            num_pages = max(1, min(num_pages, max_useful))
+            self.cache = PagedKVCache(self.n_layers, num_pages, self.nkv, self.D, page_size, dtype, self.device)
+        self.sessions = SessionManager(self.cache, max_sessions, self.max_seq_len, state=self.state)
         self.use_graphs = (self.device.type == "cuda") if use_graphs is None else bool(use_graphs)
         self.use_graphs = self.use_graphs and self.device.type == "cuda" and cfg.model_type != "gpt2" and \
             os.environ.get("MPAMD_GRAPHS", "1") != "0"
@@ -201,7 +215,7 @@ class StageExecutor:
         self._hook_owner = None
         self.last_graphed = self.last_hooked = False
         # MFMA flash attention for prefill steps (csrc/attention_mfma.hip)
-        self._attn_mfma_prefill = cfg.model_type != "gpt2" and cfg.head_dim in (64, 128)
+        self._attn_mfma_prefill = cfg.model_type != "gpt2" and not cfg.hybrid and cfg.head_dim in (64, 128)
         # GQA decode: the whole group of a kv head in the MFMA rows (2x the VALU kernel at nrep 8)
         # MHA decode stays on the flash-decoding kernel: forcing it onto the MFMA kernel (15 of 16
         # MFMA rows idle) measured 11005 vs 13617 tok/s at 64 sessions and 13847 vs 16248 at 128
@@ -251,6 +265,7 @@ class StageExecutor:
         # layers' GEMMs - dense bf16 or W8A16 Llama stages without TP (MoE / W8A8 / TP keep the
         # norm kernels)
         self._fused = (self.device.type == "cuda" and cfg.model_type != "gpt2" and not cfg.is_moe and
+                       not cfg.hybrid and
                        self._tp is None and (not weights.fp8 or self._w8) and ops.gemm_policy() != "hipblaslt" and
                        os.environ.get("MPAMD_FUSED_NORM", "1") != "0" and
                        all(d % 128 == 0 for d in (cfg.hidden_size, cfg.q_dim, cfg.intermediate_size)))
@@ -261,6 +276,7 @@ class StageExecutor:
         # unit RMSNorm weight for > 64-row decode steps over norm-folded packed weights (made
         # here, not inside a hipGraph capture)
         self._ones = torch.ones(cfg.hidden_size, dtype=self.dtype, device=self.device) if self._fused else None
+        self._hybrid = HybridStage(self) if cfg.hybrid else None
         if self.device.type == "cuda":
             ops.require_native()
             if cfg.model_type != "gpt2" and ops.gemm_policy() != "hipblaslt":
@@ -271,7 +287,9 @@ class StageExecutor:
                 ops.gemm_workspace(self.device)  # allocated before any hipGraph capture
                 ops.attention_counters(self.device)
                 ops.load_kernel_table()  # the committed per-shape kernel choices (ops.KERNEL_TABLE)
-                if ops.autotune_mode() != "off":
+                if cfg.hybrid:
+                    self._hybrid.autotune()
+                elif ops.autotune_mode() != "off":
                     H, F = cfg.hidden_size, cfg.intermediate_size
                     shapes = [] if (weights.fp8 or not weights.layers) else \
                         [(cfg.q_dim + 2 * cfg.kv_dim, H, 0), (H, cfg.q_dim, 0), (2 * F, H, 1), (H, F, 0)]
@@ -303,6 +321,28 @@ class StageExecutor:
                     f"kv_pages={num_pages} x {page_size} tokens ({self.cache.nbytes / 2**30:.2f} GiB) "
                     f"graphs={self.use_graphs}")
 
+    def _init_hybrid_memory(self, budget: int, page_size: int, max_sessions: int, max_useful: int,
+                            num_pages: Optional[int] = None) -> int:
+        """Recurrent states (one slot per session) come out of the cache budget first, pages get the rest."""
+        specs = [lay.spec for lay in self.w.layers]
+        rec = [(sp.heads, sp.dim, sp.vdim) for sp in specs if sp.recurrent]
+        att = [(sp.kv_heads, sp.dim) for sp in specs if not sp.recurrent]
+        if rec:
+            self.state = RecurrentState(rec, max_sessions, self.device)
+            budget -= self.state.nbytes
+        per_page = SharedKVCache.page_bytes(att, page_size, torch.empty((), dtype=self.dtype).element_size())
+        if num_pages is None:
+            num_pages = min(max_useful, int(budget // per_page)) if per_page else max_useful
+        if num_pages < 1:
+            raise ValueError("the cache budget does not hold the recurrent states and one page")
+        self.cache = SharedKVCache(att, num_pages, page_size, self.dtype, self.device)
+        return num_pages
+
+    @property
+    def hidden_dtype(self) -> torch.dtype:
+        """Element type of the hidden states a stage takes in and hands on (hybrid decoders: the fp32 stream)."""
+        return torch.float32 if self.cfg.hybrid else self.dtype
+
     # ================================================================== planning
     def plan(self, seqs: Sequence[Tuple[str, int]], *, reset: Sequence[bool] = (), max_length: Optional[int] = None,
              starts: Optional[Sequence[int]] = None) -> Plan:
@@ -320,8 +360,8 @@ class StageExecutor:
             s = self.sessions.open(sid, max_length)
             if reset and reset[i]:
                 self.sessions.reset(sid)
-            if starts is not None and starts[i] is not None and starts[i] < s.length:
-                s.length = int(starts[i])
+            if starts is not None and starts[i] is not None:
+                self.sessions.rewind(s, int(starts[i]))
             self.sessions.reserve(s, s.length + int(n))
             sess.append(s)
             ntoks[i] = n
@@ -350,6 +390,7 @@ class StageExecutor:
                 d32 = h32[: 2 * T + S].clone()
             return d64, d32
 
+        hp = self._hybrid.plan(ntoks, st, [s.row for s in sess]) if self._hybrid is not None and not is_decode else None
         qb = sb = fb = None
         fa_waves = 4
         if self.device.type == "cuda" and not is_decode and self._attn_fa:
@@ -360,7 +401,7 @@ class StageExecutor:
             if self._attn_grouped:
                 sb = torch.from_numpy(ops.query_superblocks(ntoks, self.nh // self.nkv)).to(self.device,
                                                                                               non_blocking=True)
-        return Plan(sess, ntoks, st, T, max_ctx, is_decode, n64, n32, qb, sb, fb, fa_waves, _upload=upload)
+        return Plan(sess, ntoks, st, T, max_ctx, is_decode, n64, n32, qb, sb, fb, fa_waves, hp, _upload=upload)
 
     def commit(self, plan: Plan) -> None:
         for s, n in zip(plan.sessions, plan.ntoks):
@@ -375,10 +416,15 @@ class StageExecutor:
         Steps larger than ``max_tokens_per_step`` run as consecutive chunks (chunked prefill,
         upstream Petals TransformerBackend.inference_step): a long prompt is split at token
         boundaries, later pieces attend to the KV the earlier pieces wrote.
+        ``logit_rows`` (last stage): flat token rows of the step whose logits are returned instead of
+        every sequence's last one (the step must fit ``max_tokens_per_step``).
         """
         T = sum(int(n) for _, n in seqs)
         prompts = plan_kw.pop("prompts", None)
         hook_owner = plan_kw.pop("hook_owner", None)
+        logit_rows = plan_kw.pop("logit_rows", None)
+        if logit_rows is not None and not (self.is_last and T <= self.max_tokens):
+            raise ValueError("logit_rows needs a last stage and a step within max_tokens_per_step")
         if prompts is not None and not any(p is not None for p in prompts):
             prompts = None
         if T > self.max_tokens:
@@ -386,6 +432,8 @@ class StageExecutor:
                 raise ValueError("deep prompts need the step to fit max_tokens_per_step")
             return self._forward_chunked(seqs, x, **plan_kw)
         plan = self.plan(seqs, **plan_kw)
+        if logit_rows is not None:
+            plan.logit_rows = torch.tensor(list(logit_rows), dtype=torch.int32, device=self.device)
         out = self.run(plan, x, prompt=self._prompt_rows(seqs, prompts) if prompts is not None else None,
                        hook_owner=hook_owner)
         self.commit(plan)
@@ -456,10 +504,11 @@ class StageExecutor:
     def run(self, plan: Plan, x: torch.Tensor, prompt=None, hook_owner=None) -> torch.Tensor:
         if plan.T == 0:
             H = self.cfg.hidden_size
-            return torch.empty(0, self.cfg.vocab_size if self.is_last else H, dtype=self.dtype, device=self.device)
+            return torch.empty(0, self.cfg.vocab_size if self.is_last else H,
+                               dtype=self.dtype if self.is_last else self.hidden_dtype, device=self.device)
         x = x.to(self.device)
-        if not self.is_first and x.dtype != self.dtype:
-            x = x.to(self.dtype)
+        if not self.is_first and x.dtype != self.hidden_dtype:
+            x = x.to(self.hidden_dtype)
         ev = None
         if self.timing and self.device.type == "cuda":
             ev = (torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True))
@@ -469,6 +518,11 @@ class StageExecutor:
             hooked = self.graph_hook is not None and hook_owner is not None and hook_owner is self._hook_owner
             out = self._run_graph(plan, x, hooked, owner=hook_owner)
             self.last_graphed, self.last_hooked = True, hooked
+            if plan.logit_rows is not None:  # (the captured step computes every row's logits)
+                out = out.index_select(0, plan.logit_rows)
+        elif self._hybrid is not None:
+            out = self._hybrid.forward(x, plan.positions, plan.slots, plan.q_seq, plan.q_ctx, plan.last_rows, plan.T,
+                                       plan=plan.hybrid, span=self._hybrid.span(plan.max_ctx), prompt=prompt)
         elif self.cfg.model_type == "gpt2":
             out = self._forward_gpt2(plan, x, prompt=prompt)
         else:
@@ -772,7 +826,7 @@ class StageExecutor:
                 if self.is_first:
                     x = torch.randint(0, self.cfg.vocab_size, (n,), device=self.device)
                 else:
-                    x = (0.1 * torch.randn(n, self.cfg.hidden_size, device=self.device)).to(self.dtype)
+                    x = (0.1 * torch.randn(n, self.cfg.hidden_size, device=self.device)).to(self.hidden_dtype)
                 try:
                     self.forward([(sid, n)], x, reset=[True])
                 except Exception as e:  # noqa: BLE001 - e.g. no KV room for n tokens: warm what fits
@@ -810,7 +864,7 @@ class StageExecutor:
                 if self.is_first:
                     x = torch.randint(0, self.cfg.vocab_size, (T,), device=self.device, generator=gen)
                 else:
-                    x = (0.1 * torch.randn(T, H, device=self.device, generator=gen)).to(self.dtype)
+                    x = (0.1 * torch.randn(T, H, device=self.device, generator=gen)).to(self.hidden_dtype)
                 out = self.forward([(s, prompt_len) for s in sids], x, reset=[True] * batch)
                 if self.is_last:
                     self._warm_sampler(out)
@@ -823,7 +877,7 @@ class StageExecutor:
                     if self.is_first:
                         x = torch.randint(0, self.cfg.vocab_size, (batch,), device=self.device, generator=gen)
                     else:
-                        x = (0.1 * torch.randn(batch, H, device=self.device, generator=gen)).to(self.dtype)
+                        x = (0.1 * torch.randn(batch, H, device=self.device, generator=gen)).to(self.hidden_dtype)
                     out = self.forward([(s, 1) for s in sids], x)
                     if self.is_last:
                         self._warm_sampler(out)
@@ -869,7 +923,7 @@ class StageExecutor:
             if self.is_first:
                 x = torch.randint(0, cfg.vocab_size, (B,), device=self.device, generator=gen)
             else:
-                x = (0.1 * torch.randn(B, H, device=self.device, generator=gen)).to(self.dtype)
+                x = (0.1 * torch.randn(B, H, device=self.device, generator=gen)).to(self.hidden_dtype)
             self.forward([(s, 1) for s in sids], x)
 
         t = {True: 0.0, False: 0.0}
@@ -1110,6 +1164,8 @@ class StageExecutor:
         (``graph_input``)."""
         B = self._bucket(T)
         ctxb = min(self._ctx_bucket(max_ctx), self._ctx_bucket(self.max_seq_len))
+        if self._hybrid is not None:  # (keys a query can see, 0) stands for the attention partition
+            return (B, self._hybrid.span(ctxb), 0, False, bool(hooked), int(tag), int(slot))
         part = ops.attention_partition(B, self.nkv, ctxb, min_part=self._attn_min_part)
         return (B, part[0], part[1], self._qkv_fold(B), bool(hooked), int(tag), int(slot))
 
@@ -1234,6 +1290,13 @@ class StageExecutor:
         self._graphs.clear()
 
 
+def _decode_step(ex: StageExecutor, x, positions, slots, q_seq, q_ctx, last_rows, T, part):
+    """The step a decode graph records: every row one token, ``part`` the attention partition of the graph key."""
+    if ex._hybrid is not None:
+        return ex._hybrid.forward(x, positions, slots, q_seq, q_ctx, last_rows, T, span=part[0])
+    return ex._forward_llama(x, positions, slots, q_seq, q_ctx, last_rows, T, 0, part, decode=True)
+
+
 class _DecodeGraph:
     """A captured decode step for a fixed (batch bucket, attention partition).
 
@@ -1244,11 +1307,11 @@ class _DecodeGraph:
 
     def __init__(self, ex: StageExecutor, B: int, part: Tuple[int, int], pool, hook=None):
         self.ex, self.B, self.part = ex, B, part
-        dev, H, dt = ex.device, ex.cfg.hidden_size, ex.dtype
+        dev, H = ex.device, ex.cfg.hidden_size
         if ex.is_first:
             self.x = torch.zeros(B, dtype=torch.long, device=dev)
         else:
-            self.x = torch.zeros(B, H, dtype=dt, device=dev)
+            self.x = torch.zeros(B, H, dtype=ex.hidden_dtype, device=dev)
         nbytes = 16 * B + 12 * B  # int64 [2, B] + int32 [3 B]
         self.blob = torch.zeros(nbytes, dtype=torch.uint8, device=dev)
         self.meta64 = self.blob[: 16 * B].view(torch.int64).view(2, B)
@@ -1270,18 +1333,18 @@ class _DecodeGraph:
         self.bufs: dict = {}
         self.done_ev = None  # end of the last replay on the compute stream (graph_input)
         args = (self.x, self.meta64[0], self.meta64[1], self.meta32[:B], self.meta32[B:2 * B], self.meta32[2 * B:], B,
-                0, part)
+                part)
         s = torch.cuda.Stream()
         s.wait_stream(torch.cuda.current_stream())
         with torch.cuda.stream(s):
             for _ in range(2):  # warm up (allocator, hipBLASLt heuristics) outside capture
-                ex._forward_llama(*args, decode=True)
+                _decode_step(ex, *args)
         torch.cuda.current_stream().wait_stream(s)
         self.graph = torch.cuda.CUDAGraph()
         # thread-local capture: another thread's stream work (a channel receive posted outside the
         # executor lock) neither breaks this capture nor fails because of it
         with torch.cuda.graph(self.graph, pool=pool, capture_error_mode="thread_local"):
-            self.out = ex._forward_llama(*args, decode=True)
+            self.out = _decode_step(ex, *args)
             if hook is not None:  # recorded only: the warm-up runs above never call it
                 hook(self.out)
         self.mark_replayed()  # the warm-up runs read ``x``: a receive into it waits for them

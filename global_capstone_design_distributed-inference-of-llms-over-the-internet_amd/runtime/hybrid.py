@@ -1,0 +1,170 @@
+"""Forward step of the hybrid decoders inside a StageExecutor (``ModelConfig.layers``).
+
+The residual stream is fp32 and lives in one buffer; a sublayer reads its activation copy ``xb`` and its
+RMS-normed, layer-scaled output is added to it:
+
+    z = xb W_in^T          one fused input projection per mixer
+    y = mixer(z) W_o^T     hgrn2: recurrence + head norm; attention: norms + cache write, attention + gate
+    res += rms(y) n1 ; xb = res
+    y = relu2(xb W_up^T) W_down^T
+    res += rms(y) n2 ; xb = res
+
+Activations feeding a decode-sized GEMM stay in the packed MFMA-fragment layout where the shape has a native
+GEMM (``ops.native_gemm_ok``); other shapes, prompts and fp32 run the library GEMM on row-major activations.
+Keys of attention layers live in the executor's paged cache, recurrent states in its ``RecurrentState``.
+"""
+from __future__ import annotations
+
+import math
+from typing import Optional
+
+import torch
+
+from .. import ops
+from ..ops import hybrid as hops
+
+
+class HybridStage:
+    """Layer loop of one stage; ``ex`` owns the weights, the cache, the states and the plans."""
+
+    def __init__(self, ex):
+        self.ex = ex
+        cfg = ex.cfg
+        self.W, self.eps = cfg.hidden_size, cfg.rms_norm_eps
+        self.inv = hops.position_frequencies(self.W, ex.device)
+        # per-layer cache / state index: attention layers count in the paged cache, recurrent ones in the states
+        self.index, na, nr = [], 0, 0
+        for lay in ex.w.layers:
+            if lay.spec.recurrent:
+                self.index.append(nr)
+                nr += 1
+            else:
+                self.index.append(na)
+                na += 1
+        self.max_chunk = max([lay.spec.chunk for lay in ex.w.layers if not lay.spec.recurrent], default=1)
+
+    def autotune(self) -> None:
+        """Decode-GEMM kernel choices for this stage's shapes (none while tuning is off)."""
+        if ops.autotune_mode() == "off":
+            return
+        shapes = {(w.shape[0], w.shape[1], 0) for lay in self.ex.w.layers
+                  for w, wp in ((getattr(lay, n), getattr(lay, n + "_p")) for n in lay.GEMMS) if wp is not None}
+        if self.ex.w.lm_head_p is not None:
+            shapes.add((self.ex.w.lm_head.shape[0], self.W, 0))
+        # (small products are launch-bound whatever kernel runs them)
+        ops.autotune_gemm([s for s in sorted(shapes) if s[0] * s[1] >= 1 << 22], self.ex.device)
+
+    # ------------------------------------------------------------------ GEMMs
+    def _packed(self, T: int, w, wp) -> bool:
+        """Does the GEMM over ``w`` take a packed T-row activation?"""
+        return (wp is not None and self.ex.device.type == "cuda" and ops.gemm_policy() != "hipblaslt" and
+                ops.native_gemm_ok(T, w.shape[0], w.shape[1], 0))
+
+    def _act(self, e, name: str, T: int, K: int, packed: bool):
+        if packed:
+            return e(f"{name}_p{K}", (ops.packed_numel(T, K),))
+        return e(f"{name}_{K}", (T, K))
+
+    def _mm(self, x, w, wp, T: int, packed: bool, out):
+        if packed:
+            return ops.linear(x, None, wp=wp, a_rows=T, out=out)
+        return ops.linear(x, w, out=out)
+
+    def _add(self, y_in, w, wp, packed: bool, T: int, res, n, xb, xb_packed: bool, e):
+        """res += rms(y_in w^T) n, xb = res.  A packed projection with a split-K form hands its fp32 slabs
+        straight to the norm kernel (no reduce launch, no rounding of y)."""
+        if packed and ops.rwk_split(T, w.shape[0], w.shape[1]) > 0:
+            y = ops.linear_partials(y_in, T, wp=wp, out=e("y", (T, self.W)))
+        else:
+            y = self._mm(y_in, w, wp, T, packed, e("y", (T, self.W)))
+        hops.residual_norm(y, res, n, self.eps, xb, packed=xb_packed)
+
+    # ------------------------------------------------------------------ the step
+    def forward(self, x, positions, slots, q_seq, q_ctx, last_rows, T, bufs: Optional[dict] = None, plan=None,
+                span: int = 0, prompt=None):
+        """``plan``: the ragged step's ``plan`` (None: a decode step, every row one token); ``span``: most keys a
+        query sees.  Returns the fp32
+        residual rows [T, W] (non-last stage) or the logits of ``last_rows``."""
+        ex, W, eps = self.ex, self.W, self.eps
+        dev, dt = ex.device, ex.dtype
+        layers = ex.w.layers
+        cache: dict = {} if bufs is None else bufs
+
+        def e(name, shape, dtype=dt):
+            t = cache.get(name)
+            if t is None or tuple(t.shape) != tuple(shape) or t.dtype != dtype:
+                t = cache[name] = torch.empty(shape, dtype=dtype, device=dev)
+            return t
+
+        def entry(i):  # (packed?, buffer) of the activation that layer i's input projection reads
+            pk = i < len(layers) and self._packed(T, layers[i].w_in, layers[i].w_in_p)
+            return pk, self._act(e, "xb", T, W, pk)
+
+        res = torch.empty(T, W, dtype=torch.float32, device=dev)
+        pk, xb = entry(0)
+        if ex.is_first:
+            hops.embed_pos(x, ex.w.embed, positions, self.inv, res, xb, packed=pk)
+        else:
+            res.copy_(x)
+            self._copy_in(res, xb, pk, T)
+        table = ex.sessions.table_dev
+        for i, lay in enumerate(layers):
+            sp = lay.spec
+            if prompt is not None:  # deep prompt: the block input += prompt[i]
+                res.index_add_(0, prompt[0], prompt[1][i].float())
+                self._copy_in(res, xb, pk, T)
+            z = self._mm(xb, lay.w_in, lay.w_in_p, T, pk, e(f"z{sp.in_rows}", (T, sp.in_rows)))
+            pko = self._packed(T, lay.w_o, lay.w_o_p)
+            o = self._act(e, "o", T, sp.out_cols, pko)
+            if sp.recurrent:
+                hops.hgrn2(z, lay.f_bias, lay.f_lower, lay.o_norm, ex.state.layer(self.index[i]), q_seq, q_ctx, o, eps,
+                           plan=plan, packed=pko)
+            else:
+                kv, rk = ex.cache.layer(self.index[i])
+                qn = e(f"qn{sp.out_cols}", (T, sp.out_cols))
+                hops.talk_prep(z, lay.w_qk, qn, kv, rk, slots, eps)
+                hops.talk_attention(z, qn, lay.talk, kv, rk, table, q_seq, q_ctx, o, sp.chunk, sp.scale, packed=pko)
+            if sp.ff:
+                pku = self._packed(T, lay.w_up, lay.w_up_p)
+                xu = self._act(e, "xb", T, W, pku)
+                self._add(o, lay.w_o, lay.w_o_p, pko, T, res, lay.n1, xu, pku, e)
+                u = self._mm(xu, lay.w_up, lay.w_up_p, T, pku, e(f"u{sp.ff}", (T, sp.ff)))
+                pkd = self._packed(T, lay.w_down, lay.w_down_p)
+                a = hops.relu2(u, self._act(e, "act", T, sp.ff, pkd), packed=pkd)
+                pk, xb = entry(i + 1)
+                self._add(a, lay.w_down, lay.w_down_p, pkd, T, res, lay.n2, xb, pk, e)
+            else:
+                pk, xb = entry(i + 1)
+                self._add(o, lay.w_o, lay.w_o_p, pko, T, res, lay.n1, xb, pk, e)
+        if not ex.is_last:
+            return res
+        S, V = last_rows.numel(), ex.cfg.vocab_size
+        head = ex.w.lm_head
+        if S == 0:
+            return torch.empty(0, V, dtype=dt, device=dev)
+        pkh = self._packed(S, head, ex.w.lm_head_p)
+        fn = hops.rows_norm(res, last_rows, ex.w.final_norm, eps, self._act(e, "fn", S, W, pkh), packed=pkh)
+        logits = self._mm(fn, head, ex.w.lm_head_p, S, pkh, torch.empty(S, head.shape[0], dtype=dt, device=dev))
+        return logits[:, :V]
+
+    def _copy_in(self, res, xb, packed: bool, T: int) -> None:
+        y = res.to(self.ex.dtype)
+        if packed:
+            ops.pack_act(y, out=xb)
+        else:
+            xb.copy_(y)
+
+    # ------------------------------------------------------------------ plans
+    def plan(self, ntoks, starts, rows) -> dict:
+        """Device description of a ragged step (not one token per session)."""
+        import numpy as np
+
+        n = np.asarray(ntoks, dtype=np.int64)
+        off = np.concatenate([[0], np.cumsum(n)[:-1]])
+        keep = n > 0
+        seg = torch.from_numpy(np.stack([off[keep], n[keep]]).astype(np.int32))
+        return {"seg": seg.to(self.ex.device, non_blocking=True)}
+
+    def span(self, max_ctx: int) -> int:
+        """Most keys a decode query of context <= max_ctx can see."""
+        return max(1, min(int(max_ctx), self.max_chunk))

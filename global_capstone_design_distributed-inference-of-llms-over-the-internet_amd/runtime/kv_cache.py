@@ -105,5 +105,46 @@ class PagedKVCache:
         return max(budget, 0)
 
 
+class SharedKVCache:
+    """Paged cache of attention layers whose values are their projected keys: one raw row per token and kv head,
+    ``rows[l] : [num_pages, nkv_l, page_size, head_dim_l]``, plus ``rk[l] : [num_pages, page_size]`` fp32, the
+    reciprocal root mean square of the token's whole key row.  Layers may differ in kv heads and head size.
+    Same page ids, allocator and block tables as ``PagedKVCache``."""
+
+    def __init__(self, shapes, num_pages: int, page_size: int = 64, dtype=torch.bfloat16, device="cpu"):
+        """``shapes``: (kv heads, head size) of every attention layer."""
+        assert page_size & (page_size - 1) == 0, "page_size must be a power of two"
+        self.shapes = [tuple(s) for s in shapes]
+        self.num_layers = len(self.shapes)
+        self.num_pages = num_pages
+        self.page_size = page_size
+        self.dtype = dtype
+        self.device = torch.device(device)
+        self.rows = [torch.zeros(num_pages, n, page_size, d, dtype=dtype, device=self.device) for n, d in self.shapes]
+        self.rk = [torch.zeros(num_pages, page_size, dtype=torch.float32, device=self.device) for _ in self.shapes]
+        self.allocator = PageAllocator(num_pages)
+
+    def layer(self, i: int):
+        return self.rows[i], self.rk[i]
+
+    def copy_pages(self, src: List[int], dst: List[int]) -> None:
+        si = torch.tensor(src, dtype=torch.long, device=self.device)
+        di = torch.tensor(dst, dtype=torch.long, device=self.device)
+        for t in self.rows + self.rk:
+            t.index_copy_(0, di, t.index_select(0, si))
+
+    @staticmethod
+    def page_bytes(shapes, page_size: int, elt_bytes: int) -> int:
+        return sum(page_size * (n * d * elt_bytes + 4) for n, d in shapes)
+
+    @property
+    def bytes_per_page(self) -> int:
+        return self.page_bytes(self.shapes, self.page_size, torch.tensor([], dtype=self.dtype).element_size())
+
+    @property
+    def nbytes(self) -> int:
+        return self.bytes_per_page * self.num_pages
+
+
 def pages_needed(num_tokens: int, page_size: int) -> int:
     return int(math.ceil(num_tokens / page_size)) if num_tokens > 0 else 0

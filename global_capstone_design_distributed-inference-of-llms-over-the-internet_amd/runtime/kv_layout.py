@@ -35,6 +35,11 @@ def bloom_to_llama(k: torch.Tensor, v: torch.Tensor, batch_size: int) -> KV:
     return k.permute(0, 2, 1).reshape(batch_size, h, t, d), v.reshape(batch_size, h, t, d)
 
 
+def _dense_only(cache) -> None:
+    if not hasattr(cache, "k"):
+        raise ValueError("dense (k, v) export / import needs separate key and value caches")
+
+
 def _layer_ids(cache, layers: Optional[Sequence[int]]) -> List[int]:
     return list(range(cache.num_layers)) if layers is None else list(layers)
 
@@ -42,6 +47,7 @@ def _layer_ids(cache, layers: Optional[Sequence[int]]) -> List[int]:
 def export_session_kv(cache, session, layers: Optional[Sequence[int]] = None,
                       length: Optional[int] = None) -> List[KV]:
     """Dense per-layer ``(k, v)`` of one session, LLaMA layout ``[1, kvh, T, hd]``."""
+    _dense_only(cache)
     t = session.length if length is None else int(length)
     if t > session.length:
         raise ValueError(f"session holds {session.length} tokens, asked for {t}")
@@ -64,6 +70,7 @@ def import_session_kv(sessions, sid: str, kv: Sequence[KV], max_length: Optional
     ``kv`` has one ``(k, v)`` per cache layer, each ``[1, kvh, T, hd]``. Returns the session.
     """
     cache = sessions.cache
+    _dense_only(cache)
     if len(kv) != cache.num_layers:
         raise ValueError(f"expected {cache.num_layers} layers, got {len(kv)}")
     t = kv[0][0].shape[2]

@@ -34,8 +34,10 @@ class SessionState:
 
 class SessionManager:
     def __init__(self, cache: PagedKVCache, max_sessions: int = 256, max_seq_len: int = 4096,
-                 ttl_seconds: float = 600.0):
+                 ttl_seconds: float = 600.0, state=None):
+        """``state``: the stage's ``RecurrentState`` (None when it has no recurrent layer)."""
         self.cache = cache
+        self.state = state
         self.page_size = cache.page_size
         self.max_sessions = max_sessions
         self.max_seq_len = max_seq_len
@@ -128,6 +130,8 @@ class SessionManager:
                 self.table[d.row, : len(new)] = new
                 d.pages = list(new)
                 self._dirty = True
+            if self.state is not None:
+                self.state.copy_row(s.row, d.row)
             d.length = s.length
             d.generated = list(s.generated)
             d.last_used = time.monotonic()
@@ -153,6 +157,16 @@ class SessionManager:
             for sid in dead:
                 self.close(sid)
             return len(dead)
+
+    def rewind(self, s: SessionState, start: int) -> None:
+        """Continue ``s`` from position ``start`` (a retried or replayed step).  Cached keys past it are
+        overwritten; recurrent state has no past, so such a session can only go back to its first token."""
+        if start >= s.length:
+            return
+        if self.state is not None and start > 0:
+            raise ValueError(f"session {s.sid[:8]}: recurrent state at {s.length} tokens cannot be rewound to {start}; "
+                             f"replay the session from its first token")
+        s.length = int(start)
 
     # ------------------------------------------------------------------ pages
     def reserve(self, s: SessionState, total_len: int) -> None:

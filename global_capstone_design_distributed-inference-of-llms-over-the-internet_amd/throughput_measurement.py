@@ -55,7 +55,7 @@ def _measure_compute(executor, sids, batch, n_warmup, n_steps, rounds, H, dev) -
         if executor.is_first:
             x = torch.randint(0, executor.cfg.vocab_size, (batch,), device=dev)
         else:
-            x = torch.randn(batch, H, device=dev).to(executor.dtype)
+            x = torch.randn(batch, H, device=dev).to(executor.hidden_dtype)
         seqs = [(s, 1) for s in sids]
         for _ in range(n_warmup):
             executor.forward(seqs, x)
@@ -91,7 +91,7 @@ def measure_forward_throughput(executor, n_tokens: int = 1024, n_steps: int = 3)
     if executor.is_first:
         x = torch.randint(0, executor.cfg.vocab_size, (n_tokens,), device=dev)
     else:
-        x = torch.randn(n_tokens, H, device=dev).to(executor.dtype)
+        x = torch.randn(n_tokens, H, device=dev).to(executor.hidden_dtype)
     sid = f"__probe_fwd_{uuid.uuid4().hex[:8]}"
     lock = getattr(executor, "exec_lock", None) or contextlib.nullcontext()
     with lock:
