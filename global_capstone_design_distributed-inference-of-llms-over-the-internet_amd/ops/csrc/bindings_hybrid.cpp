@@ -21,6 +21,15 @@ int mp_talk_attention(const void* z, int64_t zs, const void* qn, const float* ta
                       const int32_t* bt, int bt_stride, const int32_t* q_seq, const int32_t* q_ctx, void* out, int n,
                       int H, int G, int D, int page_log2, int chunk, float scale, int packed_mt, int f32,
                       hipStream_t stream);
+int mp_hgrn2_chunk(const void* z, int64_t zs, const float* bias, const float* lower, const float* norm, float* state,
+                   const int32_t* q_seq, const int32_t* q_ctx, void* out, int H, int D, int V, float eps,
+                   const int32_t* seg, int nseg, const int32_t* multi, int nm, float* ws, float* wdec, int packed_mt,
+                   int f32, hipStream_t stream);
+int mp_talk_block(int H, int G, int D);
+int mp_talk_mfma(const void* z, int64_t zs, const void* qn, const float* talk, const void* cache, const float* rk,
+                 const int32_t* bt, int bt_stride, const int32_t* q_seq, const int32_t* q_ctx, void* out, int n, int H,
+                 int G, int D, int page_log2, int chunk, float scale, const int32_t* blk, int nblk, int PS, int NP,
+                 float* part, int packed_mt, hipStream_t stream);
 }
 
 namespace {
@@ -168,6 +177,36 @@ void hgrn2_scan(const at::Tensor& z, const at::Tensor& bias, const at::Tensor& l
                "hgrn2_scan");
 }
 
+// seg [4, nseg] (first token, tokens, state source, state target), multi [4, nm] (first slot, slots, first token, -):
+// csrc/hgrn2.hip.  ``slots``: workspace slots the segments name.
+void hgrn2_chunk(const at::Tensor& z, const at::Tensor& bias, const at::Tensor& lower, const at::Tensor& norm,
+                 at::Tensor& state, const at::Tensor& q_seq, const at::Tensor& q_ctx, at::Tensor& out, double eps,
+                 const at::Tensor& seg, const c10::optional<at::Tensor>& multi, int64_t slots,
+                 const c10::optional<at::Tensor>& ws, int64_t packed) {
+  const Hgrn2Shape s = check_hgrn2(z, bias, state);
+  const int mt = check_out(out, s.T, s.H * s.V, s.f32, packed, "out");
+  MP_CHECK(seg.dim() == 2 && seg.size(0) == 4, "seg int32 [4, nseg]");
+  const int64_t nseg = seg.size(1);
+  const int32_t* mp = nullptr;
+  int64_t nm = 0;
+  float *wp = nullptr, *wd = nullptr;
+  if (multi.has_value() && multi->numel()) {
+    MP_CHECK(multi->dim() == 2 && multi->size(0) == 4 && ws.has_value(), "multi int32 [4, nm] with a workspace");
+    nm = multi->size(1);
+    mp = i32_vec(*multi, 4 * nm, "multi");
+    MP_CHECK(ws->is_cuda() && ws->scalar_type() == at::kFloat && ws->is_contiguous() &&
+                 ws->numel() >= slots * s.H * s.D * (s.V + 1), "ws: fp32 [slots H D (V + 1)]");
+    wp = ws->data_ptr<float>();
+    wd = wp + slots * s.H * s.D * s.V;
+  }
+  check_launch(mp_hgrn2_chunk(z.data_ptr(), z.stride(0), f32_vec(bias, s.H * s.D, "bias"),
+                              f32_vec(lower, s.H * s.D, "lower"), f32_vec(norm, s.V, "norm"), state.data_ptr<float>(),
+                              i32_vec(q_seq, s.T, "q_seq"), i32_vec(q_ctx, s.T, "q_ctx"), out.data_ptr(), s.H, s.D,
+                              s.V, (float)eps, i32_vec(seg, 4 * nseg, "seg"), nseg, mp, nm, wp, wd, mt, s.f32,
+                              cur_stream()),
+               "hgrn2_chunk");
+}
+
 struct TalkShape {
   int f32, page_log2;
   int64_t T, H, G, D;
@@ -215,6 +254,41 @@ void talk_attention(const at::Tensor& z, const at::Tensor& qn, const at::Tensor&
                "talk_attention");
 }
 
+int64_t talk_block(int64_t H, int64_t G, int64_t D) { return mp_talk_block((int)H, (int)G, (int)D); }
+
+// blk: int32 [2, nblk] query blocks of a prompt step, or none: one-token rows, the context in ``parts`` splits of
+// ``part_size`` keys (``ws`` when parts > 1)
+void talk_mfma(const at::Tensor& z, const at::Tensor& qn, const at::Tensor& talk, const at::Tensor& cache,
+               const at::Tensor& rk, const at::Tensor& bt, const at::Tensor& q_seq, const at::Tensor& q_ctx,
+               at::Tensor& out, int64_t chunk, double scale, const c10::optional<at::Tensor>& blk, int64_t part_size,
+               int64_t parts, const c10::optional<at::Tensor>& ws, int64_t packed) {
+  const TalkShape s = check_talk(z, qn, cache, rk);
+  MP_CHECK(!s.f32, "talk_mfma is bf16");
+  MP_CHECK(chunk >= 1 && chunk < (1ll << 31), "chunk");
+  MP_CHECK(bt.is_cuda() && bt.dim() == 2 && bt.scalar_type() == at::kInt && bt.stride(1) == 1, "block table int32");
+  const int mt = check_out(out, s.T, s.H * s.D, s.f32, packed, "out");
+  const int32_t* bp = nullptr;
+  int64_t nb = 0;
+  if (blk.has_value()) {
+    MP_CHECK(blk->dim() == 2 && blk->size(0) == 2, "blk int32 [2, nblk]");
+    nb = blk->size(1);
+    bp = i32_vec(*blk, 2 * nb, "blk");
+    if (nb == 0) return;
+  }
+  float* wp = nullptr;
+  if (parts > 1) {
+    MP_CHECK(ws.has_value() && ws->is_cuda() && ws->scalar_type() == at::kFloat && ws->is_contiguous() &&
+                 ws->numel() >= parts * s.T * s.H * (s.D + 2), "ws: fp32 [parts T H (D + 2)]");
+    wp = ws->data_ptr<float>();
+  }
+  check_launch(mp_talk_mfma(z.data_ptr(), z.stride(0), qn.data_ptr(), f32_vec(talk, s.H * s.H, "talk"),
+                            cache.data_ptr(), rk.data_ptr<float>(), bt.data_ptr<int32_t>(), bt.stride(0),
+                            i32_vec(q_seq, s.T, "q_seq"), i32_vec(q_ctx, s.T, "q_ctx"), out.data_ptr(), s.T, s.H, s.G,
+                            s.D, s.page_log2, (int)chunk, (float)scale, bp, nb, (int)part_size, (int)parts, wp, mt,
+                            cur_stream()),
+               "talk_mfma");
+}
+
 }  // namespace
 
 TORCH_LIBRARY_FRAGMENT(mpamd, m) {
@@ -230,6 +304,13 @@ TORCH_LIBRARY_FRAGMENT(mpamd, m) {
   m.def(
       "talk_attention(Tensor z, Tensor qn, Tensor talk, Tensor cache, Tensor rk, Tensor bt, Tensor q_seq, "
       "Tensor q_ctx, Tensor(a!) out, int chunk, float scale, int packed) -> ()");
+  m.def(
+      "hgrn2_chunk(Tensor z, Tensor bias, Tensor lower, Tensor norm, Tensor(a!) state, Tensor q_seq, Tensor q_ctx, "
+      "Tensor(b!) out, float eps, Tensor seg, Tensor? multi, int slots, Tensor? ws, int packed) -> ()");
+  m.def("talk_block(int H, int G, int D) -> int", &talk_block);
+  m.def(
+      "talk_mfma(Tensor z, Tensor qn, Tensor talk, Tensor cache, Tensor rk, Tensor bt, Tensor q_seq, Tensor q_ctx, "
+      "Tensor(a!) out, int chunk, float scale, Tensor? blk, int part_size, int parts, Tensor? ws, int packed) -> ()");
 }
 
 TORCH_LIBRARY_IMPL(mpamd, CUDA, m) {
@@ -240,4 +321,6 @@ TORCH_LIBRARY_IMPL(mpamd, CUDA, m) {
   m.impl("hgrn2_scan", &hgrn2_scan);
   m.impl("talk_prep", &talk_prep);
   m.impl("talk_attention", &talk_attention);
+  m.impl("hgrn2_chunk", &hgrn2_chunk);
+  m.impl("talk_mfma", &talk_mfma);
 }

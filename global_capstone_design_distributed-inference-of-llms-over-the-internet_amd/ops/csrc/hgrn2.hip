@@ -13,6 +13,8 @@
 #include "common.h"
 #include "act_io.h"
 
+#include <type_traits>
+
 namespace mp {
 
 __device__ __forceinline__ float sigmoid_f(float x) { return 1.f / (1.f + expf(-x)); }
@@ -99,7 +101,342 @@ static int launch_scan(const Hgrn2Args& a, const int32_t* seg, int nseg, int n, 
   return (int)hipGetLastError();
 }
 
+// ---------------------------------------------------------------------------------------
+// Prompts.  A segment's tokens are taken 16 at a time by one workgroup per (segment, head), the state in
+// registers across the blocks (wave w holds VT 16-column tiles of V for all of D, in the MFMA accumulator
+// layout).  With P(a, b] = prod_{a < t <= b} f_t per channel, a block of 16 is
+//
+//   O  = (q_i P(-1, i]) S  +  tril(A) v        A_ij = sum_d q_i k_j P(j, i]
+//   S <- diag(P(-1, 15]) S + (k_j P(j, 15])^T v
+//
+// every product of gates being a product of numbers <= 1: nothing is divided, no logarithm is taken, and a
+// gate of 0 is as good as any other.  A's strictly lower part splits by the highest bit in which i and j
+// differ: with L = 8, 4, 2, 1 and m the start of the upper half of their common 2L-block,
+// P(j, i] = P(j, m - 1] P(m - 1, i], so ONE table M_L (row t = q_t P(m-1, t] in upper halves,
+// k_t P(t, m-1] in lower ones) gives all pairs of that level as the masked product M_L M_L^T; the four
+// waves take a level each.  All products run on v_mfma_f32_16x16x4_f32.
+//
+// seg [4, nseg]: first token, tokens, source and target of the state (-1: the session's slot, s >= 0: slot s
+// of the workspace).  Long prompts are cut into segments so that all CUs work: a STATE pass leaves every
+// segment's own contribution (and decay) in the next segment's slot, hgrn2_prefix_kernel turns the slots
+// into initial states, and the full pass starts from them.
+__device__ __forceinline__ f32x4 mfma_f32(float a, float b, const f32x4& c) {
+  return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
+}
+
+// sum over the 16 lanes of each row of the wave, in every lane
+__device__ __forceinline__ float row16_sum(float v) {
+  v += dppf<0xB1>(v, 0.f);
+  v += dppf<0x4E>(v, 0.f);
+  v += dppf<0x141>(v, 0.f);
+  v += dppf<0x140>(v, 0.f);
+  return v;
+}
+
+template <typename T, int DT, int VT, bool STATE>
+__global__ __launch_bounds__(256, DT * VT > 32 ? 1 : 2) void hgrn2_chunk_kernel(Hgrn2Args a,
+                                                                                const int32_t* __restrict__ seg,
+                                                                                int nseg, float* __restrict__ ws,
+                                                                                float* __restrict__ wdec) {
+  constexpr int DC = DT * 16, DP = DC + 4;
+  constexpr int NTAB = STATE ? 1 : 6;
+  constexpr int TKE = STATE ? 0 : 5, TQB = 4;
+  constexpr bool SPLIT = !STATE && 2 * DC <= 256;  // two thread groups share the gate tables
+  __shared__ __attribute__((aligned(16))) float tab[NTAB][16][DP];
+  __shared__ __attribute__((aligned(16))) float dec[DC];
+  __shared__ __attribute__((aligned(16))) float ap[STATE ? 1 : 4][16][20];
+  __shared__ float dred[4][16], rss[4][16];
+
+  const int h = blockIdx.x, sg = blockIdx.y, tid = threadIdx.x, lane = tid & 63;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int c16 = lane & 15, g4 = lane >> 4;
+  const int tok0 = seg[sg], ntok = seg[nseg + sg], src = seg[2 * nseg + sg], dst = seg[3 * nseg + sg];
+  if (ntok <= 0 || (STATE && dst < 0)) return;
+  const int D = a.D, V = a.V, HD = a.H * D, row = a.q_seq[tok0];
+  const bool fresh = src < 0 && a.q_ctx[tok0] <= 1;
+  const int64_t blk = (int64_t)D * V;
+
+  f32x4 S[DT][VT];
+  {
+    const float* sp = src < 0 ? a.state + ((int64_t)row * a.H + h) * blk : ws + ((int64_t)src * a.H + h) * blk;
+    const bool zero = STATE || fresh;
+#pragma unroll
+    for (int m = 0; m < DT; ++m)
+#pragma unroll
+      for (int v = 0; v < VT; ++v)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int d = 16 * m + 4 * g4 + r, col = (w * VT + v) * 16 + c16;
+          S[m][v][r] = !zero && d < D && col < V ? sp[(int64_t)d * V + col] : 0.f;
+        }
+  }
+
+  const int grp = tid / DC, ch = tid - grp * DC;  // gate channel of this thread
+  const bool gact = grp < (SPLIT ? 2 : 1), gch = gact && ch < D;
+  const float lo = gch ? a.lower[h * D + ch] : 0.f, bi = gch ? a.bias[h * D + ch] : 0.f;
+  const T* zq = (const T*)a.z + h * D + ch;
+  const T* zf = zq + HD;
+  const T* zv = (const T*)a.z + 2 * HD + (int64_t)h * V;
+  float run = 1.f;  // decay of the whole segment (STATE)
+
+  T rq[16], rf[16];  // raw gate inputs of the next block, in flight across the MFMAs
+  T rv[VT][4];
+  auto fetch = [&](int b) {
+#pragma unroll
+    for (int t = 0; t < 16; ++t) {
+      const int64_t o = (int64_t)(tok0 + min(b + t, ntok - 1)) * a.zs;
+      if (gch) {
+        if constexpr (!STATE) rq[t] = zq[o];
+        rf[t] = zf[o];
+      }
+    }
+#pragma unroll
+    for (int v = 0; v < VT; ++v) {
+      const int col = (w * VT + v) * 16 + c16;
+#pragma unroll
+      for (int s = 0; s < 4; ++s)
+        rv[v][s] = col < V ? zv[(int64_t)(tok0 + min(b + 4 * g4 + s, ntok - 1)) * a.zs + col] : (T)0;
+    }
+  };
+  fetch(0);
+  for (int b = 0; b < ntok; b += 16) {
+    const int nb = min(16, ntok - b);
+    if (gact) {
+      float q[16], f[16];
+#pragma unroll
+      for (int t = 0; t < 16; ++t) {
+        const bool ok = gch && t < nb;  // past the end: f = 1, k = 0, q = 0
+        if constexpr (!STATE) {
+          const float x = to_f(rq[t]);
+          q[t] = ok ? x * sigmoid_f(x) : 0.f;
+        }
+        f[t] = ok ? lo + (1.f - lo) * sigmoid_f(to_f(rf[t]) + bi) : 1.f;
+      }
+      auto level = [&](int ti, auto lc) {
+        constexpr int L = decltype(lc)::value;
+#pragma unroll
+        for (int base = 0; base < 16; base += 2 * L) {
+          float p = 1.f;
+#pragma unroll
+          for (int t = base + L - 1; t >= base; --t) {
+            tab[ti][t][ch] = (1.f - f[t]) * p;
+            p *= f[t];
+          }
+          p = 1.f;
+#pragma unroll
+          for (int t = base + L; t < base + 2 * L; ++t) {
+            p *= f[t];
+            tab[ti][t][ch] = q[t] * p;
+          }
+        }
+      };
+      if constexpr (!STATE) {
+        if (grp == 0) {
+          level(0, std::integral_constant<int, 8>());
+          level(1, std::integral_constant<int, 4>());
+          level(2, std::integral_constant<int, 2>());
+#pragma unroll
+          for (int t = 0; t < 16; ++t) {
+            const float x = wave_sum(q[t] * (1.f - f[t]));
+            if (lane == 0) dred[w][t] = x;
+          }
+        }
+      }
+      if (!SPLIT || grp == 1) {
+        if constexpr (!STATE) {
+          level(3, std::integral_constant<int, 1>());
+          float p = 1.f;
+#pragma unroll
+          for (int t = 0; t < 16; ++t) {
+            p *= f[t];
+            tab[TQB][t][ch] = q[t] * p;
+          }
+        }
+        float p = 1.f;
+#pragma unroll
+        for (int t = 15; t >= 0; --t) {
+          tab[TKE][t][ch] = (1.f - f[t]) * p;
+          p *= f[t];
+        }
+        dec[ch] = p;
+        run *= p;
+      }
+    }
+    float vr[VT][4];
+#pragma unroll
+    for (int v = 0; v < VT; ++v)
+#pragma unroll
+      for (int s = 0; s < 4; ++s) vr[v][s] = 4 * g4 + s < nb ? to_f(rv[v][s]) : 0.f;
+    if (b + 16 < ntok) fetch(b + 16);
+    __syncthreads();
+
+    f32x4 O[VT];
+    if constexpr (!STATE) {
+      f32x4 sc = (f32x4)(0.f), sc2 = (f32x4)(0.f);
+#pragma unroll
+      for (int v = 0; v < VT; ++v) O[v] = (f32x4)(0.f);
+#pragma unroll
+      for (int m = 0; m < DT; ++m) {
+        const f32x4 x = *reinterpret_cast<const f32x4*>(&tab[w][c16][16 * m + 4 * g4]);
+        const f32x4 y = *reinterpret_cast<const f32x4*>(&tab[TQB][c16][16 * m + 4 * g4]);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          if (r & 1) sc2 = mfma_f32(x[r], x[r], sc2);
+          else sc = mfma_f32(x[r], x[r], sc);
+#pragma unroll
+          for (int v = 0; v < VT; ++v) O[v] = mfma_f32(y[r], S[m][v][r], O[v]);
+        }
+      }
+      const int lw = 3 - w;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int i = 4 * g4 + r, j = c16;
+        const bool pair = (i >> (lw + 1)) == (j >> (lw + 1)) && ((i >> lw) & 1) && !((j >> lw) & 1);
+        ap[w][i][j] = pair ? sc[r] + sc2[r] : 0.f;
+      }
+      __syncthreads();
+      f32x4 A = (f32x4)(0.f);
+#pragma unroll
+      for (int k = 0; k < 4; ++k) A += *reinterpret_cast<const f32x4*>(&ap[k][c16][4 * g4]);
+      float dg = 0.f;
+#pragma unroll
+      for (int k = 0; k < 4; ++k)
+        if (k * 64 < DC) dg += dred[k][c16];
+#pragma unroll
+      for (int s = 0; s < 4; ++s) {
+        const float x = 4 * g4 + s == c16 ? dg : A[s];
+#pragma unroll
+        for (int v = 0; v < VT; ++v) O[v] = mfma_f32(x, vr[v][s], O[v]);
+      }
+    }
+#pragma unroll
+    for (int m = 0; m < DT; ++m) {
+      const f32x4 p = *reinterpret_cast<const f32x4*>(&dec[16 * m + 4 * g4]);
+      float k[4];
+#pragma unroll
+      for (int s = 0; s < 4; ++s) k[s] = tab[TKE][4 * g4 + s][16 * m + c16];
+#pragma unroll
+      for (int v = 0; v < VT; ++v) {
+        S[m][v] *= p;
+#pragma unroll
+        for (int s = 0; s < 4; ++s) S[m][v] = mfma_f32(k[s], vr[v][s], S[m][v]);
+      }
+    }
+    if constexpr (!STATE) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        float x = 0.f;
+#pragma unroll
+        for (int v = 0; v < VT; ++v) x += O[v][r] * O[v][r];  // (columns past V hold zeros)
+        x = row16_sum(x);
+        if (c16 == 0) rss[w][4 * g4 + r] = x;
+      }
+    }
+    __syncthreads();
+    if constexpr (!STATE) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int i = 4 * g4 + r;
+        const float ss = rss[0][i] + rss[1][i] + rss[2][i] + rss[3][i];
+        const float sc = 1.f / sqrtf(ss / (float)V + a.eps);
+#pragma unroll
+        for (int v = 0; v < VT; ++v) {
+          const int col = (w * VT + v) * 16 + c16;
+          if (i < nb && col < V)
+            st_act((T*)a.out, tok0 + b + i, h * V + col, a.H * V, a.packed_mt, O[v][r] * sc * a.norm[col]);
+        }
+      }
+    }
+  }
+  if (!STATE && dst >= 0) return;  // (the next segment's workgroup owns the state from here)
+  float* sp = dst < 0 ? a.state + ((int64_t)row * a.H + h) * blk : ws + ((int64_t)dst * a.H + h) * blk;
+#pragma unroll
+  for (int m = 0; m < DT; ++m)
+#pragma unroll
+    for (int v = 0; v < VT; ++v)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int d = 16 * m + 4 * g4 + r, col = (w * VT + v) * 16 + c16;
+        if (d < D && col < V) sp[(int64_t)d * V + col] = S[m][v][r];
+      }
+  if (STATE && grp == 0 && ch < D) wdec[((int64_t)dst * a.H + h) * D + ch] = run;
+}
+
+// multi [4, nm]: first slot, slots, first token, unused.  Slot i holds segment i-1's contribution (i > 0):
+// every slot becomes its segment's initial state.
+__global__ __launch_bounds__(256) void hgrn2_prefix_kernel(Hgrn2Args a, const int32_t* __restrict__ multi, int nm,
+                                                           float* __restrict__ ws, const float* __restrict__ wdec) {
+  const int64_t blk = (int64_t)a.D * a.V;
+  const int64_t e = blockIdx.x * (int64_t)256 + threadIdx.x;
+  if (e >= blk) return;
+  const int h = blockIdx.y, s = blockIdx.z;
+  const int slot = multi[s], n = multi[nm + s], tok0 = multi[2 * nm + s];
+  const int d = (int)(e / a.V);
+  float p = a.q_ctx[tok0] <= 1 ? 0.f : a.state[((int64_t)a.q_seq[tok0] * a.H + h) * blk + e];
+  float* x = ws + ((int64_t)slot * a.H + h) * blk + e;
+  const float* f = wdec + ((int64_t)slot * a.H + h) * a.D + d;
+  const int64_t xs = (int64_t)a.H * blk, fs = (int64_t)a.H * a.D;
+  x[0] = p;
+  for (int i = 1; i < n; i += 4) {  // four slots' loads in flight
+    float u[4], g[4];
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const int j = min(i + k, n - 1);
+      u[k] = x[j * xs];
+      g[k] = f[j * fs];
+    }
+#pragma unroll
+    for (int k = 0; k < 4; ++k)
+      if (i + k < n) {
+        p = g[k] * p + u[k];
+        x[(i + k) * xs] = p;
+      }
+  }
+}
+
+template <typename T, bool STATE>
+static int launch_chunk(const Hgrn2Args& a, const int32_t* seg, int nseg, float* ws, float* wdec, hipStream_t stream) {
+#define MP_HC(DT_, VT_)                                                                                            \
+  hipLaunchKernelGGL((hgrn2_chunk_kernel<T, DT_, VT_, STATE>), dim3(a.H, nseg), dim3(256), 0, stream, a, seg, nseg, \
+                     ws, wdec)
+  const int dt = (a.D + 15) / 16, vt = (a.V + 63) / 64;
+  if (dt > 16 || vt > 4) return -1;
+  if (dt <= 4) {
+    if (vt <= 1) MP_HC(4, 1); else if (vt <= 2) MP_HC(4, 2); else MP_HC(4, 4);
+  } else if (dt <= 8) {
+    if (vt <= 1) MP_HC(8, 1); else if (vt <= 2) MP_HC(8, 2); else MP_HC(8, 4);
+  } else {
+    if (vt <= 2) MP_HC(16, 2); else MP_HC(16, 4);
+  }
+#undef MP_HC
+  return (int)hipGetLastError();
+}
+
 }  // namespace mp
+
+// seg [4, nseg] (all of the step), multi [4, nm] (sequences cut into several segments; ws / wdec hold their slots)
+extern "C" int mp_hgrn2_chunk(const void* z, int64_t zs, const float* bias, const float* lower, const float* norm,
+                              float* state, const int32_t* q_seq, const int32_t* q_ctx, void* out, int H, int D, int V,
+                              float eps, const int32_t* seg, int nseg, const int32_t* multi, int nm, float* ws,
+                              float* wdec, int packed_mt, int f32, hipStream_t stream) {
+  using namespace mp;
+  (void)hipGetLastError();
+  if (nseg == 0) return 0;
+  if (nseg > 65535 || nm > 65535 || H > 65535) return -1;
+  const Hgrn2Args a{z, zs, bias, lower, norm, state, q_seq, q_ctx, out, H, D, V, packed_mt, eps};
+  int rc;
+  if (nm > 0) {
+    rc = f32 ? launch_chunk<float, true>(a, seg, nseg, ws, wdec, stream)
+             : launch_chunk<bf16_t, true>(a, seg, nseg, ws, wdec, stream);
+    if (rc) return rc;
+    hipLaunchKernelGGL(hgrn2_prefix_kernel, dim3((unsigned)(((int64_t)D * V + 255) / 256), H, nm), dim3(256), 0, stream,
+                       a, multi, nm, ws, wdec);
+    rc = (int)hipGetLastError();
+    if (rc) return rc;
+  }
+  return f32 ? launch_chunk<float, false>(a, seg, nseg, ws, wdec, stream)
+             : launch_chunk<bf16_t, false>(a, seg, nseg, ws, wdec, stream);
+}
 
 extern "C" int mp_hgrn2_scan(const void* z, int64_t zs, const float* bias, const float* lower, const float* norm,
                              float* state, const int32_t* q_seq, const int32_t* q_ctx, void* out, int H, int D, int V,

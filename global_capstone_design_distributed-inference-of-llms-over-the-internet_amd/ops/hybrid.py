@@ -6,6 +6,7 @@ activation in the packed decode-GEMM layout.
 """
 from __future__ import annotations
 
+import numpy as np
 import torch
 
 from . import reference as ref
@@ -74,9 +75,49 @@ def hgrn2(z, bias, lower, norm, state, q_seq, q_ctx, out, eps, plan=None, packed
     (``HybridStage.plan``)."""
     if not _native(z):
         return _put(out, rh.hgrn2(z, bias, lower, norm, state, q_seq, q_ctx, eps), packed)
-    torch.ops.mpamd.hgrn2_scan(z, bias, lower, norm, state, q_seq, q_ctx, out, float(eps),
-                               None if plan is None else plan["seg"], int(packed))
+    _, H, D, V = state.shape
+    if plan is None:
+        torch.ops.mpamd.hgrn2_scan(z, bias, lower, norm, state, q_seq, q_ctx, out, float(eps), None, int(packed))
+    elif D <= CHUNK_MAX and V <= CHUNK_MAX and not plan.get("scan"):
+        slots = plan["slots"]
+        ws = torch.empty(slots * H * D * (V + 1), dtype=torch.float32, device=z.device) if slots else None
+        torch.ops.mpamd.hgrn2_chunk(z, bias, lower, norm, state, q_seq, q_ctx, out, float(eps), plan["seg"],
+                                    plan["multi"], slots, ws, int(packed))
+    else:
+        torch.ops.mpamd.hgrn2_scan(z, bias, lower, norm, state, q_seq, q_ctx, out, float(eps), plan["seqs"],
+                                   int(packed))
     return out
+
+
+# largest head sizes of the chunk form (csrc/hgrn2.hip hgrn2_chunk_kernel)
+CHUNK_MAX = 256
+
+
+def hgrn2_plan(ntoks, heads: int, n_cu: int = 256, seg_tokens: int = None):
+    """Segments of a ragged step for the chunk form: int32 ``seqs`` [2, n] (first flat token, tokens of every
+    sequence that brings any), ``seg`` [4, nseg], ``multi`` [4, nm] and the number of workspace slots
+    (csrc/hgrn2.hip).  Sequences are cut so that about two workgroups per CU exist, at whole 16-token blocks."""
+    n = np.asarray(ntoks, dtype=np.int64)
+    off = np.concatenate([[0], np.cumsum(n)[:-1]])
+    keep = n > 0
+    off, n = off[keep], n[keep]
+    if seg_tokens is None:
+        want = max(1, -(-2 * n_cu // max(heads, 1)))  # segments over the whole step
+        seg_tokens = max(128, 16 * (-(-int(n.sum()) // want) // 16))
+    seg, multi, slots = [], [], 0
+    for o, c in zip(off.tolist(), n.tolist()):
+        k = max(1, -(-c // seg_tokens)) if c > seg_tokens * 3 // 2 else 1
+        per = 16 * -(-c // (16 * k))
+        k = -(-c // per)
+        if k == 1:
+            seg.append((o, c, -1, -1))
+            continue
+        multi.append((slots, k, o, 0))
+        for i in range(k):
+            seg.append((o + i * per, min(per, c - i * per), slots + i, slots + i + 1 if i < k - 1 else -1))
+        slots += k
+    mk = lambda v, r: np.ascontiguousarray(np.asarray(v, dtype=np.int32).reshape(-1, r).T)  # noqa: E731
+    return {"seqs": np.stack([off, n]).astype(np.int32), "seg": mk(seg, 4), "multi": mk(multi, 4), "slots": slots}
 
 
 def talk_prep(z, wqk, qn, cache, rk, slots, eps):
@@ -87,10 +128,43 @@ def talk_prep(z, wqk, qn, cache, rk, slots, eps):
     torch.ops.mpamd.talk_prep(z, wqk, qn, cache, rk, slots, float(eps))
 
 
-def talk_attention(z, qn, talk, cache, rk, table, q_seq, q_ctx, out, chunk, scale, packed=False):
-    """Chunked talking-heads attention with the output gate of ``z``."""
+def talk_block(H: int, G: int, D: int) -> int:
+    """Tokens of a prompt's query block on the MFMA form (0: shape not covered)."""
+    return int(torch.ops.mpamd.talk_block(int(H), int(G), int(D)))
+
+
+def talk_blocks(ntoks, tokens: int):
+    """Query blocks of a ragged step: int32 [2, nblk] (first flat token, tokens)."""
+    out, off = [], 0
+    for n in ntoks:
+        for k in range(0, int(n), tokens):
+            out.append((off + k, min(tokens, int(n) - k)))
+        off += int(n)
+    return np.ascontiguousarray(np.asarray(out, dtype=np.int32).reshape(-1, 2).T)
+
+
+def talk_parts(rows: int, H: int, G: int, D: int, span: int, n_cu: int = 256):
+    """(keys per split, splits) of a decode step whose queries see at most ``span`` keys: about two workgroups per
+    CU, no split under 128 keys.  (The first split starts on a 32-key boundary at or before the first key.)"""
+    span = int(span) + 31
+    want = max(1, 2 * n_cu // max(1, rows))
+    n = max(1, min(want, span // 128))
+    ps = 32 * -(-span // (32 * n))
+    return ps, -(-span // ps)
+
+
+def talk_attention(z, qn, talk, cache, rk, table, q_seq, q_ctx, out, chunk, scale, packed=False, blocks=None,
+                   parts=None, ws=None):
+    """Chunked talking-heads attention with the output gate of ``z``.  On the GPU the MFMA form runs when
+    ``blocks`` (prompt steps: ``talk_blocks`` on the device) or ``parts`` (decode: ``talk_parts``, ``ws`` fp32
+    scratch) is given, else the form for any shape and element type."""
     if not _native(z):
         return _put(out, rh.talk_attention(z, qn, talk, cache, rk, table, q_seq, q_ctx, chunk, scale), packed)
+    if blocks is not None or parts is not None:
+        ps, np_ = parts if blocks is None else (0, 1)
+        torch.ops.mpamd.talk_mfma(z, qn, talk, cache, rk, table, q_seq, q_ctx, out, int(chunk), float(scale), blocks,
+                                  int(ps), int(np_), ws, int(packed))
+        return out
     torch.ops.mpamd.talk_attention(z, qn, talk, cache, rk, table, q_seq, q_ctx, out, int(chunk), float(scale),
                                    int(packed))
     return out

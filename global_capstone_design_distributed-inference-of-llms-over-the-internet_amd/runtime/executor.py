@@ -276,9 +276,10 @@ class StageExecutor:
         # unit RMSNorm weight for > 64-row decode steps over norm-folded packed weights (made
         # here, not inside a hipGraph capture)
         self._ones = torch.ones(cfg.hidden_size, dtype=self.dtype, device=self.device) if self._fused else None
-        self._hybrid = HybridStage(self) if cfg.hybrid else None
         if self.device.type == "cuda":
             ops.require_native()
+        self._hybrid = HybridStage(self) if cfg.hybrid else None
+        if self.device.type == "cuda":
             if cfg.model_type != "gpt2" and ops.gemm_policy() != "hipblaslt":
                 weights.pack_for_decode(fold_norms=self._fused)
                 if self._fused and not all(getattr(L, "folded", False) for L in weights.layers):
@@ -390,7 +391,7 @@ class StageExecutor:
                 d32 = h32[: 2 * T + S].clone()
             return d64, d32
 
-        hp = self._hybrid.plan(ntoks, st, [s.row for s in sess]) if self._hybrid is not None and not is_decode else None
+        hp = self._hybrid.plan(ntoks) if self._hybrid is not None and not is_decode else None
         qb = sb = fb = None
         fa_waves = 4
         if self.device.type == "cuda" and not is_decode and self._attn_fa:

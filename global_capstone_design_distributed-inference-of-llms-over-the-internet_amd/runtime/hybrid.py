@@ -41,6 +41,15 @@ class HybridStage:
             else:
                 self.index.append(na)
                 na += 1
+        # query-block tokens of each attention shape's MFMA form (0: the any-shape form)
+        self.talk_block = {}
+        for lay in ex.w.layers:
+            sp = lay.spec
+            if not sp.recurrent and ex.device.type == "cuda":
+                ok = ex.dtype == torch.bfloat16 and ex.cache.page_size >= 32
+                self.talk_block[(sp.heads, sp.kv_heads, sp.dim)] = \
+                    hops.talk_block(sp.heads, sp.kv_heads, sp.dim) if ok else 0
+        self.rec_heads = min([lay.spec.heads for lay in ex.w.layers if lay.spec.recurrent], default=0)
         self.max_chunk = max([lay.spec.chunk for lay in ex.w.layers if not lay.spec.recurrent], default=1)
 
     def autotune(self) -> None:
@@ -123,7 +132,16 @@ class HybridStage:
                 kv, rk = ex.cache.layer(self.index[i])
                 qn = e(f"qn{sp.out_cols}", (T, sp.out_cols))
                 hops.talk_prep(z, lay.w_qk, qn, kv, rk, slots, eps)
-                hops.talk_attention(z, qn, lay.talk, kv, rk, table, q_seq, q_ctx, o, sp.chunk, sp.scale, packed=pko)
+                tb = self.talk_block.get((sp.heads, sp.kv_heads, sp.dim), 0)
+                blocks = parts = ws = None
+                if tb and plan is not None:
+                    blocks = plan["blocks"][tb]
+                elif tb:
+                    parts = hops.talk_parts(T, sp.heads, sp.kv_heads, sp.dim, min(span, sp.chunk), ex._n_cu)
+                    if parts[1] > 1:
+                        ws = e("talk_ws", (parts[1] * T * sp.heads * (sp.dim + 2),), torch.float32)
+                hops.talk_attention(z, qn, lay.talk, kv, rk, table, q_seq, q_ctx, o, sp.chunk, sp.scale, packed=pko,
+                                    blocks=blocks, parts=parts, ws=ws)
             if sp.ff:
                 pku = self._packed(T, lay.w_up, lay.w_up_p)
                 xu = self._act(e, "xb", T, W, pku)
@@ -155,15 +173,17 @@ class HybridStage:
             xb.copy_(y)
 
     # ------------------------------------------------------------------ plans
-    def plan(self, ntoks, starts, rows) -> dict:
+    def plan(self, ntoks) -> dict:
         """Device description of a ragged step (not one token per session)."""
-        import numpy as np
-
-        n = np.asarray(ntoks, dtype=np.int64)
-        off = np.concatenate([[0], np.cumsum(n)[:-1]])
-        keep = n > 0
-        seg = torch.from_numpy(np.stack([off[keep], n[keep]]).astype(np.int32))
-        return {"seg": seg.to(self.ex.device, non_blocking=True)}
+        if self.ex.device.type != "cuda":
+            return {}
+        up = lambda a: torch.from_numpy(a).to(self.ex.device, non_blocking=True)  # noqa: E731
+        p = {"blocks": {tb: up(hops.talk_blocks(ntoks, tb)) for tb in set(self.talk_block.values()) if tb}}
+        if self.rec_heads:
+            h = hops.hgrn2_plan(ntoks, self.rec_heads, self.ex._n_cu)
+            p.update(seqs=up(h["seqs"]), seg=up(h["seg"]), multi=up(h["multi"]) if h["slots"] else None,
+                     slots=h["slots"])
+        return p
 
     def span(self, max_ctx: int) -> int:
         """Most keys a decode query of context <= max_ctx can see."""
