@@ -310,7 +310,15 @@ def main(argv=None):
     ap.add_argument("--phase2-inject", default="none", choices=["none", "init", "run"],
                     help="test hook: make the second phase fail on the last stage rank at communicator set-up "
                          "(init) or in the middle of its timed steps (run)")
+    ap.add_argument("--layer-bench", nargs="?", const="2048,4096", default=None, metavar="WIDTHS",
+                    help="instead of the headline workload: prefill / decode throughput of the hybrid decoder's layers "
+                         "beside the closest uniform model at these widths (one GPU, one JSON line)")
+    ap.add_argument("--layer-bench-layers", type=int, default=8)
     a = ap.parse_args(argv)
+    if a.layer_bench:
+        from src.layer_bench import main as layer_bench_main
+
+        return layer_bench_main(a.layer_bench, a.layer_bench_layers)
 
     from src import ops
     from src.models.config import resolve_model

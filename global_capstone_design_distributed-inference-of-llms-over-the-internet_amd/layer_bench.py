@@ -1,0 +1,124 @@
+"""Prefill and decode throughput of a hybrid decoder's layers beside the closest uniform family at equal size.
+
+``python bench.py --layer-bench`` (one GPU): for every width, an 8-layer Kafunex stage (three recurrent layers, then
+one attention layer) and an 8-layer Llama stage of the same width, query / kv heads, head size and feed-forward
+parameters, both bf16 with random weights, run in turn on the same executor code: prompts of several shapes, then
+decode steps (hipGraph replays) at several batch sizes.  One JSON line.
+"""
+from __future__ import annotations
+
+import json
+import statistics
+
+import torch
+
+from .models.config import LayerSpec, ModelConfig, hybrid_config
+from .models.weights import random_stage_weights
+from .runtime.executor import StageExecutor
+
+VOCAB = 32000
+PREFILL = ((1, 8192), (8, 1024), (64, 128))
+DECODE = (1, 16, 64)
+
+
+def configs(width: int, layers: int):
+    """(hybrid, uniform) model configs of one width: head size 128, four query heads per kv head."""
+    H = width // 128
+    G = max(1, H // 4)
+    ff_glu = 128 * (7 * width // 2 // 128)             # gated feed-forward of the uniform model: 3 matrices
+    ff = 128 * (3 * ff_glu // 2 // 128)                 # equal parameters in 2 matrices
+    rec = LayerSpec("hgrn2", H, 128, 128, ff)
+    att = LayerSpec("attention", H, 128, 128, ff, G, 1024, 128 ** -0.5)
+    hyb = hybrid_config("kafunex", VOCAB, width, 1e-6, [att if i % 4 == 3 else rec for i in range(layers)],
+                        f"kafunex-w{width}")
+    uni = ModelConfig(vocab_size=VOCAB, hidden_size=width, intermediate_size=ff_glu, num_hidden_layers=layers,
+                      num_attention_heads=H, num_key_value_heads=G, head_dim=128, max_position_embeddings=16384,
+                      name=f"llama-w{width}")
+    return hyb, uni
+
+
+class Side:
+    def __init__(self, cfg, device, max_len: int):
+        w = random_stage_weights(cfg, 0, cfg.num_hidden_layers, has_embed=True, has_head=True, device=device, seed=1)
+        self.cfg, self.device = cfg, device
+        self.ex = StageExecutor(cfg, w, device, kv_cache_bytes=24 << 30, max_sessions=max(DECODE),
+                                max_seq_len=max_len, max_tokens_per_step=8192, warmup=False)
+        self.gen = torch.Generator(device=device).manual_seed(7)
+
+    def ids(self, n):
+        return torch.randint(0, self.cfg.vocab_size, (n,), device=self.device, generator=self.gen)
+
+    def prefill(self, batch, length):
+        return self.ex.forward([(f"s{i}", length) for i in range(batch)], self.ids(batch * length),
+                               reset=[True] * batch)
+
+    def decode(self, batch):
+        return self.ex.forward([(f"s{i}", 1) for i in range(batch)], self.ids(batch))
+
+    def close(self):
+        for s in list(self.ex.sessions.sessions):
+            self.ex.sessions.close(s)
+
+
+def _ms(fn, iters: int) -> float:
+    e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+    e0.record()
+    for _ in range(iters):
+        fn()
+    e1.record()
+    e1.synchronize()
+    return e0.elapsed_time(e1) / iters
+
+
+def _in_turn(sides, call, iters: int, rounds: int):
+    """Median ms per call of every side, the sides timed alternately."""
+    t = {k: [] for k in sides}
+    for k, s in sides.items():
+        call(s)
+        call(s)
+    for _ in range(rounds):
+        for k, s in sides.items():
+            t[k].append(_ms(lambda: call(s), iters))
+    return {k: statistics.median(v) for k, v in t.items()}
+
+
+def run(widths, layers: int = 8, ctx: int = 1024, device="cuda:0", steps: int = 16, rounds: int = 3, log=None) -> dict:
+    out = []
+    with torch.no_grad():
+        for width in widths:
+            sides = {c.name.split("-")[0]: Side(c, device, 8704) for c in configs(width, layers)}
+            row = {"width": width, "layers": layers, "prefill": [], "decode": []}
+            for b, n in PREFILL:
+                ms = _in_turn(sides, lambda s: s.prefill(b, n), 3, rounds)
+                row["prefill"].append({"batch": b, "tokens": n, "ms": {k: round(v, 3) for k, v in ms.items()},
+                                       "tokens_per_s": {k: round(1e3 * b * n / v) for k, v in ms.items()}})
+                for s in sides.values():
+                    s.close()
+                if log:
+                    log(f"width {width} prefill {b} x {n}: {row['prefill'][-1]['ms']}")
+            for b in DECODE:
+                for s in sides.values():
+                    for i in range(0, b, 8192 // ctx):
+                        m = min(8192 // ctx, b - i)
+                        s.ex.forward([(f"s{i + j}", ctx) for j in range(m)], s.ids(m * ctx), reset=[True] * m)
+                ms = _in_turn(sides, lambda s: s.decode(b), steps, rounds)
+                row["decode"].append({"batch": b, "context": ctx, "ms": {k: round(v, 4) for k, v in ms.items()},
+                                      "tokens_per_s": {k: round(1e3 * b / v) for k, v in ms.items()}})
+                for s in sides.values():
+                    s.close()
+                if log:
+                    log(f"width {width} decode batch {b}: {row['decode'][-1]['ms']}")
+            out.append(row)
+            del sides
+            torch.cuda.empty_cache()
+    return {"metric": "layer_bench", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic", "rows": out}
+
+
+def main(widths: str, layers: int = 8) -> int:
+    import sys
+
+    if not torch.cuda.is_available():
+        raise SystemExit("--layer-bench needs a GPU")
+    rec = run([int(w) for w in widths.split(",")], layers, log=lambda m: print(m, file=sys.stderr, flush=True))
+    print(json.dumps(rec), flush=True)
+    return 0

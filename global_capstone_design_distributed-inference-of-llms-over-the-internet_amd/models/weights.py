@@ -142,6 +142,7 @@ class HybridLayer:
     o_norm: Optional[torch.Tensor] = None    # hgrn2 [vdim]
     w_qk: Optional[torch.Tensor] = None      # attention [heads * dim]: query norm x its kv head's key norm
     talk: Optional[torch.Tensor] = None      # attention [heads, heads]
+    sigma: Optional[torch.Tensor] = None     # attention [heads]: talk @ the heads' distance slopes
     w_in_p: Optional[torch.Tensor] = None
     w_o_p: Optional[torch.Tensor] = None
     w_up_p: Optional[torch.Tensor] = None
@@ -378,6 +379,9 @@ def _hybrid_layer(spec: LayerSpec, width: int, get, device, dtype) -> HybridLaye
         kn = f32("mix.k.norm").view(spec.kv_heads, 1, spec.dim)
         kn = kn.expand(spec.kv_heads, spec.heads // spec.kv_heads, spec.dim).reshape(-1)
         lay.w_qk, lay.talk = (f32("mix.q.norm") * kn).contiguous(), f32("mix.talk")
+        from ..ops.hybrid import talk_sigma
+
+        lay.sigma = talk_sigma(lay.talk)
     return lay
 
 

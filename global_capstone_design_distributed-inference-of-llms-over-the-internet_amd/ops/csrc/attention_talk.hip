@@ -12,6 +12,7 @@
 //   talk_attn_kernel    any shape and both element types: one workgroup per query token
 //   talk_mfma_kernel    bf16, head size <= 128: prompts and decode on MFMA, the head mixing folded into
 //                       the queries
+//   talk_xchg_kernel    the same for many heads: raw scores exchanged through LDS, mixed by another MFMA
 //   talk_merge_kernel   merges the context splits of a decode step, applies the gate
 #include "common.h"
 #include "act_io.h"
@@ -24,6 +25,7 @@ struct TalkArgs {
   void* qn;              // [T, H D] q'
   const float* wqk;      // [H D] query norm weight x the kv head's key norm weight
   const float* talk;     // [H, H]
+  const float* sigma;    // [H] the mixed slopes, talk @ slope
   void* cache;           // [pages, G, page, D]
   float* rk;             // [pages, page]
   const int64_t* slots;
@@ -35,31 +37,40 @@ struct TalkArgs {
   float scale, eps;
 };
 
-template <typename T>
-__global__ __launch_bounds__(256) void talk_prep_kernel(TalkArgs a) {
+// VEC columns a thread and step; NT threads (decode rows are few: more threads, one round of loads)
+template <typename T, int VEC, int NT>
+__global__ __launch_bounds__(NT) void talk_prep_kernel(TalkArgs a) {
   __shared__ float red[16];
   const int t = blockIdx.x, HD = a.H * a.D, GD = a.G * a.D;
   const int64_t slot = a.slots[t];
   if (slot < 0) return;
   const T* z = (const T*)a.z + (int64_t)t * a.zs;
   float sq = 0.f, sk = 0.f;
-  for (int i = threadIdx.x; i < HD; i += 256) {
-    const float x = ld_f(z, i);
-    sq += x * x;
-  }
-  for (int i = threadIdx.x; i < GD; i += 256) {
-    const float x = ld_f(z, HD + i);
-    sk += x * x;
+  for (int i = threadIdx.x * VEC; i < HD + GD; i += NT * VEC) {
+    float x[VEC], s = 0.f;
+    ld_vec<VEC>(z + i, x);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) s += x[j] * x[j];
+    if (i < HD) sq += s;
+    else sk += s;
   }
   sq = block_sum(sq, red);
   sk = block_sum(sk, red);
   const float rq = 1.f / sqrtf(sq / (float)HD + a.eps);
-  for (int i = threadIdx.x; i < HD; i += 256)
-    from_f(ld_f(z, i) * rq * a.wqk[i], ((T*)a.qn)[(int64_t)t * HD + i]);
   const int64_t pg = slot >> a.page_log2, off = slot & ((1 << a.page_log2) - 1);
-  for (int i = threadIdx.x; i < GD; i += 256) {
-    const int c = i / a.D, d = i - c * a.D;
-    ((T*)a.cache)[(((pg * a.G + c) << a.page_log2) + off) * a.D + d] = z[HD + i];
+  for (int i = threadIdx.x * VEC; i < HD + GD; i += NT * VEC) {
+    float x[VEC];
+    ld_vec<VEC>(z + i, x);
+    if (i < HD) {
+      float g[VEC];
+      ld_vec<VEC>(a.wqk + i, g);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) x[j] *= rq * g[j];
+      st_vec<VEC>((T*)a.qn + (int64_t)t * HD + i, x);
+    } else {
+      const int c = (i - HD) / a.D, d = i - HD - c * a.D;
+      st_vec<VEC>((T*)a.cache + (((pg * a.G + c) << a.page_log2) + off) * a.D + d, x);
+    }
   }
   if (threadIdx.x == 0) a.rk[slot] = 1.f / sqrtf(sk / (float)GD + a.eps);
 }
@@ -187,6 +198,47 @@ __device__ __forceinline__ unsigned pk2_bf(float a, float b) {
 }
 
 constexpr int TM_KEYS = 32;
+// log2 units a row's maximum may grow before its sums are rescaled (weights reach 2^8, their sums are fp32)
+constexpr float TM_GROW = 8.f;
+
+// first of the 4 head columns in accumulator tile t of lane group g4 (the key tile's column order)
+__device__ __forceinline__ int tm_col(int t, int g4) {
+  return 32 * (t >> 1) + 16 * (g4 & 1) + 8 * (t & 1) + 4 * (g4 >> 1);
+}
+
+// A query row's result: normalised, gated and stored, or left as this split's (maximum, sum, sums).
+// PERM: accumulator tile t holds the columns tm_col(t, g4), else 16 t + 4 g4.
+template <int DH, bool PERM>
+__device__ __forceinline__ void talk_store(const TalkArgs& a, float* __restrict__ part, int T, int p, int t, int h, int g4,
+                                           float m, float ls, const f32x4 (&o)[2 * DH]) {
+  const int D = a.D, HD = a.H * D;
+  if (part != nullptr) {  // split context: [NP][T][H][D] sums, then [NP][T][H][2] (max, sum)
+    const int64_t pr = ((int64_t)p * T + t) * a.H + h;
+#pragma unroll
+    for (int k = 0; k < 2 * DH; ++k) {
+      const int d = PERM ? tm_col(k, g4) : 16 * k + 4 * g4;
+      if (d < D) *reinterpret_cast<f32x4*>(part + pr * D + d) = o[k];
+    }
+    if (g4 == 0) {
+      float* ml = part + (int64_t)gridDim.z * T * HD + pr * 2;
+      ml[0] = m;
+      ml[1] = ls;
+    }
+    return;
+  }
+  const float inv = 1.f / ls;
+  const bf16_t* gate = (const bf16_t*)a.z + (int64_t)t * a.zs + HD + a.G * D + h * D;
+#pragma unroll
+  for (int k = 0; k < 2 * DH; ++k) {
+    const int d = PERM ? tm_col(k, g4) : 16 * k + 4 * g4;
+    if (d < D) {
+      float x[4];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) x[r] = o[k][r] * inv / (1.f + __expf(-bf2f(gate[d + r])));
+      st_act_vec<4>((bf16_t*)a.out, t, h * D + d, HD, a.packed_mt, x);
+    }
+  }
+}
 
 // DH: 32-column slices per head (Dp = 32 DH); KF: slices of the wide key the kernel is built for
 // (G DH <= KF, the rest zero); NW waves; UPW units per wave
@@ -223,6 +275,8 @@ __global__ __launch_bounds__(NW * 64, KF * UPW > 32 ? 1 : 2) void talk_mfma_kern
 #pragma unroll
   for (int u = 0; u < UPW; ++u) {
     const int unit = ((int)blockIdx.y * NW + w) * UPW + u;
+#pragma unroll
+    for (int f = 0; f < KF; ++f) q[u][f] = (u16x8)(0);
     const int c = unit < units ? unit / nrb : 0;
     const int row = (unit < units ? unit - c * nrb : 0) * 16 + c16;
     const bool ok = unit < units && row < ntok * rep;
@@ -235,28 +289,64 @@ __global__ __launch_bounds__(NW * 64, KF * UPW > 32 ? 1 : 2) void talk_mfma_kern
     l[u] = 0.f;
 #pragma unroll
     for (int t = 0; t < 2 * DH; ++t) o[u][t] = (f32x4)(0.f);
-    const float* tr = a.talk + row_h[u] * H;
-    float sg = 0.f;
-    for (int g = 0; g < H; ++g) sg += tr[g] * exp2f(-8.f * (float)(g + 1) / (float)H);
-    sig[u] = sg * LOG2E;
+    sig[u] = a.sigma[row_h[u]] * LOG2E;
+  }
+
+  // The mixed queries: per row block, its tokens' query rows go to LDS as a [32][wide] tile (row = token x group
+  // member g, column = kv head c, d) and u^T = Q^T T^T runs on MFMA, T^T block-diagonal over the tokens.  The
+  // accumulator leaves lane group g4 with d = 4 g4 + r of both 16-column halves of a slice, so that is the
+  // order in which the key tile keeps a slice's columns.
+  {
+    bf16_t* qt = kt[1];
+    for (int rb = 0; rb < nrb; ++rb) {
+      const int t0 = rb * 16 / rep, t1 = min((rb * 16 + 15) / rep, ntok - 1), nr = (t1 - t0 + 1) * rep;
+      if (rb > 0) __syncthreads();
 #pragma unroll
-    for (int f = 0; f < KF; ++f) {
-      const int cc = f / DH, d = (f % DH) * 32 + 8 * g4;
-      float x[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-      if (ok && cc < G && d < D) {
-        const bf16_t* qp = (const bf16_t*)a.qn + (int64_t)row_t[u] * HD + cc * rep * D + d;
-        for (int g = 0; g < rep; ++g) {
-          const u16x8 v = *reinterpret_cast<const u16x8*>(qp + g * D);
-          const float t = tr[cc * rep + g];
+      for (int k = 0; k < CPT; ++k) {
+        const int x = tid + NT * k, kr = x / (WC / 8), col = (x % (WC / 8)) * 8;
+        const int c = col / DP, d = col % DP;
+        if (kr < TM_KEYS)
+          *reinterpret_cast<u16x8*>(qt + kr * STR + col) =
+              kr < nr && c < G && d < D
+                  ? *reinterpret_cast<const u16x8*>((const bf16_t*)a.qn + (int64_t)(tok0 + t0 + kr / rep) * HD +
+                                                    (c * rep + kr % rep) * D + d)
+                  : (u16x8)(0);
+      }
+      __syncthreads();
 #pragma unroll
-          for (int j = 0; j < 8; ++j) x[j] += t * bf2f(v[j]);
+      for (int u = 0; u < UPW; ++u) {
+        const int unit = ((int)blockIdx.y * NW + w) * UPW + u;
+        if (unit >= units || unit % nrb != rb) continue;  // (uniform over the wave)
+        const float* tr = a.talk + row_h[u] * H;
+        const int mt = row_t[u] - tok0 - t0;  // this lane's token within the block
+        const bf16_t* qb = qt + (8 * g4 + (c16 >> 2)) * STR + 4 * (c16 & 3);
+#pragma unroll
+        for (int c = 0; c < KF / DH; ++c) {
+          u16x8 tb = (u16x8)(0);
+          if (c < G && row_t[u] >= 0) {
+#pragma unroll
+            for (int j = 0; j < 8; ++j) {
+              const int g = 8 * g4 + j - mt * rep;
+              if (g >= 0 && g < rep) tb[j] = f2bf(tr[c * rep + g]);
+            }
+          }
+#pragma unroll
+          for (int f = c * DH; f < (c + 1) * DH; ++f) {
+            f32x4 x[2];
+#pragma unroll
+            for (int half = 0; half < 2; ++half) {
+              const bf16_t* p0 = qb + 32 * f + 16 * half;
+              const u16x4 v0 = lds_tr4(p0), v1 = lds_tr4(p0 + 4 * STR);
+              const u16x8 va = {v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
+              x[half] = mfma_bf(va, tb, (f32x4)(0.f));
+            }
+            u32x4_t pk = {pk2_bf(x[0][0], x[0][1]), pk2_bf(x[0][2], x[0][3]), pk2_bf(x[1][0], x[1][1]),
+                          pk2_bf(x[1][2], x[1][3])};
+            asm volatile("" : "+v"(pk));  // packed here: four registers a slice stay live, not eight
+            q[u][f] = __builtin_bit_cast(u16x8, pk);
+          }
         }
       }
-      u32x4_t pk;
-#pragma unroll
-      for (int j = 0; j < 4; ++j) pk[j] = pk2_bf(x[2 * j], x[2 * j + 1]);
-      asm volatile("" : "+v"(pk));  // packed here: four registers a slice stay live, not eight
-      q[u][f] = __builtin_bit_cast(u16x8, pk);
     }
   }
 
@@ -278,7 +368,12 @@ __global__ __launch_bounds__(NW * 64, KF * UPW > 32 ? 1 : 2) void talk_mfma_kern
 #pragma unroll
     for (int k = 0; k < CPT; ++k) {
       const int x = tid + NT * k, key = x / (WC / 8), col = (x % (WC / 8)) * 8;
-      if (key < TM_KEYS) *reinterpret_cast<u16x8*>(&kt[buf][key * STR + col]) = kreg[k];
+      if (key < TM_KEYS) {  // column d of a slice at 8 (d % 16 / 4) + 4 (d / 16) + d % 4
+        const int i = (col >> 3) & 3;
+        bf16_t* kp = &kt[buf][key * STR + (col & ~31) + 16 * (i & 1) + 4 * (i >> 1)];
+        *reinterpret_cast<u16x4*>(kp) = (u16x4){kreg[k][0], kreg[k][1], kreg[k][2], kreg[k][3]};
+        *reinterpret_cast<u16x4*>(kp + 8) = (u16x4){kreg[k][4], kreg[k][5], kreg[k][6], kreg[k][7]};
+      }
     }
     if (tid < TM_KEYS) rks[buf][tid] = rreg * a.scale * LOG2E;
   };
@@ -321,7 +416,7 @@ __global__ __launch_bounds__(NW * 64, KF * UPW > 32 ? 1 : 2) void talk_mfma_kern
         }
       lm = fmaxf(lm, __shfl_xor(lm, 16, 64));
       lm = fmaxf(lm, __shfl_xor(lm, 32, 64));
-      if (__any(lm > m[u])) {
+      if (__any(lm > m[u] + TM_GROW)) {
         const float mn = fmaxf(m[u], lm);
         const float al = mn == -INFINITY ? 1.f : __builtin_amdgcn_exp2f(m[u] - mn);
         l[u] *= al;
@@ -340,7 +435,7 @@ __global__ __launch_bounds__(NW * 64, KF * UPW > 32 ? 1 : 2) void talk_mfma_kern
           ph[4 * sub + r] = f2bf(x);
           pl[4 * sub + r] = f2bf(x - bf2f(ph[4 * sub + r]));
         }
-      // V^T: lane c16 of group g4 needs column d = 16 t + c16 of keys 4 g4 .. + 3 (+ 16)
+      // V^T: lane c16 of group g4 needs tile column 16 t + c16 of keys 4 g4 .. + 3 (+ 16)
       const bf16_t* vb = tb + (4 * g4 + (c16 >> 2)) * STR + uc[u] * DP + 4 * (c16 & 3);
 #pragma unroll
       for (int t = 0; t < 2 * DH; ++t) {
@@ -359,33 +454,255 @@ __global__ __launch_bounds__(NW * 64, KF * UPW > 32 ? 1 : 2) void talk_mfma_kern
     ls += __shfl_xor(ls, 16, 64);
     ls += __shfl_xor(ls, 32, 64);
     if (row_t[u] < 0) continue;
-    const int t = row_t[u], h = row_h[u];
-    if (part != nullptr) {  // split context: [NP][T][H][D] sums, then [NP][T][H][2] (max, sum)
-      const int64_t pr = ((int64_t)p * T + t) * H + h;
-      float* po = part + pr * D;
+    f32x4 y[2 * DH];
 #pragma unroll
-      for (int k = 0; k < 2 * DH; ++k)
-        if (16 * k + 4 * g4 < D) *reinterpret_cast<f32x4*>(po + 16 * k + 4 * g4) = o[u][k];
-      if (g4 == 0) {
-        float* ml = part + (int64_t)gridDim.z * T * HD + pr * 2;
-        ml[0] = m[u];
-        ml[1] = ls;
-      }
-      continue;
+    for (int k = 0; k < 2 * DH; ++k) y[k] = o[u][k];
+    talk_store<DH, true>(a, part, T, p, row_t[u], row_h[u], g4, m[u], ls, y);
+  }
+}
+
+// ---------------------------------------------------------------------------------------
+// MFMA form for many heads (up to 8 kv heads, 32 query heads): the fold above multiplies the QK work by G, so
+// here the raw scores are made once, exchanged through LDS and mixed by another MFMA:
+//
+//   wave w streams kv head c = w / (8 / G) alone: K fragments go from global memory to registers (the A operand
+//   of S^T = K q'^T) and from there to a wave-private LDS tile, which the PV product reads transposed;
+//   raw scores, r_j applied, go to LDS as fp32 S[token][key][head];
+//   M^T[key, h] = sum_g S^T[key, g] T[h, g] per (token, 16 keys): S splits exactly into three bf16 terms
+//   (24 bits), T is bf16 as it comes from the checkpoint;
+//   mixed scores return through LDS M[token, head][key]; softmax and O^T += V^T P^T as above.
+//
+// Two barriers per 32 keys; everything else is private to a wave.
+constexpr int TX_NW = 8;
+
+__device__ __forceinline__ u16x8 split_bf(float (&x)[8]) {  // leading bf16 of every x, x <- the remainder (exact)
+  u16x8 h;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) {
+    h[j] = f2bf(x[j]);
+    x[j] -= bf2f(h[j]);
+  }
+  return h;
+}
+
+struct TalkXchg {  // LDS layout (floats): S at 0, M at m_off, the waves' key tiles (bf16) at k_off
+  int hp, s_tok, m_tok, m_off, k_off, nwc, tb;  // (s_tok, m_tok: pitch of a token, padded against bank conflicts)
+};
+
+template <int DH, int UPW>
+__global__ __launch_bounds__(TX_NW * 64, 2) void talk_xchg_kernel(TalkArgs a, TalkXchg x, const int32_t* __restrict__ blk,
+                                                                  int nblk, int PS, float* __restrict__ part, int T) {
+  constexpr int STR = 32 * DH + 8, MS = TM_KEYS + 4;
+  extern __shared__ __attribute__((aligned(16))) float sm[];
+  const int tid = threadIdx.x, lane = tid & 63, c16 = lane & 15, g4 = lane >> 4;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int H = a.H, G = a.G, D = a.D, HD = H * D, rep = H / G;
+  const int bx = blk ? nblk - 1 - (int)blockIdx.x : (int)blockIdx.x;
+  const int tok0 = blk ? blk[bx] : bx, ntok = blk ? blk[nblk + bx] : 1;
+  const int hi = a.q_ctx[tok0 + ntok - 1];
+  if (hi <= 0) return;
+  const int lo = (a.q_ctx[tok0] - 1) / a.chunk * a.chunk;
+  const int p = blockIdx.z, s_lo = (lo & ~(TM_KEYS - 1)) + p * PS, s_hi = PS > 0 ? min(hi, s_lo + PS) : hi;
+  const int32_t* bt = a.bt + (int64_t)a.q_seq[tok0] * a.bt_stride;
+  const int pmask = (1 << a.page_log2) - 1;
+  constexpr float LOG2E = 1.44269504088896340736f;
+  const float sl2 = a.scale * LOG2E;
+  float* sS = sm;
+  float* sM = sm + x.m_off;
+  bf16_t* kt = reinterpret_cast<bf16_t*>(sm + x.k_off) + w * TM_KEYS * STR;
+  const int c = min(w / x.nwc, G - 1);
+  const bool streams = w / x.nwc < G && ((w % x.nwc) * UPW) * 16 < ntok * rep;  // this wave has rows
+
+  int khi[UPW], klo[UPW], row_t[UPW], row_h[UPW];
+  float sig[UPW], m[UPW], l[UPW];
+  u16x8 q[UPW][DH];
+  f32x4 o[UPW][2 * DH];
+#pragma unroll
+  for (int u = 0; u < UPW; ++u) {
+    const int row = ((w % x.nwc) * UPW + u) * 16 + c16;
+    const bool ok = streams && row < ntok * rep;
+    row_t[u] = ok ? row / rep : -1;
+    row_h[u] = c * rep + row % rep;
+    khi[u] = ok ? a.q_ctx[tok0 + row_t[u]] : 0;
+    klo[u] = ok ? (khi[u] - 1) / a.chunk * a.chunk : 0;
+    sig[u] = a.sigma[row_h[u]] * LOG2E;
+    m[u] = -INFINITY;
+    l[u] = 0.f;
+#pragma unroll
+    for (int t = 0; t < 2 * DH; ++t) o[u][t] = (f32x4)(0.f);
+#pragma unroll
+    for (int f = 0; f < DH; ++f) {
+      const int d = 32 * f + 8 * g4;
+      q[u][f] = ok && d < D ? *reinterpret_cast<const u16x8*>((const bf16_t*)a.qn + (int64_t)(tok0 + row_t[u]) * HD +
+                                                             row_h[u] * D + d)
+                            : (u16x8)(0);
     }
-    const float inv = 1.f / ls;
-    const bf16_t* gate = (const bf16_t*)a.z + (int64_t)t * a.zs + HD + G * D + h * D;
+  }
+  u16x8 tb[2];  // T^T: column h = 16 hb + c16, k = g = 8 g4 + j
 #pragma unroll
-    for (int k = 0; k < 2 * DH; ++k) {
-      const int d = 16 * k + 4 * g4;
-      if (d < D) {
-        float x[4];
+  for (int hb = 0; hb < 2; ++hb)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) x[r] = o[u][k][r] * inv / (1.f + __expf(-bf2f(gate[d + r])));
-        st_act_vec<4>((bf16_t*)a.out, t, h * D + d, HD, a.packed_mt, x);
+    for (int j = 0; j < 8; ++j) {
+      const int h = 16 * hb + c16, g = 8 * g4 + j;
+      tb[hb][j] = h < H && g < H ? f2bf(a.talk[h * H + g]) : (bf16_t)0;
+    }
+
+  u16x8 kf[2][DH];
+  f32x4 rr[2];
+  auto fetch = [&](int64_t pg, int s0) {
+    const int off = s0 & pmask;
+    const bf16_t* base = (const bf16_t*)a.cache + (((pg * G + c) << a.page_log2) + off) * D;
+    const float* rp = a.rk + (pg << a.page_log2) + off + 4 * g4;
+#pragma unroll
+    for (int sub = 0; sub < 2; ++sub) {
+      rr[sub] = *reinterpret_cast<const f32x4*>(rp + 16 * sub);
+#pragma unroll
+      for (int f = 0; f < DH; ++f)
+        kf[sub][f] = 32 * f + 8 * g4 < D
+                         ? *reinterpret_cast<const u16x8*>(base + (int64_t)(16 * sub + c16) * D + 32 * f + 8 * g4)
+                         : (u16x8)(0);
+    }
+  };
+  int64_t pg1 = 0;
+  if (s_lo < s_hi) {
+    if (streams) fetch(bt[s_lo >> a.page_log2], s_lo);
+    pg1 = bt[min(s_lo + TM_KEYS, s_hi - 1) >> a.page_log2];
+  }
+  for (int s0 = s_lo; s0 < s_hi; s0 += TM_KEYS) {
+    const int64_t pg2 = bt[min(s0 + 2 * TM_KEYS, s_hi - 1) >> a.page_log2];  // a tile ahead of its use
+    if (streams) {
+      if (s0 + TM_KEYS > s_hi) {  // rows past the context: stale bytes never meet a weight of 0
+#pragma unroll
+        for (int sub = 0; sub < 2; ++sub)
+#pragma unroll
+          for (int f = 0; f < DH; ++f)
+            if (s0 + 16 * sub + c16 >= s_hi) kf[sub][f] = (u16x8)(0);
+      }
+#pragma unroll
+      for (int sub = 0; sub < 2; ++sub) {
+#pragma unroll
+        for (int f = 0; f < DH; ++f)
+          *reinterpret_cast<u16x8*>(kt + (16 * sub + c16) * STR + 32 * f + 8 * g4) = kf[sub][f];
+#pragma unroll
+        for (int u = 0; u < UPW; ++u) {
+          f32x4 s = (f32x4)(0.f);
+#pragma unroll
+          for (int f = 0; f < DH; ++f) s = mfma_bf(kf[sub][f], q[u][f], s);
+          if (row_t[u] >= 0) {
+            float* sp = sS + row_t[u] * x.s_tok + (16 * sub + 4 * g4) * (x.hp + 4) + row_h[u];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) sp[r * (x.hp + 4)] = s[r] * (rr[sub][r] * sl2);
+          }
+        }
+      }
+      if (s0 + TM_KEYS < s_hi) fetch(pg1, s0 + TM_KEYS);
+      pg1 = pg2;
+    }
+    __syncthreads();
+    for (int fr = w; fr < 2 * ntok; fr += TX_NW) {  // (token, 16 keys)
+      const int t = fr >> 1, sub = fr & 1;
+      float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+      if (8 * g4 < x.hp) {
+        ld_vec<8>(sS + t * x.s_tok + (16 * sub + c16) * (x.hp + 4) + 8 * g4, v);
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+          if (8 * g4 + j >= H) v[j] = 0.f;  // (columns past H are never written)
+      }
+      const u16x8 v1 = split_bf(v), v2 = split_bf(v), v3 = split_bf(v);
+#pragma unroll
+      for (int hb = 0; hb < 2; ++hb) {
+        if (16 * hb >= H) break;
+        f32x4 y = mfma_bf(v3, tb[hb], (f32x4)(0.f));
+        y = mfma_bf(v2, tb[hb], y);
+        y = mfma_bf(v1, tb[hb], y);
+        if (16 * hb + c16 < H)
+          *reinterpret_cast<f32x4*>(sM + t * x.m_tok + (16 * hb + c16) * MS + 16 * sub + 4 * g4) = y;
+      }
+    }
+    __syncthreads();
+    if (!streams) continue;
+    u16x8 ph[UPW], pl[UPW];
+#pragma unroll
+    for (int u = 0; u < UPW; ++u) {
+      f32x4 st[2];
+      float lm = -INFINITY;
+      const float dj = (float)(s0 + 4 * g4 - (khi[u] - 1));  // key - query of this lane's first key
+      // every row of the wave sees the whole tile: no mask
+      const bool full = __all(row_t[u] < 0 || (s0 >= klo[u] && s0 + TM_KEYS <= min(khi[u], s_hi)));
+#pragma unroll
+      for (int sub = 0; sub < 2; ++sub) {
+        st[sub] = *reinterpret_cast<const f32x4*>(sM + max(row_t[u], 0) * x.m_tok + row_h[u] * MS + 16 * sub + 4 * g4);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          st[sub][r] = __builtin_fmaf(dj + (float)(16 * sub + r), sig[u], st[sub][r]);
+          if (!full) {
+            const int j = s0 + 16 * sub + 4 * g4 + r;
+            st[sub][r] = j >= klo[u] && j < khi[u] && j < s_hi ? st[sub][r] : -INFINITY;
+          }
+          lm = fmaxf(lm, st[sub][r]);
+        }
+      }
+      lm = fmaxf(lm, __shfl_xor(lm, 16, 64));
+      lm = fmaxf(lm, __shfl_xor(lm, 32, 64));
+      if (__any(lm > m[u] + TM_GROW)) {
+        const float mn = fmaxf(m[u], lm);
+        const float al = mn == -INFINITY ? 1.f : __builtin_amdgcn_exp2f(m[u] - mn);
+        l[u] *= al;
+#pragma unroll
+        for (int t = 0; t < 2 * DH; ++t) o[u][t] *= al;
+        m[u] = mn;
+      }
+      const float mu = m[u] == -INFINITY ? 0.f : m[u];
+#pragma unroll
+      for (int sub = 0; sub < 2; ++sub)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const float e = __builtin_amdgcn_exp2f(st[sub][r] - mu);
+          l[u] += e;
+          ph[u][4 * sub + r] = f2bf(e);
+          pl[u][4 * sub + r] = f2bf(e - bf2f(ph[u][4 * sub + r]));
+        }
+    }
+    const bf16_t* vb = kt + (4 * g4 + (c16 >> 2)) * STR + 4 * (c16 & 3);
+#pragma unroll
+    for (int t = 0; t < 2 * DH; ++t) {
+      const u16x4 v0 = lds_tr4(vb + 16 * t), v1 = lds_tr4(vb + 16 * STR + 16 * t);
+      const u16x8 va = {v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
+#pragma unroll
+      for (int u = 0; u < UPW; ++u) {
+        o[u][t] = mfma_bf(va, ph[u], o[u][t]);
+        o[u][t] = mfma_bf(va, pl[u], o[u][t]);
       }
     }
   }
+  if (!streams) return;
+#pragma unroll
+  for (int u = 0; u < UPW; ++u) {
+    float ls = l[u];
+    ls += __shfl_xor(ls, 16, 64);
+    ls += __shfl_xor(ls, 32, 64);
+    if (row_t[u] < 0) continue;
+    f32x4 y[2 * DH];
+#pragma unroll
+    for (int k = 0; k < 2 * DH; ++k) y[k] = o[u][k];
+    talk_store<DH, false>(a, part, T, p, tok0 + row_t[u], row_h[u], g4, m[u], ls, y);
+  }
+}
+
+static bool talk_xchg_geometry(int H, int G, int D, int upw, TalkXchg& x, size_t& lds) {
+  const int dh = D <= 32 ? 1 : D <= 64 ? 2 : 4;
+  if (D % 8 || D > 128 || H > 32 || G < 1 || G > TX_NW || TX_NW % G || H % G) return false;
+  const int rep = H / G;
+  x.nwc = TX_NW / G;
+  x.tb = 16 * x.nwc * upw / rep;
+  if (x.tb < 1) return false;
+  x.hp = (H + 7) / 8 * 8;
+  x.s_tok = TM_KEYS * (x.hp + 4) + 4;
+  x.m_off = x.tb * x.s_tok;
+  x.m_tok = H * (TM_KEYS + 4) + 16;
+  x.k_off = x.m_off + x.tb * x.m_tok;
+  lds = (size_t)x.k_off * 4 + (size_t)TX_NW * TM_KEYS * (32 * dh + 8) * 2;
+  return lds <= 160 * 1024;
 }
 
 __global__ __launch_bounds__(256) void talk_merge_kernel(TalkArgs a, const float* __restrict__ part, int T, int NP) {
@@ -418,16 +735,19 @@ static bool talk_geometry(int H, int G, int D, int& dh, int& kf, int& upw, int& 
   dh = D <= 32 ? 1 : D <= 64 ? 2 : 4;
   kf = G * dh <= 4 ? 4 : G * dh <= 8 ? 8 : G * dh <= 16 ? 16 : 32;
   if (G * dh > kf) return false;
+  const int rep = H / G;
+  for (int rb = 0; rb < 16; ++rb)  // a row block's tokens must fit the 32-row query tile
+    if (((rb * 16 + 15) / rep - rb * 16 / rep + 1) * rep > TM_KEYS) return false;
   // (the widest keys: one wave per SIMD with two units' queries in its 512 registers)
-  nw = kf == 16 ? 8 : 4;
-  upw = kf == 16 ? 1 : 2;
+  nw = kf >= 16 ? 8 : 4;
+  upw = kf >= 16 ? 1 : 2;
   return true;
 }
 
 template <int DH>
 static int launch_talk_mfma(const TalkArgs& a, const int32_t* blk, int nblk, int grid_x, int tokens, int PS, int NP,
                             float* part, int T, int kf, hipStream_t stream) {
-  const int nw = kf == 16 ? 8 : 4, upw = kf == 16 ? 1 : 2;
+  const int nw = kf >= 16 ? 8 : 4, upw = kf >= 16 ? 1 : 2;
   const int units = a.G * ((tokens * (a.H / a.G) + 15) / 16);
   const dim3 grid(grid_x, (units + nw * upw - 1) / (nw * upw), NP);
 #define MP_TM(KF_, UPW_, NW_)                                                                                     \
@@ -435,7 +755,7 @@ static int launch_talk_mfma(const TalkArgs& a, const int32_t* blk, int nblk, int
   if (kf == 4) MP_TM(4, 2, 4);
   else if (kf == 8) MP_TM(8, 2, 4);
   else if (kf == 16) MP_TM(16, 1, 8);
-  else MP_TM(32, 2, 4);
+  else MP_TM(32, 1, 8);
 #undef MP_TM
   return (int)hipGetLastError();
 }
@@ -471,8 +791,17 @@ extern "C" int mp_talk_prep(const void* z, int64_t zs, void* qn, const float* wq
   TalkArgs a{};
   a.z = z, a.zs = zs, a.qn = qn, a.wqk = wqk, a.cache = cache, a.rk = rk, a.slots = slots;
   a.H = H, a.G = G, a.D = D, a.page_log2 = page_log2, a.eps = eps;
-  if (f32) hipLaunchKernelGGL(talk_prep_kernel<float>, dim3(n), dim3(256), 0, stream, a);
-  else hipLaunchKernelGGL(talk_prep_kernel<bf16_t>, dim3(n), dim3(256), 0, stream, a);
+  const bool vec = D % 8 == 0 && zs % 8 == 0;
+  if (f32) {
+    if (vec) hipLaunchKernelGGL((talk_prep_kernel<float, 8, 256>), dim3(n), dim3(256), 0, stream, a);
+    else hipLaunchKernelGGL((talk_prep_kernel<float, 1, 256>), dim3(n), dim3(256), 0, stream, a);
+  } else if (!vec) {
+    hipLaunchKernelGGL((talk_prep_kernel<bf16_t, 1, 256>), dim3(n), dim3(256), 0, stream, a);
+  } else if (n <= 256 && (H + G) * D > 2048) {
+    hipLaunchKernelGGL((talk_prep_kernel<bf16_t, 8, 1024>), dim3(n), dim3(1024), 0, stream, a);
+  } else {
+    hipLaunchKernelGGL((talk_prep_kernel<bf16_t, 8, 256>), dim3(n), dim3(256), 0, stream, a);
+  }
   return (int)hipGetLastError();
 }
 
@@ -490,39 +819,76 @@ extern "C" int mp_talk_attention(const void* z, int64_t zs, const void* qn, cons
   return f32 ? launch_talk<float>(a, n, stream) : launch_talk<bf16_t>(a, n, stream);
 }
 
-// Tokens of a prompt's query block (0: the MFMA form does not cover the shape)
-extern "C" int mp_talk_block(int H, int G, int D) {
+namespace mp {
+constexpr int TX_UPW = 2;  // prompts: two 16-row blocks per wave (one in decode)
+static bool use_xchg(int H, int G, int D, int form, int upw, TalkXchg& x, size_t& lds) {
+  // the fold costs G x the QK work: it is kept where G is small and for the shapes the exchange does not take
+  const int work = H * G * (D <= 32 ? 1 : D <= 64 ? 2 : 4);
+  return form != 1 && (form == 2 || work >= (upw == 1 ? 256 : 512)) && talk_xchg_geometry(H, G, D, upw, x, lds);
+}
+}  // namespace mp
+
+// Tokens of a prompt's query block (0: the MFMA forms do not cover the shape).  form 0: by shape, 1: the folded
+// form, 2: the exchange form where it applies
+extern "C" int mp_talk_block(int H, int G, int D, int form) {
   using namespace mp;
+  TalkXchg x;
+  size_t lds;
+  if (use_xchg(H, G, D, form, TX_UPW, x, lds)) return x.tb;
   int dh, kf, upw, nw;
   if (!talk_geometry(H, G, D, dh, kf, upw, nw)) return 0;
-  const int rep = H / G, nrb = nw * upw / G > 1 ? nw * upw / G : 1;
+  const int rep = H / G;
+  int nrb = nw * upw / G > 1 ? nw * upw / G : 1;
+  nrb = nrb > 16 ? 16 : nrb;
   const int tb = 16 * nrb / rep;
   return tb < 1 ? 1 : tb > 64 ? 64 : tb;
 }
 
 // blk [2, nblk] (first token, tokens; tokens <= mp_talk_block): a prompt step; blk == null: n one-token rows, the
 // context in NP splits of PS keys (part: NP n (H D + 2 H) floats when NP > 1)
-extern "C" int mp_talk_mfma(const void* z, int64_t zs, const void* qn, const float* talk, const void* cache,
+extern "C" int mp_talk_mfma(const void* z, int64_t zs, const void* qn, const float* talk, const float* sigma,
+                            const void* cache,
                             const float* rk, const int32_t* bt, int bt_stride, const int32_t* q_seq,
                             const int32_t* q_ctx, void* out, int n, int H, int G, int D, int page_log2, int chunk,
                             float scale, const int32_t* blk, int nblk, int PS, int NP, float* part, int packed_mt,
-                            hipStream_t stream) {
+                            int form, hipStream_t stream) {
   using namespace mp;
   (void)hipGetLastError();
   if (n == 0) return 0;
   int dh, kf, upw, nw;
-  if (!talk_geometry(H, G, D, dh, kf, upw, nw) || page_log2 < 5) return -1;
+  TalkXchg x;
+  size_t lds;
+  // (decode rows: one row block per wave, so all of a kv head's query heads must fit it)
+  const bool xchg = use_xchg(H, G, D, form, blk ? TX_UPW : 1, x, lds) && mp_talk_block(H, G, D, form) > 0;
+  if (page_log2 < 5 || (!xchg && !talk_geometry(H, G, D, dh, kf, upw, nw))) return -1;
   if (NP > 1 && (PS <= 0 || PS % TM_KEYS || part == nullptr || blk != nullptr)) return -2;
   if (NP < 1 || NP > 65535) return -2;
   TalkArgs a{};
-  a.z = z, a.zs = zs, a.qn = (void*)qn, a.talk = talk, a.cache = (void*)cache, a.rk = (float*)rk, a.bt = bt;
+  a.z = z, a.zs = zs, a.qn = (void*)qn, a.talk = talk, a.sigma = sigma, a.cache = (void*)cache, a.rk = (float*)rk, a.bt = bt;
   a.bt_stride = bt_stride, a.q_seq = q_seq, a.q_ctx = q_ctx, a.out = out;
   a.H = H, a.G = G, a.D = D, a.page_log2 = page_log2, a.chunk = chunk, a.packed_mt = packed_mt, a.scale = scale;
-  const int gx = blk ? nblk : n, tokens = blk ? mp_talk_block(H, G, D) : 1;
+  const int gx = blk ? nblk : n, tokens = blk ? mp_talk_block(H, G, D, form) : 1;
   float* pp = NP > 1 ? part : nullptr;
   const int ps = NP > 1 ? PS : 0;
   int rc;
-  if (dh == 1) rc = launch_talk_mfma<1>(a, blk, nblk, gx, tokens, ps, NP, pp, n, kf, stream);
+  if (xchg) {
+    const dim3 grid(gx, 1, NP);
+#define MP_TX(DH_, UPW_)                                                                                              \
+  {                                                                                                                   \
+    (void)hipFuncSetAttribute((const void*)talk_xchg_kernel<DH_, UPW_>, hipFuncAttributeMaxDynamicSharedMemorySize,  \
+                              (int)lds);                                                                             \
+    hipLaunchKernelGGL((talk_xchg_kernel<DH_, UPW_>), grid, dim3(TX_NW * 64), lds, stream, a, x, blk, nblk, ps, pp, n); \
+  }
+    if (D <= 32) {
+      if (blk) MP_TX(1, TX_UPW) else MP_TX(1, 1)
+    } else if (D <= 64) {
+      if (blk) MP_TX(2, TX_UPW) else MP_TX(2, 1)
+    } else {
+      if (blk) MP_TX(4, TX_UPW) else MP_TX(4, 1)
+    }
+#undef MP_TX
+    rc = (int)hipGetLastError();
+  } else if (dh == 1) rc = launch_talk_mfma<1>(a, blk, nblk, gx, tokens, ps, NP, pp, n, kf, stream);
   else if (dh == 2) rc = launch_talk_mfma<2>(a, blk, nblk, gx, tokens, ps, NP, pp, n, kf, stream);
   else rc = launch_talk_mfma<4>(a, blk, nblk, gx, tokens, ps, NP, pp, n, kf, stream);
   if (rc || NP == 1) return rc;

@@ -25,11 +25,12 @@ int mp_hgrn2_chunk(const void* z, int64_t zs, const float* bias, const float* lo
                    const int32_t* q_seq, const int32_t* q_ctx, void* out, int H, int D, int V, float eps,
                    const int32_t* seg, int nseg, const int32_t* multi, int nm, float* ws, float* wdec, int packed_mt,
                    int f32, hipStream_t stream);
-int mp_talk_block(int H, int G, int D);
-int mp_talk_mfma(const void* z, int64_t zs, const void* qn, const float* talk, const void* cache, const float* rk,
+int mp_talk_block(int H, int G, int D, int form);
+int mp_talk_mfma(const void* z, int64_t zs, const void* qn, const float* talk, const float* sigma, const void* cache,
+                 const float* rk,
                  const int32_t* bt, int bt_stride, const int32_t* q_seq, const int32_t* q_ctx, void* out, int n, int H,
                  int G, int D, int page_log2, int chunk, float scale, const int32_t* blk, int nblk, int PS, int NP,
-                 float* part, int packed_mt, hipStream_t stream);
+                 float* part, int packed_mt, int form, hipStream_t stream);
 }
 
 namespace {
@@ -254,14 +255,17 @@ void talk_attention(const at::Tensor& z, const at::Tensor& qn, const at::Tensor&
                "talk_attention");
 }
 
-int64_t talk_block(int64_t H, int64_t G, int64_t D) { return mp_talk_block((int)H, (int)G, (int)D); }
+int64_t talk_block(int64_t H, int64_t G, int64_t D, int64_t form) {
+  return mp_talk_block((int)H, (int)G, (int)D, (int)form);
+}
 
 // blk: int32 [2, nblk] query blocks of a prompt step, or none: one-token rows, the context in ``parts`` splits of
 // ``part_size`` keys (``ws`` when parts > 1)
-void talk_mfma(const at::Tensor& z, const at::Tensor& qn, const at::Tensor& talk, const at::Tensor& cache,
+void talk_mfma(const at::Tensor& z, const at::Tensor& qn, const at::Tensor& talk, const at::Tensor& sigma,
+               const at::Tensor& cache,
                const at::Tensor& rk, const at::Tensor& bt, const at::Tensor& q_seq, const at::Tensor& q_ctx,
                at::Tensor& out, int64_t chunk, double scale, const c10::optional<at::Tensor>& blk, int64_t part_size,
-               int64_t parts, const c10::optional<at::Tensor>& ws, int64_t packed) {
+               int64_t parts, const c10::optional<at::Tensor>& ws, int64_t packed, int64_t form) {
   const TalkShape s = check_talk(z, qn, cache, rk);
   MP_CHECK(!s.f32, "talk_mfma is bf16");
   MP_CHECK(chunk >= 1 && chunk < (1ll << 31), "chunk");
@@ -282,10 +286,11 @@ void talk_mfma(const at::Tensor& z, const at::Tensor& qn, const at::Tensor& talk
     wp = ws->data_ptr<float>();
   }
   check_launch(mp_talk_mfma(z.data_ptr(), z.stride(0), qn.data_ptr(), f32_vec(talk, s.H * s.H, "talk"),
+                            f32_vec(sigma, s.H, "sigma"),
                             cache.data_ptr(), rk.data_ptr<float>(), bt.data_ptr<int32_t>(), bt.stride(0),
                             i32_vec(q_seq, s.T, "q_seq"), i32_vec(q_ctx, s.T, "q_ctx"), out.data_ptr(), s.T, s.H, s.G,
                             s.D, s.page_log2, (int)chunk, (float)scale, bp, nb, (int)part_size, (int)parts, wp, mt,
-                            cur_stream()),
+                            (int)form, cur_stream()),
                "talk_mfma");
 }
 
@@ -307,10 +312,11 @@ TORCH_LIBRARY_FRAGMENT(mpamd, m) {
   m.def(
       "hgrn2_chunk(Tensor z, Tensor bias, Tensor lower, Tensor norm, Tensor(a!) state, Tensor q_seq, Tensor q_ctx, "
       "Tensor(b!) out, float eps, Tensor seg, Tensor? multi, int slots, Tensor? ws, int packed) -> ()");
-  m.def("talk_block(int H, int G, int D) -> int", &talk_block);
+  m.def("talk_block(int H, int G, int D, int form) -> int", &talk_block);
   m.def(
-      "talk_mfma(Tensor z, Tensor qn, Tensor talk, Tensor cache, Tensor rk, Tensor bt, Tensor q_seq, Tensor q_ctx, "
-      "Tensor(a!) out, int chunk, float scale, Tensor? blk, int part_size, int parts, Tensor? ws, int packed) -> ()");
+      "talk_mfma(Tensor z, Tensor qn, Tensor talk, Tensor sigma, Tensor cache, Tensor rk, Tensor bt, Tensor q_seq, Tensor q_ctx, "
+      "Tensor(a!) out, int chunk, float scale, Tensor? blk, int part_size, int parts, Tensor? ws, int packed, "
+      "int form) -> ()");
 }
 
 TORCH_LIBRARY_IMPL(mpamd, CUDA, m) {

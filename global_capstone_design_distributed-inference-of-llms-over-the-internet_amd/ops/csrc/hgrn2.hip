@@ -17,7 +17,17 @@
 
 namespace mp {
 
-__device__ __forceinline__ float sigmoid_f(float x) { return 1.f / (1.f + expf(-x)); }
+// sigmoid(x) and sigmoid(-x) (its own value, not a difference from 1: a gate near 1 writes little, but exactly)
+__device__ __forceinline__ void sigmoid2(float x, float& s, float& c) {
+  const float e = __builtin_amdgcn_exp2f(fminf(-1.44269504088896340736f * x, 120.f));  // (finite: e s stays a number)
+  s = __builtin_amdgcn_rcpf(1.f + e);
+  c = e * s;
+}
+__device__ __forceinline__ float silu_f(float x) {
+  float s, c;
+  sigmoid2(x, s, c);
+  return x * s;
+}
 
 struct Hgrn2Args {
   const void* z;
@@ -33,9 +43,10 @@ struct Hgrn2Args {
 // seg == null: blockIdx.y is one row of one token (q_ctx 0: a padding row).  seg: [3, nseg] (tok0, ntok, ..)
 template <typename T, int VEC>
 __global__ __launch_bounds__(256) void hgrn2_scan_kernel(Hgrn2Args a, const int32_t* __restrict__ seg, int nseg) {
-  extern __shared__ float sm[];  // q[D], f[D], red[256 * VEC], red16[16]
+  constexpr int PRE = 16;
+  extern __shared__ float sm[];  // q[D], f[D], k[D], red[256 * VEC], red16[16]
   const int h = blockIdx.x, D = a.D, V = a.V, tid = threadIdx.x;
-  float *sq = sm, *sf = sm + D, *red = sm + 2 * D, *r16 = red + 256 * VEC;
+  float *sq = sm, *sf = sm + D, *sk = sm + 2 * D, *red = sm + 3 * D, *r16 = red + 256 * VEC;
   const int tok0 = seg ? seg[blockIdx.y] : (int)blockIdx.y;
   const int ntok = seg ? seg[nseg + blockIdx.y] : 1;
   const int ctx0 = a.q_ctx[tok0];
@@ -46,12 +57,21 @@ __global__ __launch_bounds__(256) void hgrn2_scan_kernel(Hgrn2Args a, const int3
   const bool act = g < ng;
   for (int t = tok0; t < tok0 + ntok; ++t) {
     const T* z = (const T*)a.z + (int64_t)t * a.zs;
+    // the first PRE state rows of this thread are on their way while the gates are made
+    float pre[PRE][VEC];
+    if (act) {
+#pragma unroll
+      for (int i = 0; i < PRE; ++i) ld_vec<VEC>(S + (int64_t)min(g + i * ng, D - 1) * V + c, pre[i]);
+    }
     const bool fresh = t == tok0 && ctx0 == 1;  // a sequence's first token: the slot's old state does not count
     for (int d = tid; d < D; d += 256) {
       const float zq = ld_f(z, h * D + d), zf = ld_f(z, a.H * D + h * D + d);
       const float lo = a.lower[h * D + d];
-      sq[d] = zq * sigmoid_f(zq);
-      sf[d] = lo + (1.f - lo) * sigmoid_f(zf + a.bias[h * D + d]);
+      float s, c;
+      sigmoid2(zf + a.bias[h * D + d], s, c);
+      sq[d] = silu_f(zq);
+      sf[d] = lo + (1.f - lo) * s;
+      sk[d] = (1.f - lo) * c;
     }
     __syncthreads();
     float o[VEC], v[VEC];
@@ -60,17 +80,23 @@ __global__ __launch_bounds__(256) void hgrn2_scan_kernel(Hgrn2Args a, const int3
     if (act) {
 #pragma unroll
       for (int j = 0; j < VEC; ++j) v[j] = ld_f(z, (int64_t)2 * a.H * D + h * V + c + j);
-#pragma unroll 8
-      for (int d = g; d < D; d += ng) {
-        float s[VEC];
-        ld_vec<VEC>(S + (int64_t)d * V + c, s);
-        const float f = sf[d], k = 1.f - f, qd = sq[d];
+      auto row = [&](int d, float (&s)[VEC]) {
+        const float f = sf[d], k = sk[d], qd = sq[d];
 #pragma unroll
         for (int j = 0; j < VEC; ++j) {
           s[j] = (fresh ? 0.f : f * s[j]) + k * v[j];
           o[j] += qd * s[j];
         }
         st_vec<VEC>(S + (int64_t)d * V + c, s);
+      };
+#pragma unroll
+      for (int i = 0; i < PRE; ++i)
+        if (g + i * ng < D) row(g + i * ng, pre[i]);
+#pragma unroll 4
+      for (int d = g + PRE * ng; d < D; d += ng) {
+        float s[VEC];
+        ld_vec<VEC>(S + (int64_t)d * V + c, s);
+        row(d, s);
       }
 #pragma unroll
       for (int j = 0; j < VEC; ++j) red[g * V + c + j] = o[j];
@@ -94,7 +120,7 @@ template <typename T>
 static int launch_scan(const Hgrn2Args& a, const int32_t* seg, int nseg, int n, hipStream_t stream) {
   const int vec = a.V % 4 == 0 ? 4 : 1;
   if (a.V / vec > 256) return -1;
-  const size_t lds = (2 * a.D + 256 * vec + 16) * sizeof(float);
+  const size_t lds = (3 * a.D + 256 * vec + 16) * sizeof(float);
   if (lds > 60000) return -1;
   if (vec == 4) hipLaunchKernelGGL((hgrn2_scan_kernel<T, 4>), dim3(a.H, n), dim3(256), lds, stream, a, seg, nseg);
   else hipLaunchKernelGGL((hgrn2_scan_kernel<T, 1>), dim3(a.H, n), dim3(256), lds, stream, a, seg, nseg);
@@ -114,7 +140,7 @@ static int launch_scan(const Hgrn2Args& a, const int32_t* seg, int nseg, int n, 
 // differ: with L = 8, 4, 2, 1 and m the start of the upper half of their common 2L-block,
 // P(j, i] = P(j, m - 1] P(m - 1, i], so ONE table M_L (row t = q_t P(m-1, t] in upper halves,
 // k_t P(t, m-1] in lower ones) gives all pairs of that level as the masked product M_L M_L^T; the four
-// waves take a level each.  All products run on v_mfma_f32_16x16x4_f32.
+// waves take a level each, and a quarter of the channels of the diagonal.  All products run on v_mfma_f32_16x16x4_f32.
 //
 // seg [4, nseg]: first token, tokens, source and target of the state (-1: the session's slot, s >= 0: slot s
 // of the workspace).  Long prompts are cut into segments so that all CUs work: a STATE pass leaves every
@@ -139,13 +165,13 @@ __global__ __launch_bounds__(256, DT * VT > 32 ? 1 : 2) void hgrn2_chunk_kernel(
                                                                                 int nseg, float* __restrict__ ws,
                                                                                 float* __restrict__ wdec) {
   constexpr int DC = DT * 16, DP = DC + 4;
-  constexpr int NTAB = STATE ? 1 : 6;
-  constexpr int TKE = STATE ? 0 : 5, TQB = 4;
-  constexpr bool SPLIT = !STATE && 2 * DC <= 256;  // two thread groups share the gate tables
+  constexpr int NC = DC > 128 ? 2 : 1;  // gate channels of a thread
+  constexpr int NTAB = STATE ? 1 : 7;
+  constexpr int TKE = STATE ? 0 : 5, TQB = 4, TQK = 6;
   __shared__ __attribute__((aligned(16))) float tab[NTAB][16][DP];
   __shared__ __attribute__((aligned(16))) float dec[DC];
   __shared__ __attribute__((aligned(16))) float ap[STATE ? 1 : 4][16][20];
-  __shared__ float dred[4][16], rss[4][16];
+  __shared__ float rss[4][16];
 
   const int h = blockIdx.x, sg = blockIdx.y, tid = threadIdx.x, lane = tid & 63;
   const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -171,108 +197,141 @@ __global__ __launch_bounds__(256, DT * VT > 32 ? 1 : 2) void hgrn2_chunk_kernel(
         }
   }
 
-  const int grp = tid / DC, ch = tid - grp * DC;  // gate channel of this thread
-  const bool gact = grp < (SPLIT ? 2 : 1), gch = gact && ch < D;
-  const float lo = gch ? a.lower[h * D + ch] : 0.f, bi = gch ? a.bias[h * D + ch] : 0.f;
-  const T* zq = (const T*)a.z + h * D + ch;
-  const T* zf = zq + HD;
-  const T* zv = (const T*)a.z + 2 * HD + (int64_t)h * V;
-  float run = 1.f;  // decay of the whole segment (STATE)
+  // gates: neighbouring lanes share a channel, the even one takes tokens 0..7 of a block, the odd one 8..15
+  const int half = tid & 1, ch0 = tid >> 1;
+  float lo[NC], bi[NC], run[NC];
+  unsigned oq[NC];  // element offset of the channel's first token of this half, from the block's first row
+#pragma unroll
+  for (int k = 0; k < NC; ++k) {
+    const int ch = ch0 + 128 * k;
+    lo[k] = ch < D ? a.lower[h * D + ch] : 0.f;
+    bi[k] = ch < D ? a.bias[h * D + ch] : 0.f;
+    run[k] = 1.f;  // decay of the whole segment (STATE)
+    oq[k] = (unsigned)(8 * half * a.zs + h * D + min(ch, D - 1));
+  }
+  unsigned ov[VT];
+  float nw[VT];
+#pragma unroll
+  for (int v = 0; v < VT; ++v) {
+    const int col = (w * VT + v) * 16 + c16;
+    ov[v] = (unsigned)(4 * g4 * a.zs + 2 * HD + h * V + min(col, V - 1));
+    nw[v] = !STATE && col < V ? a.norm[col] : 0.f;
+  }
 
-  T rq[16], rf[16];  // raw gate inputs of the next block, in flight across the MFMAs
+  T rq[NC][8], rf[NC][8];  // raw gate inputs of the next block, in flight across the MFMAs
   T rv[VT][4];
   auto fetch = [&](int b) {
+    const T* z0 = (const T*)a.z + (int64_t)(tok0 + b) * a.zs;
+    if (b + 16 <= ntok) {
 #pragma unroll
-    for (int t = 0; t < 16; ++t) {
-      const int64_t o = (int64_t)(tok0 + min(b + t, ntok - 1)) * a.zs;
-      if (gch) {
-        if constexpr (!STATE) rq[t] = zq[o];
-        rf[t] = zf[o];
+      for (int t = 0; t < 8; ++t) {
+        const T* zt = z0 + t * a.zs;  // (uniform base, 32-bit lane offset)
+#pragma unroll
+        for (int k = 0; k < NC; ++k) {
+          if constexpr (!STATE) rq[k][t] = zt[oq[k]];
+          rf[k][t] = zt[oq[k] + HD];
+        }
       }
-    }
-#pragma unroll
-    for (int v = 0; v < VT; ++v) {
-      const int col = (w * VT + v) * 16 + c16;
 #pragma unroll
       for (int s = 0; s < 4; ++s)
-        rv[v][s] = col < V ? zv[(int64_t)(tok0 + min(b + 4 * g4 + s, ntok - 1)) * a.zs + col] : (T)0;
+#pragma unroll
+        for (int v = 0; v < VT; ++v) rv[v][s] = (z0 + s * a.zs)[ov[v]];
+      return;
     }
+    const int last = ntok - 1 - b;  // the tail block: rows past the end re-read the last one, unused
+#pragma unroll
+    for (int t = 0; t < 8; ++t)
+#pragma unroll
+      for (int k = 0; k < NC; ++k) {
+        const T* zt = z0 + (int64_t)(min(8 * half + t, last) - 8 * half) * a.zs + oq[k];
+        if constexpr (!STATE) rq[k][t] = zt[0];
+        rf[k][t] = zt[HD];
+      }
+#pragma unroll
+    for (int s = 0; s < 4; ++s)
+#pragma unroll
+      for (int v = 0; v < VT; ++v) rv[v][s] = (z0 + (int64_t)(min(4 * g4 + s, last) - 4 * g4) * a.zs)[ov[v]];
   };
   fetch(0);
   for (int b = 0; b < ntok; b += 16) {
     const int nb = min(16, ntok - b);
-    if (gact) {
-      float q[16], f[16];
+    if (ch0 < DC) {
 #pragma unroll
-      for (int t = 0; t < 16; ++t) {
-        const bool ok = gch && t < nb;  // past the end: f = 1, k = 0, q = 0
+      for (int kk = 0; kk < NC; ++kk) {
+        const int ch = ch0 + 128 * kk;
+        float q[8], f[8], k[8];
+#pragma unroll
+        for (int t = 0; t < 8; ++t) {
+          const bool ok = ch < D && 8 * half + t < nb;  // past the end: f = 1, k = 0, q = 0
+          if constexpr (!STATE) q[t] = ok ? silu_f(to_f(rq[kk][t])) : 0.f;
+          float s, c;
+          sigmoid2(to_f(rf[kk][t]) + bi[kk], s, c);
+          f[t] = ok ? lo[kk] + (1.f - lo[kk]) * s : 1.f;
+          k[t] = ok ? (1.f - lo[kk]) * c : 0.f;
+        }
+        const int r0 = 8 * half;
         if constexpr (!STATE) {
-          const float x = to_f(rq[t]);
-          q[t] = ok ? x * sigmoid_f(x) : 0.f;
-        }
-        f[t] = ok ? lo + (1.f - lo) * sigmoid_f(to_f(rf[t]) + bi) : 1.f;
-      }
-      auto level = [&](int ti, auto lc) {
-        constexpr int L = decltype(lc)::value;
+          auto level = [&](int ti, auto lc) {
+            constexpr int L = decltype(lc)::value;
 #pragma unroll
-        for (int base = 0; base < 16; base += 2 * L) {
-          float p = 1.f;
+            for (int base = 0; base < 8; base += 2 * L) {
+              float p = 1.f;
 #pragma unroll
-          for (int t = base + L - 1; t >= base; --t) {
-            tab[ti][t][ch] = (1.f - f[t]) * p;
-            p *= f[t];
-          }
-          p = 1.f;
+              for (int t = base + L - 1; t >= base; --t) {
+                tab[ti][r0 + t][ch] = k[t] * p;
+                p *= f[t];
+              }
+              p = 1.f;
 #pragma unroll
-          for (int t = base + L; t < base + 2 * L; ++t) {
-            p *= f[t];
-            tab[ti][t][ch] = q[t] * p;
-          }
-        }
-      };
-      if constexpr (!STATE) {
-        if (grp == 0) {
-          level(0, std::integral_constant<int, 8>());
+              for (int t = base + L; t < base + 2 * L; ++t) {
+                p *= f[t];
+                tab[ti][r0 + t][ch] = q[t] * p;
+              }
+            }
+          };
           level(1, std::integral_constant<int, 4>());
           level(2, std::integral_constant<int, 2>());
-#pragma unroll
-          for (int t = 0; t < 16; ++t) {
-            const float x = wave_sum(q[t] * (1.f - f[t]));
-            if (lane == 0) dred[w][t] = x;
-          }
-        }
-      }
-      if (!SPLIT || grp == 1) {
-        if constexpr (!STATE) {
           level(3, std::integral_constant<int, 1>());
-          float p = 1.f;
 #pragma unroll
-          for (int t = 0; t < 16; ++t) {
-            p *= f[t];
-            tab[TQB][t][ch] = q[t] * p;
+          for (int t = 0; t < 8; ++t) tab[TQK][r0 + t][ch] = q[t] * k[t];
+        }
+        // products within the half: fw[t] = P up to and with t, bw[t] = P after t
+        float fw[8], bw[8];
+        fw[0] = f[0];
+        bw[7] = 1.f;
+#pragma unroll
+        for (int t = 1; t < 8; ++t) {
+          fw[t] = fw[t - 1] * f[t];
+          bw[7 - t] = bw[8 - t] * f[8 - t];
+        }
+        const float other = dppf<0xB1>(fw[7], 0.f);  // the neighbour lane's half
+        const float fp = half ? other : 1.f, bp = half ? 1.f : other;
+#pragma unroll
+        for (int t = 0; t < 8; ++t) {
+          const float x = k[t] * bw[t];
+          if constexpr (!STATE) {
+            const float y = q[t] * fw[t];
+            tab[0][r0 + t][ch] = half ? y : x;  // level 8: upper tokens forward, lower ones backward
+            tab[TQB][r0 + t][ch] = y * fp;
           }
+          tab[TKE][r0 + t][ch] = x * bp;
         }
-        float p = 1.f;
-#pragma unroll
-        for (int t = 15; t >= 0; --t) {
-          tab[TKE][t][ch] = (1.f - f[t]) * p;
-          p *= f[t];
-        }
-        dec[ch] = p;
-        run *= p;
+        const float all = fw[7] * other;
+        if (half == 0) dec[ch] = all;
+        run[kk] *= all;
       }
     }
     float vr[VT][4];
 #pragma unroll
     for (int v = 0; v < VT; ++v)
 #pragma unroll
-      for (int s = 0; s < 4; ++s) vr[v][s] = 4 * g4 + s < nb ? to_f(rv[v][s]) : 0.f;
+      for (int s = 0; s < 4; ++s) vr[v][s] = 4 * g4 + s < nb && (w * VT + v) * 16 + c16 < V ? to_f(rv[v][s]) : 0.f;
     if (b + 16 < ntok) fetch(b + 16);
     __syncthreads();
 
     f32x4 O[VT];
     if constexpr (!STATE) {
-      f32x4 sc = (f32x4)(0.f), sc2 = (f32x4)(0.f);
+      f32x4 sc = (f32x4)(0.f), dg = (f32x4)(0.f);
 #pragma unroll
       for (int v = 0; v < VT; ++v) O[v] = (f32x4)(0.f);
 #pragma unroll
@@ -281,10 +340,14 @@ __global__ __launch_bounds__(256, DT * VT > 32 ? 1 : 2) void hgrn2_chunk_kernel(
         const f32x4 y = *reinterpret_cast<const f32x4*>(&tab[TQB][c16][16 * m + 4 * g4]);
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          if (r & 1) sc2 = mfma_f32(x[r], x[r], sc2);
-          else sc = mfma_f32(x[r], x[r], sc);
+          sc = mfma_f32(x[r], x[r], sc);
 #pragma unroll
           for (int v = 0; v < VT; ++v) O[v] = mfma_f32(y[r], S[m][v][r], O[v]);
+        }
+        if ((m & 3) == w) {  // the diagonal q_i . k_i: a quarter of the channels each
+          const f32x4 u = *reinterpret_cast<const f32x4*>(&tab[TQK][c16][16 * m + 4 * g4]);
+#pragma unroll
+          for (int r = 0; r < 4; ++r) dg = mfma_f32(u[r], 1.f, dg);
         }
       }
       const int lw = 3 - w;
@@ -292,22 +355,16 @@ __global__ __launch_bounds__(256, DT * VT > 32 ? 1 : 2) void hgrn2_chunk_kernel(
       for (int r = 0; r < 4; ++r) {
         const int i = 4 * g4 + r, j = c16;
         const bool pair = (i >> (lw + 1)) == (j >> (lw + 1)) && ((i >> lw) & 1) && !((j >> lw) & 1);
-        ap[w][i][j] = pair ? sc[r] + sc2[r] : 0.f;
+        ap[w][i][j] = pair ? sc[r] : i == j ? dg[r] : 0.f;
       }
       __syncthreads();
       f32x4 A = (f32x4)(0.f);
 #pragma unroll
       for (int k = 0; k < 4; ++k) A += *reinterpret_cast<const f32x4*>(&ap[k][c16][4 * g4]);
-      float dg = 0.f;
 #pragma unroll
-      for (int k = 0; k < 4; ++k)
-        if (k * 64 < DC) dg += dred[k][c16];
+      for (int s = 0; s < 4; ++s)
 #pragma unroll
-      for (int s = 0; s < 4; ++s) {
-        const float x = 4 * g4 + s == c16 ? dg : A[s];
-#pragma unroll
-        for (int v = 0; v < VT; ++v) O[v] = mfma_f32(x, vr[v][s], O[v]);
-      }
+        for (int v = 0; v < VT; ++v) O[v] = mfma_f32(A[s], vr[v][s], O[v]);
     }
 #pragma unroll
     for (int m = 0; m < DT; ++m) {
@@ -334,16 +391,18 @@ __global__ __launch_bounds__(256, DT * VT > 32 ? 1 : 2) void hgrn2_chunk_kernel(
     }
     __syncthreads();
     if constexpr (!STATE) {
+      const float inv_v = 1.f / (float)V;
+      T* ob = (T*)a.out + (int64_t)(tok0 + b) * a.H * V + h * V;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int i = 4 * g4 + r;
-        const float ss = rss[0][i] + rss[1][i] + rss[2][i] + rss[3][i];
-        const float sc = 1.f / sqrtf(ss / (float)V + a.eps);
+        const float sc = rsqrtf((rss[0][i] + rss[1][i] + rss[2][i] + rss[3][i]) * inv_v + a.eps);
 #pragma unroll
         for (int v = 0; v < VT; ++v) {
           const int col = (w * VT + v) * 16 + c16;
-          if (i < nb && col < V)
-            st_act((T*)a.out, tok0 + b + i, h * V + col, a.H * V, a.packed_mt, O[v][r] * sc * a.norm[col]);
+          if (i >= nb || col >= V) continue;
+          if (a.packed_mt > 0) st_act((T*)a.out, tok0 + b + i, h * V + col, a.H * V, a.packed_mt, O[v][r] * sc * nw[v]);
+          else from_f(O[v][r] * sc * nw[v], ob[(unsigned)(i * a.H * V + col)]);
         }
       }
     }
@@ -359,7 +418,11 @@ __global__ __launch_bounds__(256, DT * VT > 32 ? 1 : 2) void hgrn2_chunk_kernel(
         const int d = 16 * m + 4 * g4 + r, col = (w * VT + v) * 16 + c16;
         if (d < D && col < V) sp[(int64_t)d * V + col] = S[m][v][r];
       }
-  if (STATE && grp == 0 && ch < D) wdec[((int64_t)dst * a.H + h) * D + ch] = run;
+  if (STATE && half == 0) {
+#pragma unroll
+    for (int k = 0; k < NC; ++k)
+      if (ch0 + 128 * k < D) wdec[((int64_t)dst * a.H + h) * D + ch0 + 128 * k] = run[k];
+  }
 }
 
 // multi [4, nm]: first slot, slots, first token, unused.  Slot i holds segment i-1's contribution (i > 0):

@@ -42,8 +42,8 @@ __global__ __launch_bounds__(256) void embed_pos_kernel(const int64_t* __restric
 }
 
 // SRC: 0 = rows of T, 1 = S fp32 slabs, 2 = no y: out rows = rms(res[rows]) * w (rows_norm)
-template <typename T, int VEC, int MAXC, int SRC>
-__global__ __launch_bounds__(256) void residual_norm_kernel(const T* __restrict__ y, int64_t ys,
+template <typename T, int VEC, int MAXC, int SRC, int NT>
+__global__ __launch_bounds__(NT) void residual_norm_kernel(const T* __restrict__ y, int64_t ys,
                                                             const float* __restrict__ part, int S, int64_t slab,
                                                             float* __restrict__ res, const float* __restrict__ w,
                                                             T* __restrict__ xb, const int32_t* __restrict__ rows,
@@ -56,7 +56,7 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(const T* __restrict_
   float ss = 0.f;
 #pragma unroll
   for (int k = 0; k < MAXC; ++k) {
-    const int c = min((int)threadIdx.x + 256 * k, nch - 1) * VEC;
+    const int c = min((int)threadIdx.x + NT * k, nch - 1) * VEC;
     ld_vec<VEC>(res + (int64_t)row * W + c, r[k]);
     ld_vec<VEC>(w + c, g[k]);
     if constexpr (SRC == 0) {
@@ -64,11 +64,15 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(const T* __restrict_
     } else if constexpr (SRC == 1) {
 #pragma unroll
       for (int j = 0; j < VEC; ++j) v[k][j] = 0.f;
-      for (int s = 0; s < S; ++s) {
-        float p[VEC];
-        ld_vec<VEC>(part + s * slab + (int64_t)row * ys + c, p);
+      for (int s = 0; s < S; s += 4) {  // four slabs' loads in flight, added in slab order
+        float p[4][VEC];
 #pragma unroll
-        for (int j = 0; j < VEC; ++j) v[k][j] += p[j];
+        for (int i = 0; i < 4; ++i) ld_vec<VEC>(part + min(s + i, S - 1) * slab + (int64_t)row * ys + c, p[i]);
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (s + i < S)
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) v[k][j] += p[i][j];
       }
     } else {
 #pragma unroll
@@ -77,13 +81,13 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(const T* __restrict_
   }
 #pragma unroll
   for (int k = 0; k < MAXC; ++k)
-    if ((int)threadIdx.x + 256 * k < nch)
+    if ((int)threadIdx.x + NT * k < nch)
 #pragma unroll
       for (int j = 0; j < VEC; ++j) ss += v[k][j] * v[k][j];
   const float sc = 1.f / sqrtf(block_sum(ss, red) / (float)W + eps);
 #pragma unroll
   for (int k = 0; k < MAXC; ++k) {
-    const int ch = threadIdx.x + 256 * k;
+    const int ch = threadIdx.x + NT * k;
     if (ch >= nch) continue;
     float o[VEC];
 #pragma unroll
@@ -116,20 +120,23 @@ template <typename T, int SRC>
 static int launch_residual_norm(const void* y, int64_t ys, const float* part, int S, int64_t slab, float* res,
                                 const float* w, void* xb, const int32_t* rows, int n, int W, float eps, int packed_mt,
                                 hipStream_t stream) {
-#define MP_RN(VEC_, MAXC_)                                                                                           \
-  hipLaunchKernelGGL((residual_norm_kernel<T, VEC_, MAXC_, SRC>), dim3(n), dim3(256), 0, stream, (const T*)y, ys,     \
+#define MP_RN(VEC_, MAXC_, NT_)                                                                                     \
+  hipLaunchKernelGGL((residual_norm_kernel<T, VEC_, MAXC_, SRC, NT_>), dim3(n), dim3(NT_), 0, stream, (const T*)y, ys, \
                      part, S, slab, res, w, (T*)xb, rows, W, eps, packed_mt)
   if (W % 4 == 0 && (SRC == 2 || ys % 4 == 0)) {
-    const int per = (W / 4 + 255) / 256;
-    if (per <= 1) MP_RN(4, 1);
-    else if (per <= 2) MP_RN(4, 2);
-    else if (per <= 4) MP_RN(4, 4);
-    else if (per <= 8) MP_RN(4, 8);
-    else if (per <= 16) MP_RN(4, 16);
+    const int ch = W / 4;
+    if (n <= 256 && ch > 256 && ch <= 2048) {  // few rows: latency is what there is to save
+      if (ch <= 1024) MP_RN(4, 1, 1024);
+      else MP_RN(4, 2, 1024);
+    } else if (ch <= 256) MP_RN(4, 1, 256);
+    else if (ch <= 512) MP_RN(4, 2, 256);
+    else if (ch <= 1024) MP_RN(4, 4, 256);
+    else if (ch <= 2048) MP_RN(4, 8, 256);
+    else if (ch <= 4096) MP_RN(4, 16, 256);
     else return -1;
   } else {
     if (W > 16 * 256) return -1;
-    MP_RN(1, 16);
+    MP_RN(1, 16, 256);
   }
 #undef MP_RN
   return (int)hipGetLastError();

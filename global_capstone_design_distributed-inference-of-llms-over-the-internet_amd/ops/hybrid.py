@@ -128,9 +128,23 @@ def talk_prep(z, wqk, qn, cache, rk, slots, eps):
     torch.ops.mpamd.talk_prep(z, wqk, qn, cache, rk, slots, float(eps))
 
 
+# MFMA form of the attention: 0 = by shape, 1 = mixing folded into the queries, 2 = scores exchanged through LDS
+TALK_FORM = 0
+
+
 def talk_block(H: int, G: int, D: int) -> int:
-    """Tokens of a prompt's query block on the MFMA form (0: shape not covered)."""
-    return int(torch.ops.mpamd.talk_block(int(H), int(G), int(D)))
+    """Tokens of a prompt's query block on the MFMA forms (0: shape not covered)."""
+    return int(torch.ops.mpamd.talk_block(int(H), int(G), int(D), TALK_FORM))
+
+
+def talk_slopes(H: int) -> torch.Tensor:
+    """fp32 [H]: the heads' distance slopes, 2^(-8 (h + 1) / H)."""
+    return torch.exp2(-8.0 * torch.arange(1, H + 1, dtype=torch.float64) / H).float()
+
+
+def talk_sigma(talk: torch.Tensor) -> torch.Tensor:
+    """fp32 [H]: the slopes after the heads' mixing."""
+    return (talk.double() @ talk_slopes(talk.shape[0]).to(talk.device).double()).float()
 
 
 def talk_blocks(ntoks, tokens: int):
@@ -153,17 +167,17 @@ def talk_parts(rows: int, H: int, G: int, D: int, span: int, n_cu: int = 256):
     return ps, -(-span // ps)
 
 
-def talk_attention(z, qn, talk, cache, rk, table, q_seq, q_ctx, out, chunk, scale, packed=False, blocks=None,
-                   parts=None, ws=None):
+def talk_attention(z, qn, talk, cache, rk, table, q_seq, q_ctx, out, chunk, scale, packed=False, sigma=None,
+                   blocks=None, parts=None, ws=None):
     """Chunked talking-heads attention with the output gate of ``z``.  On the GPU the MFMA form runs when
     ``blocks`` (prompt steps: ``talk_blocks`` on the device) or ``parts`` (decode: ``talk_parts``, ``ws`` fp32
-    scratch) is given, else the form for any shape and element type."""
+    scratch) is given, with ``sigma`` = talk @ slopes (``talk_sigma``), else the form for any shape and element type."""
     if not _native(z):
         return _put(out, rh.talk_attention(z, qn, talk, cache, rk, table, q_seq, q_ctx, chunk, scale), packed)
     if blocks is not None or parts is not None:
         ps, np_ = parts if blocks is None else (0, 1)
-        torch.ops.mpamd.talk_mfma(z, qn, talk, cache, rk, table, q_seq, q_ctx, out, int(chunk), float(scale), blocks,
-                                  int(ps), int(np_), ws, int(packed))
+        torch.ops.mpamd.talk_mfma(z, qn, talk, sigma, cache, rk, table, q_seq, q_ctx, out, int(chunk), float(scale), blocks,
+                                  int(ps), int(np_), ws, int(packed), TALK_FORM)
         return out
     torch.ops.mpamd.talk_attention(z, qn, talk, cache, rk, table, q_seq, q_ctx, out, int(chunk), float(scale),
                                    int(packed))

@@ -141,7 +141,7 @@ class HybridStage:
                     if parts[1] > 1:
                         ws = e("talk_ws", (parts[1] * T * sp.heads * (sp.dim + 2),), torch.float32)
                 hops.talk_attention(z, qn, lay.talk, kv, rk, table, q_seq, q_ctx, o, sp.chunk, sp.scale, packed=pko,
-                                    blocks=blocks, parts=parts, ws=ws)
+                                    sigma=lay.sigma, blocks=blocks, parts=parts, ws=ws)
             if sp.ff:
                 pku = self._packed(T, lay.w_up, lay.w_up_p)
                 xu = self._act(e, "xb", T, W, pku)
