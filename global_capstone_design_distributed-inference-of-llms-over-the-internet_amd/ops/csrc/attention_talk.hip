@@ -283,7 +283,8 @@ __global__ __launch_bounds__(NW * 64, KF * UPW > 32 ? 1 : 2) void talk_mfma_kern
     uc[u] = c;
     row_t[u] = ok ? tok0 + row / rep : -1;
     row_h[u] = c * rep + row % rep;
-    khi[u] = ok ? a.q_ctx[row_t[u]] : 0;
+    const int ctx = a.q_ctx[ok ? row_t[u] : tok0];
+    khi[u] = ok ? ctx : 0;
     klo[u] = ok ? (khi[u] - 1) / a.chunk * a.chunk : 0;
     m[u] = -INFINITY;
     l[u] = 0.f;
@@ -301,16 +302,21 @@ __global__ __launch_bounds__(NW * 64, KF * UPW > 32 ? 1 : 2) void talk_mfma_kern
     for (int rb = 0; rb < nrb; ++rb) {
       const int t0 = rb * 16 / rep, t1 = min((rb * 16 + 15) / rep, ntok - 1), nr = (t1 - t0 + 1) * rep;
       if (rb > 0) __syncthreads();
+      // (clamped, unconditional loads: all in flight together)
+      u16x8 qreg[CPT];
+#pragma unroll
+      for (int k = 0; k < CPT; ++k) {
+        const int x = tid + NT * k, kr = min(x / (WC / 8), nr - 1), col = (x % (WC / 8)) * 8;
+        const int c = min(col / DP, G - 1), d = min(col % DP, D - 8);
+        qreg[k] = *reinterpret_cast<const u16x8*>((const bf16_t*)a.qn + (int64_t)(tok0 + t0 + kr / rep) * HD +
+                                                  (c * rep + kr % rep) * D + d);
+      }
 #pragma unroll
       for (int k = 0; k < CPT; ++k) {
         const int x = tid + NT * k, kr = x / (WC / 8), col = (x % (WC / 8)) * 8;
-        const int c = col / DP, d = col % DP;
         if (kr < TM_KEYS)
           *reinterpret_cast<u16x8*>(qt + kr * STR + col) =
-              kr < nr && c < G && d < D
-                  ? *reinterpret_cast<const u16x8*>((const bf16_t*)a.qn + (int64_t)(tok0 + t0 + kr / rep) * HD +
-                                                    (c * rep + kr % rep) * D + d)
-                  : (u16x8)(0);
+              kr < nr && col / DP < G && col % DP < D ? qreg[k] : (u16x8)(0);
       }
       __syncthreads();
 #pragma unroll
@@ -322,13 +328,12 @@ __global__ __launch_bounds__(NW * 64, KF * UPW > 32 ? 1 : 2) void talk_mfma_kern
         const bf16_t* qb = qt + (8 * g4 + (c16 >> 2)) * STR + 4 * (c16 & 3);
 #pragma unroll
         for (int c = 0; c < KF / DH; ++c) {
-          u16x8 tb = (u16x8)(0);
-          if (c < G && row_t[u] >= 0) {
+          u16x8 tb;
 #pragma unroll
-            for (int j = 0; j < 8; ++j) {
-              const int g = 8 * g4 + j - mt * rep;
-              if (g >= 0 && g < rep) tb[j] = f2bf(tr[c * rep + g]);
-            }
+          for (int j = 0; j < 8; ++j) {
+            const int g = 8 * g4 + j - mt * rep;
+            const float t = tr[min(c, G - 1) * rep + min(max(g, 0), rep - 1)];
+            tb[j] = c < G && row_t[u] >= 0 && g >= 0 && g < rep ? f2bf(t) : (bf16_t)0;
           }
 #pragma unroll
           for (int f = c * DH; f < (c + 1) * DH; ++f) {
@@ -357,12 +362,12 @@ __global__ __launch_bounds__(NW * 64, KF * UPW > 32 ? 1 : 2) void talk_mfma_kern
     const bf16_t* base = (const bf16_t*)a.cache + ((pg * G) << a.page_log2) * D + (int64_t)(s0 & pmask) * D;
 #pragma unroll
     for (int k = 0; k < CPT; ++k) {
-      const int x = tid + NT * k, key = x / (WC / 8), col = (x % (WC / 8)) * 8;
-      const int c = col / DP, d = col % DP;
-      const bool ok = key < TM_KEYS && c < G && d < D && s0 + key < s_hi;
-      kreg[k] = ok ? *reinterpret_cast<const u16x8*>(base + (((int64_t)c << a.page_log2) + key) * D + d) : (u16x8)(0);
+      // clamped, unconditional: a column past the head meets a 0 in u, a row past the context is masked
+      const int x = tid + NT * k, key = min(x / (WC / 8), s_hi - 1 - s0), col = (x % (WC / 8)) * 8;
+      const int c = min(col / DP, G - 1), d = min(col % DP, D - 8);
+      kreg[k] = *reinterpret_cast<const u16x8*>(base + (((int64_t)c << a.page_log2) + min(key, TM_KEYS - 1)) * D + d);
     }
-    if (tid < TM_KEYS) rreg = s0 + tid < s_hi ? a.rk[(pg << a.page_log2) + (s0 & pmask) + tid] : 0.f;
+    rreg = a.rk[(pg << a.page_log2) + (s0 & pmask) + min(min(tid, TM_KEYS - 1), s_hi - 1 - s0)];
   };
   auto stash = [&](int buf) {
 #pragma unroll
@@ -523,7 +528,8 @@ __global__ __launch_bounds__(TX_NW * 64, 2) void talk_xchg_kernel(TalkArgs a, Ta
     const bool ok = streams && row < ntok * rep;
     row_t[u] = ok ? row / rep : -1;
     row_h[u] = c * rep + row % rep;
-    khi[u] = ok ? a.q_ctx[tok0 + row_t[u]] : 0;
+    const int ctx = a.q_ctx[tok0 + max(row_t[u], 0)];
+    khi[u] = ok ? ctx : 0;
     klo[u] = ok ? (khi[u] - 1) / a.chunk * a.chunk : 0;
     sig[u] = a.sigma[row_h[u]] * LOG2E;
     m[u] = -INFINITY;
@@ -533,9 +539,9 @@ __global__ __launch_bounds__(TX_NW * 64, 2) void talk_xchg_kernel(TalkArgs a, Ta
 #pragma unroll
     for (int f = 0; f < DH; ++f) {
       const int d = 32 * f + 8 * g4;
-      q[u][f] = ok && d < D ? *reinterpret_cast<const u16x8*>((const bf16_t*)a.qn + (int64_t)(tok0 + row_t[u]) * HD +
-                                                             row_h[u] * D + d)
-                            : (u16x8)(0);
+      const u16x8 v = *reinterpret_cast<const u16x8*>((const bf16_t*)a.qn + (int64_t)(tok0 + max(row_t[u], 0)) * HD +
+                                                      row_h[u] * D + min(d, D - 8));
+      q[u][f] = ok && d < D ? v : (u16x8)(0);
     }
   }
   u16x8 tb[2];  // T^T: column h = 16 hb + c16, k = g = 8 g4 + j
@@ -544,7 +550,8 @@ __global__ __launch_bounds__(TX_NW * 64, 2) void talk_xchg_kernel(TalkArgs a, Ta
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
       const int h = 16 * hb + c16, g = 8 * g4 + j;
-      tb[hb][j] = h < H && g < H ? f2bf(a.talk[h * H + g]) : (bf16_t)0;
+      const float t = a.talk[min(h, H - 1) * H + min(g, H - 1)];
+      tb[hb][j] = h < H && g < H ? f2bf(t) : (bf16_t)0;
     }
 
   u16x8 kf[2][DH];
@@ -558,9 +565,9 @@ __global__ __launch_bounds__(TX_NW * 64, 2) void talk_xchg_kernel(TalkArgs a, Ta
       rr[sub] = *reinterpret_cast<const f32x4*>(rp + 16 * sub);
 #pragma unroll
       for (int f = 0; f < DH; ++f)
-        kf[sub][f] = 32 * f + 8 * g4 < D
-                         ? *reinterpret_cast<const u16x8*>(base + (int64_t)(16 * sub + c16) * D + 32 * f + 8 * g4)
-                         : (u16x8)(0);
+        // clamped: a column past the head meets a 0 in q', a row past the context is masked
+        kf[sub][f] = *reinterpret_cast<const u16x8*>(base + min(16 * sub + c16, s_hi - 1 - s0) * D +
+                                                     min(32 * f + 8 * g4, D - 8));
     }
   };
   int64_t pg1 = 0;
@@ -571,13 +578,6 @@ __global__ __launch_bounds__(TX_NW * 64, 2) void talk_xchg_kernel(TalkArgs a, Ta
   for (int s0 = s_lo; s0 < s_hi; s0 += TM_KEYS) {
     const int64_t pg2 = bt[min(s0 + 2 * TM_KEYS, s_hi - 1) >> a.page_log2];  // a tile ahead of its use
     if (streams) {
-      if (s0 + TM_KEYS > s_hi) {  // rows past the context: stale bytes never meet a weight of 0
-#pragma unroll
-        for (int sub = 0; sub < 2; ++sub)
-#pragma unroll
-          for (int f = 0; f < DH; ++f)
-            if (s0 + 16 * sub + c16 >= s_hi) kf[sub][f] = (u16x8)(0);
-      }
 #pragma unroll
       for (int sub = 0; sub < 2; ++sub) {
 #pragma unroll
@@ -599,49 +599,54 @@ __global__ __launch_bounds__(TX_NW * 64, 2) void talk_xchg_kernel(TalkArgs a, Ta
       pg1 = pg2;
     }
     __syncthreads();
-    for (int fr = w; fr < 2 * ntok; fr += TX_NW) {  // (token, 16 keys)
-      const int t = fr >> 1, sub = fr & 1;
-      float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-      if (8 * g4 < x.hp) {
-        ld_vec<8>(sS + t * x.s_tok + (16 * sub + c16) * (x.hp + 4) + 8 * g4, v);
+    for (int f0 = w; f0 < 2 * ntok; f0 += 2 * TX_NW) {  // (token, 16 keys), two at a time
+      float v[2][8];
 #pragma unroll
-        for (int j = 0; j < 8; ++j)
-          if (8 * g4 + j >= H) v[j] = 0.f;  // (columns past H are never written)
+      for (int i = 0; i < 2; ++i) {
+        const int fr = min(f0 + i * TX_NW, 2 * ntok - 1);
+        ld_vec<8>(sS + (fr >> 1) * x.s_tok + (16 * (fr & 1) + c16) * (x.hp + 4) + min(8 * g4, x.hp - 8), v[i]);
       }
-      const u16x8 v1 = split_bf(v), v2 = split_bf(v), v3 = split_bf(v);
 #pragma unroll
-      for (int hb = 0; hb < 2; ++hb) {
-        if (16 * hb >= H) break;
-        f32x4 y = mfma_bf(v3, tb[hb], (f32x4)(0.f));
-        y = mfma_bf(v2, tb[hb], y);
-        y = mfma_bf(v1, tb[hb], y);
-        if (16 * hb + c16 < H)
-          *reinterpret_cast<f32x4*>(sM + t * x.m_tok + (16 * hb + c16) * MS + 16 * sub + 4 * g4) = y;
+      for (int i = 0; i < 2; ++i)
+#pragma unroll
+        for (int j = 0; j < 8; ++j) v[i][j] = 8 * g4 + j < H ? v[i][j] : 0.f;  // (columns past H are never written)
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        const int fr = f0 + i * TX_NW;
+        const u16x8 v1 = split_bf(v[i]), v2 = split_bf(v[i]), v3 = split_bf(v[i]);
+#pragma unroll
+        for (int hb = 0; hb < 2; ++hb) {
+          f32x4 y = mfma_bf(v3, tb[hb], (f32x4)(0.f));
+          y = mfma_bf(v2, tb[hb], y);
+          y = mfma_bf(v1, tb[hb], y);
+          if (16 * hb + c16 < H && fr < 2 * ntok)
+            *reinterpret_cast<f32x4*>(sM + (fr >> 1) * x.m_tok + (16 * hb + c16) * MS + 16 * (fr & 1) + 4 * g4) = y;
+        }
       }
     }
     __syncthreads();
     if (!streams) continue;
     u16x8 ph[UPW], pl[UPW];
+    f32x4 sc[UPW][2];
+#pragma unroll
+    for (int u = 0; u < UPW; ++u)
+#pragma unroll
+      for (int sub = 0; sub < 2; ++sub)
+        sc[u][sub] = *reinterpret_cast<const f32x4*>(sM + max(row_t[u], 0) * x.m_tok + row_h[u] * MS + 16 * sub + 4 * g4);
 #pragma unroll
     for (int u = 0; u < UPW; ++u) {
-      f32x4 st[2];
+      f32x4 (&st)[2] = sc[u];
       float lm = -INFINITY;
       const float dj = (float)(s0 + 4 * g4 - (khi[u] - 1));  // key - query of this lane's first key
-      // every row of the wave sees the whole tile: no mask
-      const bool full = __all(row_t[u] < 0 || (s0 >= klo[u] && s0 + TM_KEYS <= min(khi[u], s_hi)));
+      const int k0 = klo[u] - s0 - 4 * g4, k1 = min(khi[u], s_hi) - s0 - 4 * g4;
 #pragma unroll
-      for (int sub = 0; sub < 2; ++sub) {
-        st[sub] = *reinterpret_cast<const f32x4*>(sM + max(row_t[u], 0) * x.m_tok + row_h[u] * MS + 16 * sub + 4 * g4);
+      for (int sub = 0; sub < 2; ++sub)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          st[sub][r] = __builtin_fmaf(dj + (float)(16 * sub + r), sig[u], st[sub][r]);
-          if (!full) {
-            const int j = s0 + 16 * sub + 4 * g4 + r;
-            st[sub][r] = j >= klo[u] && j < khi[u] && j < s_hi ? st[sub][r] : -INFINITY;
-          }
+          const float y = __builtin_fmaf(dj + (float)(16 * sub + r), sig[u], st[sub][r]);
+          st[sub][r] = 16 * sub + r >= k0 && 16 * sub + r < k1 ? y : -INFINITY;
           lm = fmaxf(lm, st[sub][r]);
         }
-      }
       lm = fmaxf(lm, __shfl_xor(lm, 16, 64));
       lm = fmaxf(lm, __shfl_xor(lm, 32, 64));
       if (__any(lm > m[u] + TM_GROW)) {
