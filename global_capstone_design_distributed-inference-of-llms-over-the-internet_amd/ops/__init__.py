@@ -205,11 +205,11 @@ def _covered(name: str, M: int, N: int, K: int, epilogue: int) -> bool:
     if name == "rw":  # widths the launcher does not build fall back to the other kernels by itself
         return True
     if name == "rwk":  # split-K ring + reduce launch: plain / residual / fused-norm producer epilogues
-        return epilogue != 1 and N % 2048 == 0
+        return epilogue not in (1, 4) and N % 2048 == 0
     if name == "rwki":  # the same with an in-launch combine (M <= 64)
-        return epilogue != 1 and N % 2048 == 0 and M <= 64
+        return epilogue not in (1, 4) and N % 2048 == 0 and M <= 64
     if name == "rwr":  # row-split ring: 2 or 4 row tiles split over a workgroup pair
-        return epilogue != 1 and N % 2048 == 0 and (M + 15) // 16 in (2, 4)
+        return epilogue not in (1, 4) and N % 2048 == 0 and (M + 15) // 16 in (2, 4)
     if name == "t2d":  # row blocks x column groups: more than 64 rows only (picked by linear itself)
         return 64 < M <= 256 and t2d_ok(M, N, K, epilogue, epilogue == 1)
     return _lds_covered(name, M, N, K, epilogue)
@@ -393,26 +393,26 @@ def autotune_gemm(shapes, device, ms=(4, 16, 32, 48, 64), iters: int = 24, round
                     _SK_CHOICE[(_m_bucket(M), N, K, int(epi))] = "pk"
                     continue
                 xp = pack_act(torch.randn(M, K, device=device).to(torch.bfloat16))
-                y = torch.empty(packed_numel(M, ncols) if epi == 1 else M * ncols, dtype=torch.bfloat16,
+                y = torch.empty(packed_numel(M, ncols) if epi in (1, 4) else M * ncols, dtype=torch.bfloat16,
                                 device=device)
                 res = torch.zeros(M, N, dtype=torch.bfloat16, device=device) if epi in (2, 3) else None
                 extra = {}
                 if epi == 3:  # fused-norm producer: packed copy + per-row sum of squares
                     extra = dict(ap_out=torch.zeros(packed_numel(M, N), dtype=torch.bfloat16, device=device),
                                  ss_out=norm_stats_buffer(device)[0], ss_zero=norm_stats_buffer(device)[0])
-                out = y if epi == 1 else (res if epi == 3 else y.view(M, ncols))
+                out = y if epi in (1, 4) else (res if epi == 3 else y.view(M, ncols))
                 t = {k: float("inf") for k in cands}
                 for _ in range(rounds):
                     for mode in cands:
                         _GEMM_SK = mode
                         for i in range(2):
                             linear(xp, None, out=out, epilogue=epi, residual=res, wp=wps[i % copies], a_rows=M,
-                                   out_packed=epi == 1, **extra)
+                                   out_packed=epi in (1, 4), **extra)
                         e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
                         e0.record()
                         for i in range(iters):
                             linear(xp, None, out=out, epilogue=epi, residual=res, wp=wps[i % copies], a_rows=M,
-                                   out_packed=epi == 1, **extra)
+                                   out_packed=epi in (1, 4), **extra)
                         e1.record()
                         e1.synchronize()
                         t[mode] = min(t[mode], e0.elapsed_time(e1) / iters)
@@ -426,12 +426,12 @@ def autotune_gemm(shapes, device, ms=(4, 16, 32, 48, 64), iters: int = 24, round
                         _GEMM_SK = mode
                         for i in range(2):
                             linear(xp, None, out=out, epilogue=epi, residual=res, wp=wps[i % copies], a_rows=M,
-                                   out_packed=epi == 1, **extra)
+                                   out_packed=epi in (1, 4), **extra)
                         e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
                         e0.record()
                         for i in range(iters):
                             linear(xp, None, out=out, epilogue=epi, residual=res, wp=wps[i % copies], a_rows=M,
-                                   out_packed=epi == 1, **extra)
+                                   out_packed=epi in (1, 4), **extra)
                         e1.record()
                         e1.synchronize()
                         tr[mode] = min(tr[mode], e0.elapsed_time(e1) / iters)
@@ -865,9 +865,18 @@ def add(a, b, out=None):
     return out
 
 
+def _aligned_rows(x):
+    """``x`` [R, V] with the 16-byte row pitch the logits kernels read (a copy only for other pitches)."""
+    if x.stride(0) % 8 == 0 and x.stride(1) == 1:
+        return x
+    rows = torch.empty(x.shape[0], -(-x.shape[1] // 8) * 8, dtype=x.dtype, device=x.device)
+    return rows[:, : x.shape[1]].copy_(x)
+
+
 def argmax(logits, out=None):
     if not _native(logits):
         return ref.argmax(logits, out=out)
+    logits = _aligned_rows(logits)
     if out is None:
         out = torch.empty(logits.shape[0], dtype=torch.long, device=logits.device)
     torch.ops.mpamd.argmax(logits, out)
@@ -884,6 +893,9 @@ def sample(logits, temps, top_ps, top_ks, rep_pens, recent, recent_len, seeds, w
             ref.push_history(recent, recent_len, out)
         return out
     R, V = logits.shape
+    if logits.dtype == torch.float32:  # a 32-bit model: the sampling kernel reads bf16 rows
+        logits = _aligned_rows(logits.to(torch.bfloat16))
+    logits = _aligned_rows(logits)
     if out is None:
         out = torch.empty(R, dtype=torch.long, device=logits.device)
     if workspace is None:
@@ -945,6 +957,8 @@ def t2d_ok(M: int, N: int, K: int, epilogue: int = 0, out_packed: bool = False) 
 def native_gemm_ok(M: int, N: int, K: int, epilogue: int = 0, out_packed: bool = False) -> bool:
     if not (K % 128 == 0 and N % (32 if epilogue == 1 else 16) == 0):
         return False
+    if epilogue == 4:  # (squared relu: the kernels of up to 64 rows)
+        return 0 < M <= 64
     if 64 < M <= wide_rows():
         return wide_gemm_ok(M, N, K, epilogue, out_packed)
     return 0 < M <= 64
@@ -967,11 +981,11 @@ def linear(x, w, out=None, epilogue=0, residual=None, policy=None, wp=None, a_ro
            gate=None, ss_in=None, eps=0.0, ap_out=None, ss_out=None, ss_zero=None):
     """y = epilogue(x @ w^T). epilogue 0: none; 1: SwiGLU (16-row interleaved gate/up w); 2: + residual;
     3: fused-norm producer (``residual`` updated in place to bf16(y + residual), also written packed to
-    ``ap_out``, per-row sum of squares added to ``ss_out``; ``ss_zero`` is cleared).
+    ``ap_out``, per-row sum of squares added to ``ss_out``; ``ss_zero`` is cleared); 4: max(y, 0)^2.
 
     ``wp`` is the packed copy of ``w`` (``pack_weight``); the native decode GEMM needs it.
     ``a_rows`` (int) says ``x`` is a PACKED activation holding that many rows (decode path);
-    ``out_packed`` (SwiGLU only) writes the output packed for the next GEMM.
+    ``out_packed`` (epilogues 1 and 4) writes the output packed for the next GEMM.
     ``ss_in`` (fused-norm consumer): ``x`` is the raw residual stream, ``w`` has the RMSNorm weight
     folded into its columns, and row r of the product is scaled by rsqrt(ss_in[r] / K + eps).
     """
@@ -1026,6 +1040,8 @@ def linear(x, w, out=None, epilogue=0, residual=None, policy=None, wp=None, a_ro
         return swiglu(y, out=out)
     if epilogue == 2:
         return add(y, residual, out=out)
+    if epilogue == 4:
+        return hybrid.relu2(y, torch.empty_like(y) if out is None else out)
     if out is not None:
         out.copy_(y)
         return out

@@ -27,7 +27,7 @@ int mp_paged_attention(const void* q, int64_t q_stride, const void* kc, const vo
 int mp_embedding(const int64_t* ids, const void* table, void* out, int T, int H, int64_t vocab, hipStream_t stream);
 int mp_swiglu(const void* gu, void* out, int64_t T, int F, hipStream_t stream);
 int mp_add(const void* a, const void* b, void* y, int64_t n, hipStream_t stream);
-int mp_argmax(const void* logits, int64_t stride, int R, int V, int64_t* out, hipStream_t stream);
+int mp_argmax(const void* logits, int64_t stride, int R, int V, int64_t* out, int f32, hipStream_t stream);
 int mp_sample(const void* logits, int64_t stride, int R, int V, const float* temps, const float* top_ps,
               const int32_t* top_ks, const float* rep_pens, int32_t* recent, int recent_stride, int32_t* recent_len,
               const int64_t* seeds, float* ws, int64_t* out, int update, hipStream_t stream);
@@ -475,11 +475,13 @@ void add(const at::Tensor& a, const at::Tensor& b, at::Tensor& y) {
 }
 
 void argmax(const at::Tensor& logits, at::Tensor& out) {
-  check_bf16_cuda(logits, "logits");
+  const bool f32 = logits.scalar_type() == at::kFloat;
+  if (!f32) check_bf16_cuda(logits, "logits");
+  MP_CHECK(logits.is_cuda(), "logits must be on the GPU");
   check_rows(logits, "logits");
   MP_CHECK(out.scalar_type() == at::kLong && out.numel() == logits.size(0), "out int64 [R]");
   check_launch(mp_argmax(logits.data_ptr(), logits.stride(0), logits.size(0), logits.size(1),
-                         out.data_ptr<int64_t>(), cur_stream()),
+                         out.data_ptr<int64_t>(), f32, cur_stream()),
                "argmax");
 }
 
@@ -530,7 +532,7 @@ void gemm(const at::Tensor& x, const at::Tensor& wp, at::Tensor& y, const c10::o
   }
   const int ncols = epilogue == 1 ? N / 2 : N;
   if (opk) {
-    MP_CHECK(epilogue == 1 && y.is_contiguous() && y.numel() >= packed_numel(M, ncols), "packed y");
+    MP_CHECK((epilogue == 1 || epilogue == 4) && y.is_contiguous() && y.numel() >= packed_numel(M, ncols), "packed y");
   } else {
     check_rows(y, "y");
     MP_CHECK(y.size(0) == M && y.size(1) == ncols, "y shape");
@@ -544,8 +546,8 @@ void gemm(const at::Tensor& x, const at::Tensor& wp, at::Tensor& y, const c10::o
     rp = residual->data_ptr();
     rs = residual->stride(0);
   }
-  MP_CHECK(epilogue < 2 || rp != nullptr, "residual epilogue needs residual");
-  MP_CHECK(epilogue >= 0 && epilogue <= 3, "epilogue");
+  MP_CHECK(epilogue < 2 || epilogue == 4 || rp != nullptr, "residual epilogue needs residual");
+  MP_CHECK(epilogue >= 0 && epilogue <= 4, "epilogue");
   void* app = nullptr;
   if (ap.has_value()) {
     check_bf16_cuda(*ap, "ap");
@@ -613,7 +615,7 @@ void gemm_w8(const at::Tensor& x, const at::Tensor& wq, const at::Tensor& wsc, a
   MP_CHECK(x.is_contiguous() && x.numel() >= packed_numel(M, K), "packed x too small");
   const int ncols = epilogue == 1 ? N / 2 : N;
   if (opk) {
-    MP_CHECK(epilogue == 1 && y.is_contiguous() && y.numel() >= packed_numel(M, ncols), "packed y");
+    MP_CHECK((epilogue == 1 || epilogue == 4) && y.is_contiguous() && y.numel() >= packed_numel(M, ncols), "packed y");
   } else {
     check_rows(y, "y");
     MP_CHECK(y.size(0) == M && y.size(1) == ncols, "y shape");
@@ -774,7 +776,7 @@ void gemm_fp8(const at::Tensor& a8, const at::Tensor& as, const at::Tensor& wq, 
   check_bf16_cuda(y, "y");
   const int ncols = epilogue == 1 ? N / 2 : N;
   if (out_packed) {
-    MP_CHECK(epilogue == 1 && y.is_contiguous() && y.numel() >= packed_numel(M, ncols), "packed y");
+    MP_CHECK((epilogue == 1 || epilogue == 4) && y.is_contiguous() && y.numel() >= packed_numel(M, ncols), "packed y");
   } else {
     check_rows(y, "y");
     MP_CHECK(y.size(0) == M && y.size(1) == ncols, "y shape");

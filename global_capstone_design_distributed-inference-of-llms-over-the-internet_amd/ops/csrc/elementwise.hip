@@ -4,6 +4,7 @@
 // temperature <= 0 branch of reference src/rpc_handler.py:331-336).
 // All bf16 traffic is 16 B per lane.
 #include "common.h"
+#include "act_io.h"
 
 namespace mp {
 
@@ -55,25 +56,27 @@ __global__ __launch_bounds__(256) void add_kernel(const bf16_t* __restrict__ a, 
   }
 }
 
-// First maximum of each row (torch.argmax tie rule). logits bf16 [R, V], row stride given.
-__global__ __launch_bounds__(256) void argmax_kernel(const bf16_t* __restrict__ logits, int64_t stride, int V,
+// First maximum of each row (torch.argmax tie rule). logits bf16 or fp32 [R, V], row stride given.
+template <typename T>
+__global__ __launch_bounds__(256) void argmax_kernel(const T* __restrict__ logits, int64_t stride, int V,
                                                      int64_t* __restrict__ out) {
   __shared__ float sv[4];
   __shared__ int si[4];
-  const bf16_t* row = logits + (int64_t)blockIdx.x * stride;
+  const T* row = logits + (int64_t)blockIdx.x * stride;
   float best = -INFINITY;
   int bi = 0x7fffffff;
   const int nv = V / 8;
   for (int c = threadIdx.x; c < nv; c += blockDim.x) {
-    const u16x8 v = *reinterpret_cast<const u16x8*>(row + c * 8);
+    float v[8];
+    ld_vec<8>(row + c * 8, v);
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
-      const float f = bf2f(v[j]);
+      const float f = v[j];
       if (f > best) { best = f; bi = c * 8 + j; }
     }
   }
   for (int i = nv * 8 + threadIdx.x; i < V; i += blockDim.x) {
-    const float f = bf2f(row[i]);
+    const float f = to_f(row[i]);
     if (f > best || (f == best && i < bi)) { best = f; bi = i; }
   }
 #pragma unroll
@@ -131,10 +134,11 @@ extern "C" int mp_add(const void* a, const void* b, void* y, int64_t n, hipStrea
   return (int)hipGetLastError();
 }
 
-extern "C" int mp_argmax(const void* logits, int64_t stride, int R, int V, int64_t* out, hipStream_t stream) {
+extern "C" int mp_argmax(const void* logits, int64_t stride, int R, int V, int64_t* out, int f32, hipStream_t stream) {
   using namespace mp;
   if (R == 0) return 0;
   if (stride % 8) return -1;
-  hipLaunchKernelGGL(argmax_kernel, dim3(R), dim3(256), 0, stream, (const bf16_t*)logits, stride, V, out);
+  if (f32) hipLaunchKernelGGL(argmax_kernel<float>, dim3(R), dim3(256), 0, stream, (const float*)logits, stride, V, out);
+  else hipLaunchKernelGGL(argmax_kernel<bf16_t>, dim3(R), dim3(256), 0, stream, (const bf16_t*)logits, stride, V, out);
   return (int)hipGetLastError();
 }

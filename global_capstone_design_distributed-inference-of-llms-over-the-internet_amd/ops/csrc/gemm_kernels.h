@@ -27,7 +27,8 @@
 //     output N/2 columns); 2 = y = bf16(bf16(acc) + residual); 3 = the residual-stream
 //     producer of the fused-norm decode path: r = bf16(bf16(acc) + residual) stored in place
 //     (row-major) AND packed (the next GEMM's A operand), and sum(r^2) per row accumulated
-//     into an fp32 vector with atomics (16 lanes reduce a row first).
+//     into an fp32 vector with atomics (16 lanes reduce a row first); 4 = max(acc, 0)^2,
+//     row-major or packed (M <= 64).
 //   * RMSNorm folded away (EpiArgs::ss_in): the consumer GEMMs (qkv, gate/up) read the RAW
 //     residual stream with the norm weight folded into their packed weight columns
 //     (W' = W diag(g)), and scale accumulator row r by rsqrt(ss[r] / H + eps) in the
@@ -387,6 +388,9 @@ __global__ __launch_bounds__(512) void gemm_packed_kernel(const bf16_t* __restri
         float v = s * row_scale<EPI>(ep, rs_lds, row);
         if constexpr (EPI == 3) {
           epi3_store(ep, y, y_stride, row, col, v, c, rpre[j]);
+        } else if constexpr (EPI == 4) {
+          v = fmaxf(v, 0.f);
+          y[OPK ? apk_off(row, col, MT) : (int64_t)row * y_stride + col] = f2bf(v * v);
         } else {
           if constexpr (EPI == 2) v = round_bf(v) + bf2f(res[(int64_t)row * res_stride + col]);
           y[(int64_t)row * y_stride + col] = f2bf(v);
@@ -416,6 +420,9 @@ static int launch_gemm(const void* x, int64_t xs, const void* w, void* y, int64_
   if (epi == 1) {
     if (ntiles % 2) return -2;
     if (opk) { MP_APK(2, 1, true) } else { MP_APK(2, 1, false) }
+  } else if (epi == 4) {
+    if (two) { if (opk) { MP_APK(2, 4, true) } else { MP_APK(2, 4, false) } }
+    else { if (opk) { MP_APK(1, 4, true) } else { MP_APK(1, 4, false) } }
   } else if (opk) {
     return -3;  // packed output only for the SwiGLU epilogue (it feeds the down projection)
   } else if (epi == 2) {
@@ -493,6 +500,9 @@ __device__ __forceinline__ void tile_epilogue(int mt, int tile, const f32x4& v, 
     } else if constexpr (EPI == 3) {
       const bf16_t rv = rpv != nullptr ? (*rpv)[r] : res[(int64_t)row * rs + tile * 16 + c];
       epi3_store(ep, y, ys, row, tile * 16 + c, v[r] * sc, c, rv);
+    } else if constexpr (EPI == 4) {
+      const float o = fmaxf(v[r], 0.f);
+      y[OPK ? apk_off(row, tile * 16 + c, ep.mt_out) : (int64_t)row * ys + tile * 16 + c] = f2bf(o * o);
     } else {
       const int col = tile * 16 + c;
       float o = v[r] * sc;
@@ -646,7 +656,7 @@ static int launch_gemm_lds_cfg(const void* x, const void* w, void* y, int64_t ys
     const int ntiles = N / 16;
     const bool opk = flags & 2;
     if (ntiles % (CH * NT) || K % 64) return 1;
-    if (opk && epi != 1) return -3;
+    if (opk && epi != 1 && epi != 4) return -3;
     const dim3 grid(ntiles / (CH * NT));
 #define MP_LL(EPI_, OPK_)                                                                                      \
   hipLaunchKernelGGL((gemm_lds_kernel<MT, NT, CH, EPI_, OPK_>), grid, dim3(512), 0, stream, (const bf16_t*)x,   \
@@ -657,6 +667,8 @@ static int launch_gemm_lds_cfg(const void* x, const void* w, void* y, int64_t ys
       } else {
         return 1;
       }
+    } else if (epi == 4) {
+      if (opk) { MP_LL(4, true); } else { MP_LL(4, false); }
     } else if (epi == 2) {
       MP_LL(2, false);
     } else if (epi == 3) {
@@ -929,6 +941,8 @@ static int launch_gemm_sk_cfg(const void* x, void* y, int64_t ys, const void* w,
     } else {
       return 1;
     }
+  } else if (epi == 4) {
+    if (opk) { MP_SK(4, true); } else { MP_SK(4, false); }
   } else if (opk) {
     return -3;
   } else if (epi == 2) {
@@ -1216,6 +1230,8 @@ static int launch_gemm_rw_cfg(const void* x, const void* w, void* y, int64_t ys,
     } else {
       return 1;
     }
+  } else if (epi == 4) {
+    if (opk) { MP_RW(4, true); } else { MP_RW(4, false); }
   } else if (opk) {
     return -3;
   } else if (epi == 2) {

@@ -217,6 +217,8 @@ def linear(x, w, out=None, epilogue=0, residual=None, ss_in=None, inv_k=0.0, eps
         y = swiglu(y)
     elif epilogue == 2:
         y = add(y, residual)
+    elif epilogue == 4:
+        y = torch.clamp(y.float(), min=0).pow(2).to(x.dtype)
     if out is not None:
         out.copy_(y)
         return out

@@ -56,8 +56,8 @@ class HybridStage:
         """Decode-GEMM kernel choices for this stage's shapes (none while tuning is off)."""
         if ops.autotune_mode() == "off":
             return
-        shapes = {(w.shape[0], w.shape[1], 0) for lay in self.ex.w.layers
-                  for w, wp in ((getattr(lay, n), getattr(lay, n + "_p")) for n in lay.GEMMS) if wp is not None}
+        shapes = {(getattr(lay, n).shape[0], getattr(lay, n).shape[1], 4 if n == "w_up" else 0)
+                  for lay in self.ex.w.layers for n in lay.GEMMS if getattr(lay, n + "_p") is not None}
         if self.ex.w.lm_head_p is not None:
             shapes.add((self.ex.w.lm_head.shape[0], self.W, 0))
         # (small products are launch-bound whatever kernel runs them)
@@ -146,9 +146,13 @@ class HybridStage:
                 pku = self._packed(T, lay.w_up, lay.w_up_p)
                 xu = self._act(e, "xb", T, W, pku)
                 self._add(o, lay.w_o, lay.w_o_p, pko, T, res, lay.n1, xu, pku, e)
-                u = self._mm(xu, lay.w_up, lay.w_up_p, T, pku, e(f"u{sp.ff}", (T, sp.ff)))
                 pkd = self._packed(T, lay.w_down, lay.w_down_p)
-                a = hops.relu2(u, self._act(e, "act", T, sp.ff, pkd), packed=pkd)
+                a = self._act(e, "act", T, sp.ff, pkd)
+                if pku and ops.native_gemm_ok(T, sp.ff, W, 4):  # the squared relu in the GEMM's epilogue
+                    ops.linear(xu, None, wp=lay.w_up_p, a_rows=T, out=a, epilogue=4, out_packed=pkd)
+                else:
+                    u = self._mm(xu, lay.w_up, lay.w_up_p, T, pku, e(f"u{sp.ff}", (T, sp.ff)))
+                    hops.relu2(u, a, packed=pkd)
                 pk, xb = entry(i + 1)
                 self._add(a, lay.w_down, lay.w_down_p, pkd, T, res, lay.n2, xb, pk, e)
             else:
