@@ -66,8 +66,10 @@ def kv_cache_bytes_per_block(cfg: ModelConfig, tokens: Optional[int] = None, dty
 
 def auto_num_blocks(cfg: ModelConfig, free_bytes: Optional[int] = None, dtype=torch.bfloat16,
                     quant_type: Optional[str] = None, attn_cache_tokens: Optional[int] = None,
-                    reserve_bytes: int = 2 << 30, device=None, total_blocks: Optional[int] = None) -> int:
-    """How many blocks this GPU can serve: floor((free - reserve) / (block + KV per block)).
+                    reserve_bytes: int = 2 << 30, device=None, total_blocks: Optional[int] = None,
+                    max_sessions: int = 256) -> int:
+    """How many blocks this GPU can serve: floor((free - reserve) / (block + KV per block)), with a recurrent
+    state slot per session where the model has them.
 
     ``free_bytes`` defaults to the device's free memory (``torch.cuda.mem_get_info``); on a
     CPU host the caller must pass it.  The result is clamped to [1, total_blocks].
@@ -78,6 +80,7 @@ def auto_num_blocks(cfg: ModelConfig, free_bytes: Optional[int] = None, dtype=to
         free_bytes = torch.cuda.mem_get_info(torch.device(device))[0]
     per_block = get_block_size(cfg, "memory", dtype, quant_type) + kv_cache_bytes_per_block(cfg, attn_cache_tokens,
                                                                                            dtype)
+    per_block += max_sessions * cfg.state_bytes_per_session_per_layer()
     n = int((int(free_bytes) - int(reserve_bytes)) // per_block)
     total = cfg.num_hidden_layers if total_blocks is None else int(total_blocks)
     return max(1, min(n, total))

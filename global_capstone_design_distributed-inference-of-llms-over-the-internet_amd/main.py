@@ -659,7 +659,8 @@ def run_stage_server_with_load_balancing(args, device, cuts: List[int], stop: Op
     if args.num_blocks is None and getattr(args, "auto_num_blocks", False) and device.type == "cuda":
         from .block_utils import auto_num_blocks
 
-        num_blocks = auto_num_blocks(cfg, dtype=dtype, device=device, total_blocks=total - min_block)
+        num_blocks = auto_num_blocks(cfg, dtype=dtype, device=device, total_blocks=total - min_block,
+                                     max_sessions=args.max_sessions)
         logger.info(f"auto num_blocks = {num_blocks}")
     else:
         num_blocks = args.num_blocks or 4

@@ -7,7 +7,7 @@ resolves to, in order:
 
 1. a local directory holding a Hugging Face ``config.json`` (weights are then read
    from its safetensors shards, see ``models.weights``);
-2. a built-in preset for the configurations named in BASELINE.json / SURVEY.md
+2. a built-in preset for the configurations of the reference's benchmarks
    (Llama-2-7B, Llama-3(.1)-8B, Llama-3-70B, GPT-2) plus tiny test models.
 
 The GPU box has no network, so presets are used with synthetic random-init weights.
@@ -132,7 +132,7 @@ class ModelConfig:
         return self.num_attention_heads // self.num_key_value_heads
 
     def layer_param_bytes(self, bytes_per_param: float = 2.0) -> int:
-        """Weights of one decoder block (survey V11 `get_block_size`)."""
+        """Weights of one decoder block (upstream `get_block_size`)."""
         H, F = self.hidden_size, self.intermediate_size
         if self.hybrid:  # layers differ: the mean
             n = sum(sp.param_count(H) for sp in self.layers) / max(len(self.layers), 1)
@@ -148,6 +148,12 @@ class ModelConfig:
             n = sum(sp.kv_elems * bytes_per_elt + 4 for sp in self.layers if not sp.recurrent)
             return -(-n // max(len(self.layers), 1))
         return 2 * self.kv_dim * bytes_per_elt
+
+    def state_bytes_per_session_per_layer(self) -> int:
+        """fp32 recurrent state of one session, averaged over the layers (0 for the uniform families)."""
+        if not self.hybrid:
+            return 0
+        return -(-sum(sp.state_elems * 4 for sp in self.layers) // max(len(self.layers), 1))
 
     def validate(self) -> None:
         if self.model_type not in SUPPORTED_TYPES:

@@ -363,6 +363,8 @@ def _hybrid_layer(spec: LayerSpec, width: int, get, device, dtype) -> HybridLaye
     raw = {}
     for name, shape in _hybrid_names(spec, width).items():
         t = get(name)
+        if shape == () and t.numel() == 1:
+            t = t.reshape(())
         if tuple(t.shape) != shape:
             raise ValueError(f"{name}: shape {tuple(t.shape)}, expected {shape}")
         raw[name] = t.to(device)

@@ -34,7 +34,7 @@ from ..models.weights import LlamaLayer, StageWeights, interleave_gate_up, split
 
 
 def check_tp(cfg: ModelConfig, tp: int) -> None:
-    if cfg.model_type == "gpt2":
+    if cfg.model_type == "gpt2" or cfg.hybrid:
         raise ValueError("tensor parallelism supports the LLaMA-family (llama/mistral/mixtral) blocks only")
     for name, v in (("num_attention_heads", cfg.num_attention_heads), ("num_key_value_heads", cfg.num_key_value_heads)):
         if v % tp:

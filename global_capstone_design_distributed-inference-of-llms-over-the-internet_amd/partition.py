@@ -65,7 +65,7 @@ def stage_cost_model(cfg, *, batch: int = 64, ctx: int = 256, fp8: bool = False)
     tail's extras) - what a pipeline stage actually streams from HBM:
 
     * block: its weights (1 byte per projection weight on the fp8 W8A16 path, else 2) + the
-      micro-batch's KV (``batch`` sessions x ``ctx`` tokens) + 5 launches;
+      micro-batch's KV (``batch`` sessions x ``ctx`` tokens) and recurrent state + 5 launches;
     * head: the embedding gather (``batch`` rows: negligible, the table is not streamed);
     * tail: final norm + ``lm_head`` (bf16, also in fp8 mode) on the last rows + the sampler,
       which makes several passes over ``batch`` x vocab fp32 logits.
@@ -76,6 +76,7 @@ def stage_cost_model(cfg, *, batch: int = 64, ctx: int = 256, fp8: bool = False)
     else:
         wbytes = cfg.layer_param_bytes(2.0)
     kv = batch * ctx * cfg.kv_bytes_per_token_per_layer(2)
+    kv += 2 * batch * cfg.state_bytes_per_session_per_layer()  # recurrent state: read and written back
     block = (wbytes + kv) / STREAM_BPS + 5 * LAUNCH_S
     head = batch * H * 2 / STREAM_BPS + LAUNCH_S
     tail = (V * H * 2 + batch * V * 4 * 4) / STREAM_BPS + SAMPLER_FIXED_S + 3 * LAUNCH_S

@@ -15,7 +15,10 @@ Replaces the reference's Stage0 / StageSegment / StageLast modules
   sequence only (the reference projects every prefill position, src/llama_partition.py:470).
 
 Attention is causal for prefill (the reference's optimized layer gets no mask and is
-NOT causal: src/llama_partition.py:118 -> petals/llama/block.py:136-137; see SURVEY §7.2).
+NOT causal: src/llama_partition.py:118 -> petals/llama/block.py:136-137).
+
+Hybrid decoders (``ModelConfig.layers``: layers that differ, some recurrent) plug their own layer loop, cache and
+states into the same planning, session, graph and stage code (runtime/hybrid.py).
 """
 from __future__ import annotations
 
@@ -815,7 +818,7 @@ class StageExecutor:
         """Run throwaway prefill steps at start-up so the first real request does not pay the
         first-call costs of its shapes (hipBLASLt algorithm selection for the row-major GEMMs,
         first launches of the prefill kernels): a cold 64 x 128-token prefill round took 4x
-        the warm one (VERDICT r2).  One single-sequence prefill per size (default: the step
+        the warm one.  One single-sequence prefill per size (default: the step
         capacity, 2048 and 512 tokens); the probe session is closed afterwards."""
         cap = min(self.max_tokens, self.max_seq_len - 1)
         sizes = sorted({int(n) for n in (sizes or (cap, 2048, 512)) if 128 < int(n) <= cap}, reverse=True)
@@ -1303,8 +1306,8 @@ class _DecodeGraph:
 
     Its metadata lives in ONE device blob (positions, slots | q_seq, q_ctx, last_rows) that a
     replay refills with a single host-to-device copy from a double-buffered pinned staging
-    blob, padded for the bucket (padding rows: slot -1, context 0): round 1 issued six small
-    copies / fills per step (profiles/r2_decode_step_*.txt)."""
+    blob, padded for the bucket (padding rows: slot -1, context 0): six small copies / fills per
+    step otherwise (profiles/r2_decode_step_*.txt)."""
 
     def __init__(self, ex: StageExecutor, B: int, part: Tuple[int, int], pool, hook=None):
         self.ex, self.B, self.part = ex, B, part

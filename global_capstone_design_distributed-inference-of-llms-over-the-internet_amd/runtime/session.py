@@ -1,7 +1,7 @@
 """Per-stage session table over the paged KV cache.
 
 Reference: the stage handler keeps ``self._kv_cache[session_id]`` forever
-(reference src/rpc_handler.py:70,266; "no eviction") and ignores
+(reference src/rpc_handler.py:70,266; no eviction) and ignores
 ``max_length``.  Here a session owns a row of a block table and a list of KV pages;
 ``max_length`` is enforced, pages are returned on close, and idle sessions expire after
 a TTL (``evict_expired``) so a crashed client cannot leak HBM.

@@ -190,7 +190,7 @@ def get_server_throughput(executor, network_bandwidth_mbps: Optional[float] = No
             return FALLBACK_THROUGHPUT
         if cache is not None:
             cache.put(key, {"compute_rps": compute, "measured_at": time.time()})
-    elt = torch.tensor([], dtype=executor.dtype).element_size()
+    elt = torch.tensor([], dtype=executor.hidden_dtype).element_size()
     network = estimate_network_throughput(executor.cfg.hidden_size, elt, network_bandwidth_mbps) * (1 - relay_penalty)
     final = min(compute, network)
     logger.info(f"Server throughput: compute={compute:.2f} rps, network={network:.2f} rps, final={final:.2f} rps")

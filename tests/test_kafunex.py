@@ -68,8 +68,25 @@ def test_wrong_tensor_shape_is_refused(tmp_path):
 
 
 def test_offload_and_tensor_split_are_refused(model):
+    from src.parallel.tensor_parallel import check_tp
+
     with pytest.raises(ValueError, match="resident"):
         U.executor(model[2], "cpu", "fp32", offload=True)
+    with pytest.raises(ValueError, match="tensor parallelism"):
+        check_tp(resolve_model(model[2]), 2)
+
+
+def test_block_sizes_count_the_recurrent_state():
+    from src.block_utils import auto_num_blocks
+    from src.partition import balanced_splits, stage_cost_model
+
+    c = resolve_model("kafunex-7b")
+    state = c.state_bytes_per_session_per_layer()
+    assert state == 32 * 128 * 128 * 4 * 3 // 4
+    lots, none = (auto_num_blocks(c, 20 << 30, max_sessions=n) for n in (2048, 0))
+    assert lots < none
+    assert stage_cost_model(c, batch=64)[0] > stage_cost_model(c, batch=1)[0]
+    assert len(balanced_splits(c, 4)) == 3
 
 
 def test_preset_runs_with_random_weights():
