@@ -3,7 +3,8 @@
 ``python bench.py --layer-bench`` (one GPU): for every width, an 8-layer Kafunex stage (three recurrent layers, then
 one attention layer) and an 8-layer Llama stage of the same width, query / kv heads, head size and feed-forward
 parameters, both bf16 with random weights, run in turn on the same executor code: prompts of several shapes, then
-decode steps (hipGraph replays) at several batch sizes.  One JSON line.
+decode steps (hipGraph replays) at several batch sizes, at contexts that end inside a 1024-token attention chunk (a
+query then sees as many keys on both sides).  One JSON line.
 """
 from __future__ import annotations
 
@@ -82,7 +83,7 @@ def _in_turn(sides, call, iters: int, rounds: int):
     return {k: statistics.median(v) for k, v in t.items()}
 
 
-def run(widths, layers: int = 8, ctx: int = 1024, device="cuda:0", steps: int = 16, rounds: int = 3, log=None) -> dict:
+def run(widths, layers: int = 8, ctx: int = 896, device="cuda:0", steps: int = 16, rounds: int = 3, log=None) -> dict:
     out = []
     with torch.no_grad():
         for width in widths:

@@ -701,6 +701,7 @@ static bool talk_xchg_geometry(int H, int G, int D, int upw, TalkXchg& x, size_t
   x.nwc = TX_NW / G;
   x.tb = 16 * x.nwc * upw / rep;
   if (x.tb < 1) return false;
+  if (upw == 1) x.tb = 1;  // decode: one token a workgroup
   x.hp = (H + 7) / 8 * 8;
   x.s_tok = TM_KEYS * (x.hp + 4) + 4;
   x.m_off = x.tb * x.s_tok;
@@ -718,9 +719,11 @@ __global__ __launch_bounds__(256) void talk_merge_kernel(TalkArgs a, const float
   for (int e = (blockIdx.y * 256 + threadIdx.x) * 4; e < HD; e += gridDim.y * 1024) {
     const int h = e / a.D;
     float mx = -INFINITY;
+#pragma unroll 8
     for (int p = 0; p < NP; ++p) mx = fmaxf(mx, ml[(((int64_t)p * T + t) * a.H + h) * 2]);
     f32x4 acc = (f32x4)(0.f);
     float l = 0.f;
+#pragma unroll 4
     for (int p = 0; p < NP; ++p) {
       const int64_t pr = ((int64_t)p * T + t) * a.H + h;
       const float f = __builtin_amdgcn_exp2f(ml[pr * 2] - mx);  // (an empty split: exp2(-inf) = 0)

@@ -158,11 +158,11 @@ def talk_blocks(ntoks, tokens: int):
 
 
 def talk_parts(rows: int, H: int, G: int, D: int, span: int, n_cu: int = 256):
-    """(keys per split, splits) of a decode step whose queries see at most ``span`` keys: about two workgroups per
-    CU, no split under 128 keys.  (The first split starts on a 32-key boundary at or before the first key.)"""
+    """(keys per split, splits) of a decode step whose queries see at most ``span`` keys: one workgroup per CU
+    (what fits one), no split under 64 keys.  (The first split starts on a 32-key boundary at or before the first key.)"""
     span = int(span) + 31
-    want = max(1, 2 * n_cu // max(1, rows))
-    n = max(1, min(want, span // 128))
+    want = max(1, n_cu // max(1, rows))
+    n = max(1, min(want, span // 64))
     ps = 32 * -(-span // (32 * n))
     return ps, -(-span // ps)
 
