@@ -135,7 +135,7 @@ REC_TOL = {"bf16": dict(atol=4e-2, rtol=2e-2), "fp32": dict(atol=3e-4, rtol=3e-4
 
 
 @pytest.mark.parametrize("dt", sorted(DTYPES))
-@pytest.mark.parametrize("H,D,V", [(2, 16, 16), (3, 48, 32), (2, 20, 33), (1, 1, 1), (2, 64, 128), (2, 128, 128),
+@pytest.mark.parametrize("H,D,V", [(2, 16, 16), (3, 40, 32), (2, 20, 33), (1, 1, 1), (2, 64, 128), (2, 128, 128),
                                    (1, 100, 200), (1, 256, 64), (1, 200, 256)])
 @pytest.mark.parametrize("form", ["chunk", "segments", "scan"])
 def test_recurrence_prompts(dt, H, D, V, form):
@@ -150,7 +150,7 @@ def test_recurrence_prompts(dt, H, D, V, form):
 
 
 @pytest.mark.parametrize("dt", sorted(DTYPES))
-@pytest.mark.parametrize("H,D,V", [(2, 16, 16), (3, 48, 32), (2, 20, 33), (2, 128, 128), (1, 300, 64)])
+@pytest.mark.parametrize("H,D,V", [(2, 16, 16), (3, 40, 32), (2, 20, 33), (2, 128, 128), (1, 300, 64)])
 def test_recurrence_decode(dt, H, D, V):
     n, starts = 9, [0, 3, 0, 1, 7, 20, 1, 1, 2]
     case = rec_case([1] * n, H, D, V, dt, starts)
@@ -250,7 +250,7 @@ def form(request, monkeypatch):
     return request.param
 
 
-SHAPES = [(4, 2, 64), (1, 1, 32), (6, 3, 48), (8, 1, 128), (16, 4, 128), (32, 8, 128), (32, 4, 64), (12, 4, 96),
+SHAPES = [(4, 2, 80), (1, 1, 32), (2, 2, 64), (6, 3, 48), (8, 1, 128), (16, 4, 128), (32, 8, 128), (32, 4, 64), (12, 4, 96),
           (24, 8, 40), (10, 2, 8), (16, 16, 32), (20, 5, 64)]
 PROMPTS = ([70, 2, 1, 130, 33], [0, 30, 63, 64, 100])
 
@@ -265,7 +265,7 @@ def test_attention_prompts(H, G, D, chunk, form):
 
 
 @pytest.mark.parametrize("dt", sorted(DTYPES))
-@pytest.mark.parametrize("H,G,D", [(4, 2, 64), (1, 1, 1), (6, 3, 20), (3, 1, 130), (32, 32, 128), (64, 8, 128)])
+@pytest.mark.parametrize("H,G,D", [(4, 2, 80), (1, 1, 1), (6, 3, 20), (3, 1, 130), (32, 32, 128), (64, 8, 128)])
 def test_attention_any_shape(dt, H, G, D):
     ntoks, starts = [20, 1, 2, 40], [0, 30, 63, 64]
     a, *rest = att_case(ntoks, starts, H, G, D, dt)
@@ -292,7 +292,7 @@ def test_attention_decode(H, G, D, chunk, split, form):
                                       (149, 100, True), (150, 100, False), (127, 100, True), (128, 127, True)])
 def test_a_standing_out_key_at_a_chunk_edge(i, j, seen, form):
     """Chunks of 50, pages and key tiles at 64 and 32: in a prompt and decoded, the key counts exactly in its chunk."""
-    H, G, D, chunk = 4, 2, 64, 50
+    H, G, D, chunk = 4, 2, 80, 50
     for ntoks, starts in (([i + 1], [0]), ([1], [i])):
         res = []
         for flip in (1, -1):
@@ -305,8 +305,8 @@ def test_a_standing_out_key_at_a_chunk_edge(i, j, seen, form):
                 pg, off = int(a["table"][1, j // 64]), j % 64
                 a["cache"][pg, :, off] *= -1
             parts = None if starts == [0] else hops.talk_parts(1, H, G, D, chunk)
-            got = run_att(a, H, G, D, ntoks, chunk, 1.0, form, parts)[-1]
-            close(got, att_oracle(seqs, ntoks, *rest, H, G, D, chunk, 1.0)[-1], TOL["bf16"])
+            got = run_att(a, H, G, D, ntoks, chunk, 0.3, form, parts)[-1]
+            close(got, att_oracle(seqs, ntoks, *rest, H, G, D, chunk, 0.3)[-1], TOL["bf16"])
             res.append(got.float())
         assert ((res[0] - res[1]).abs().max() > 0.2) == seen
 
