@@ -16,11 +16,14 @@ from __future__ import annotations
 
 import dataclasses
 import json
+import math
 import os
 from typing import Callable, Dict, Optional, Tuple
 
-SUPPORTED_TYPES = ("llama", "mistral", "mixtral", "gpt2", "kafunex")
-MIXERS = ("attention", "hgrn2")
+SUPPORTED_TYPES = ("llama", "mistral", "mixtral", "gpt2", "kafunex", "fubapel")
+MIXERS = ("attention", "hgrn2", "latent_attention", "mlstm", "retention")
+RECURRENT = ("hgrn2", "mlstm", "retention")
+FEED_FORWARDS = ("relu2", "clamped_glu")
 
 
 @dataclasses.dataclass(frozen=True)
@@ -29,7 +32,9 @@ class LayerSpec:
     the width of its feed-forward (0 = none).  Layers of one model may differ in every field.
 
     ``attention``: chunked talking-heads attention whose values are the projected keys; ``hgrn2``: the
-    gated linear recurrence (no kv heads, no mask, no scale)."""
+    gated linear recurrence (no kv heads, no mask, no scale); ``latent_attention``: keys and values are made from
+    one cached latent per token, plus a rotated key part that all heads share; ``mlstm``: matrix memory with
+    exponential gates; ``retention``: linear attention with a fixed decay per head."""
     mixer: str
     heads: int
     dim: int
@@ -38,16 +43,33 @@ class LayerSpec:
     kv_heads: int = 0
     chunk: int = 0
     scale: float = 1.0
+    ffn: str = "relu2"                      # feed-forward: squared relu, or the clamped gated form
+    limit: float = 0.0                      # clamped_glu: bound of its two inputs
+    q_rank: int = 0                         # latent_attention: size of the queries' latent
+    kv_rank: int = 0                        # latent_attention: size of the keys' and values' latent
+    rot_dim: int = 0                        # latent_attention: rotated part of a query / key head
+    rot_dims: int = 0                       # rotary: dimensions that turn
+    rot_base: float = 10000.0
+    decay: Tuple[float, ...] = ()           # retention: one factor per head
+    gate_cap: float = 0.0                   # mlstm: soft cap of the gates' inputs
+    source: Optional[int] = None            # checkpoint layer whose weights these are (None: its own place)
 
     @property
     def recurrent(self) -> bool:
-        return self.mixer == "hgrn2"
+        return self.mixer in RECURRENT
 
     @property
     def in_rows(self) -> int:
-        """Rows of the fused input projection: [q | f | v] or [q | k | gate]."""
-        if self.recurrent:
+        """Rows of the fused input projection: [q | f | v], [q | k | gate], [q latent | kv latent | rotated key],
+        [q | k | v | gate] or that and the two log gates, filled up to a whole GEMM tile."""
+        if self.mixer == "hgrn2":
             return self.heads * (2 * self.dim + self.vdim)
+        if self.mixer == "latent_attention":
+            return self.q_rank + self.kv_rank + self.rot_dim
+        if self.mixer == "retention":
+            return 2 * self.heads * (self.dim + self.vdim)
+        if self.mixer == "mlstm":
+            return 16 * -(-2 * self.heads * (self.dim + self.vdim + 1) // 16)
         return (2 * self.heads + self.kv_heads) * self.dim
 
     @property
@@ -55,26 +77,61 @@ class LayerSpec:
         return self.heads * self.vdim
 
     @property
-    def kv_elems(self) -> int:
-        """Cached elements per token (one shared key/value row)."""
-        return 0 if self.recurrent else self.kv_heads * self.dim
+    def q_rows(self) -> int:
+        """latent_attention: rows of the query up-projection."""
+        return self.heads * (self.dim + self.rot_dim)
+
+    @property
+    def cache_row(self) -> Optional[Tuple[int, int, bool]]:
+        """Cached rows of a token: (rows, size, with an fp32 scale beside them); None without a cache."""
+        if self.recurrent:
+            return None
+        if self.mixer == "latent_attention":
+            return 1, self.kv_rank + self.rot_dim, False
+        return self.kv_heads, self.dim, True
+
+    @property
+    def state_shapes(self) -> Tuple[Tuple[int, ...], ...]:
+        """fp32 state of one session; mlstm: the matrix, and per head its normalizer and running maximum."""
+        if not self.recurrent:
+            return ()
+        mat = (self.heads, self.dim, self.vdim)
+        return (mat, (self.heads, self.dim + 1)) if self.mixer == "mlstm" else (mat,)
+
+    def cache_bytes(self, elt_bytes: int) -> int:
+        """Cached bytes per token."""
+        if self.recurrent:
+            return 0
+        n, d, scaled = self.cache_row
+        return n * d * elt_bytes + (4 if scaled else 0)
 
     @property
     def state_elems(self) -> int:
         """fp32 state elements per session."""
-        return self.heads * self.dim * self.vdim if self.recurrent else 0
+        return sum(math.prod(s) for s in self.state_shapes)
 
     def param_count(self, width: int) -> int:
-        n = width * (self.in_rows + self.out_cols + 2 * self.ff) + 2 * width
-        if self.recurrent:
-            return n + 2 * self.heads * self.dim + self.vdim
-        return n + (self.heads + self.kv_heads) * self.dim + self.heads * self.heads
+        n = width * (self.in_rows + self.out_cols + (3 if self.ffn == "clamped_glu" else 2) * self.ff) + 2 * width
+        H, D, V = self.heads, self.dim, self.vdim
+        if self.mixer == "hgrn2":
+            return n + 2 * H * D + V
+        if self.mixer == "latent_attention":
+            return n + self.q_rows * self.q_rank + H * (D + V) * self.kv_rank + self.q_rank + self.kv_rank + H
+        if self.mixer == "mlstm":
+            return n + H * (V + 2)
+        if self.mixer == "retention":
+            return n
+        return n + (H + self.kv_heads) * D + H * H
 
     def validate(self) -> None:
         if self.mixer not in MIXERS:
             raise ValueError(f"unsupported mixer {self.mixer!r}; supported: {MIXERS}")
+        if self.ffn not in FEED_FORWARDS:
+            raise ValueError(f"unsupported feed-forward {self.ffn!r}; supported: {FEED_FORWARDS}")
         if min(self.heads, self.dim, self.vdim) < 1 or self.ff < 0:
             raise ValueError(f"bad layer sizes: {self}")
+        if self.ff and self.ffn == "clamped_glu" and not self.limit > 0:
+            raise ValueError("the clamped feed-forward needs a limit > 0")
         if self.mixer == "attention":
             if self.kv_heads < 1 or self.heads % self.kv_heads:
                 raise ValueError("attention heads must be a multiple of kv_heads")
@@ -82,6 +139,21 @@ class LayerSpec:
                 raise ValueError("the values are the keys: vdim must equal dim")
             if self.chunk < 1:
                 raise ValueError("attention needs a mask size >= 1")
+        if self.mixer == "latent_attention":
+            if min(self.q_rank, self.kv_rank, self.rot_dim) < 1:
+                raise ValueError("latent attention needs q_rank, kv_rank and rot_dim >= 1")
+            if self.rot_dims != self.rot_dim:
+                raise ValueError("latent attention turns its whole rotated part: rot.dims must equal rot_dim")
+        if self.mixer == "retention" and len(self.decay) != self.heads:
+            raise ValueError("retention needs one decay per head")
+        if self.mixer == "retention" and not all(d >= 0 for d in self.decay):
+            raise ValueError("retention needs decays >= 0")
+        if self.mixer == "mlstm" and not self.gate_cap > 0:
+            raise ValueError("mlstm needs a gate_cap > 0")
+        if self.mixer in ("latent_attention", "retention"):
+            whole = self.rot_dim if self.mixer == "latent_attention" else self.dim
+            if self.rot_dims % 2 or not 0 <= self.rot_dims <= whole:
+                raise ValueError(f"rot.dims must be even and at most {whole}")
 
 
 @dataclasses.dataclass
@@ -110,6 +182,12 @@ class ModelConfig:
     sliding_window: Optional[int] = None
     # hybrid decoders: one LayerSpec per layer (None = the uniform families above)
     layers: Optional[Tuple[LayerSpec, ...]] = None
+    # hybrid decoders' residual stream: where a sublayer is normed (its output, "post", or its input, "pre"), the norm
+    # ("rms" / "layer"), the factor of a sublayer's output, and whether the embedding adds positions
+    stream: str = "post"
+    norm: str = "rms"
+    residual_mult: float = 1.0
+    embed_positions: bool = True
 
     @property
     def hybrid(self) -> bool:
@@ -144,8 +222,8 @@ class ModelConfig:
         return int(n * bytes_per_param)
 
     def kv_bytes_per_token_per_layer(self, bytes_per_elt: int = 2) -> int:
-        if self.hybrid:  # shared key/value rows + one fp32 per attention layer, averaged over the layers
-            n = sum(sp.kv_elems * bytes_per_elt + 4 for sp in self.layers if not sp.recurrent)
+        if self.hybrid:  # shared rows (and scales) of the attention layers, averaged over the layers
+            n = sum(sp.cache_bytes(bytes_per_elt) for sp in self.layers)
             return -(-n // max(len(self.layers), 1))
         return 2 * self.kv_dim * bytes_per_elt
 
@@ -161,6 +239,8 @@ class ModelConfig:
         if self.hybrid:
             if len(self.layers) != self.num_hidden_layers:
                 raise ValueError("layers must list every layer")
+            if self.stream not in ("post", "pre") or self.norm not in ("rms", "layer"):
+                raise ValueError(f"unsupported residual stream: {self.stream!r}, {self.norm!r}")
             for sp in self.layers:
                 sp.validate()
             return
@@ -215,15 +295,15 @@ class ModelConfig:
 
 
 def hybrid_config(model_type: str, vocab: int, width: int, eps: float, layers, name: str,
-                  max_positions: int = 32768) -> ModelConfig:
-    """A hybrid decoder's ModelConfig.  The uniform fields (heads, kv heads, head size, ff) describe its
+                  max_positions: int = 32768, **stream) -> ModelConfig:
+    """A hybrid decoder's ModelConfig; ``stream``: its residual stream's fields.  The uniform fields (heads, kv heads, head size, ff) describe its
     first attention layer, else its first layer: estimates and announcements read them, kernels do not."""
     layers = tuple(layers)
     ref = next((sp for sp in layers if not sp.recurrent), layers[0])
     return ModelConfig(model_type=model_type, vocab_size=vocab, hidden_size=width, intermediate_size=ref.ff,
                        num_hidden_layers=len(layers), num_attention_heads=ref.heads,
                        num_key_value_heads=ref.kv_heads or ref.heads, head_dim=ref.dim, rms_norm_eps=eps,
-                       max_position_embeddings=max_positions, name=name, layers=layers)
+                       max_position_embeddings=max_positions, name=name, layers=layers, **stream)
 
 
 def _kafunex_config(d: dict, name: str) -> ModelConfig:
@@ -243,13 +323,72 @@ def _kafunex_config(d: dict, name: str) -> ModelConfig:
     return hybrid_config("kafunex", int(d["vocab"]), int(d["width"]), float(d["norm"]["eps"]), layers, name)
 
 
+def looped(layers, loop: Optional[dict]) -> list:
+    """Layer runs of a model whose layers ``start`` .. ``stop`` - 1 run ``times`` times in a row: every run is a layer
+    of its own (cache or state, place in a stage) that names the checkpoint layer it takes its weights from."""
+    runs = [dataclasses.replace(sp, source=i) for i, sp in enumerate(layers)]
+    if loop is None:
+        return runs
+    a, b, n = int(loop["start"]), int(loop["stop"]), int(loop["times"])
+    if not 0 <= a <= b <= len(runs) or n < 1:
+        raise ValueError(f"bad loop {loop} over {len(runs)} layers")
+    return runs[:a] + runs[a:b] * n + runs[b:]
+
+
+def _fubapel_config(d: dict, name: str) -> ModelConfig:
+    layers = []
+    for i, e in enumerate(d["layers"]):
+        m, mlp = e["mixer"], e.get("mlp")
+        kw = {"ffn": "clamped_glu"}
+        if mlp is not None:
+            if mlp.get("kind", "dense") != "dense":
+                raise ValueError(f"layer {i}: unsupported feed-forward kind {mlp['kind']!r}")
+            kw.update(ff=int(mlp["ff"]), limit=float(mlp["limit"]))
+        if "rot" in m:
+            kw.update(rot_dims=int(m["rot"]["dims"]), rot_base=float(m["rot"]["base"]))
+        if e["type"] == "latent_attention":
+            kw.update(q_rank=int(m["q_rank"]), kv_rank=int(m["kv_rank"]), rot_dim=int(m["rot_dim"]),
+                      scale=float(m["scale"]))
+        elif e["type"] == "retention":
+            kw.update(decay=tuple(float(x) for x in m["decay"]))
+        elif e["type"] == "mlstm":
+            kw.update(gate_cap=float(m["gate_cap"]))
+        else:
+            raise ValueError(f"layer {i}: unsupported mixer {e['type']!r}; supported: {MIXERS}")
+        layers.append(LayerSpec(e["type"], int(m["heads"]), int(m["dim"]), int(m["vdim"]), **kw))
+    return hybrid_config("fubapel", int(d["vocab"]), int(d["width"]), float(d["norm"]["eps"]),
+                         looped(layers, d.get("loop")), name, stream="pre", norm="layer",
+                         residual_mult=float(d["residual_mult"]), embed_positions=False)
+
+
 # config.json "architecture" -> reader (the other families are told apart by Hugging Face's "model_type")
-ARCHITECTURES: Dict[str, Callable[[dict, str], ModelConfig]] = {"Kafunex": _kafunex_config}
+ARCHITECTURES: Dict[str, Callable[[dict, str], ModelConfig]] = {"Kafunex": _kafunex_config,
+                                                                     "Fubapel": _fubapel_config}
 
 
 def _kafunex_preset(name, vocab, width, ff, groups, rec, att) -> ModelConfig:
     """``groups`` x [three recurrent layers, one attention layer]."""
     return hybrid_config("kafunex", vocab, width, 1e-6, ((rec,) * 3 + (att,)) * groups, name)
+
+
+def _fubapel_preset(name, vocab, width, ff, loop, mla, mem, ret, groups) -> ModelConfig:
+    """``groups`` x [retention, latent attention, mLSTM, latent attention]; the attention layers have the feed-forward."""
+    return hybrid_config("fubapel", vocab, width, 1e-6, looped((ret, mla, mem, mla) * groups, loop), name, stream="pre",
+                         norm="layer", residual_mult=0.5, embed_positions=False)
+
+
+def _latent(heads, dim, vdim, rot, q_rank, kv_rank, ff, limit=7.0) -> LayerSpec:
+    return LayerSpec("latent_attention", heads, dim, vdim, ff, scale=(dim + rot) ** -0.5, ffn="clamped_glu", limit=limit,
+                     q_rank=q_rank, kv_rank=kv_rank, rot_dim=rot, rot_dims=rot)
+
+
+def _retention(heads, dim, vdim) -> LayerSpec:
+    return LayerSpec("retention", heads, dim, vdim, ffn="clamped_glu", rot_dims=dim,
+                     decay=tuple(1.0 - 2.0 ** (-5.0 - 4.0 * h / heads) for h in range(heads)))
+
+
+def _mlstm(heads, dim, vdim, cap=15.0) -> LayerSpec:
+    return LayerSpec("mlstm", heads, dim, vdim, ffn="clamped_glu", gate_cap=cap)
 
 
 PRESETS = {
@@ -258,6 +397,11 @@ PRESETS = {
                                     LayerSpec("attention", 4, 32, 32, 256, 2, 40, 32 ** -0.5)),
     "kafunex-7b": _kafunex_preset("kafunex-7b", 32000, 4096, 16384, 8, LayerSpec("hgrn2", 32, 128, 128, 16384),
                                   LayerSpec("attention", 32, 128, 128, 16384, 8, 1024, 128 ** -0.5)),
+    "tiny-fubapel": _fubapel_preset("tiny-fubapel", 640, 128, 256, {"start": 1, "stop": 3, "times": 2},
+                                    _latent(4, 32, 24, 8, 80, 64, 256), _mlstm(2, 32, 48), _retention(4, 16, 32), 1),
+    "fubapel-7b": _fubapel_preset("fubapel-7b", 32000, 4096, 14336, {"start": 4, "stop": 8, "times": 2},
+                                  _latent(32, 128, 128, 64, 1536, 512, 14336), _mlstm(16, 256, 256),
+                                  _retention(32, 128, 128), 8),
     "llama2-7b": ModelConfig(name="llama2-7b"),
     "llama3-8b": ModelConfig(vocab_size=128256, intermediate_size=14336, num_key_value_heads=8,
                              rope_theta=500000.0, max_position_embeddings=8192, bos_token_id=128000,

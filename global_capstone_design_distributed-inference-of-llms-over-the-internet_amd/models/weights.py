@@ -128,13 +128,13 @@ class GPT2Layer:
 @dataclasses.dataclass
 class HybridLayer:
     """A layer of a hybrid decoder.  GEMM weights have the stage's dtype; norms, gates and mixing matrices
-    are fp32.  ``w_in`` fuses the mixer's input projections ([q | f | v] or [q | k | gate]); ``*_p`` are the
+    are fp32.  ``w_in`` fuses the mixer's input projections (``LayerSpec.in_rows``); ``*_p`` are the
     fragment-native copies for the decode GEMM where the shape allows one."""
     spec: LayerSpec
     w_in: torch.Tensor                       # [in_rows, W]
     w_o: torch.Tensor                        # [W, heads * vdim]
-    n1: torch.Tensor                         # [W] mixer output norm gain x layer scale
-    w_up: Optional[torch.Tensor] = None      # [ff, W]
+    n1: torch.Tensor                         # [W] norm gain of the mixer's output x layer scale, or of its input
+    w_up: Optional[torch.Tensor] = None      # [ff, W]; gated: [2 ff, W] gate and up rows in blocks of ``ffn_block``
     w_down: Optional[torch.Tensor] = None    # [W, ff]
     n2: Optional[torch.Tensor] = None        # [W]
     f_bias: Optional[torch.Tensor] = None    # hgrn2 [heads * dim]
@@ -143,12 +143,23 @@ class HybridLayer:
     w_qk: Optional[torch.Tensor] = None      # attention [heads * dim]: query norm x its kv head's key norm
     talk: Optional[torch.Tensor] = None      # attention [heads, heads]
     sigma: Optional[torch.Tensor] = None     # attention [heads]: talk @ the heads' distance slopes
+    q_norm: Optional[torch.Tensor] = None    # latent_attention [q_rank]
+    c_norm: Optional[torch.Tensor] = None    # latent_attention [kv_rank]
+    w_uq: Optional[torch.Tensor] = None      # latent_attention [heads * (dim + rot_dim), q_rank]
+    w_uk: Optional[torch.Tensor] = None      # latent_attention [heads, kv_rank, dim]: a query head into latent space
+    w_uv: Optional[torch.Tensor] = None      # latent_attention [heads, vdim, kv_rank]: a head's latent sum to its value
+    w_ukv: Optional[torch.Tensor] = None     # latent_attention [heads * (dim + vdim), kv_rank]: keys and values, by head
+    sink: Optional[torch.Tensor] = None      # latent_attention [heads]
+    log_decay: Optional[torch.Tensor] = None  # retention [heads]: log2 of the decay
+    gate_bias: Optional[torch.Tensor] = None  # mlstm [2, heads]: input and forget gate
+    ffn_block: int = 0                       # gated feed-forward: rows of a gate / up block of ``w_up``
     w_in_p: Optional[torch.Tensor] = None
     w_o_p: Optional[torch.Tensor] = None
     w_up_p: Optional[torch.Tensor] = None
     w_down_p: Optional[torch.Tensor] = None
+    w_uq_p: Optional[torch.Tensor] = None
 
-    GEMMS = ("w_in", "w_o", "w_up", "w_down")
+    GEMMS = ("w_in", "w_o", "w_up", "w_down", "w_uq")
 
 
 @dataclasses.dataclass
@@ -342,26 +353,50 @@ def _random_gpt2_layer(cfg: ModelConfig, idx: int, device, dtype, seed: int) -> 
 
 
 # ------------------------------------------------------------------ hybrid decoders
-def _hybrid_names(spec: LayerSpec, width: int) -> Dict[str, tuple]:
+def _hybrid_names(spec: LayerSpec, cfg: ModelConfig) -> Dict[str, tuple]:
     """Checkpoint tensors of one layer (after its 'l<i>.' prefix) -> shape."""
-    n: Dict[str, tuple] = {"norm1": (), "ls1": (width,)}
+    width = cfg.hidden_size
+    norm = (width,) if cfg.stream == "pre" else ()
+    scaled = cfg.stream == "post"  # post-norm streams have a layer scale per sublayer
+    n: Dict[str, tuple] = {"norm1": norm}
     H, D, V = spec.heads, spec.dim, spec.vdim
-    if spec.recurrent:
+    if spec.mixer == "hgrn2":
         n.update({"mix.q": (H * D, width), "mix.f": (H * D, width), "mix.f.b": (H * D,), "mix.lower": (H * D,),
                   "mix.v": (H * V, width), "mix.norm": (V,), "mix.o": (width, H * V)})
+    elif spec.mixer == "latent_attention":
+        C, R, Q = spec.kv_rank, spec.rot_dim, spec.q_rank
+        n.update({"mix.dq": (Q, width), "mix.dq.norm": (Q,), "mix.uq": (H * (D + R), Q), "mix.dkv": (C + R, width),
+                  "mix.dkv.norm": (C,), "mix.uk": (H * D, C), "mix.uv": (H * V, C), "mix.sink": (H,),
+                  "mix.o": (width, H * V)})
+    elif spec.mixer in ("retention", "mlstm"):
+        n.update({"mix.q": (H * D, width), "mix.k": (H * D, width), "mix.v": (H * V, width), "mix.g": (H * V, width),
+                  "mix.o": (width, H * V)})
+        if spec.mixer == "mlstm":
+            n.update({"mix.norm": (H * V,), "mix.i": (H, width), "mix.i.b": (H,), "mix.f": (H, width), "mix.f.b": (H,)})
     else:
         KD = spec.kv_heads * D
         n.update({"mix.q": (H * D, width), "mix.k": (KD, width), "mix.q.norm": (H * D,), "mix.k.norm": (KD,),
                   "mix.talk": (H, H), "mix.g": (H * D, width), "mix.o": (width, H * D)})
     if spec.ff:
-        n.update({"mlp.up": (spec.ff, width), "mlp.down": (width, spec.ff), "norm2": (), "ls2": (width,)})
+        n.update({"mlp.up": (spec.ff, width), "mlp.down": (width, spec.ff), "norm2": norm})
+        if spec.ffn == "clamped_glu":
+            n["mlp.gate"] = (spec.ff, width)
+    if scaled:
+        n["ls1"] = (width,)
+        if spec.ff:
+            n["ls2"] = (width,)
     return n
 
 
-def _hybrid_layer(spec: LayerSpec, width: int, get, device, dtype) -> HybridLayer:
+# a mixer's input projections in the order in which ``w_in`` fuses them
+_IN_PARTS = {"hgrn2": ("q", "f", "v"), "attention": ("q", "k", "g"), "latent_attention": ("dq", "dkv"),
+             "retention": ("q", "k", "v", "g"), "mlstm": ("q", "k", "v", "g", "i", "f")}
+
+
+def _hybrid_layer(spec: LayerSpec, cfg: ModelConfig, get, device, dtype) -> HybridLayer:
     """``get(name)``: checkpoint tensor of this layer (any device / dtype)."""
     raw = {}
-    for name, shape in _hybrid_names(spec, width).items():
+    for name, shape in _hybrid_names(spec, cfg).items():
         t = get(name)
         if shape == () and t.numel() == 1:
             t = t.reshape(())
@@ -370,13 +405,31 @@ def _hybrid_layer(spec: LayerSpec, width: int, get, device, dtype) -> HybridLaye
         raw[name] = t.to(device)
     f32 = lambda n: raw[n].float().contiguous()  # noqa: E731
     g = lambda n: raw[n].to(dtype).contiguous()  # noqa: E731
-    parts = ("mix.q", "mix.f", "mix.v") if spec.recurrent else ("mix.q", "mix.k", "mix.g")
-    lay = HybridLayer(spec, torch.cat([raw[p].to(dtype) for p in parts], 0).contiguous(), g("mix.o"),
-                      f32("norm1") * f32("ls1"))
+    gain = lambda n, ls: f32(n) * f32(ls) if ls in raw else f32(n)  # noqa: E731
+    w_in = torch.cat([raw["mix." + p].to(dtype) for p in _IN_PARTS[spec.mixer]], 0)
+    pad = spec.in_rows - w_in.shape[0]
+    if pad:
+        w_in = torch.cat([w_in, w_in.new_zeros(pad, w_in.shape[1])], 0)
+    lay = HybridLayer(spec, w_in.contiguous(), g("mix.o"), gain("norm1", "ls1"))
     if spec.ff:
-        lay.w_up, lay.w_down, lay.n2 = g("mlp.up"), g("mlp.down"), f32("norm2") * f32("ls2")
-    if spec.recurrent:
+        lay.w_up, lay.w_down, lay.n2 = g("mlp.up"), g("mlp.down"), gain("norm2", "ls2")
+        if spec.ffn == "clamped_glu":
+            lay.ffn_block = GU_BLOCK if spec.ff % GU_BLOCK == 0 else spec.ff
+            gate = g("mlp.gate")
+            lay.w_up = interleave_gate_up(gate, lay.w_up) if lay.ffn_block == GU_BLOCK else torch.cat([gate, lay.w_up], 0)
+    H, D, V = spec.heads, spec.dim, spec.vdim
+    if spec.mixer == "hgrn2":
         lay.f_bias, lay.f_lower, lay.o_norm = f32("mix.f.b"), f32("mix.lower"), f32("mix.norm")
+    elif spec.mixer == "latent_attention":
+        C = spec.kv_rank
+        lay.q_norm, lay.c_norm, lay.w_uq, lay.sink = f32("mix.dq.norm"), f32("mix.dkv.norm"), g("mix.uq"), f32("mix.sink")
+        uk, uv = g("mix.uk").view(H, D, C), g("mix.uv").view(H, V, C)
+        lay.w_uk, lay.w_uv = uk.transpose(1, 2).contiguous(), uv
+        lay.w_ukv = torch.cat([uk, uv], 1).reshape(H * (D + V), C).contiguous()
+    elif spec.mixer == "retention":
+        lay.log_decay = torch.log2(torch.tensor(spec.decay, dtype=torch.float64)).clamp(min=-1e30).float().to(device)
+    elif spec.mixer == "mlstm":
+        lay.o_norm, lay.gate_bias = f32("mix.norm"), torch.stack([f32("mix.i.b"), f32("mix.f.b")])
     else:
         kn = f32("mix.k.norm").view(spec.kv_heads, 1, spec.dim)
         kn = kn.expand(spec.kv_heads, spec.heads // spec.kv_heads, spec.dim).reshape(-1)
@@ -390,16 +443,19 @@ def _hybrid_layer(spec: LayerSpec, width: int, get, device, dtype) -> HybridLaye
 def random_hybrid_tensors(cfg: ModelConfig, idx: int, device="cpu", dtype=torch.bfloat16,
                           seed: int = 0) -> Dict[str, torch.Tensor]:
     """Synthetic checkpoint tensors of layer ``idx`` (names without the layer prefix)."""
-    g = _gen(device, seed * 100003 + idx + 1)
-    spec, W = cfg.layers[idx], cfg.hidden_size
+    spec = cfg.layers[idx]
+    src = idx if spec.source is None else spec.source
+    g = _gen(device, seed * 100003 + src + 1)
     out = {}
-    for name, shape in _hybrid_names(spec, W).items():
+    for name, shape in _hybrid_names(spec, cfg).items():
         if name.endswith("norm") or name in ("norm1", "norm2", "ls1", "ls2"):
             t = torch.ones(shape, device=device)
         elif name == "mix.talk":
             t = torch.eye(shape[0], device=device) + _randn(shape, g, device, torch.float32, 0.3 / shape[0] ** 0.5)
         elif name == "mix.f.b":  # forget gates near 1: the state remembers
             t = 2.0 + _randn(shape, g, device, torch.float32, 1.0)
+        elif name in ("mix.i.b", "mix.sink"):
+            t = _randn(shape, g, device, torch.float32, 1.0)
         elif name == "mix.lower":
             t = torch.empty(shape, device=device).uniform_(0.0, 0.9, generator=g)
         else:
@@ -408,9 +464,21 @@ def random_hybrid_tensors(cfg: ModelConfig, idx: int, device="cpu", dtype=torch.
     return out
 
 
+def _hybrid_layers(cfg: ModelConfig, start: int, end: int, make) -> List[HybridLayer]:
+    """Layers [start, end): runs of one checkpoint layer share one object, so its weights are held once."""
+    made: Dict[int, HybridLayer] = {}
+    out = []
+    for i in range(start, end):
+        src = i if cfg.layers[i].source is None else cfg.layers[i].source
+        if src not in made:
+            made[src] = make(i, src)
+        out.append(made[src])
+    return out
+
+
 def _random_hybrid_layer(cfg: ModelConfig, idx: int, device, dtype, seed: int) -> HybridLayer:
     raw = random_hybrid_tensors(cfg, idx, device, dtype, seed)
-    return _hybrid_layer(cfg.layers[idx], cfg.hidden_size, raw.__getitem__, device, dtype)
+    return _hybrid_layer(cfg.layers[idx], cfg, raw.__getitem__, device, dtype)
 
 
 def _pad_rows(w: torch.Tensor, m: int) -> torch.Tensor:
@@ -424,10 +492,10 @@ def random_stage_weights(cfg: ModelConfig, start: int, end: int, *, has_embed: b
     """``fp8``: quantize each block as soon as it is generated (bf16 copies dropped), so a
     70B stage never holds its full bf16 weights."""
     device = torch.device(device)
-    mk = _random_hybrid_layer if cfg.hybrid else \
-        _random_gpt2_layer if cfg.model_type == "gpt2" else _random_llama_layer
-    layers = []
-    for i in range(start, end):
+    mk = _random_gpt2_layer if cfg.model_type == "gpt2" else _random_llama_layer
+    layers = _hybrid_layers(cfg, start, end, lambda i, _: _random_hybrid_layer(cfg, i, device, dtype, seed)) \
+        if cfg.hybrid else []
+    for i in range(start, end) if not cfg.hybrid else ():
         lay = mk(cfg, i, device, dtype, seed)
         if fp8 and isinstance(lay, LlamaLayer):
             one = StageWeights(cfg, i, i + 1, [lay])
@@ -538,13 +606,14 @@ def load_stage_weights(cfg: ModelConfig, path: str, start: int, end: int, *, has
     layers: List = []
     if cfg.hybrid:
         W = cfg.hidden_size
-        for i in range(start, end):
-            layers.append(_hybrid_layer(cfg.layers[i], W, lambda n, p=f"l{i}.": ck.get(p + n), dev, dtype))
+        layers = _hybrid_layers(cfg, start, end, lambda i, src: _hybrid_layer(
+            cfg.layers[i], cfg, lambda n: ck.get(f"l{src}.{n}"), dev, dtype))
         sw = StageWeights(cfg, start, end, layers)
         if has_embed:
             sw.embed = t("embed").contiguous()
         if has_head:
-            sw.final_norm = ck.get("final.norm").to(dev).float().reshape(1).repeat(W)
+            fn = ck.get("final.norm").to(dev).float().reshape(-1)
+            sw.final_norm = fn.expand(W).contiguous()  # (one gain for all, or one each)
             sw.lm_head = _pad_rows(t("head"), 16).contiguous()
         return sw
     if cfg.model_type == "gpt2":

@@ -978,8 +978,9 @@ def unpack_weight(wp: torch.Tensor) -> torch.Tensor:
 
 
 def linear(x, w, out=None, epilogue=0, residual=None, policy=None, wp=None, a_rows=None, out_packed=False,
-           gate=None, ss_in=None, eps=0.0, ap_out=None, ss_out=None, ss_zero=None):
-    """y = epilogue(x @ w^T). epilogue 0: none; 1: SwiGLU (16-row interleaved gate/up w); 2: + residual;
+           gate=None, ss_in=None, eps=0.0, ap_out=None, ss_out=None, ss_zero=None, glu_limit=0.0):
+    """y = epilogue(x @ w^T). epilogue 0: none; 1: SwiGLU (16-row interleaved gate/up w), or with ``glu_limit`` > 0
+    the clamped gate g sigmoid(1.702 g) (u + 1), g <= limit, |u| <= limit; 2: + residual;
     3: fused-norm producer (``residual`` updated in place to bf16(y + residual), also written packed to
     ``ap_out``, per-row sum of squares added to ``ss_out``; ``ss_zero`` is cleared); 4: max(y, 0)^2.
 
@@ -995,7 +996,7 @@ def linear(x, w, out=None, epilogue=0, residual=None, policy=None, wp=None, a_ro
             x = ref.unpack_act(x, a_rows, K)
         y = ref.linear(x, w if w is not None else unpack_weight(wp), out=None if out_packed or epilogue == 3 else out,
                        epilogue=epilogue, residual=residual, ss_in=ss_in, inv_k=1.0 / K, eps=eps, ap_out=ap_out,
-                       ss_out=ss_out, ss_zero=ss_zero)
+                       ss_out=ss_out, ss_zero=ss_zero, glu_limit=glu_limit)
         return ref.pack_act(y, out=out) if out_packed else y
     if a_rows is not None:
         M = int(a_rows)
@@ -1024,7 +1025,7 @@ def linear(x, w, out=None, epilogue=0, residual=None, policy=None, wp=None, a_ro
         flags = 1 | (2 if out_packed else 0) | _kflags(kern) | (262144 if kern == "t2d" and T2D_GL else 0)
         ws = gemm_workspace(x.device) if _base(kern) in ("sk", "rwk", "rwki", "t2d") else None
         torch.ops.mpamd.gemm(x, wp, out, residual, int(epilogue), M, flags, ws, gate, ap_out, ss_out, ss_zero, ss_in,
-                             1.0 / K, float(eps))
+                             1.0 / K, float(eps), float(glu_limit))
         return out
     if epilogue == 3 or ss_in is not None:
         raise RuntimeError(f"the fused-norm epilogues need the native decode GEMM (M={M}, N={N}, K={K})")
@@ -1036,6 +1037,9 @@ def linear(x, w, out=None, epilogue=0, residual=None, policy=None, wp=None, a_ro
             out.shape == (M, N) and x.dim() == 2:
         return torch.mm(x, w.t(), out=out)  # hipBLASLt straight into the caller's buffer (no copy)
     y = torch.nn.functional.linear(x, w)  # hipBLASLt
+    if epilogue == 1 and glu_limit > 0:
+        out = torch.empty(M, N // 2, dtype=y.dtype, device=y.device) if out is None else out
+        return mixers.clamped_glu(y, out, GU_BLOCK, glu_limit)
     if epilogue == 1:
         return swiglu(y, out=out)
     if epilogue == 2:
@@ -1466,4 +1470,4 @@ def autotune_w8(shapes, device, ms=(4, 16, 32, 48, 64), iters: int = 12, rounds:
 
 
 # the hybrid decoders' ops (imported last: they dispatch through this module)
-from . import hybrid  # noqa: E402,F401
+from . import hybrid, mixers  # noqa: E402,F401

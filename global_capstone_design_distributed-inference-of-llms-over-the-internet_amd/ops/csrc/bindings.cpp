@@ -56,7 +56,7 @@ int mp_gemm_t2d_ok(int M, int N, int K, int epilogue, int out_packed, int with_w
 int mp_quant_rows_fp8(const void* x, int64_t xs, void* a8, float* scale, int M, int K, hipStream_t stream);
 int mp_gemm_bf16(const void* x, int64_t x_stride, const void* w, void* y, int64_t y_stride, const void* res,
                  int64_t res_stride, int M, int N, int K, int epilogue, int flags, void* ws, const int* gate,
-                 void* ap, void* ss_out, void* ss_zero, const void* ss_in, float inv_k, float eps,
+                 void* ap, void* ss_out, void* ss_zero, const void* ss_in, float inv_k, float eps, float glu_limit,
                  hipStream_t stream);
 int mp_gemm_ss_elems();
 int mp_gemm_w8(const void* x, const void* wq, const float* wsc, void* y, int64_t y_stride, const void* res,
@@ -513,7 +513,7 @@ void gemm(const at::Tensor& x, const at::Tensor& wp, at::Tensor& y, const c10::o
           int64_t epilogue, int64_t M_, int64_t flags, const c10::optional<at::Tensor>& workspace,
           const c10::optional<at::Tensor>& gate, const c10::optional<at::Tensor>& ap,
           const c10::optional<at::Tensor>& ss_out, const c10::optional<at::Tensor>& ss_zero,
-          const c10::optional<at::Tensor>& ss_in, double inv_k, double eps) {
+          const c10::optional<at::Tensor>& ss_in, double inv_k, double eps, double glu_limit) {
   check_bf16_cuda(x, "x");
   check_bf16_cuda(wp, "wp");
   check_bf16_cuda(y, "y");
@@ -572,7 +572,7 @@ void gemm(const at::Tensor& x, const at::Tensor& wp, at::Tensor& y, const c10::o
   }
   check_launch(mp_gemm_bf16(x.data_ptr(), apk ? 0 : x.stride(0), wp.data_ptr(), y.data_ptr(), opk ? 0 : y.stride(0),
                             rp, rs, M, N, K, (int)epilogue, (int)flags, ws, gp, app, sso, ssz, ssi, (float)inv_k,
-                            (float)eps, cur_stream()),
+                            (float)eps, (float)glu_limit, cur_stream()),
                "gemm");
 }
 
@@ -854,7 +854,7 @@ TORCH_LIBRARY(mpamd, m) {
   m.def(
       "gemm(Tensor x, Tensor wp, Tensor(a!) y, Tensor? residual, int epilogue, int M, int flags, "
       "Tensor(b!)? workspace=None, Tensor? gate=None, Tensor(c!)? ap=None, Tensor(d!)? ss_out=None, "
-      "Tensor(e!)? ss_zero=None, Tensor? ss_in=None, float inv_k=0., float eps=0.) -> ()");
+      "Tensor(e!)? ss_zero=None, Tensor? ss_in=None, float inv_k=0., float eps=0., float glu_limit=0.) -> ()");
   m.def(
       "gemm_w8(Tensor x, Tensor wq, Tensor wsc, Tensor(a!) y, Tensor? residual, int epilogue, int M, int flags, "
       "Tensor(b!)? workspace=None, Tensor(c!)? ap=None, Tensor(d!)? ss_out=None, Tensor(e!)? ss_zero=None, "

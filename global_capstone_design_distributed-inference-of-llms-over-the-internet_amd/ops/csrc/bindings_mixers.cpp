@@ -1,0 +1,287 @@
+// torch custom-op registrations (namespace `mpamd`) of the pre-norm decoders' kernels: residual stream with input
+// norms, scalar-decay linear attention, latent attention.  Same rules as bindings.cpp: outputs come from the caller,
+// launches go to the current stream, shapes and dtypes are checked here.
+#include "bind_check.h"
+
+extern "C" {
+int mp_stream_norm(int src, const void* y, int64_t ys, const float* part, int S, int64_t slab, const int64_t* ids,
+                   int64_t vocab, const int32_t* rows, float* res, const float* w, void* x, int n, int W, float mult,
+                   float eps, int center, int packed_mt, int f32, hipStream_t stream);
+int mp_clamped_glu(const void* x, int64_t xs, void* out, int64_t M, int F, int B, float limit, int packed_mt, int f32,
+                   hipStream_t stream);
+int mp_linear_scan(int kind, const void* z, int64_t zs, const float* rope, int rot, const float* decay,
+                   const float* bias, const float* norm, float* state, float* aux, const int32_t* q_seq,
+                   const int32_t* q_ctx, void* out, int H, int D, int V, float cap, float eps, float qs, float ks,
+                   const int32_t* seg, int nseg, int n, int packed_mt, int f32, hipStream_t stream);
+int mp_latent_prep(const void* z, int64_t zs, const float* qw, const float* cw, void* cq, void* cache,
+                   const int64_t* slots, const int32_t* q_ctx, const float* rope, int n, int Q, int C, int R, float eps,
+                   int packed_q, int f32, hipStream_t stream);
+int mp_latent_block(int H, int D, int R, int V, int C, int page_log2);
+int mp_latent_attention(int form, const void* q, int64_t qs, const void* uk, const void* uv, const float* sink,
+                        const float* rope, const void* cache, const int32_t* bt, int bt_stride, const int32_t* q_seq,
+                        const int32_t* q_ctx, void* u, void* oc, void* out, int T, int H, int D, int R, int V, int C,
+                        int page_log2, float scale, const int32_t* rows, int n, const int32_t* blk, int nblk, int PS,
+                        int NP, float* part, int packed_mt, int f32, hipStream_t stream);
+}
+
+namespace {
+
+typedef c10::optional<at::Tensor> opt_tensor;
+
+void check_res(const at::Tensor& res, int64_t n, int64_t W) {
+  check_rows(res, n, W, "res");
+  MP_CHECK(res.scalar_type() == at::kFloat && res.is_contiguous(), "res: fp32 contiguous");
+}
+
+// res += mult * y, x = norm(res) * w.  y: [n, W] rows, fp32 [S, n, W] slabs, or none
+void add_norm(const opt_tensor& y, at::Tensor& res, const opt_tensor& w, const opt_tensor& x, double mult, double eps,
+              int64_t center, int64_t packed) {
+  const int64_t n = res.size(0), W = res.size(1);
+  check_res(res, n, W);
+  int f32 = 0, mt = 0;
+  const float* wp = nullptr;
+  void* xp = nullptr;
+  if (w.has_value()) {
+    MP_CHECK(x.has_value(), "x is missing");
+    f32 = act_type(*x, "x");
+    mt = check_out(*x, n, W, f32, packed, "x");
+    wp = f32_vec(*w, W, "w");
+    xp = x->data_ptr();
+  }
+  int src = 2, S = 0;
+  const void* yp = nullptr;
+  int64_t ys = W;
+  const float* part = nullptr;
+  if (y.has_value() && y->dim() == 3) {
+    MP_CHECK(y->is_cuda() && y->scalar_type() == at::kFloat && y->is_contiguous() && y->size(1) == n && y->size(2) == W,
+             "slabs: fp32 [S, n, W]");
+    src = 1, S = y->size(0), part = y->data_ptr<float>();
+    MP_CHECK(!f32, "slabs go with bf16 activations");
+  } else if (y.has_value()) {
+    const int yf = act_type(*y, "y");
+    MP_CHECK(xp == nullptr || yf == f32, "y: element types differ");
+    f32 = yf;
+    check_rows(*y, n, W, "y");
+    src = 0, yp = y->data_ptr(), ys = y->stride(0);
+  }
+  check_launch(mp_stream_norm(src, yp, ys, part, S, n * W, nullptr, 0, nullptr, res.data_ptr<float>(), wp, xp, n, W,
+                              (float)mult, (float)eps, (int)center, mt, f32, cur_stream()),
+               "add_norm");
+}
+
+void embed_norm(const at::Tensor& ids, const at::Tensor& table, at::Tensor& res, const at::Tensor& w, at::Tensor& x,
+                double eps, int64_t center, int64_t packed) {
+  const int f32 = act_type(table, "table");
+  const int64_t n = ids.numel(), W = table.size(1);
+  MP_CHECK(table.dim() == 2 && table.is_contiguous(), "table [vocab, W]");
+  MP_CHECK(reinterpret_cast<uintptr_t>(table.data_ptr()) % 16 == 0, "table must be 16-B aligned");
+  check_res(res, n, W);
+  const int mt = check_out(x, n, W, f32, packed, "x");
+  check_launch(mp_stream_norm(3, table.data_ptr(), W, nullptr, 0, 0, i64_vec(ids, n, "ids"), table.size(0), nullptr,
+                              res.data_ptr<float>(), f32_vec(w, W, "w"), x.data_ptr(), n, W, 1.f, (float)eps,
+                              (int)center, mt, f32, cur_stream()),
+               "embed_norm");
+}
+
+// out[i] = norm(res[rows[i]]) * w
+void rows_stream_norm(const at::Tensor& res, const at::Tensor& rows, const at::Tensor& w, at::Tensor& out, double eps,
+                      int64_t center, int64_t packed) {
+  const int f32 = act_type(out, "out");
+  const int64_t n = rows.numel(), W = res.size(1);
+  check_res(res, 0, W);
+  const int mt = check_out(out, n, W, f32, packed, "out");
+  check_launch(mp_stream_norm(2, nullptr, W, nullptr, 0, 0, nullptr, 0, i32_vec(rows, n, "rows"), res.data_ptr<float>(),
+                              f32_vec(w, W, "w"), out.data_ptr(), n, W, 0.f, (float)eps, (int)center, mt, f32,
+                              cur_stream()),
+               "rows_stream_norm");
+}
+
+void clamped_glu(const at::Tensor& x, at::Tensor& out, int64_t block, double limit, int64_t packed) {
+  const int f32 = act_type(x, "x");
+  const int64_t n = x.size(0), F = x.size(1) / 2;
+  check_rows(x, n, 2 * F, "x");
+  MP_CHECK(block >= 1 && F % block == 0, "gate / up blocks must divide the feed-forward width");
+  const int mt = check_out(out, n, F, f32, packed, "out");
+  check_launch(mp_clamped_glu(x.data_ptr(), x.stride(0), out.data_ptr(), n, F, block, (float)limit, mt, f32, cur_stream()),
+               "clamped_glu");
+}
+
+struct LinShape {
+  int f32, mlstm;
+  int64_t T, H, D, V;
+  int rot;
+  const float *rope, *decay, *bias, *norm;
+  float* aux;
+};
+// kind 0: retention (rope [positions, rot], decay [H]); 1: mLSTM (bias [2, H], norm [H V], aux [rows, H, D + 1])
+LinShape check_linear(int64_t kind, const at::Tensor& z, const opt_tensor& rope, const opt_tensor& decay,
+                      const opt_tensor& bias, const opt_tensor& norm, const at::Tensor& state, const opt_tensor& aux) {
+  LinShape s{};
+  MP_CHECK(kind == 0 || kind == 1, "kind");
+  s.mlstm = (int)kind;
+  s.f32 = act_type(z, "z");
+  MP_CHECK(state.is_cuda() && state.dim() == 4 && state.scalar_type() == at::kFloat && state.is_contiguous(),
+           "state: fp32 [rows, H, D, V]");
+  s.T = z.size(0), s.H = state.size(1), s.D = state.size(2), s.V = state.size(3);
+  const int64_t need = 2 * s.H * (s.D + s.V) + (s.mlstm ? 2 * s.H : 0);
+  MP_CHECK(z.dim() == 2 && z.size(1) >= need, "z columns");
+  check_rows(z, s.T, z.size(1), "z");
+  if (s.mlstm) {
+    MP_CHECK(bias.has_value() && norm.has_value() && aux.has_value(), "mlstm: bias, norm and aux");
+    s.bias = f32_vec(*bias, 2 * s.H, "bias");
+    s.norm = f32_vec(*norm, s.H * s.V, "norm");
+    s.aux = const_cast<float*>(f32_vec(*aux, state.size(0) * s.H * (s.D + 1), "aux"));
+  } else {
+    MP_CHECK(rope.has_value() && decay.has_value(), "retention: rope and decay");
+    MP_CHECK(rope->is_cuda() && rope->dim() == 2 && rope->scalar_type() == at::kFloat && rope->is_contiguous(), "rope");
+    s.rot = rope->size(1);
+    MP_CHECK(s.rot % 2 == 0 && s.rot <= s.D, "rope: an even number of columns, at most D");
+    s.rope = rope->data_ptr<float>();
+    s.decay = f32_vec(*decay, s.H, "decay");
+  }
+  return s;
+}
+
+void linear_scan(int64_t kind, const at::Tensor& z, const opt_tensor& rope, const opt_tensor& decay,
+                 const opt_tensor& bias, const opt_tensor& norm, at::Tensor& state, const opt_tensor& aux,
+                 const at::Tensor& q_seq, const at::Tensor& q_ctx, at::Tensor& out, double cap, double eps, double qs,
+                 double ks, const opt_tensor& seg, int64_t packed) {
+  const LinShape s = check_linear(kind, z, rope, decay, bias, norm, state, aux);
+  const int mt = check_out(out, s.T, s.H * s.V, s.f32, packed, "out");
+  const int32_t* sp = nullptr;
+  int64_t nseg = 0;
+  if (seg.has_value()) {
+    MP_CHECK(seg->dim() == 2 && seg->size(0) >= 2, "seg int32 [2+, nseg]");
+    nseg = seg->size(1);
+    sp = i32_vec(*seg, 2 * nseg, "seg");
+  }
+  check_launch(mp_linear_scan(s.mlstm, z.data_ptr(), z.stride(0), s.rope, s.rot, s.decay, s.bias, s.norm,
+                              state.data_ptr<float>(), s.aux, i32_vec(q_seq, s.T, "q_seq"), i32_vec(q_ctx, s.T, "q_ctx"),
+                              out.data_ptr(), s.H, s.D, s.V, (float)cap, (float)eps, (float)qs, (float)ks, sp, nseg,
+                              sp ? nseg : s.T, mt, s.f32, cur_stream()),
+               "linear_scan");
+}
+
+int page_log2_of(const at::Tensor& cache, int f32) {
+  check_act(cache, f32, "cache");
+  MP_CHECK(cache.dim() == 4 && cache.is_contiguous() && cache.size(1) == 1, "cache [pages, 1, page, C + R]");
+  MP_CHECK(reinterpret_cast<uintptr_t>(cache.data_ptr()) % 16 == 0, "cache must be 16-B aligned");
+  const int64_t page = cache.size(2);
+  MP_CHECK((page & (page - 1)) == 0, "page size must be a power of two");
+  int l = 0;
+  while ((1ll << l) < page) ++l;
+  return l;
+}
+
+void latent_prep(const at::Tensor& z, const at::Tensor& qw, const at::Tensor& cw, at::Tensor& cq, at::Tensor& cache,
+                 const at::Tensor& slots, const at::Tensor& q_ctx, const at::Tensor& rope, double eps, int64_t packed) {
+  const int f32 = act_type(z, "z");
+  page_log2_of(cache, f32);
+  const int64_t n = z.size(0), Q = qw.numel(), C = cw.numel(), R = cache.size(3) - C;
+  MP_CHECK(R >= 2 && R % 2 == 0, "the rotated part has an even size");
+  check_rows(z, n, Q + C + R, "z");
+  MP_CHECK(rope.is_cuda() && rope.dim() == 2 && rope.scalar_type() == at::kFloat && rope.is_contiguous() &&
+               rope.size(1) == R, "rope: fp32 [positions, R]");
+  const int mt = check_out(cq, n, Q, f32, packed, "cq");
+  check_launch(mp_latent_prep(z.data_ptr(), z.stride(0), f32_vec(qw, Q, "qw"), f32_vec(cw, C, "cw"), cq.data_ptr(),
+                              cache.data_ptr(), i64_vec(slots, n, "slots"), i32_vec(q_ctx, n, "q_ctx"),
+                              rope.data_ptr<float>(), n, Q, C, R, (float)eps, mt, f32, cur_stream()),
+               "latent_prep");
+}
+
+int64_t latent_block(int64_t H, int64_t D, int64_t R, int64_t V, int64_t C, int64_t page) {
+  int l = 0;
+  while ((1ll << l) < page) ++l;
+  return mp_latent_block((int)H, (int)D, (int)R, (int)V, (int)C, l);
+}
+
+// uk [H, C, D], uv [H, V, C].  form 1: u [T, H, C + R] and oc [T, H, C] are scratch, ``rows`` / ``blk`` choose the
+// token rows (none: all), the context goes in ``parts`` splits of ``part_size`` keys (``ws`` when parts > 1)
+void latent_attention(const at::Tensor& q, const at::Tensor& uk, const at::Tensor& uv, const at::Tensor& sink,
+                      const at::Tensor& rope, const at::Tensor& cache, const at::Tensor& bt, const at::Tensor& q_seq,
+                      const at::Tensor& q_ctx, at::Tensor& out, double scale, int64_t form, const opt_tensor& u,
+                      const opt_tensor& oc, const opt_tensor& rows, const opt_tensor& blk, int64_t part_size,
+                      int64_t parts, const opt_tensor& ws, int64_t packed) {
+  const int f32 = act_type(q, "q");
+  const int pl2 = page_log2_of(cache, f32);
+  check_act(uk, f32, "uk");
+  check_act(uv, f32, "uv");
+  MP_CHECK(uk.dim() == 3 && uk.is_contiguous() && uv.dim() == 3 && uv.is_contiguous() && uk.size(0) == uv.size(0) &&
+               uk.size(1) == uv.size(2), "uk [H, C, D], uv [H, V, C]");
+  const int64_t T = q.size(0), H = uk.size(0), C = uk.size(1), D = uk.size(2), V = uv.size(1), R = cache.size(3) - C;
+  MP_CHECK(R >= 2 && R % 2 == 0, "the rotated part has an even size");
+  check_rows(q, T, H * (D + R), "q");
+  MP_CHECK(rope.is_cuda() && rope.dim() == 2 && rope.scalar_type() == at::kFloat && rope.is_contiguous() &&
+               rope.size(1) == R, "rope: fp32 [positions, R]");
+  MP_CHECK(bt.is_cuda() && bt.dim() == 2 && bt.scalar_type() == at::kInt && bt.stride(1) == 1, "block table int32");
+  const int mt = check_out(out, T, H * V, f32, packed, "out");
+  void *up = nullptr, *op = nullptr;
+  float* wp = nullptr;
+  const int32_t *rp = nullptr, *bp = nullptr;
+  int64_t n = T, nb = 0;
+  if (form == 1) {
+    MP_CHECK(!f32 && u.has_value() && oc.has_value(), "the MFMA form is bf16 and needs u and oc");
+    check_act(*u, 0, "u");
+    check_act(*oc, 0, "oc");
+    MP_CHECK(u->is_contiguous() && u->numel() >= T * H * (C + R) && oc->is_contiguous() && oc->numel() >= T * H * C,
+             "u [T, H, C + R], oc [T, H, C]");
+    up = u->data_ptr(), op = oc->data_ptr();
+    if (rows.has_value()) {
+      n = rows->numel();
+      rp = i32_vec(*rows, n, "rows");
+    }
+    if (blk.has_value()) {
+      MP_CHECK(blk->dim() == 2 && blk->size(0) == 2, "blk int32 [2, nblk]");
+      nb = blk->size(1);
+      bp = i32_vec(*blk, 2 * nb, "blk");
+      if (nb == 0) return;
+    }
+    if (parts > 1) {
+      MP_CHECK(ws.has_value() && ws->is_cuda() && ws->scalar_type() == at::kFloat && ws->is_contiguous() &&
+                   ws->numel() >= parts * T * H * (C + 2), "ws: fp32 [parts T H (C + 2)]");
+      wp = ws->data_ptr<float>();
+    }
+  }
+  check_launch(mp_latent_attention((int)form, q.data_ptr(), q.stride(0), uk.data_ptr(), uv.data_ptr(),
+                                   f32_vec(sink, H, "sink"), rope.data_ptr<float>(), cache.data_ptr(),
+                                   bt.data_ptr<int32_t>(), bt.stride(0), i32_vec(q_seq, T, "q_seq"),
+                                   i32_vec(q_ctx, T, "q_ctx"), up, op, out.data_ptr(), T, H, D, R, V, C, pl2, (float)scale,
+                                   rp, n, bp, nb, (int)part_size, (int)parts, wp, mt, f32, cur_stream()),
+               "latent_attention");
+}
+
+}  // namespace
+
+TORCH_LIBRARY_FRAGMENT(mpamd, m) {
+  m.def(
+      "add_norm(Tensor? y, Tensor(a!) res, Tensor? w, Tensor(b!)? x, float mult, float eps, int center, int packed) -> "
+      "()");
+  m.def(
+      "embed_norm(Tensor ids, Tensor table, Tensor(a!) res, Tensor w, Tensor(b!) x, float eps, int center, int packed) "
+      "-> ()");
+  m.def(
+      "rows_stream_norm(Tensor res, Tensor rows, Tensor w, Tensor(a!) out, float eps, int center, int packed) -> ()");
+  m.def("clamped_glu(Tensor x, Tensor(a!) out, int block, float limit, int packed) -> ()");
+  m.def(
+      "linear_scan(int kind, Tensor z, Tensor? rope, Tensor? decay, Tensor? bias, Tensor? norm, Tensor(a!) state, "
+      "Tensor(b!)? aux, Tensor q_seq, Tensor q_ctx, Tensor(c!) out, float cap, float eps, float qs, float ks, Tensor? "
+      "seg, int packed) -> ()");
+  m.def(
+      "latent_prep(Tensor z, Tensor qw, Tensor cw, Tensor(a!) cq, Tensor(b!) cache, Tensor slots, Tensor q_ctx, Tensor "
+      "rope, float eps, int packed) -> ()");
+  m.def("latent_block(int H, int D, int R, int V, int C, int page) -> int", &latent_block);
+  m.def(
+      "latent_attention(Tensor q, Tensor uk, Tensor uv, Tensor sink, Tensor rope, Tensor cache, Tensor bt, Tensor q_seq, "
+      "Tensor q_ctx, Tensor(a!) out, float scale, int form, Tensor(b!)? u, Tensor(c!)? oc, Tensor? rows, Tensor? blk, "
+      "int part_size, int parts, Tensor(d!)? ws, int packed) -> ()");
+}
+
+TORCH_LIBRARY_IMPL(mpamd, CUDA, m) {
+  m.impl("add_norm", &add_norm);
+  m.impl("embed_norm", &embed_norm);
+  m.impl("rows_stream_norm", &rows_stream_norm);
+  m.impl("clamped_glu", &clamped_glu);
+  m.impl("linear_scan", &linear_scan);
+  m.impl("latent_prep", &latent_prep);
+  m.impl("latent_attention", &latent_attention);
+}

@@ -74,13 +74,14 @@ extern "C" int64_t mp_gemm_workspace_bytes() {
 extern "C" int mp_gemm_bf16(const void* x, int64_t x_stride, const void* w, void* y, int64_t y_stride,
                             const void* res, int64_t res_stride, int M, int N, int K, int epilogue, int flags,
                             void* ws, const int* gate, void* ap, void* ss_out, void* ss_zero, const void* ss_in,
-                            float inv_k, float eps, hipStream_t stream) {
+                            float inv_k, float eps, float glu_limit, hipStream_t stream) {
   (void)hipGetLastError();  // an earlier non-mpamd HIP call's stale error is not this launch's
   using namespace mp;
   if (M == 0) return 0;
   if (epilogue == 3 && (ap == nullptr || res == nullptr)) return -5;
   EpiArgs ep{(bf16_t*)ap, (u64*)ss_out, (u64*)ss_zero, (const u64*)ss_in, inv_k, eps, (M + 15) / 16};
   ep.rot = (flags >> 10) & 1;
+  ep.glu_limit = glu_limit;
   if (M > 256 || K % (32 * GU_MAX) || N % 16 || ((flags & 1) == 0 && x_stride % 8)) return -1;
   int rc;
   if (M > 64) {  // 65..256 rows: gemm_wide.hip (split-K ring / balanced ring, packed A, no gate)

@@ -98,7 +98,19 @@ struct EpiArgs {
   const float* wsc;    // fp8 weights (W8A16 kernels): per-output-column dequantization scales
   int rot = 0;         // rotate each workgroup's k walk (rw_krot; flags bit 10, chosen per shape)
   const uint8_t* xsc = nullptr;  // MX activations (gemm_mx.hip): e8m0 block scales [K/128][MT][64]
+  float glu_limit = 0.f;  // EPI 1, > 0: the clamped gate (glu_epilogue) in place of SwiGLU
 };
+
+// EPI 1 value of a gate / up pair of accumulators.  SwiGLU rounds where the unfused path rounds; the clamped gate
+// g sigmoid(1.702 g) (u + 1), g <= limit, |u| <= limit, stays fp32 until its store.
+__device__ __forceinline__ bf16_t glu_epilogue(const EpiArgs& ep, float g, float u) {
+  if (ep.glu_limit > 0.f) {
+    const float a = fminf(g, ep.glu_limit), b = fminf(fmaxf(u, -ep.glu_limit), ep.glu_limit);
+    return f2bf(a / (1.f + __expf(-1.702f * a)) * (b + 1.f));
+  }
+  const float gg = round_bf(g);
+  return f2bf(round_bf(gg / (1.f + __expf(-gg))) * round_bf(u));
+}
 
 // fp8 (OCP e4m3) weight fragment -> bf16 MFMA B operand (exact: every e4m3 value is a bf16
 // value): the W8A16 form of the ring kernels streams 1 byte per weight and keeps bf16
@@ -377,10 +389,8 @@ __global__ __launch_bounds__(512) void gemm_packed_kernel(const bf16_t* __restri
       if (row < M) {
         const int ncol = ((nt0 + t) >> 1) * 16 + c;
         const float sc = row_scale<EPI>(ep, rs_lds, row);
-        const float gg = round_bf(s * sc);
-        const float a = round_bf(gg / (1.f + __expf(-gg)));
         const int64_t yo = OPK ? apk_off(row, ncol, MT) : (int64_t)row * y_stride + ncol;
-        y[yo] = f2bf(a * round_bf(up * sc));
+        y[yo] = glu_epilogue(ep, s * sc, up * sc);
       }
     } else {
       if (row < M) {  // uniform over the 16 lanes of a row: sum16 in epi3_store is safe
@@ -493,10 +503,8 @@ __device__ __forceinline__ void tile_epilogue(int mt, int tile, const f32x4& v, 
     const float sc = row_scale<EPI>(ep, rsl, row);
     if constexpr (EPI == 1) {
       const int ncol = (tile >> 1) * 16 + c;
-      const float gg = round_bf(v[r] * sc);
-      const float a = round_bf(gg / (1.f + __expf(-gg)));
       const int64_t yo = OPK ? apk_off(row, ncol, ep.mt_out) : (int64_t)row * ys + ncol;
-      y[yo] = f2bf(a * round_bf(up[r] * sc));
+      y[yo] = glu_epilogue(ep, v[r] * sc, up[r] * sc);
     } else if constexpr (EPI == 3) {
       const bf16_t rv = rpv != nullptr ? (*rpv)[r] : res[(int64_t)row * rs + tile * 16 + c];
       epi3_store(ep, y, ys, row, tile * 16 + c, v[r] * sc, c, rv);

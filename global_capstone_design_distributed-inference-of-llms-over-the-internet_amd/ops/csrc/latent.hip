@@ -1,0 +1,543 @@
+// Latent attention over a paged cache of latents, gfx950.
+//
+// A token's cache row is its latent c (C values, RMS-normed) and one rotated key part r (R values) that all heads
+// share.  Head h's key is [U_h c | r], its value W_h c, its query [a | b] (a: D unrotated, b: R rotated values):
+//   s(i, j) = (a_i . U_h c_j + b_i . r_j) scale          p = exp(s) / (exp(sink_h) + sum_j exp(s))
+// over all j <= i.  Both products move to the query side, a . U c = (U^T a) . c and sum_j p_j W c_j = W sum_j p_j c_j,
+// so every head reads the same cached row, as key (all of it) and as value (its first C columns):
+//   u_i = [U_h^T a_i | b_i]  (C + R)      s = (u_i . row_j) scale      o_i = W_h sum_j p_j c_j
+// Scores and weights are fp32.
+//
+//   latent_prep_kernel    norms of a projected row [q latent | c | r], r turned, cache write
+//   latent_any_kernel     any shape and both element types: one workgroup per (query token, head)
+//   latent_query_kernel   u, by MFMA: 16 rows of a head at a time
+//   latent_attn_kernel    the core on MFMA: rows = (token, head) against 64-key tiles of the cache, split contexts
+//   latent_value_kernel   merges the splits, applies the sink, W_h by MFMA
+#include "common.h"
+#include "act_io.h"
+
+namespace mp {
+
+struct LatentArgs {
+  const void* z;          // prep: [T, zs] projected rows
+  int64_t zs;
+  const float *qw, *cw;   // norm weights of the q latent [Q] and of c [C]
+  void* cq;               // [T, Q] row-major or packed
+  int Q, packed_q;
+  const void* q;          // [T, qs] queries, head by head [D | R]
+  int64_t qs;
+  const void *uk, *uv;    // [H, C, D], [H, V, C]
+  const float* sink;      // [H]
+  const float* rope;      // [positions, R], cosines then sines
+  void* cache;            // [pages, page, C + R]
+  const int64_t* slots;
+  const int32_t* bt;
+  int bt_stride;
+  const int32_t *q_seq, *q_ctx;
+  const int32_t* rows;    // token rows to work on (null: all)
+  void* u;                // [T, H, C + R]
+  void* oc;               // [T, H, C]
+  void* out;              // [T, H V] row-major or packed
+  int T, H, D, R, V, C, page_log2, packed_mt;
+  float scale, eps;
+};
+
+constexpr float LOG2E_F = 1.44269504088896340736f;
+
+template <typename T>
+__global__ __launch_bounds__(256) void latent_prep_kernel(LatentArgs a) {
+  __shared__ float red[16];
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const int64_t slot = a.slots[t];
+  if (slot < 0) return;
+  const T* z = (const T*)a.z + (int64_t)t * a.zs;
+  float sq = 0.f, sc = 0.f;
+  for (int i = tid; i < a.Q; i += 256) {
+    const float x = to_f(z[i]);
+    sq += x * x;
+  }
+  for (int i = tid; i < a.C; i += 256) {
+    const float x = to_f(z[a.Q + i]);
+    sc += x * x;
+  }
+  sq = 1.f / sqrtf(block_sum(sq, red) / (float)a.Q + a.eps);
+  sc = 1.f / sqrtf(block_sum(sc, red) / (float)a.C + a.eps);
+  for (int i = tid; i < a.Q; i += 256) st_act((T*)a.cq, t, i, a.Q, a.packed_q, to_f(z[i]) * sq * a.qw[i]);
+  T* row = (T*)a.cache + slot * (a.C + a.R);
+  for (int i = tid; i < a.C; i += 256) from_f(to_f(z[a.Q + i]) * sc * a.cw[i], row[i]);
+  const float* cs = a.rope + (int64_t)(a.q_ctx[t] - 1) * a.R;
+  const int half = a.R >> 1;
+  const T* zr = z + a.Q + a.C;
+  for (int i = tid; i < half; i += 256) {
+    const float x = to_f(zr[i]), y = to_f(zr[i + half]), c = cs[i], s = cs[half + i];
+    from_f(x * c - y * s, row[a.C + i]);
+    from_f(y * c + x * s, row[a.C + half + i]);
+  }
+}
+
+// dynamic LDS: u [C + R], acc [C], p [256], row ids [256] (as int), red [16]
+template <typename T>
+__global__ __launch_bounds__(256) void latent_any_kernel(LatentArgs a) {
+  extern __shared__ float sm[];
+  const int t = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
+  const int ctx = a.q_ctx[t];
+  if (ctx <= 0) return;
+  const int D = a.D, R = a.R, C = a.C, V = a.V, KW = C + R, half = R >> 1;
+  float *u = sm, *acc = u + KW, *p = acc + C, *red = p + 512;
+  int* rid = (int*)(p + 256);
+  const T* q = (const T*)a.q + (int64_t)t * a.qs + (int64_t)h * (D + R);
+  const T* uk = (const T*)a.uk + (int64_t)h * C * D;
+  for (int c = tid; c < C; c += 256) {
+    float s = 0.f;
+    for (int d = 0; d < D; ++d) s += to_f(q[d]) * to_f(uk[(int64_t)c * D + d]);
+    u[c] = s;
+  }
+  const float* cs = a.rope + (int64_t)(ctx - 1) * R;
+  for (int i = tid; i < half; i += 256) {
+    const float x = to_f(q[D + i]), y = to_f(q[D + half + i]), c = cs[i], s = cs[half + i];
+    u[C + i] = x * c - y * s;
+    u[C + half + i] = y * c + x * s;
+  }
+  __syncthreads();
+  for (int c = tid; c < C; c += 256) acc[c] = 0.f;
+  const int32_t* bt = a.bt + (int64_t)a.q_seq[t] * a.bt_stride;
+  const int pmask = (1 << a.page_log2) - 1;
+  float m = fmaxf(a.sink[h], -1e30f), l = 1.f;  // the sink's own term
+  for (int j0 = 0; j0 < ctx; j0 += 256) {
+    const int n = min(256, ctx - j0), j = j0 + tid;
+    float s = -INFINITY;
+    if (tid < n) {
+      const int64_t r = ((int64_t)bt[j >> a.page_log2] << a.page_log2) + (j & pmask);
+      rid[tid] = (int)r;
+      const T* kp = (const T*)a.cache + r * KW;
+      s = 0.f;
+      for (int d = 0; d < KW; ++d) s += u[d] * to_f(kp[d]);
+      s *= a.scale;
+    }
+    const float mx = fmaxf(m, block_max(s, red)), f = expf(m - mx), e = tid < n ? expf(s - mx) : 0.f;
+    p[tid] = e;
+    l = l * f + block_sum(e, red);
+    m = mx;
+    __syncthreads();
+    for (int c = tid; c < C; c += 256) {
+      float x = acc[c] * f;
+      for (int k = 0; k < n; ++k) x += p[k] * to_f(((const T*)a.cache)[(int64_t)rid[k] * KW + c]);
+      acc[c] = x;
+    }
+    __syncthreads();
+  }
+  const float inv = 1.f / l;
+  const T* uv = (const T*)a.uv + (int64_t)h * V * C;
+  const int lane = tid & 63;
+  for (int v = tid >> 6; v < V; v += 4) {
+    float x = 0.f;
+    for (int c = lane; c < C; c += 64) x += acc[c] * inv * to_f(uv[(int64_t)v * C + c]);
+    x = wave_sum(x);
+    if (lane == 0) st_act((T*)a.out, t, h * V + v, a.H * V, a.packed_mt, x);
+  }
+}
+
+// ---------------------------------------------------------------------------------------
+// MFMA forms (bf16): C a multiple of 32 up to 512, D and R of 8, V of 4, pages of 64 tokens or more.
+typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8_l;
+typedef short s16x4_l __attribute__((ext_vector_type(4)));
+__device__ __forceinline__ f32x4 mfma_l(const u16x8& a, const u16x8& b, const f32x4& c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_l, a), __builtin_bit_cast(bf16x8_l, b), c, 0,
+                                                 0, 0);
+}
+__device__ __forceinline__ u16x4 lds_tr(const bf16_t* p) {
+  const s16x4_l v = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4_l*)(p));
+  return __builtin_bit_cast(u16x4, v);
+}
+__device__ __forceinline__ u16x4 pack4(float a, float b, float c, float d) { return (u16x4){f2bf(a), f2bf(b), f2bf(c), f2bf(d)}; }
+
+// u rows of head blockIdx.y for 16 token rows; the four waves take 16-column tiles of C, blockIdx.z splits them
+__global__ __launch_bounds__(256) void latent_query_kernel(LatentArgs a, int n) {
+  const int tid = threadIdx.x, lane = tid & 63, c16 = lane & 15, g4 = lane >> 4;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int h = blockIdx.y, D = a.D, R = a.R, C = a.C, KW = C + R;
+  const int i = blockIdx.x * 16 + c16;
+  const int t = i < n ? (a.rows ? a.rows[i] : i) : -1;
+  const bf16_t* q = (const bf16_t*)a.q + (int64_t)max(t, 0) * a.qs + (int64_t)h * (D + R);
+  u16x8 qf[8];
+#pragma unroll
+  for (int f = 0; f < 8; ++f) {
+    const int d = 32 * f + 8 * g4;
+    const u16x8 x = *reinterpret_cast<const u16x8*>(q + min(d, D - 8));
+    qf[f] = t >= 0 && d < D ? x : (u16x8)(0);
+  }
+  bf16_t* u = (bf16_t*)a.u + ((int64_t)max(t, 0) * a.H + h) * KW;
+  for (int ct = blockIdx.z * 4 + w; ct * 16 < C; ct += 4 * gridDim.z) {
+    const bf16_t* wk = (const bf16_t*)a.uk + ((int64_t)h * C + ct * 16 + c16) * D;
+    f32x4 x = (f32x4)(0.f);
+#pragma unroll
+    for (int f = 0; f < 8; ++f) {
+      if (32 * f >= D) break;
+      x = mfma_l(*reinterpret_cast<const u16x8*>(wk + min(32 * f + 8 * g4, D - 8)), qf[f], x);
+    }
+    if (t >= 0) *reinterpret_cast<u16x4*>(u + ct * 16 + 4 * g4) = pack4(x[0], x[1], x[2], x[3]);
+  }
+  if (blockIdx.z == 0 && t >= 0 && a.q_ctx[t] > 0) {
+    const float* cs = a.rope + (int64_t)(a.q_ctx[t] - 1) * R;
+    const int half = R >> 1;
+    for (int k = w * 4 + g4; k < half; k += 16) {
+      const float x = bf2f(q[D + k]), y = bf2f(q[D + half + k]), c = cs[k], s = cs[half + k];
+      u[C + k] = f2bf(x * c - y * s);
+      u[C + half + k] = f2bf(y * c + x * s);
+    }
+  }
+}
+
+constexpr int LT_KEYS = 64, LT_PS = LT_KEYS + 8;
+constexpr float LT_GROW = 8.f;  // log2 units a row's maximum may grow before its sums are rescaled
+
+// A workgroup owns up to 16 RT query rows (token-major x heads) of one sequence.  Per 64-key tile wave w makes the
+// scores of keys 16 w .. + 15 for all rows (S^T = rows u^T: a lane owns one query row), the row maxima meet in LDS,
+// the weights go to LDS as hi + lo bf16 (32-bit in effect), and wave w adds them into its 16 CW of the C value
+// columns (O^T += c^T P^T, c^T by transposed reads of the same tile).  The next tile is in flight in registers.
+template <int RT, int CW>
+__global__ __launch_bounds__(256) void latent_attn_kernel(LatentArgs a, const int32_t* __restrict__ blk, int nblk, int PS,
+                                                          float* __restrict__ part) {
+  constexpr int KPT = 2 * CW + 2;  // 16-B chunks of a tile per thread: C + R <= 64 CW + 64
+  extern __shared__ __attribute__((aligned(16))) bf16_t ls[];
+  const int tid = threadIdx.x, lane = tid & 63, c16 = lane & 15, g4 = lane >> 4;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int H = a.H, C = a.C, KW = C + a.R, KF = (KW + 31) >> 5, STR = 32 * KF + 8;
+  bf16_t *kt = ls, *qt = kt + LT_KEYS * STR, *ph = qt + 16 * RT * STR, *pl = ph + 16 * RT * LT_PS;
+  float* wred = (float*)(pl + 16 * RT * LT_PS);  // [4][16 RT]
+
+  const int bx = blk ? nblk - 1 - (int)blockIdx.x : (int)blockIdx.x;  // (later tokens see more keys: first)
+  const int tok0 = blk ? blk[bx] : bx, ntok = blk ? blk[nblk + bx] : 1;
+  const int hi = a.q_ctx[tok0 + ntok - 1];
+  if (hi <= 0) return;
+  const int h0 = blockIdx.y * 16 * RT, hg = min(H - h0, 16 * RT), nrow = ntok * hg;
+  const int p = blockIdx.z, s_lo = p * PS, s_hi = PS > 0 ? min(hi, s_lo + PS) : hi;
+  const int32_t* bt = a.bt + (int64_t)a.q_seq[tok0] * a.bt_stride;
+  const int pmask = (1 << a.page_log2) - 1;
+  const int cpr = KW >> 3;  // chunks per cache row
+  const float rcp = 1.f / (float)cpr, sl2 = a.scale * LOG2E_F;
+
+  // query rows, zero past the row count and past KW; the tile's own columns past KW
+  for (int x = tid; x < 16 * RT * 4 * KF; x += 256) {
+    const int r = x / (4 * KF), col = (x - r * 4 * KF) * 8;
+    const int rr = min(r, nrow - 1);
+    const bf16_t* src = (const bf16_t*)a.u + ((int64_t)(tok0 + rr / hg) * H + h0 + rr % hg) * KW;
+    const u16x8 v = *reinterpret_cast<const u16x8*>(src + min(col, KW - 8));
+    *reinterpret_cast<u16x8*>(qt + r * STR + col) = r < nrow && col < KW ? v : (u16x8)(0);
+  }
+  if (KW & 31)
+    for (int x = tid; x < LT_KEYS * (4 * KF - cpr); x += 256) {
+      const int r = x / (4 * KF - cpr), col = KW + (x - r * (4 * KF - cpr)) * 8;
+      *reinterpret_cast<u16x8*>(kt + r * STR + col) = (u16x8)(0);
+    }
+
+  int khi[RT];
+  float m[RT], l[RT];
+  f32x4 o[RT][CW];
+#pragma unroll
+  for (int r = 0; r < RT; ++r) {
+    const int row = 16 * r + c16;
+    khi[r] = row < nrow ? min(a.q_ctx[tok0 + row / hg], s_hi) : 0;
+    m[r] = -INFINITY;
+    l[r] = 0.f;
+#pragma unroll
+    for (int t = 0; t < CW; ++t) o[r][t] = (f32x4)(0.f);
+  }
+
+  u16x8 kreg[KPT];
+  auto fetch = [&](int s0) {  // a tile's rows are consecutive in the page; past the context the last row repeats
+    const bf16_t* base = (const bf16_t*)a.cache + (((int64_t)bt[s0 >> a.page_log2] << a.page_log2) + (s0 & pmask)) * KW;
+    const int lastc = min(LT_KEYS, s_hi - s0) * cpr - 1;
+#pragma unroll
+    for (int k = 0; k < KPT; ++k) kreg[k] = *reinterpret_cast<const u16x8*>(base + min(tid + 256 * k, lastc) * 8);
+  };
+  auto stash = [&]() {
+#pragma unroll
+    for (int k = 0; k < KPT; ++k) {
+      const int x = tid + 256 * k, key = (int)(((float)x + 0.5f) * rcp);
+      if (key < LT_KEYS) *reinterpret_cast<u16x8*>(kt + key * STR + (x - key * cpr) * 8) = kreg[k];
+    }
+  };
+
+  if (s_lo < s_hi) fetch(s_lo);
+  for (int s0 = s_lo; s0 < s_hi; s0 += LT_KEYS) {
+    stash();
+    if (s0 + LT_KEYS < s_hi) fetch(s0 + LT_KEYS);
+    __syncthreads();
+    f32x4 st[RT];
+#pragma unroll
+    for (int r = 0; r < RT; ++r) st[r] = (f32x4)(0.f);
+    const bf16_t *kp = kt + (16 * w + c16) * STR + 8 * g4, *qp = qt + c16 * STR + 8 * g4;
+#pragma unroll 2
+    for (int f = 0; f < KF; ++f) {
+      const u16x8 ka = *reinterpret_cast<const u16x8*>(kp + 32 * f);
+#pragma unroll
+      for (int r = 0; r < RT; ++r) st[r] = mfma_l(ka, *reinterpret_cast<const u16x8*>(qp + 16 * r * STR + 32 * f), st[r]);
+    }
+#pragma unroll
+    for (int r = 0; r < RT; ++r) {
+      float lm = -INFINITY;
+#pragma unroll
+      for (int k = 0; k < 4; ++k) {
+        st[r][k] = s0 + 16 * w + 4 * g4 + k < khi[r] ? st[r][k] * sl2 : -INFINITY;
+        lm = fmaxf(lm, st[r][k]);
+      }
+      lm = fmaxf(lm, __shfl_xor(lm, 16, 64));
+      lm = fmaxf(lm, __shfl_xor(lm, 32, 64));
+      if (g4 == 0) wred[w * 16 * RT + 16 * r + c16] = lm;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int r = 0; r < RT; ++r) {
+      float lm = wred[16 * r + c16];
+#pragma unroll
+      for (int k = 1; k < 4; ++k) lm = fmaxf(lm, wred[k * 16 * RT + 16 * r + c16]);
+      if (__any(lm > m[r] + LT_GROW)) {  // (every wave sees the same maxima: the same decision)
+        const float mn = fmaxf(m[r], lm), al = mn == -INFINITY ? 1.f : __builtin_amdgcn_exp2f(m[r] - mn);
+        l[r] *= al;
+#pragma unroll
+        for (int t = 0; t < CW; ++t) o[r][t] *= al;
+        m[r] = mn;
+      }
+      const float mu = m[r] == -INFINITY ? 0.f : m[r];
+      float x[4];
+#pragma unroll
+      for (int k = 0; k < 4; ++k) {
+        x[k] = __builtin_amdgcn_exp2f(st[r][k] - mu);
+        l[r] += x[k];
+      }
+      const u16x4 xh = pack4(x[0], x[1], x[2], x[3]);
+      const int off = (16 * r + c16) * LT_PS + 16 * w + 4 * g4;
+      *reinterpret_cast<u16x4*>(ph + off) = xh;
+      *reinterpret_cast<u16x4*>(pl + off) =
+          pack4(x[0] - bf2f(xh[0]), x[1] - bf2f(xh[1]), x[2] - bf2f(xh[2]), x[3] - bf2f(xh[3]));
+    }
+    __syncthreads();
+#pragma unroll
+    for (int kb = 0; kb < 2; ++kb) {
+      u16x8 bh[RT], bl[RT];
+#pragma unroll
+      for (int r = 0; r < RT; ++r) {
+        const int off = (16 * r + c16) * LT_PS + 32 * kb + 8 * g4;
+        bh[r] = *reinterpret_cast<const u16x8*>(ph + off);
+        bl[r] = *reinterpret_cast<const u16x8*>(pl + off);
+      }
+      // c^T: lane c16 of group g4 needs column 16 tile + c16 of keys 32 kb + 8 g4 .. + 7
+      const bf16_t* vb = kt + (32 * kb + 8 * g4 + (c16 >> 2)) * STR + 4 * (c16 & 3);
+#pragma unroll
+      for (int t = 0; t < CW; ++t) {
+        const int ct = w * CW + t;
+        if (ct * 16 >= C) break;  // (uniform)
+        const u16x4 v0 = lds_tr(vb + 16 * ct), v1 = lds_tr(vb + 4 * STR + 16 * ct);
+        const u16x8 va = {v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
+#pragma unroll
+        for (int r = 0; r < RT; ++r) {
+          o[r][t] = mfma_l(va, bh[r], o[r][t]);
+          o[r][t] = mfma_l(va, bl[r], o[r][t]);
+        }
+      }
+    }
+    __syncthreads();
+  }
+#pragma unroll
+  for (int r = 0; r < RT; ++r) {
+    float x = l[r];
+    x += __shfl_xor(x, 16, 64);
+    x += __shfl_xor(x, 32, 64);
+    if (g4 == 0) wred[w * 16 * RT + 16 * r + c16] = x;
+  }
+  __syncthreads();
+#pragma unroll
+  for (int r = 0; r < RT; ++r) {
+    const int row = 16 * r + c16;
+    if (row >= nrow) continue;
+    float ll = 0.f;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) ll += wred[k * 16 * RT + row];
+    const int h = h0 + row % hg;
+    const int64_t th = (int64_t)(tok0 + row / hg) * H + h;
+    if (part != nullptr) {  // split context: [NP][T H][C] sums, then [NP][T H][2] (maximum, sum)
+      const int64_t TH = (int64_t)a.T * H;
+      float* po = part + ((int64_t)p * TH + th) * C;
+#pragma unroll
+      for (int t = 0; t < CW; ++t)
+        if ((w * CW + t) * 16 < C) *reinterpret_cast<f32x4*>(po + (w * CW + t) * 16 + 4 * g4) = o[r][t];
+      if (w == 0 && g4 == 0) {
+        float* ml = part + (int64_t)gridDim.z * TH * C + ((int64_t)p * TH + th) * 2;
+        ml[0] = m[r];
+        ml[1] = ll;
+      }
+      continue;
+    }
+    const float sk = fmaxf(a.sink[h] * LOG2E_F, -1e30f), mf = fmaxf(m[r], sk);
+    const float f = __builtin_amdgcn_exp2f(m[r] - mf), inv = f / (ll * f + __builtin_amdgcn_exp2f(sk - mf));
+    bf16_t* po = (bf16_t*)a.oc + th * C;
+#pragma unroll
+    for (int t = 0; t < CW; ++t)
+      if ((w * CW + t) * 16 < C)
+        *reinterpret_cast<u16x4*>(po + (w * CW + t) * 16 + 4 * g4) =
+            pack4(o[r][t][0] * inv, o[r][t][1] * inv, o[r][t][2] * inv, o[r][t][3] * inv);
+  }
+}
+
+// values of head blockIdx.y for 16 token rows: the latent sums go to LDS (merged over NP splits when part is given),
+// then each wave makes 16-column tiles of V
+__global__ __launch_bounds__(256) void latent_value_kernel(LatentArgs a, int n, const float* __restrict__ part, int NP) {
+  extern __shared__ __attribute__((aligned(16))) bf16_t ls[];  // [16][C + 8]
+  const int tid = threadIdx.x, lane = tid & 63, c16 = lane & 15, g4 = lane >> 4;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int h = blockIdx.y, H = a.H, C = a.C, V = a.V, STR = C + 8;
+  {
+    const int r = tid >> 4, i = blockIdx.x * 16 + r;  // 16 threads a row
+    const int t = i < n ? (a.rows ? a.rows[i] : i) : -1;
+    const bool live = t >= 0 && a.q_ctx[max(t, 0)] > 0;
+    const int64_t TH = (int64_t)a.T * H, th = (int64_t)max(t, 0) * H + h;
+    if (part == nullptr) {
+      for (int c = (tid & 15) * 8; c < C; c += 128) {
+        const u16x8 x = *reinterpret_cast<const u16x8*>((const bf16_t*)a.oc + th * C + c);
+        *reinterpret_cast<u16x8*>(ls + r * STR + c) = live ? x : (u16x8)(0);
+      }
+    } else {
+      const float* ml = part + (int64_t)NP * TH * C + th * 2;
+      const float sk = fmaxf(a.sink[h] * LOG2E_F, -1e30f);
+      float m = sk;
+      if (live)
+        for (int p = 0; p < NP; ++p) m = fmaxf(m, ml[p * TH * 2]);
+      float l = __builtin_amdgcn_exp2f(sk - m);
+      if (live)
+        for (int p = 0; p < NP; ++p) l += ml[p * TH * 2 + 1] * __builtin_amdgcn_exp2f(ml[p * TH * 2] - m);
+      const float inv = 1.f / l;
+      for (int c = (tid & 15) * 8; c < C; c += 128) {
+        float x[8];
+#pragma unroll
+        for (int k = 0; k < 8; ++k) x[k] = 0.f;
+        if (live)
+          for (int p0 = 0; p0 < NP; p0 += 4) {  // four splits' loads in flight
+            float y[4][8], f[4];
+#pragma unroll
+            for (int k = 0; k < 4; ++k) {
+              const int p = min(p0 + k, NP - 1);
+              ld_vec<8>(part + ((int64_t)p * TH + th) * C + c, y[k]);
+              f[k] = p0 + k < NP ? __builtin_amdgcn_exp2f(ml[p * TH * 2] - m) * inv : 0.f;
+            }
+#pragma unroll
+            for (int k = 0; k < 4; ++k)
+#pragma unroll
+              for (int e = 0; e < 8; ++e) x[e] += f[k] * y[k][e];
+          }
+        st_vec<8>(ls + r * STR + c, x);
+      }
+    }
+  }
+  __syncthreads();
+  const int i = blockIdx.x * 16 + c16;
+  const int t = i < n ? (a.rows ? a.rows[i] : i) : -1;
+  for (int vt = blockIdx.z * 4 + w; vt * 16 < V; vt += 4 * gridDim.z) {
+    const bf16_t* wv = (const bf16_t*)a.uv + ((int64_t)h * V + min(vt * 16 + c16, V - 1)) * C + 8 * g4;
+    f32x4 x = (f32x4)(0.f);
+#pragma unroll 4
+    for (int f = 0; f < C >> 5; ++f)
+      x = mfma_l(*reinterpret_cast<const u16x8*>(wv + 32 * f),
+                 *reinterpret_cast<const u16x8*>(ls + c16 * STR + 32 * f + 8 * g4), x);
+    const int v = vt * 16 + 4 * g4;
+    if (t >= 0 && v < V) {
+      const float y[4] = {x[0], x[1], x[2], x[3]};
+      st_act_vec<4>((bf16_t*)a.out, t, h * V + v, H * V, a.packed_mt, y);
+    }
+  }
+}
+
+// row tiles of a workgroup (0: the MFMA forms do not cover the shape) and its LDS; rows: query rows that there are
+static int latent_geometry(int H, int D, int R, int V, int C, int page_log2, int rows, int& cw, size_t& lds) {
+  if (page_log2 < 6 || D % 8 || R % 8 || V % 4 || C % 32 || C > 512 || D > 256) return 0;
+  cw = C <= 128 ? 2 : C <= 256 ? 4 : 8;
+  if (C + R > 64 * cw + 64) return 0;
+  const int str = (C + R + 31) / 32 * 32 + 8;
+  for (int rt = rows > 32 ? 4 : rows > 16 ? 2 : 1; rt; rt >>= 1) {
+    lds = (size_t)(LT_KEYS + 16 * rt) * str * 2 + 2 * 16 * rt * LT_PS * 2 + 4 * 16 * rt * 4;
+    if (lds <= 160 * 1024) return rt;
+  }
+  return 0;
+}
+
+}  // namespace mp
+
+extern "C" int mp_latent_prep(const void* z, int64_t zs, const float* qw, const float* cw, void* cq, void* cache,
+                              const int64_t* slots, const int32_t* q_ctx, const float* rope, int n, int Q, int C, int R,
+                              float eps, int packed_q, int f32, hipStream_t stream) {
+  using namespace mp;
+  (void)hipGetLastError();
+  if (n == 0) return 0;
+  LatentArgs a{};
+  a.z = z, a.zs = zs, a.qw = qw, a.cw = cw, a.cq = cq, a.cache = cache, a.slots = slots, a.q_ctx = q_ctx, a.rope = rope;
+  a.Q = Q, a.C = C, a.R = R, a.eps = eps, a.packed_q = packed_q;
+  if (f32) hipLaunchKernelGGL(latent_prep_kernel<float>, dim3(n), dim3(256), 0, stream, a);
+  else hipLaunchKernelGGL(latent_prep_kernel<bf16_t>, dim3(n), dim3(256), 0, stream, a);
+  return (int)hipGetLastError();
+}
+
+// Tokens of a query block of the MFMA form (0: it does not cover the shape)
+extern "C" int mp_latent_block(int H, int D, int R, int V, int C, int page_log2) {
+  int cw;
+  size_t lds;
+  const int rt = mp::latent_geometry(H, D, R, V, C, page_log2, 64, cw, lds);
+  return rt == 0 ? 0 : 16 * rt / H > 1 ? 16 * rt / H : 1;
+}
+
+// form 0: any shape.  form 1: MFMA over the rows ``rows`` (n of them, null: all T rows) in the blocks ``blk`` [2, nblk]
+// (null: every row its own block), the context in NP splits of PS keys (part: NP T H (C + 2) floats when NP > 1).
+extern "C" int mp_latent_attention(int form, const void* q, int64_t qs, const void* uk, const void* uv, const float* sink,
+                                   const float* rope, const void* cache, const int32_t* bt, int bt_stride,
+                                   const int32_t* q_seq, const int32_t* q_ctx, void* u, void* oc, void* out, int T, int H,
+                                   int D, int R, int V, int C, int page_log2, float scale, const int32_t* rows, int n,
+                                   const int32_t* blk, int nblk, int PS, int NP, float* part, int packed_mt, int f32,
+                                   hipStream_t stream) {
+  using namespace mp;
+  (void)hipGetLastError();
+  if (T == 0 || n == 0) return 0;
+  LatentArgs a{};
+  a.q = q, a.qs = qs, a.uk = uk, a.uv = uv, a.sink = sink, a.rope = rope, a.cache = (void*)cache, a.bt = bt;
+  a.bt_stride = bt_stride, a.q_seq = q_seq, a.q_ctx = q_ctx, a.u = u, a.oc = oc, a.out = out, a.rows = rows;
+  a.T = T, a.H = H, a.D = D, a.R = R, a.V = V, a.C = C, a.page_log2 = page_log2, a.packed_mt = packed_mt;
+  a.scale = scale;
+  if (form == 0) {
+    const size_t lds = (size_t)(C + R + C + 512 + 16) * sizeof(float);
+    if (lds > 60000 || H > 65535) return -1;
+    if (f32) hipLaunchKernelGGL(latent_any_kernel<float>, dim3(T, H), dim3(256), lds, stream, a);
+    else hipLaunchKernelGGL(latent_any_kernel<bf16_t>, dim3(T, H), dim3(256), lds, stream, a);
+    return (int)hipGetLastError();
+  }
+  int cw;
+  size_t lds;
+  const int tb = blk ? mp_latent_block(H, D, R, V, C, page_log2) : 1;
+  const int rt = f32 ? 0 : latent_geometry(H, D, R, V, C, page_log2, tb * H, cw, lds);
+  if (rt == 0 || qs % 8) return -1;
+  if (NP < 1 || NP > 65535 || (NP > 1 && (PS <= 0 || PS % LT_KEYS || part == nullptr))) return -2;
+  const int nb16 = (n + 15) / 16;
+  const int ctiles = (C / 16 + 3) / 4, vtiles = ((V + 15) / 16 + 3) / 4;
+  const int zq = nb16 * H >= 1024 ? 1 : ctiles, zv = nb16 * H >= 1024 ? 1 : vtiles;
+  hipLaunchKernelGGL(latent_query_kernel, dim3(nb16, H, zq), dim3(256), 0, stream, a, n);
+  int rc = (int)hipGetLastError();
+  if (rc) return rc;
+  const dim3 grid(blk ? nblk : T, (H + 16 * rt - 1) / (16 * rt), NP);
+  float* pp = NP > 1 ? part : nullptr;
+  const int ps = NP > 1 ? PS : 0;
+#define MP_LA(RT_, CW_)                                                                                               \
+  {                                                                                                                   \
+    if (lds > 65536)                                                                                                  \
+      (void)hipFuncSetAttribute((const void*)latent_attn_kernel<RT_, CW_>, hipFuncAttributeMaxDynamicSharedMemorySize, \
+                                (int)lds);                                                                            \
+    hipLaunchKernelGGL((latent_attn_kernel<RT_, CW_>), grid, dim3(256), lds, stream, a, blk, nblk, ps, pp);            \
+  }
+#define MP_LAC(CW_)            \
+  if (rt == 1) MP_LA(1, CW_)   \
+  else if (rt == 2) MP_LA(2, CW_) \
+  else MP_LA(4, CW_)
+  if (cw == 2) { MP_LAC(2) } else if (cw == 4) { MP_LAC(4) } else { MP_LAC(8) }
+#undef MP_LAC
+#undef MP_LA
+  rc = (int)hipGetLastError();
+  if (rc) return rc;
+  hipLaunchKernelGGL(latent_value_kernel, dim3(nb16, H, zv), dim3(256), 16 * (C + 8) * 2, stream, a, n, pp, NP);
+  return (int)hipGetLastError();
+}

@@ -1,0 +1,193 @@
+// Bandwidth-bound kernels of pre-norm decoders with a 32-bit residual stream.
+//
+//   stream_norm   res[t] += mult * y[t], then x[t] = norm(res[t]) * w for the next sublayer
+//                 y: activation rows, the S fp32 split-K slabs of the projection that made it, rows of the
+//                 embedding table (res[t] = table[id]), or none
+//                 norm: centred (layer norm: mean and variance) or not (root mean square); w == null: no x
+//   clamped_glu   out = g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit)
+//
+// x feeds the next GEMM: row-major, or the packed decode-GEMM layout (common.h apk_off) when packed_mt > 0.
+#include "common.h"
+#include "act_io.h"
+
+namespace mp {
+
+struct StreamArgs {
+  const void* y;          // SRC 0: [n, ys] rows; SRC 3: the table [vocab, W]
+  int64_t ys;
+  const float* part;      // SRC 1: [S][n][ys]
+  int S;
+  int64_t slab;
+  const int64_t* ids;     // SRC 3
+  int64_t vocab;
+  const int32_t* rows;    // SRC 2: x[i] comes from res[rows[i]]
+  float* res;
+  const float* w;
+  void* x;
+  int W, packed_mt, center;
+  float mult, eps;
+};
+
+enum { SRC_ROWS = 0, SRC_SLABS = 1, SRC_NONE = 2, SRC_TABLE = 3 };
+
+template <typename T, int VEC, int MAXC, int SRC, int NT>
+__global__ __launch_bounds__(NT) void stream_norm_kernel(StreamArgs a) {
+  __shared__ float red[16];
+  const int orow = blockIdx.x, W = a.W;
+  const int row = SRC == SRC_NONE && a.rows != nullptr ? a.rows[orow] : orow;
+  const int nch = W / VEC;
+  float v[MAXC][VEC], g[MAXC][VEC];
+  int64_t id = 0;
+  if constexpr (SRC == SRC_TABLE) {
+    id = a.ids[orow];
+    if (id < 0 || id >= a.vocab) id = 0;  // never read out of bounds; the host validates ids
+  }
+  float sum = 0.f;
+#pragma unroll
+  for (int k = 0; k < MAXC; ++k) {
+    const int ch = (int)threadIdx.x + NT * k;
+    const int c = min(ch, nch - 1) * VEC;
+    if (a.w != nullptr) ld_vec<VEC>(a.w + c, g[k]);
+    if constexpr (SRC == SRC_TABLE) {
+      ld_vec<VEC>((const T*)a.y + id * W + c, v[k]);
+    } else {
+      ld_vec<VEC>(a.res + (int64_t)row * W + c, v[k]);
+      if constexpr (SRC == SRC_ROWS) {
+        float y[VEC];
+        ld_vec<VEC>((const T*)a.y + (int64_t)row * a.ys + c, y);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) v[k][j] += a.mult * y[j];
+      } else if constexpr (SRC == SRC_SLABS) {
+        float y[VEC];
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) y[j] = 0.f;
+        for (int s = 0; s < a.S; s += 4) {  // four slabs' loads in flight, added in slab order
+          float p[4][VEC];
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+            ld_vec<VEC>(a.part + min(s + i, a.S - 1) * a.slab + (int64_t)row * a.ys + c, p[i]);
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+            if (s + i < a.S)
+#pragma unroll
+              for (int j = 0; j < VEC; ++j) y[j] += p[i][j];
+        }
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) v[k][j] += a.mult * y[j];
+      }
+    }
+    if (ch < nch) {
+      if constexpr (SRC != SRC_NONE) st_vec<VEC>(a.res + (int64_t)row * W + c, v[k]);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) sum += v[k][j];
+    }
+  }
+  if (a.w == nullptr) return;  // (uniform)
+  const float mean = a.center ? block_sum(sum, red) / (float)W : 0.f;
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < MAXC; ++k)
+    if ((int)threadIdx.x + NT * k < nch)
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) {
+        v[k][j] -= mean;
+        ss += v[k][j] * v[k][j];
+      }
+  const float sc = 1.f / sqrtf(block_sum(ss, red) / (float)W + a.eps);
+#pragma unroll
+  for (int k = 0; k < MAXC; ++k) {
+    const int ch = (int)threadIdx.x + NT * k;
+    if (ch >= nch) continue;
+    float o[VEC];
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) o[j] = v[k][j] * sc * g[k][j];
+    st_act_vec<VEC>((T*)a.x, orow, ch * VEC, W, a.packed_mt, o);
+  }
+}
+
+template <typename T, int SRC>
+static int launch_stream_norm(const StreamArgs& a, int n, hipStream_t stream) {
+#define MP_SN(VEC_, MAXC_, NT_) \
+  hipLaunchKernelGGL((stream_norm_kernel<T, VEC_, MAXC_, SRC, NT_>), dim3(n), dim3(NT_), 0, stream, a)
+  const int W = a.W;
+  if (W % 4 == 0 && a.ys % 4 == 0) {
+    const int ch = W / 4;
+    if (n <= 256 && ch > 256 && ch <= 2048) {  // few rows: latency is what there is to save
+      if (ch <= 1024) MP_SN(4, 1, 1024);
+      else MP_SN(4, 2, 1024);
+    } else if (ch <= 256) MP_SN(4, 1, 256);
+    else if (ch <= 512) MP_SN(4, 2, 256);
+    else if (ch <= 1024) MP_SN(4, 4, 256);
+    else if (ch <= 2048) MP_SN(4, 8, 256);
+    else if (ch <= 4096) MP_SN(4, 16, 256);
+    else return -1;
+  } else {
+    if (W > 16 * 256) return -1;
+    MP_SN(1, 16, 256);
+  }
+#undef MP_SN
+  return (int)hipGetLastError();
+}
+
+constexpr float GLU_ALPHA = 1.702f;
+
+// x rows: gate and up columns in alternating blocks of B (B == F: all gates, then all ups)
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void clamped_glu_kernel(const T* __restrict__ x, int64_t xs, T* __restrict__ out,
+                                                          int64_t M, int F, int B, float limit, int packed_mt) {
+  const int nch = F / VEC;
+  const int64_t n = M * nch;
+  for (int64_t i = blockIdx.x * (int64_t)blockDim.x + threadIdx.x; i < n; i += (int64_t)gridDim.x * blockDim.x) {
+    const int64_t t = i / nch;
+    const int c = (int)(i - t * nch) * VEC;
+    const T* p = x + t * xs + (int64_t)(c / B) * 2 * B + c % B;
+    float g[VEC], u[VEC];
+    ld_vec<VEC>(p, g);
+    ld_vec<VEC>(p + B, u);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      const float a = fminf(g[j], limit), b = fminf(fmaxf(u[j], -limit), limit);
+      g[j] = a / (1.f + expf(-GLU_ALPHA * a)) * (b + 1.f);
+    }
+    st_act_vec<VEC>(out, (int)t, c, F, packed_mt, g);
+  }
+}
+
+}  // namespace mp
+
+// src: SRC_* above
+extern "C" int mp_stream_norm(int src, const void* y, int64_t ys, const float* part, int S, int64_t slab,
+                              const int64_t* ids, int64_t vocab, const int32_t* rows, float* res, const float* w,
+                              void* x, int n, int W, float mult, float eps, int center, int packed_mt, int f32,
+                              hipStream_t stream) {
+  using namespace mp;
+  (void)hipGetLastError();
+  if (n == 0) return 0;
+  const StreamArgs a{y, ys, part, S, slab, ids, vocab, rows, res, w, x, W, packed_mt, center, mult, eps};
+  switch (src) {
+    case SRC_ROWS: return f32 ? launch_stream_norm<float, 0>(a, n, stream) : launch_stream_norm<bf16_t, 0>(a, n, stream);
+    case SRC_SLABS: return f32 ? -2 : launch_stream_norm<bf16_t, 1>(a, n, stream);
+    case SRC_NONE: return f32 ? launch_stream_norm<float, 2>(a, n, stream) : launch_stream_norm<bf16_t, 2>(a, n, stream);
+    default: return f32 ? launch_stream_norm<float, 3>(a, n, stream) : launch_stream_norm<bf16_t, 3>(a, n, stream);
+  }
+}
+
+extern "C" int mp_clamped_glu(const void* x, int64_t xs, void* out, int64_t M, int F, int B, float limit, int packed_mt,
+                              int f32, hipStream_t stream) {
+  using namespace mp;
+  (void)hipGetLastError();
+  if (M == 0) return 0;
+  const int vec = F % 8 == 0 && B % 8 == 0 && xs % 8 == 0 ? 8 : 1;
+  int64_t g = (M * (F / vec) + 255) / 256;
+  const dim3 grid((unsigned)(g > 8192 ? 8192 : g));
+#define MP_CG(T_, V_)                                                                                              \
+  hipLaunchKernelGGL((clamped_glu_kernel<T_, V_>), grid, dim3(256), 0, stream, (const T_*)x, xs, (T_*)out, M, F, B, \
+                     limit, packed_mt)
+  if (f32) {
+    if (vec == 8) MP_CG(float, 8); else MP_CG(float, 1);
+  } else {
+    if (vec == 8) MP_CG(bf16_t, 8); else MP_CG(bf16_t, 1);
+  }
+#undef MP_CG
+  return (int)hipGetLastError();
+}

@@ -1,0 +1,129 @@
+"""Ops of the pre-norm decoders: residual stream with input norms, clamped gated feed-forward, scalar-decay linear
+attention (retention, mLSTM) and latent attention.
+
+Same dispatch rule as the package: GPU tensors run the HIP kernels (csrc/pre_norm.hip, csrc/linear_attn.hip,
+csrc/latent.hip), CPU tensors the plain-PyTorch forms of ``reference_mixers``.  ``packed`` writes an activation in the
+packed decode-GEMM layout.
+"""
+from __future__ import annotations
+
+import numpy as np
+import torch
+
+from . import reference_mixers as rm
+from .hybrid import _native, _put
+
+
+def rope_table(base: float, dims: int, positions: int, device) -> torch.Tensor:
+    """fp32 [positions, dims]: cosines, then sines, of position * base^(-2i / dims) (angles made in fp64)."""
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    a = torch.arange(positions, dtype=torch.float64)[:, None] * torch.pow(float(base), -2.0 * i / max(dims, 1))[None]
+    return torch.cat([torch.cos(a), torch.sin(a)], 1).float().to(device)
+
+
+# ------------------------------------------------------------------ residual stream
+def embed_norm(ids, table, res, w, eps, x, center=False, packed=False):
+    """res[t] = table[ids[t]] (fp32), x = norm(res) * w; ``center``: layer norm, else root mean square."""
+    if not _native(table):
+        res.copy_(table[ids.long()].float())
+        return _put(x, rm.norm(res, w, eps, center), packed)
+    torch.ops.mpamd.embed_norm(ids, table, res, w, x, float(eps), int(center), int(packed))
+    return x
+
+
+def add_norm(y, res, mult, w, eps, x, center=False, packed=False):
+    """res += mult * y, then x = norm(res) * w.  ``y``: [n, W], fp32 split-K slabs [S, n, W], or None; ``w`` None:
+    the sum alone."""
+    if not _native(res):
+        if y is not None:
+            res.add_((y.sum(0) if y.dim() == 3 else y).float() * mult)
+        return _put(x, rm.norm(res, w, eps, center), packed) if w is not None else None
+    torch.ops.mpamd.add_norm(y, res, w, x, float(mult), float(eps), int(center), int(packed))
+    return x
+
+
+def rows_norm(res, rows, w, eps, out, center=False, packed=False):
+    """out[i] = norm(res[rows[i]]) * w."""
+    if not _native(res):
+        return _put(out, rm.norm(res.index_select(0, rows.long()), w, eps, center), packed)
+    torch.ops.mpamd.rows_stream_norm(res, rows, w, out, float(eps), int(center), int(packed))
+    return out
+
+
+def clamped_glu(x, out, block, limit, packed=False):
+    """g sigmoid(1.702 g) (u + 1) with g <= limit and |u| <= limit; ``x`` [n, 2 F] in gate / up blocks of ``block``."""
+    if not _native(x):
+        return _put(out, rm.clamped_glu(x, block, limit), packed)
+    torch.ops.mpamd.clamped_glu(x, out, int(block), float(limit), int(packed))
+    return out
+
+
+# ------------------------------------------------------------------ scalar-decay linear attention
+def _scan_plan(plan):
+    return None if plan is None else plan["seqs"]
+
+
+def retention(z, rope, log_decay, state, q_seq, q_ctx, out, eps, plan=None, packed=False):
+    """Retention over a ragged step.  ``z`` [T, 2 H (D + V)] projected rows [q | k | v | gate], ``state`` [rows, H, D, V]
+    fp32 updated in place for row q_seq[t]; a token of context 1 starts from a zero state, a row of context 0 is
+    padding.  ``plan``: None = every row is one token of its own sequence (decode), else the step's device plan."""
+    if not _native(z):
+        return _put(out, rm.retention(z, rope, log_decay, state, q_seq, q_ctx, eps), packed)
+    return _linear(0, z, rope, log_decay, None, None, state, None, q_seq, q_ctx, out, 0.0, eps, 1.0,
+                   state.shape[2] ** -0.5, plan, packed)
+
+
+def mlstm(z, bias, cap, norm_w, state, aux, q_seq, q_ctx, out, eps, plan=None, packed=False):
+    """mLSTM over a ragged step, as ``retention``; z rows [q | k | v | gate | i | f], ``bias`` [2, H] of the log gates,
+    ``aux`` [rows, H, D + 1]: normalizer and running maximum."""
+    if not _native(z):
+        return _put(out, rm.mlstm(z, bias, cap, norm_w, state, aux, q_seq, q_ctx, eps), packed)
+    return _linear(1, z, None, None, bias, norm_w, state, aux, q_seq, q_ctx, out, cap, eps, state.shape[2] ** -0.5, 1.0,
+                   plan, packed)
+
+
+def _linear(kind, z, rope, decay, bias, norm_w, state, aux, q_seq, q_ctx, out, cap, eps, qs, ks, plan, packed):
+    torch.ops.mpamd.linear_scan(kind, z, rope, decay, bias, norm_w, state, aux, q_seq, q_ctx, out, float(cap), float(eps),
+                                float(qs), float(ks), _scan_plan(plan), int(packed))
+    return out
+
+
+# ------------------------------------------------------------------ latent attention
+LATENT_KEYS = 64  # keys of a tile: splits of a context are multiples of it
+
+
+def latent_prep(z, qw, cw, cq, cache, slots, q_ctx, rope, eps, packed=False):
+    """Norms of projected rows [q latent | c | rotated key]: ``cq`` gets the q latent, [c | turned key] goes to ``cache``
+    at ``slots`` (-1: skip)."""
+    if not _native(z):
+        return _put(cq, rm.latent_prep(z, qw, cw, cache, slots, q_ctx, rope, eps), packed)
+    torch.ops.mpamd.latent_prep(z, qw, cw, cq, cache, slots, q_ctx, rope, float(eps), int(packed))
+    return cq
+
+
+def latent_block(H: int, D: int, R: int, V: int, C: int, page: int) -> int:
+    """Tokens of a query block on the MFMA form (0: shape not covered)."""
+    return int(torch.ops.mpamd.latent_block(int(H), int(D), int(R), int(V), int(C), int(page)))
+
+
+def latent_parts(groups: int, span: int, n_cu: int = 256):
+    """(keys per split, splits) for ``groups`` workgroups whose queries see at most ``span`` keys: about one workgroup
+    per CU, no split under two tiles."""
+    span = max(1, int(span))
+    n = max(1, min(n_cu // max(1, groups), span // (2 * LATENT_KEYS)))
+    ps = LATENT_KEYS * -(-span // (LATENT_KEYS * n))
+    return ps, -(-span // ps)
+
+
+def latent_attention(q, uk, uv, sink, rope, cache, table, q_seq, q_ctx, out, scale, packed=False, u=None, oc=None,
+                     rows=None, blocks=None, parts=(0, 1), ws=None):
+    """Causal attention over cached latents, with a sink in the denominator.  ``q`` [T, H (D + R)], ``uk`` [H, C, D],
+    ``uv`` [H, V, C].  On the GPU the MFMA form runs when its scratch ``u`` [T, H, C + R] and ``oc`` [T, H, C] is given
+    (``rows``: token rows to work on, ``blocks`` [2, n] their query blocks; none: every row a block; ``parts``:
+    (keys per split, splits) with ``ws`` fp32 scratch), else the form for any shape and element type."""
+    if not _native(q):
+        return _put(out, rm.latent_attention(q, uk, uv, sink, rope, cache, table, q_seq, q_ctx, scale), packed)
+    torch.ops.mpamd.latent_attention(q, uk, uv, sink, rope, cache, table, q_seq, q_ctx, out, float(scale),
+                                     0 if u is None else 1, u, oc, rows, blocks, int(parts[0]), int(parts[1]), ws,
+                                     int(packed))
+    return out

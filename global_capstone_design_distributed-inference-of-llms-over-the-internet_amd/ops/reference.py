@@ -196,7 +196,7 @@ def argmax(logits, out=None):
 
 
 def linear(x, w, out=None, epilogue=0, residual=None, ss_in=None, inv_k=0.0, eps=0.0, ap_out=None, ss_out=None,
-           ss_zero=None):
+           ss_zero=None, glu_limit=0.0):
     """``ss_in``: scale row r of x @ w^T by rsqrt(ss_in[r] * inv_k + eps) (fused-norm consumer);
     epilogue 3: r = bf16(bf16(y) + residual) -> residual (in place) and ``ap_out`` (packed),
     ``ss_out[r] += sum(r^2)`` (fused-norm producer)."""
@@ -213,7 +213,11 @@ def linear(x, w, out=None, epilogue=0, residual=None, ss_in=None, inv_k=0.0, eps
         pack_act(o, out=ap_out)
         ss_out.view(SS_SHARDS, SS_ROWS)[0, : o.shape[0]] += fx_sumsq(o)
         return residual
-    if epilogue == 1:
+    if epilogue == 1 and glu_limit > 0:
+        from .reference_mixers import clamped_glu
+
+        y = clamped_glu(y, GU_BLOCK, glu_limit).to(x.dtype)
+    elif epilogue == 1:
         y = swiglu(y)
     elif epilogue == 2:
         y = add(y, residual)

@@ -1,0 +1,120 @@
+"""Plain-PyTorch implementations of the pre-norm decoders' ops (``ops/mixers.py``): the CPU data path.
+
+Token by token; math in fp32, outputs in the activation dtype (bf16 or fp32).
+"""
+from __future__ import annotations
+
+import torch
+
+GLU_ALPHA = 1.702
+
+
+def norm(x, w, eps, center):
+    x = x.float()
+    if center:
+        x = x - x.mean(-1, keepdim=True)
+    return x / torch.sqrt(x.pow(2).mean(-1, keepdim=True) + eps) * w
+
+
+def clamped_glu(x, block, limit):
+    T, F2 = x.shape
+    v = x.float().view(T, F2 // (2 * block), 2, block)
+    g, u = v[:, :, 0].reshape(T, F2 // 2), v[:, :, 1].reshape(T, F2 // 2)
+    g, u = g.clamp(max=limit), u.clamp(-limit, limit)
+    return g * torch.sigmoid(GLU_ALPHA * g) * (u + 1)
+
+
+def turn(x, table):
+    """x [..., n] fp32, table [..., dims] (cosines then sines): the first ``dims`` entries turned."""
+    dims = table.shape[-1]
+    h = dims // 2
+    c, s = table[..., :h], table[..., h:]
+    u, v = x[..., :h], x[..., h:dims]
+    return torch.cat([u * c - v * s, v * c + u * s, x[..., dims:]], -1)
+
+
+def _gated(o, g, eps):
+    return o / torch.sqrt(o.pow(2).mean(-1, keepdim=True) + eps), torch.sigmoid(g)
+
+
+def retention(z, rope, log_decay, state, q_seq, q_ctx, eps):
+    """z [T, 2 H (D + V)] in flat token order (a session's tokens in sequence); ``state`` is updated."""
+    T = z.shape[0]
+    _, H, D, V = state.shape
+    z = z.float()
+    q, k, v, g = z.split([H * D, H * D, H * V, H * V], 1)
+    cs = rope[(q_ctx.long() - 1).clamp(min=0)][:, None]
+    q, k = turn(q.reshape(T, H, D), cs), turn(k.reshape(T, H, D), cs) * D ** -0.5
+    v, decay = v.reshape(T, H, V), torch.exp2(log_decay)[:, None, None]
+    o = torch.zeros(T, H, V, device=z.device)
+    for t in range(T):
+        if int(q_ctx[t]) <= 0:
+            continue
+        S = state[int(q_seq[t])]
+        if int(q_ctx[t]) == 1:
+            S.zero_()
+        S.mul_(decay).add_(k[t].unsqueeze(-1) * v[t].unsqueeze(1))
+        o[t] = torch.einsum("hd,hdv->hv", q[t], S)
+    y, s = _gated(o, g, eps)
+    return y.reshape(T, H * V) * g * s
+
+
+def mlstm(z, bias, cap, norm_w, state, aux, q_seq, q_ctx, eps):
+    T = z.shape[0]
+    _, H, D, V = state.shape
+    z = z.float()
+    q, k, v, g, zi, zf = z[:, : 2 * H * (D + V + 1)].split([H * D, H * D, H * V, H * V, H, H], 1)
+    q, k, v = q.reshape(T, H, D) * D ** -0.5, k.reshape(T, H, D), v.reshape(T, H, V)
+    li = cap * torch.tanh((zi + bias[0]) / cap)
+    lf = torch.nn.functional.logsigmoid(cap * torch.tanh((zf + bias[1]) / cap))
+    o = torch.zeros(T, H, V, device=z.device)
+    for t in range(T):
+        if int(q_ctx[t]) <= 0:
+            continue
+        S, nm = state[int(q_seq[t])], aux[int(q_seq[t])]
+        if int(q_ctx[t]) == 1:
+            S.zero_()
+            nm.zero_()
+        n, m = nm[:, :D], nm[:, D]
+        m1 = torch.maximum(lf[t] + m, li[t])
+        a, b = torch.exp(lf[t] + m - m1), torch.exp(li[t] - m1)
+        kb = b[:, None] * k[t]
+        S.mul_(a[:, None, None]).add_(kb.unsqueeze(-1) * v[t].unsqueeze(1))
+        n.mul_(a[:, None]).add_(kb)
+        m.copy_(m1)
+        den = torch.maximum((n * q[t]).sum(-1).abs(), torch.exp(-m1)) + 1e-6
+        o[t] = torch.einsum("hd,hdv->hv", q[t], S) / den[:, None]
+    y, s = _gated(o, g, eps)
+    return y.reshape(T, H * V) * norm_w * s
+
+
+def latent_prep(z, qw, cw, cache, slots, q_ctx, rope, eps):
+    """Norms of projected rows [q latent | c | rotated key]; rows go to the cache, returns the q latent."""
+    Q, C, ps = qw.numel(), cw.numel(), cache.shape[2]
+    z = z.float()
+    row = torch.cat([norm(z[:, Q:Q + C], cw, eps, False),
+                     turn(z[:, Q + C:], rope[(q_ctx.long() - 1).clamp(min=0)])], 1).to(cache.dtype)
+    ok = slots >= 0
+    s = slots[ok]
+    cache[s // ps, 0, s % ps] = row[ok]
+    return norm(z[:, :Q], qw, eps, False)
+
+
+def latent_attention(q, uk, uv, sink, rope, cache, table, q_seq, q_ctx, scale):
+    H, C, D = uk.shape
+    V, ps, R = uv.shape[1], cache.shape[2], cache.shape[3] - C
+    T = q.shape[0]
+    q = q.float().view(T, H, D + R)
+    qr = turn(q[..., D:], rope[(q_ctx.long() - 1).clamp(min=0)][:, None])
+    u = torch.einsum("thd,hcd->thc", q[..., :D], uk.float())
+    out = torch.zeros(T, H, V, device=q.device)
+    for t in range(T):
+        n = int(q_ctx[t])
+        if n <= 0:
+            continue
+        j = torch.arange(n, device=q.device)
+        rows = cache[table[int(q_seq[t])][j // ps].long(), 0, j % ps].float()
+        s = (u[t] @ rows[:, :C].t() + qr[t] @ rows[:, C:].t()) * scale
+        p = torch.softmax(torch.cat([s, sink[:, None]], 1), -1)[:, :n]
+        out[t] = torch.einsum("hc,hvc->hv", p @ rows[:, :C], uv.float())
+    return out.reshape(T, H * V)

@@ -329,8 +329,8 @@ class StageExecutor:
                             num_pages: Optional[int] = None) -> int:
         """Recurrent states (one slot per session) come out of the cache budget first, pages get the rest."""
         specs = [lay.spec for lay in self.w.layers]
-        rec = [(sp.heads, sp.dim, sp.vdim) for sp in specs if sp.recurrent]
-        att = [(sp.kv_heads, sp.dim) for sp in specs if not sp.recurrent]
+        rec = [sp.state_shapes for sp in specs if sp.recurrent]
+        att = [sp.cache_row for sp in specs if not sp.recurrent]
         if rec:
             self.state = RecurrentState(rec, max_sessions, self.device)
             budget -= self.state.nbytes
@@ -394,7 +394,7 @@ class StageExecutor:
                 d32 = h32[: 2 * T + S].clone()
             return d64, d32
 
-        hp = self._hybrid.plan(ntoks) if self._hybrid is not None and not is_decode else None
+        hp = self._hybrid.plan(ntoks, st) if self._hybrid is not None and not is_decode else None
         qb = sb = fb = None
         fa_waves = 4
         if self.device.type == "cuda" and not is_decode and self._attn_fa:

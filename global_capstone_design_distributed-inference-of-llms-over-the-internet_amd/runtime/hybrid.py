@@ -1,27 +1,32 @@
 """Forward step of the hybrid decoders inside a StageExecutor (``ModelConfig.layers``).
 
-The residual stream is fp32 and lives in one buffer; a sublayer reads its activation copy ``xb`` and its
-RMS-normed, layer-scaled output is added to it:
+The residual stream is fp32 and lives in one buffer; a sublayer f reads an activation ``xb`` made from it.
 
-    z = xb W_in^T          one fused input projection per mixer
-    y = mixer(z) W_o^T     hgrn2: recurrence + head norm; attention: norms + cache write, attention + gate
-    res += rms(y) n1 ; xb = res
-    y = relu2(xb W_up^T) W_down^T
-    res += rms(y) n2 ; xb = res
+    post-norm streams   xb = res ;            res += rms(f(xb)) * gain
+    pre-norm streams    xb = norm(res) gain ; res += mult * f(xb)
+
+One kernel closes a sublayer: it adds the output projection (rows, or the fp32 split-K slabs of a decode GEMM) to the
+stream and writes the next sublayer's ``xb``.  A mixer is one fused input projection z = xb W_in^T, its own ops, and
+an output projection; the feed-forward is squared relu or the clamped gated form.
 
 Activations feeding a decode-sized GEMM stay in the packed MFMA-fragment layout where the shape has a native
 GEMM (``ops.native_gemm_ok``); other shapes, prompts and fp32 run the library GEMM on row-major activations.
-Keys of attention layers live in the executor's paged cache, recurrent states in its ``RecurrentState``.
+Keys and latents of attention layers live in the executor's paged cache, recurrent states in its ``RecurrentState``:
+every layer run has its own, also where a loop runs the same weights again.
 """
 from __future__ import annotations
 
-import math
 from typing import Optional
 
+import numpy as np
 import torch
 
 from .. import ops
 from ..ops import hybrid as hops
+from ..ops import mixers as mops
+
+# most bytes of fp32 partial sums of a latent attention step whose contexts are split
+LATENT_WS_BYTES = 256 << 20
 
 
 class HybridStage:
@@ -31,7 +36,8 @@ class HybridStage:
         self.ex = ex
         cfg = ex.cfg
         self.W, self.eps = cfg.hidden_size, cfg.rms_norm_eps
-        self.inv = hops.position_frequencies(self.W, ex.device)
+        self.pre, self.center, self.mult = cfg.stream == "pre", cfg.norm == "layer", cfg.residual_mult
+        self.inv = hops.position_frequencies(self.W, ex.device) if cfg.embed_positions else None
         # per-layer cache / state index: attention layers count in the paged cache, recurrent ones in the states
         self.index, na, nr = [], 0, 0
         for lay in ex.w.layers:
@@ -41,22 +47,36 @@ class HybridStage:
             else:
                 self.index.append(na)
                 na += 1
+        specs = [lay.spec for lay in ex.w.layers]
+        self.rope = {(sp.rot_base, sp.rot_dims): None for sp in specs if sp.mixer in ("retention", "latent_attention")}
+        for base, dims in self.rope:
+            self.rope[(base, dims)] = mops.rope_table(base, dims, ex.max_seq_len, ex.device)
         # query-block tokens of each attention shape's MFMA form (0: the any-shape form)
-        self.talk_block = {}
-        for lay in ex.w.layers:
-            sp = lay.spec
-            if not sp.recurrent and ex.device.type == "cuda":
-                ok = ex.dtype == torch.bfloat16 and ex.cache.page_size >= 32
+        self.talk_block, self.latent_block = {}, {}
+        for sp in specs if ex.device.type == "cuda" else ():
+            bf16 = ex.dtype == torch.bfloat16
+            if sp.mixer == "attention":
+                ok = bf16 and ex.cache.page_size >= 32
                 self.talk_block[(sp.heads, sp.kv_heads, sp.dim)] = \
                     hops.talk_block(sp.heads, sp.kv_heads, sp.dim) if ok else 0
-        self.rec_heads = min([lay.spec.heads for lay in ex.w.layers if lay.spec.recurrent], default=0)
-        self.max_chunk = max([lay.spec.chunk for lay in ex.w.layers if not lay.spec.recurrent], default=1)
+            elif sp.mixer == "latent_attention":
+                key = self._latent_key(sp)
+                self.latent_block[key] = mops.latent_block(*key, ex.cache.page_size) if bf16 else 0
+        self.rec_heads = min([sp.heads for sp in specs if sp.mixer == "hgrn2"], default=0)
+        self.lin_heads = min([sp.heads for sp in specs if sp.mixer in ("retention", "mlstm")], default=0)
+        self.max_chunk = max([sp.chunk if sp.mixer == "attention" else 1 << 30 for sp in specs if not sp.recurrent],
+                             default=1)
+
+    @staticmethod
+    def _latent_key(sp):
+        return sp.heads, sp.dim, sp.rot_dim, sp.vdim, sp.kv_rank
 
     def autotune(self) -> None:
         """Decode-GEMM kernel choices for this stage's shapes (none while tuning is off)."""
         if ops.autotune_mode() == "off":
             return
-        shapes = {(getattr(lay, n).shape[0], getattr(lay, n).shape[1], 4 if n == "w_up" else 0)
+        up = {"relu2": 4, "clamped_glu": 1}
+        shapes = {(getattr(lay, n).shape[0], getattr(lay, n).shape[1], up[lay.spec.ffn] if n == "w_up" else 0)
                   for lay in self.ex.w.layers for n in lay.GEMMS if getattr(lay, n + "_p") is not None}
         if self.ex.w.lm_head_p is not None:
             shapes.add((self.ex.w.lm_head.shape[0], self.W, 0))
@@ -79,14 +99,105 @@ class HybridStage:
             return ops.linear(x, None, wp=wp, a_rows=T, out=out)
         return ops.linear(x, w, out=out)
 
-    def _add(self, y_in, w, wp, packed: bool, T: int, res, n, xb, xb_packed: bool, e):
-        """res += rms(y_in w^T) n, xb = res.  A packed projection with a split-K form hands its fp32 slabs
-        straight to the norm kernel (no reduce launch, no rounding of y)."""
+    def _add(self, y_in, w, wp, packed: bool, T: int, res, gain, nxt, xb, xb_packed: bool, e):
+        """Close a sublayer: add y = y_in w^T to the stream and write the next sublayer's ``xb``.  ``gain``: the
+        sublayer's own norm gain, ``nxt``: the next one's (None after the last).  A packed projection with a split-K
+        form hands its fp32 slabs straight to the kernel (no reduce launch, no rounding of y)."""
         if packed and ops.rwk_split(T, w.shape[0], w.shape[1]) > 0:
             y = ops.linear_partials(y_in, T, wp=wp, out=e("y", (T, self.W)))
         else:
             y = self._mm(y_in, w, wp, T, packed, e("y", (T, self.W)))
-        hops.residual_norm(y, res, n, self.eps, xb, packed=xb_packed)
+        if self.pre:
+            mops.add_norm(y, res, self.mult, nxt, self.eps, xb if nxt is not None else None, self.center,
+                          packed=xb_packed)
+        else:
+            hops.residual_norm(y, res, gain, self.eps, xb, packed=xb_packed)
+
+    def _enter(self, res, gain, xb, packed: bool) -> None:
+        """``xb`` of a sublayer from the stream alone."""
+        if self.pre:
+            mops.add_norm(None, res, 0.0, gain, self.eps, xb, self.center, packed=packed)
+            return
+        y = res.to(self.ex.dtype)
+        if packed:
+            ops.pack_act(y, out=xb)
+        else:
+            xb.copy_(y)
+
+    # ------------------------------------------------------------------ mixers: z -> the output projection's input
+    def _hgrn2(self, i, lay, z, o, pko, m, e):
+        hops.hgrn2(z, lay.f_bias, lay.f_lower, lay.o_norm, self.ex.state.layer(self.index[i])[0], m["q_seq"], m["q_ctx"],
+                   o, self.eps, plan=m["plan"], packed=pko)
+
+    def _retention(self, i, lay, z, o, pko, m, e):
+        sp = lay.spec
+        mops.retention(z, self.rope[(sp.rot_base, sp.rot_dims)], lay.log_decay, self.ex.state.layer(self.index[i])[0],
+                       m["q_seq"], m["q_ctx"], o, self.eps, plan=m["linear"], packed=pko)
+
+    def _mlstm(self, i, lay, z, o, pko, m, e):
+        state, aux = self.ex.state.layer(self.index[i])
+        mops.mlstm(z, lay.gate_bias, lay.spec.gate_cap, lay.o_norm, state, aux, m["q_seq"], m["q_ctx"], o, self.eps,
+                   plan=m["linear"], packed=pko)
+
+    def _attention(self, i, lay, z, o, pko, m, e):
+        ex, sp, T, plan = self.ex, lay.spec, m["T"], m["plan"]
+        kv, rk = ex.cache.layer(self.index[i])
+        qn = e(f"qn{sp.out_cols}", (T, sp.out_cols))
+        hops.talk_prep(z, lay.w_qk, qn, kv, rk, m["slots"], self.eps)
+        tb = self.talk_block.get((sp.heads, sp.kv_heads, sp.dim), 0)
+        blocks = parts = ws = None
+        if tb and plan is not None:
+            blocks = plan["blocks"][tb]
+        elif tb:
+            parts = hops.talk_parts(T, sp.heads, sp.kv_heads, sp.dim, min(m["span"], sp.chunk), ex._n_cu)
+            if parts[1] > 1:
+                ws = e("talk_ws", (parts[1] * T * sp.heads * (sp.dim + 2),), torch.float32)
+        hops.talk_attention(z, qn, lay.talk, kv, rk, m["table"], m["q_seq"], m["q_ctx"], o, sp.chunk, sp.scale,
+                            packed=pko, sigma=lay.sigma, blocks=blocks, parts=parts, ws=ws)
+
+    def _latent(self, i, lay, z, o, pko, m, e):
+        ex, sp, T, plan = self.ex, lay.spec, m["T"], m["plan"]
+        kv, _ = ex.cache.layer(self.index[i])
+        rope = self.rope[(sp.rot_base, sp.rot_dims)]
+        pkq = self._packed(T, lay.w_uq, lay.w_uq_p)
+        cq = self._act(e, "cq", T, sp.q_rank, pkq)
+        mops.latent_prep(z, lay.q_norm, lay.c_norm, cq, kv, m["slots"], m["q_ctx"], rope, self.eps, packed=pkq)
+        q = self._mm(cq, lay.w_uq, lay.w_uq_p, T, pkq, e(f"q{sp.q_rows}", (T, sp.q_rows)))
+        kw = {}
+        key = self._latent_key(sp)
+        if self.latent_block.get(key, 0):
+            H, C, R = sp.heads, sp.kv_rank, sp.rot_dim
+            kw = dict(u=e("lat_u", (T, H, C + R)), oc=e("lat_oc", (T, H, C)))
+            if plan is not None:
+                kw.update(plan["latent"][key])
+            else:
+                kw["parts"] = mops.latent_parts(T * -(-H // 32), m["span"], ex._n_cu)
+            if kw["parts"][1] > 1:
+                kw["ws"] = e("lat_ws", (kw["parts"][1] * T * H * (C + 2),), torch.float32)
+        mops.latent_attention(q, lay.w_uk, lay.w_uv, lay.sink, rope, kv, m["table"], m["q_seq"], m["q_ctx"], o, sp.scale,
+                              packed=pko, **kw)
+
+    MIX = {"hgrn2": _hgrn2, "retention": _retention, "mlstm": _mlstm, "attention": _attention,
+           "latent_attention": _latent}
+
+    def _ffn(self, lay, xu, pku: bool, T: int, e):
+        """Feed-forward activation (what ``w_down`` reads) and whether it is packed."""
+        sp = lay.spec
+        pkd = self._packed(T, lay.w_down, lay.w_down_p)
+        a = self._act(e, "act", T, sp.ff, pkd)
+        rows = lay.w_up.shape[0]
+        glu = sp.ffn == "clamped_glu"
+        fused = dict(epilogue=1, glu_limit=sp.limit) if glu else dict(epilogue=4)
+        if pku and (not glu or lay.ffn_block == ops.GU_BLOCK) and \
+                ops.native_gemm_ok(T, rows, self.W, fused["epilogue"], pkd):
+            ops.linear(xu, None, wp=lay.w_up_p, a_rows=T, out=a, out_packed=pkd, **fused)  # in the GEMM's epilogue
+            return a, pkd
+        u = self._mm(xu, lay.w_up, lay.w_up_p, T, pku, e(f"u{rows}", (T, rows)))
+        if glu:
+            mops.clamped_glu(u, a, lay.ffn_block, sp.limit, packed=pkd)
+        else:
+            hops.relu2(u, a, packed=pkd)
+        return a, pkd
 
     # ------------------------------------------------------------------ the step
     def forward(self, x, positions, slots, q_seq, q_ctx, last_rows, T, bufs: Optional[dict] = None, plan=None,
@@ -109,55 +220,42 @@ class HybridStage:
             pk = i < len(layers) and self._packed(T, layers[i].w_in, layers[i].w_in_p)
             return pk, self._act(e, "xb", T, W, pk)
 
+        def first_gain(i):  # norm gain ahead of layer i's mixer (pre-norm streams)
+            return layers[i].n1 if i < len(layers) else None
+
         res = torch.empty(T, W, dtype=torch.float32, device=dev)
         pk, xb = entry(0)
-        if ex.is_first:
-            hops.embed_pos(x, ex.w.embed, positions, self.inv, res, xb, packed=pk)
-        else:
+        if not ex.is_first:
             res.copy_(x)
-            self._copy_in(res, xb, pk, T)
-        table = ex.sessions.table_dev
+            if layers:
+                self._enter(res, first_gain(0), xb, pk)
+        elif not self.pre:
+            hops.embed_pos(x, ex.w.embed, positions, self.inv, res, xb, packed=pk)
+        elif layers:
+            mops.embed_norm(x, ex.w.embed, res, first_gain(0), eps, xb, self.center, packed=pk)
+        else:
+            res.copy_(ex.w.embed[x.long()])
+        m = {"T": T, "slots": slots, "q_seq": q_seq, "q_ctx": q_ctx, "plan": plan, "span": span,
+             "linear": plan.get("linear") if plan else None, "table": ex.sessions.table_dev}
         for i, lay in enumerate(layers):
             sp = lay.spec
             if prompt is not None:  # deep prompt: the block input += prompt[i]
                 res.index_add_(0, prompt[0], prompt[1][i].float())
-                self._copy_in(res, xb, pk, T)
+                self._enter(res, first_gain(i), xb, pk)
             z = self._mm(xb, lay.w_in, lay.w_in_p, T, pk, e(f"z{sp.in_rows}", (T, sp.in_rows)))
             pko = self._packed(T, lay.w_o, lay.w_o_p)
             o = self._act(e, "o", T, sp.out_cols, pko)
-            if sp.recurrent:
-                hops.hgrn2(z, lay.f_bias, lay.f_lower, lay.o_norm, ex.state.layer(self.index[i]), q_seq, q_ctx, o, eps,
-                           plan=plan, packed=pko)
-            else:
-                kv, rk = ex.cache.layer(self.index[i])
-                qn = e(f"qn{sp.out_cols}", (T, sp.out_cols))
-                hops.talk_prep(z, lay.w_qk, qn, kv, rk, slots, eps)
-                tb = self.talk_block.get((sp.heads, sp.kv_heads, sp.dim), 0)
-                blocks = parts = ws = None
-                if tb and plan is not None:
-                    blocks = plan["blocks"][tb]
-                elif tb:
-                    parts = hops.talk_parts(T, sp.heads, sp.kv_heads, sp.dim, min(span, sp.chunk), ex._n_cu)
-                    if parts[1] > 1:
-                        ws = e("talk_ws", (parts[1] * T * sp.heads * (sp.dim + 2),), torch.float32)
-                hops.talk_attention(z, qn, lay.talk, kv, rk, table, q_seq, q_ctx, o, sp.chunk, sp.scale, packed=pko,
-                                    sigma=lay.sigma, blocks=blocks, parts=parts, ws=ws)
+            self.MIX[sp.mixer](self, i, lay, z, o, pko, m, e)
             if sp.ff:
                 pku = self._packed(T, lay.w_up, lay.w_up_p)
                 xu = self._act(e, "xb", T, W, pku)
-                self._add(o, lay.w_o, lay.w_o_p, pko, T, res, lay.n1, xu, pku, e)
-                pkd = self._packed(T, lay.w_down, lay.w_down_p)
-                a = self._act(e, "act", T, sp.ff, pkd)
-                if pku and ops.native_gemm_ok(T, sp.ff, W, 4):  # the squared relu in the GEMM's epilogue
-                    ops.linear(xu, None, wp=lay.w_up_p, a_rows=T, out=a, epilogue=4, out_packed=pkd)
-                else:
-                    u = self._mm(xu, lay.w_up, lay.w_up_p, T, pku, e(f"u{sp.ff}", (T, sp.ff)))
-                    hops.relu2(u, a, packed=pkd)
+                self._add(o, lay.w_o, lay.w_o_p, pko, T, res, lay.n1, lay.n2, xu, pku, e)
+                a, pkd = self._ffn(lay, xu, pku, T, e)
                 pk, xb = entry(i + 1)
-                self._add(a, lay.w_down, lay.w_down_p, pkd, T, res, lay.n2, xb, pk, e)
+                self._add(a, lay.w_down, lay.w_down_p, pkd, T, res, lay.n2, first_gain(i + 1), xb, pk, e)
             else:
                 pk, xb = entry(i + 1)
-                self._add(o, lay.w_o, lay.w_o_p, pko, T, res, lay.n1, xb, pk, e)
+                self._add(o, lay.w_o, lay.w_o_p, pko, T, res, lay.n1, first_gain(i + 1), xb, pk, e)
         if not ex.is_last:
             return res
         S, V = last_rows.numel(), ex.cfg.vocab_size
@@ -165,20 +263,18 @@ class HybridStage:
         if S == 0:
             return torch.empty(0, V, dtype=dt, device=dev)
         pkh = self._packed(S, head, ex.w.lm_head_p)
-        fn = hops.rows_norm(res, last_rows, ex.w.final_norm, eps, self._act(e, "fn", S, W, pkh), packed=pkh)
+        fn = self._act(e, "fn", S, W, pkh)
+        if self.pre:
+            mops.rows_norm(res, last_rows, ex.w.final_norm, eps, fn, self.center, packed=pkh)
+        else:
+            hops.rows_norm(res, last_rows, ex.w.final_norm, eps, fn, packed=pkh)
         logits = self._mm(fn, head, ex.w.lm_head_p, S, pkh, torch.empty(S, head.shape[0], dtype=dt, device=dev))
         return logits[:, :V]
 
-    def _copy_in(self, res, xb, packed: bool, T: int) -> None:
-        y = res.to(self.ex.dtype)
-        if packed:
-            ops.pack_act(y, out=xb)
-        else:
-            xb.copy_(y)
-
     # ------------------------------------------------------------------ plans
-    def plan(self, ntoks) -> dict:
-        """Device description of a ragged step (not one token per session)."""
+    def plan(self, ntoks, starts) -> dict:
+        """Device description of a ragged step (not one token per session): ``ntoks`` tokens per session after the
+        ``starts`` it already holds."""
         if self.ex.device.type != "cuda":
             return {}
         up = lambda a: torch.from_numpy(a).to(self.ex.device, non_blocking=True)  # noqa: E731
@@ -187,6 +283,20 @@ class HybridStage:
             h = hops.hgrn2_plan(ntoks, self.rec_heads, self.ex._n_cu)
             p.update(seqs=up(h["seqs"]), seg=up(h["seg"]), multi=up(h["multi"]) if h["slots"] else None,
                      slots=h["slots"])
+        if self.lin_heads:
+            h = hops.hgrn2_plan(ntoks, self.lin_heads, self.ex._n_cu)
+            p["linear"] = {"seqs": up(h["seqs"])}
+        p["latent"] = {}
+        T, span = int(np.sum(ntoks)), int(np.max(np.asarray(ntoks) + np.asarray(starts)))
+        for key, tb in self.latent_block.items():
+            if not tb:
+                continue
+            H, C = key[0], key[4]
+            blk = hops.talk_blocks(ntoks, tb)
+            ps, n = mops.latent_parts(blk.shape[1] * -(-H // 32), span, self.ex._n_cu)
+            if n * T * H * (C + 2) * 4 > LATENT_WS_BYTES:
+                ps, n = 0, 1
+            p["latent"][key] = {"blocks": up(blk), "parts": (ps, n)}
         return p
 
     def span(self, max_ctx: int) -> int:

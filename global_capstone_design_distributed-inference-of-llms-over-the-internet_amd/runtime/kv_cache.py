@@ -106,13 +106,13 @@ class PagedKVCache:
 
 
 class SharedKVCache:
-    """Paged cache of attention layers whose values are their projected keys: one raw row per token and kv head,
-    ``rows[l] : [num_pages, nkv_l, page_size, head_dim_l]``, plus ``rk[l] : [num_pages, page_size]`` fp32, the
-    reciprocal root mean square of the token's whole key row.  Layers may differ in kv heads and head size.
-    Same page ids, allocator and block tables as ``PagedKVCache``."""
+    """Paged cache of attention layers whose keys and values come from one cached row: ``rows[l] : [num_pages, n_l,
+    page_size, d_l]`` (a row per kv head, or one latent row for all heads), and where the layer asks for it one fp32
+    scale per token, ``[num_pages, page_size]``.  Layers may differ in all of it.  Same page ids, allocator and
+    block tables as ``PagedKVCache``."""
 
     def __init__(self, shapes, num_pages: int, page_size: int = 64, dtype=torch.bfloat16, device="cpu"):
-        """``shapes``: (kv heads, head size) of every attention layer."""
+        """``shapes``: (rows, row size, scaled) of every attention layer (``LayerSpec.cache_row``)."""
         assert page_size & (page_size - 1) == 0, "page_size must be a power of two"
         self.shapes = [tuple(s) for s in shapes]
         self.num_layers = len(self.shapes)
@@ -120,12 +120,16 @@ class SharedKVCache:
         self.page_size = page_size
         self.dtype = dtype
         self.device = torch.device(device)
-        self.rows = [torch.zeros(num_pages, n, page_size, d, dtype=dtype, device=self.device) for n, d in self.shapes]
-        self.rk = [torch.zeros(num_pages, page_size, dtype=torch.float32, device=self.device) for _ in self.shapes]
+        self.rows = [torch.zeros(num_pages, n, page_size, d, dtype=dtype, device=self.device)
+                     for n, d, _ in self.shapes]
+        self._rk = [torch.zeros(num_pages, page_size, dtype=torch.float32, device=self.device) if scaled else None
+                    for _, _, scaled in self.shapes]
+        self.rk = [t for t in self._rk if t is not None]
         self.allocator = PageAllocator(num_pages)
 
     def layer(self, i: int):
-        return self.rows[i], self.rk[i]
+        """(rows, scales or None) of attention layer ``i``."""
+        return self.rows[i], self._rk[i]
 
     def copy_pages(self, src: List[int], dst: List[int]) -> None:
         si = torch.tensor(src, dtype=torch.long, device=self.device)
@@ -135,7 +139,7 @@ class SharedKVCache:
 
     @staticmethod
     def page_bytes(shapes, page_size: int, elt_bytes: int) -> int:
-        return sum(page_size * (n * d * elt_bytes + 4) for n, d in shapes)
+        return sum(page_size * (n * d * elt_bytes + (4 if scaled else 0)) for n, d, scaled in shapes)
 
     @property
     def bytes_per_page(self) -> int:

@@ -1,6 +1,7 @@
 """Recurrent state of a stage's recurrent layers, one slot per session row.
 
-A recurrent layer's state replaces its KV cache: a fixed [heads, dim, vdim] fp32 block per session instead of
+A recurrent layer's state replaces its KV cache: a fixed fp32 block per session ([heads, dim, vdim], and
+what else the mixer carries) instead of
 pages that grow with the context.  Slots are the session manager's rows: a row that is handed out again needs no
 clearing, because a sequence's first token starts from a zero state whatever the slot holds.  State cannot be
 rewound: a session continues from its length or starts over.
@@ -13,13 +14,17 @@ import torch
 
 
 class RecurrentState:
-    def __init__(self, shapes: Sequence[Tuple[int, int, int]], max_sessions: int, device="cpu"):
-        """``shapes``: (heads, dim, vdim) of every recurrent layer."""
-        self.states: List[torch.Tensor] = [torch.zeros((max_sessions,) + tuple(s), dtype=torch.float32, device=device)
-                                           for s in shapes]
+    def __init__(self, shapes: Sequence[Sequence[Tuple[int, ...]]], max_sessions: int, device="cpu"):
+        """``shapes``: the shapes of every recurrent layer's tensors (the state matrix [heads, dim, vdim] first)."""
+        self.states: List[torch.Tensor] = []
+        self._layers: List[Tuple[torch.Tensor, ...]] = []
+        for lay in shapes:
+            made = tuple(torch.zeros((max_sessions,) + tuple(s), dtype=torch.float32, device=device) for s in lay)
+            self.states += made
+            self._layers.append(made)
 
-    def layer(self, i: int) -> torch.Tensor:
-        return self.states[i]
+    def layer(self, i: int) -> Tuple[torch.Tensor, ...]:
+        return self._layers[i]
 
     def copy_row(self, src: int, dst: int) -> None:
         for s in self.states:
