@@ -151,7 +151,9 @@ __device__ __forceinline__ u16x4 lds_tr(const bf16_t* p) {
 }
 __device__ __forceinline__ u16x4 pack4(float a, float b, float c, float d) { return (u16x4){f2bf(a), f2bf(b), f2bf(c), f2bf(d)}; }
 
-// u rows of head blockIdx.y for 16 token rows; the four waves take 16-column tiles of C, blockIdx.z splits them
+// u rows of head blockIdx.y for 16 token rows; the four waves take 16-column tiles of C, blockIdx.z splits them.
+// NF: 32-wide slices of D (past D the query fragment is 0 and the weight's last columns repeat: no branch)
+template <int NF>
 __global__ __launch_bounds__(256) void latent_query_kernel(LatentArgs a, int n) {
   const int tid = threadIdx.x, lane = tid & 63, c16 = lane & 15, g4 = lane >> 4;
   const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -159,9 +161,9 @@ __global__ __launch_bounds__(256) void latent_query_kernel(LatentArgs a, int n) 
   const int i = blockIdx.x * 16 + c16;
   const int t = i < n ? (a.rows ? a.rows[i] : i) : -1;
   const bf16_t* q = (const bf16_t*)a.q + (int64_t)max(t, 0) * a.qs + (int64_t)h * (D + R);
-  u16x8 qf[8];
+  u16x8 qf[NF];
 #pragma unroll
-  for (int f = 0; f < 8; ++f) {
+  for (int f = 0; f < NF; ++f) {
     const int d = 32 * f + 8 * g4;
     const u16x8 x = *reinterpret_cast<const u16x8*>(q + min(d, D - 8));
     qf[f] = t >= 0 && d < D ? x : (u16x8)(0);
@@ -169,12 +171,12 @@ __global__ __launch_bounds__(256) void latent_query_kernel(LatentArgs a, int n) 
   bf16_t* u = (bf16_t*)a.u + ((int64_t)max(t, 0) * a.H + h) * KW;
   for (int ct = blockIdx.z * 4 + w; ct * 16 < C; ct += 4 * gridDim.z) {
     const bf16_t* wk = (const bf16_t*)a.uk + ((int64_t)h * C + ct * 16 + c16) * D;
+    u16x8 wf[NF];
+#pragma unroll
+    for (int f = 0; f < NF; ++f) wf[f] = *reinterpret_cast<const u16x8*>(wk + min(32 * f + 8 * g4, D - 8));
     f32x4 x = (f32x4)(0.f);
 #pragma unroll
-    for (int f = 0; f < 8; ++f) {
-      if (32 * f >= D) break;
-      x = mfma_l(*reinterpret_cast<const u16x8*>(wk + min(32 * f + 8 * g4, D - 8)), qf[f], x);
-    }
+    for (int f = 0; f < NF; ++f) x = mfma_l(wf[f], qf[f], x);
     if (t >= 0) *reinterpret_cast<u16x4*>(u + ct * 16 + 4 * g4) = pack4(x[0], x[1], x[2], x[3]);
   }
   if (blockIdx.z == 0 && t >= 0 && a.q_ctx[t] > 0) {
@@ -326,8 +328,7 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(LatentArgs a, const in
       const bf16_t* vb = kt + (32 * kb + 8 * g4 + (c16 >> 2)) * STR + 4 * (c16 & 3);
 #pragma unroll
       for (int t = 0; t < CW; ++t) {
-        const int ct = w * CW + t;
-        if (ct * 16 >= C) break;  // (uniform)
+        const int ct = min(w * CW + t, (C >> 4) - 1);  // (a tile past C repeats the last one and is not stored)
         const u16x4 v0 = lds_tr(vb + 16 * ct), v1 = lds_tr(vb + 4 * STR + 16 * ct);
         const u16x8 va = {v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
 #pragma unroll
@@ -516,7 +517,9 @@ extern "C" int mp_latent_attention(int form, const void* q, int64_t qs, const vo
   const int nb16 = (n + 15) / 16;
   const int ctiles = (C / 16 + 3) / 4, vtiles = ((V + 15) / 16 + 3) / 4;
   const int zq = nb16 * H >= 1024 ? 1 : ctiles, zv = nb16 * H >= 1024 ? 1 : vtiles;
-  hipLaunchKernelGGL(latent_query_kernel, dim3(nb16, H, zq), dim3(256), 0, stream, a, n);
+  if (D <= 64) hipLaunchKernelGGL(latent_query_kernel<2>, dim3(nb16, H, zq), dim3(256), 0, stream, a, n);
+  else if (D <= 128) hipLaunchKernelGGL(latent_query_kernel<4>, dim3(nb16, H, zq), dim3(256), 0, stream, a, n);
+  else hipLaunchKernelGGL(latent_query_kernel<8>, dim3(nb16, H, zq), dim3(256), 0, stream, a, n);
   int rc = (int)hipGetLastError();
   if (rc) return rc;
   const dim3 grid(blk ? nblk : T, (H + 16 * rt - 1) / (16 * rt), NP);

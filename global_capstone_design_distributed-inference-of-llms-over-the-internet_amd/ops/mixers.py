@@ -59,6 +59,13 @@ def clamped_glu(x, out, block, limit, packed=False):
 
 
 # ------------------------------------------------------------------ scalar-decay linear attention
+def linear_plan(ntoks, heads: int, n_cu: int = 256, seg_tokens: int = None):
+    """Segments of a ragged step, cut at whole blocks of 32 tokens (``hybrid.hgrn2_plan``)."""
+    from .hybrid import hgrn2_plan
+
+    return hgrn2_plan(ntoks, heads, n_cu, seg_tokens)
+
+
 def _scan_plan(plan):
     return None if plan is None else plan["seqs"]
 
