@@ -13,6 +13,13 @@ int mp_linear_scan(int kind, const void* z, int64_t zs, const float* rope, int r
                    const float* bias, const float* norm, float* state, float* aux, const int32_t* q_seq,
                    const int32_t* q_ctx, void* out, int H, int D, int V, float cap, float eps, float qs, float ks,
                    const int32_t* seg, int nseg, int n, int packed_mt, int f32, hipStream_t stream);
+int64_t mp_linear_slot(int D, int V);
+int mp_linear_chunk_ok(int D, int V, int rot);
+int mp_linear_chunk(int kind, const void* z, int64_t zs, const float* rope, int rot, const float* decay,
+                    const float* bias, const float* norm, float* state, float* aux, const int32_t* q_seq,
+                    const int32_t* q_ctx, void* out, int H, int D, int V, float cap, float eps, float qs, float ks,
+                    const int32_t* seg, int nseg, const int32_t* multi, int nm, float* ws, int packed_mt,
+                    hipStream_t stream);
 int mp_latent_prep(const void* z, int64_t zs, const float* qw, const float* cw, void* cq, void* cache,
                    const int64_t* slots, const int32_t* q_ctx, const float* rope, int n, int Q, int C, int R, float eps,
                    int packed_q, int f32, hipStream_t stream);
@@ -162,6 +169,39 @@ void linear_scan(int64_t kind, const at::Tensor& z, const opt_tensor& rope, cons
                "linear_scan");
 }
 
+int64_t linear_slot(int64_t D, int64_t V) { return mp_linear_slot((int)D, (int)V); }
+bool linear_chunk_ok(int64_t D, int64_t V, int64_t rot) { return mp_linear_chunk_ok((int)D, (int)V, (int)rot) != 0; }
+
+// seg [4, nseg] (first token, tokens, state source, state target), multi [4, nm] (first slot, slots, first token, -):
+// csrc/linear_attn.hip.  ``slots``: workspace slots the segments name.
+void linear_chunk(int64_t kind, const at::Tensor& z, const opt_tensor& rope, const opt_tensor& decay,
+                  const opt_tensor& bias, const opt_tensor& norm, at::Tensor& state, const opt_tensor& aux,
+                  const at::Tensor& q_seq, const at::Tensor& q_ctx, at::Tensor& out, double cap, double eps, double qs,
+                  double ks, const at::Tensor& seg, const opt_tensor& multi, int64_t slots, const opt_tensor& ws,
+                  int64_t packed) {
+  const LinShape s = check_linear(kind, z, rope, decay, bias, norm, state, aux);
+  MP_CHECK(!s.f32, "the chunk form is bf16");
+  const int mt = check_out(out, s.T, s.H * s.V, s.f32, packed, "out");
+  MP_CHECK(seg.dim() == 2 && seg.size(0) == 4, "seg int32 [4, nseg]");
+  const int64_t nseg = seg.size(1);
+  const int32_t* mp = nullptr;
+  int64_t nm = 0;
+  float* wp = nullptr;
+  if (multi.has_value() && multi->numel()) {
+    MP_CHECK(multi->dim() == 2 && multi->size(0) == 4 && ws.has_value(), "multi int32 [4, nm] with a workspace");
+    nm = multi->size(1);
+    mp = i32_vec(*multi, 4 * nm, "multi");
+    MP_CHECK(ws->is_cuda() && ws->scalar_type() == at::kFloat && ws->is_contiguous() &&
+                 ws->numel() >= slots * s.H * mp_linear_slot(s.D, s.V), "ws: fp32, a slot per head and segment");
+    wp = ws->data_ptr<float>();
+  }
+  check_launch(mp_linear_chunk(s.mlstm, z.data_ptr(), z.stride(0), s.rope, s.rot, s.decay, s.bias, s.norm,
+                               state.data_ptr<float>(), s.aux, i32_vec(q_seq, s.T, "q_seq"), i32_vec(q_ctx, s.T, "q_ctx"),
+                               out.data_ptr(), s.H, s.D, s.V, (float)cap, (float)eps, (float)qs, (float)ks,
+                               i32_vec(seg, 4 * nseg, "seg"), nseg, mp, nm, wp, mt, cur_stream()),
+               "linear_chunk");
+}
+
 int page_log2_of(const at::Tensor& cache, int f32) {
   check_act(cache, f32, "cache");
   MP_CHECK(cache.dim() == 4 && cache.is_contiguous() && cache.size(1) == 1, "cache [pages, 1, page, C + R]");
@@ -267,6 +307,12 @@ TORCH_LIBRARY_FRAGMENT(mpamd, m) {
       "Tensor(b!)? aux, Tensor q_seq, Tensor q_ctx, Tensor(c!) out, float cap, float eps, float qs, float ks, Tensor? "
       "seg, int packed) -> ()");
   m.def(
+      "linear_chunk(int kind, Tensor z, Tensor? rope, Tensor? decay, Tensor? bias, Tensor? norm, Tensor(a!) state, "
+      "Tensor(b!)? aux, Tensor q_seq, Tensor q_ctx, Tensor(c!) out, float cap, float eps, float qs, float ks, Tensor seg, "
+      "Tensor? multi, int slots, Tensor(d!)? ws, int packed) -> ()");
+  m.def("linear_slot(int D, int V) -> int", &linear_slot);
+  m.def("linear_chunk_ok(int D, int V, int rot) -> bool", &linear_chunk_ok);
+  m.def(
       "latent_prep(Tensor z, Tensor qw, Tensor cw, Tensor(a!) cq, Tensor(b!) cache, Tensor slots, Tensor q_ctx, Tensor "
       "rope, float eps, int packed) -> ()");
   m.def("latent_block(int H, int D, int R, int V, int C, int page) -> int", &latent_block);
@@ -282,6 +328,7 @@ TORCH_LIBRARY_IMPL(mpamd, CUDA, m) {
   m.impl("rows_stream_norm", &rows_stream_norm);
   m.impl("clamped_glu", &clamped_glu);
   m.impl("linear_scan", &linear_scan);
+  m.impl("linear_chunk", &linear_chunk);
   m.impl("latent_prep", &latent_prep);
   m.impl("latent_attention", &latent_attention);
 }

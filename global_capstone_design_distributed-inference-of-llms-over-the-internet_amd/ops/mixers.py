@@ -60,14 +60,10 @@ def clamped_glu(x, out, block, limit, packed=False):
 
 # ------------------------------------------------------------------ scalar-decay linear attention
 def linear_plan(ntoks, heads: int, n_cu: int = 256, seg_tokens: int = None):
-    """Segments of a ragged step, cut at whole blocks of 32 tokens (``hybrid.hgrn2_plan``)."""
+    """Segments of a ragged step, shared with the gated recurrence (``hybrid.hgrn2_plan``)."""
     from .hybrid import hgrn2_plan
 
     return hgrn2_plan(ntoks, heads, n_cu, seg_tokens)
-
-
-def _scan_plan(plan):
-    return None if plan is None else plan["seqs"]
 
 
 def retention(z, rope, log_decay, state, q_seq, q_ctx, out, eps, plan=None, packed=False):
@@ -90,8 +86,16 @@ def mlstm(z, bias, cap, norm_w, state, aux, q_seq, q_ctx, out, eps, plan=None, p
 
 
 def _linear(kind, z, rope, decay, bias, norm_w, state, aux, q_seq, q_ctx, out, cap, eps, qs, ks, plan, packed):
-    torch.ops.mpamd.linear_scan(kind, z, rope, decay, bias, norm_w, state, aux, q_seq, q_ctx, out, float(cap), float(eps),
-                                float(qs), float(ks), _scan_plan(plan), int(packed))
+    _, H, D, V = state.shape
+    head = (kind, z, rope, decay, bias, norm_w, state, aux, q_seq, q_ctx, out, float(cap), float(eps), float(qs), float(ks))
+    if plan is not None and not plan.get("scan") and z.dtype == torch.bfloat16 and z.stride(0) % 8 == 0 and \
+            torch.ops.mpamd.linear_chunk_ok(D, V, 0 if rope is None else rope.shape[1]):
+        slots = plan["slots"]
+        ws = torch.empty(slots * H * torch.ops.mpamd.linear_slot(D, V), dtype=torch.float32, device=z.device) \
+            if slots else None
+        torch.ops.mpamd.linear_chunk(*head, plan["seg"], plan["multi"], slots, ws, int(packed))
+        return out
+    torch.ops.mpamd.linear_scan(*head, None if plan is None else plan["seqs"], int(packed))
     return out
 
 

@@ -284,8 +284,9 @@ class HybridStage:
             p.update(seqs=up(h["seqs"]), seg=up(h["seg"]), multi=up(h["multi"]) if h["slots"] else None,
                      slots=h["slots"])
         if self.lin_heads:
-            h = hops.hgrn2_plan(ntoks, self.lin_heads, self.ex._n_cu)
-            p["linear"] = {"seqs": up(h["seqs"])}
+            h = mops.linear_plan(ntoks, self.lin_heads, self.ex._n_cu)
+            p["linear"] = {"seqs": up(h["seqs"]), "seg": up(h["seg"]), "slots": h["slots"],
+                           "multi": up(h["multi"]) if h["slots"] else None}
         p["latent"] = {}
         T, span = int(np.sum(ntoks)), int(np.max(np.asarray(ntoks) + np.asarray(starts)))
         for key, tb in self.latent_block.items():
