@@ -314,11 +314,13 @@ def main(argv=None):
                     help="instead of the headline workload: prefill / decode throughput of the hybrid decoder's layers "
                          "beside the closest uniform model at these widths (one GPU, one JSON line)")
     ap.add_argument("--layer-bench-layers", type=int, default=8)
+    ap.add_argument("--layer-model", choices=("kafunex", "fubapel"), default="kafunex",
+                    help="the hybrid decoder that --layer-bench measures")
     a = ap.parse_args(argv)
     if a.layer_bench:
         from src.layer_bench import main as layer_bench_main
 
-        return layer_bench_main(a.layer_bench, a.layer_bench_layers)
+        return layer_bench_main(a.layer_bench, a.layer_bench_layers, a.layer_model)
 
     from src import ops
     from src.models.config import resolve_model

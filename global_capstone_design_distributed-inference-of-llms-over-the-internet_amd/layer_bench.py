@@ -1,10 +1,13 @@
-"""Prefill and decode throughput of a hybrid decoder's layers beside the closest uniform family at equal size.
+"""Prefill and decode throughput of a hybrid decoder's layers beside the closest other families at equal size.
 
-``python bench.py --layer-bench`` (one GPU): for every width, an 8-layer Kafunex stage (three recurrent layers, then
-one attention layer) and an 8-layer Llama stage of the same width, query / kv heads, head size and feed-forward
-parameters, both bf16 with random weights, run in turn on the same executor code: prompts of several shapes, then
-decode steps (hipGraph replays) at several batch sizes, at contexts that end inside a 1024-token attention chunk (a
-query then sees as many keys on both sides).  One JSON line.
+``python bench.py --layer-bench [--layer-model kafunex|fubapel]`` (one GPU): for every width an 8-layer stage of the
+model and of its like, of the same width, query heads, head size and feed-forward parameters, all bf16 with random
+weights, run in turn on the same executor code: prompts of several shapes, then decode steps (hipGraph replays) at
+several batch sizes, at contexts that end inside a 1024-token attention chunk (a query then sees as many keys on all
+sides).  One JSON line.
+
+* ``kafunex``: (three recurrent layers, one attention layer) x 2, beside Llama;
+* ``fubapel``: (retention, latent attention, mLSTM, latent attention) x 2, beside Kafunex and Llama.
 """
 from __future__ import annotations
 
@@ -22,11 +25,11 @@ PREFILL = ((1, 8192), (8, 1024), (64, 128))
 DECODE = (1, 16, 64)
 
 
-def configs(width: int, layers: int):
-    """(hybrid, uniform) model configs of one width: head size 128, four query heads per kv head."""
+def configs(width: int, layers: int, model: str = "kafunex"):
+    """Model configs of one width, the measured one first: head size 128, four query heads per kv head."""
     H = width // 128
     G = max(1, H // 4)
-    ff_glu = 128 * (7 * width // 2 // 128)             # gated feed-forward of the uniform model: 3 matrices
+    ff_glu = 128 * (7 * width // 2 // 128)             # gated feed-forward: 3 matrices
     ff = 128 * (3 * ff_glu // 2 // 128)                 # equal parameters in 2 matrices
     rec = LayerSpec("hgrn2", H, 128, 128, ff)
     att = LayerSpec("attention", H, 128, 128, ff, G, 1024, 128 ** -0.5)
@@ -35,14 +38,23 @@ def configs(width: int, layers: int):
     uni = ModelConfig(vocab_size=VOCAB, hidden_size=width, intermediate_size=ff_glu, num_hidden_layers=layers,
                       num_attention_heads=H, num_key_value_heads=G, head_dim=128, max_position_embeddings=16384,
                       name=f"llama-w{width}")
-    return hyb, uni
+    if model == "kafunex":
+        return hyb, uni
+    glu = dict(ff=ff_glu, ffn="clamped_glu", limit=7.0)
+    ret = LayerSpec("retention", H, 128, 128, rot_dims=128, decay=tuple(1 - 2.0 ** (-5 - h % 8) for h in range(H)), **glu)
+    mem = LayerSpec("mlstm", H, 128, 128, gate_cap=15.0, **glu)
+    mla = LayerSpec("latent_attention", H, 128, 128, scale=192 ** -0.5, q_rank=3 * width // 8, kv_rank=512, rot_dim=64,
+                    rot_dims=64, **glu)
+    fub = hybrid_config("fubapel", VOCAB, width, 1e-6, [(ret, mla, mem, mla)[i % 4] for i in range(layers)],
+                        f"fubapel-w{width}", stream="pre", norm="layer", residual_mult=0.5, embed_positions=False)
+    return fub, hyb, uni
 
 
 class Side:
     def __init__(self, cfg, device, max_len: int):
         w = random_stage_weights(cfg, 0, cfg.num_hidden_layers, has_embed=True, has_head=True, device=device, seed=1)
         self.cfg, self.device = cfg, device
-        self.ex = StageExecutor(cfg, w, device, kv_cache_bytes=24 << 30, max_sessions=max(DECODE),
+        self.ex = StageExecutor(cfg, w, device, kv_cache_bytes=16 << 30, max_sessions=max(DECODE),
                                 max_seq_len=max_len, max_tokens_per_step=8192, warmup=False)
         self.gen = torch.Generator(device=device).manual_seed(7)
 
@@ -83,11 +95,12 @@ def _in_turn(sides, call, iters: int, rounds: int):
     return {k: statistics.median(v) for k, v in t.items()}
 
 
-def run(widths, layers: int = 8, ctx: int = 896, device="cuda:0", steps: int = 16, rounds: int = 3, log=None) -> dict:
+def run(widths, layers: int = 8, ctx: int = 896, device="cuda:0", steps: int = 16, rounds: int = 3, log=None,
+        model: str = "kafunex") -> dict:
     out = []
     with torch.no_grad():
         for width in widths:
-            sides = {c.name.split("-")[0]: Side(c, device, 8704) for c in configs(width, layers)}
+            sides = {c.name.split("-")[0]: Side(c, device, 8704) for c in configs(width, layers, model)}
             row = {"width": width, "layers": layers, "prefill": [], "decode": []}
             for b, n in PREFILL:
                 ms = _in_turn(sides, lambda s: s.prefill(b, n), 3, rounds)
@@ -112,14 +125,15 @@ def run(widths, layers: int = 8, ctx: int = 896, device="cuda:0", steps: int = 1
             out.append(row)
             del sides
             torch.cuda.empty_cache()
-    return {"metric": "layer_bench", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic", "rows": out}
+    return {"metric": "layer_bench", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic", "model": model, "rows": out}
 
 
-def main(widths: str, layers: int = 8) -> int:
+def main(widths: str, layers: int = 8, model: str = "kafunex") -> int:
     import sys
 
     if not torch.cuda.is_available():
         raise SystemExit("--layer-bench needs a GPU")
-    rec = run([int(w) for w in widths.split(",")], layers, log=lambda m: print(m, file=sys.stderr, flush=True))
+    rec = run([int(w) for w in widths.split(",")], layers, log=lambda m: print(m, file=sys.stderr, flush=True),
+              model=model)
     print(json.dumps(rec), flush=True)
     return 0

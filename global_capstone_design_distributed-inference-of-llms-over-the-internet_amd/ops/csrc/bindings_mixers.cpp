@@ -29,6 +29,11 @@ int mp_latent_attention(int form, const void* q, int64_t qs, const void* uk, con
                         const int32_t* q_ctx, void* u, void* oc, void* out, int T, int H, int D, int R, int V, int C,
                         int page_log2, float scale, const int32_t* rows, int n, const int32_t* blk, int nblk, int PS,
                         int NP, float* part, int packed_mt, int f32, hipStream_t stream);
+int mp_latent_wide_ok(int D, int R, int V, int C);
+int mp_latent_gather(const void* cache, const int64_t* idx, void* out, int64_t n, int KW, hipStream_t stream);
+int mp_latent_wide(const void* q, int64_t qs, const void* kv, int64_t kvs, const void* lat, const float* sink,
+                   const float* rope, const int32_t* q_ctx, void* out, int H, int D, int R, int V, int C, float scale,
+                   const int32_t* blk, int nblk, int nw, int packed_mt, hipStream_t stream);
 }
 
 namespace {
@@ -290,6 +295,42 @@ void latent_attention(const at::Tensor& q, const at::Tensor& uk, const at::Tenso
                "latent_attention");
 }
 
+bool latent_wide_ok(int64_t D, int64_t R, int64_t V, int64_t C) {
+  return mp_latent_wide_ok((int)D, (int)R, (int)V, (int)C) != 0;
+}
+
+// out[i] = cache row idx[i] (a slot: page * page size + offset)
+void latent_gather(const at::Tensor& cache, const at::Tensor& idx, at::Tensor& out) {
+  page_log2_of(cache, 0);
+  const int64_t n = idx.numel(), KW = cache.size(3);
+  check_act(out, 0, "out");
+  MP_CHECK(out.is_contiguous() && out.numel() >= n * KW && KW % 8 == 0, "out [n, C + R]");
+  check_launch(mp_latent_gather(cache.data_ptr(), i64_vec(idx, n, "idx"), out.data_ptr(), n, KW, cur_stream()),
+               "latent_gather");
+}
+
+// Attention over every head's own keys and values: kv [N, H (D + V)] and lat [N, C + R] hold the contexts of the
+// sequences one after the other, blk int32 [3, nblk] the query blocks (first token, tokens, first context row)
+void latent_wide(const at::Tensor& q, const at::Tensor& kv, const at::Tensor& lat, const at::Tensor& sink,
+                 const at::Tensor& rope, const at::Tensor& q_ctx, at::Tensor& out, int64_t D, int64_t V, double scale,
+                 const at::Tensor& blk, int64_t waves, int64_t packed) {
+  const int64_t T = q.size(0), H = sink.numel(), R = rope.size(1), N = kv.size(0), C = lat.size(1) - R;
+  check_act(q, 0, "q");
+  check_act(kv, 0, "kv");
+  check_act(lat, 0, "lat");
+  check_rows(q, T, H * (D + R), "q");
+  check_rows(kv, N, H * (D + V), "kv");
+  MP_CHECK(lat.is_contiguous() && lat.size(0) == N && C > 0, "lat [N, C + R]");
+  MP_CHECK(rope.is_cuda() && rope.dim() == 2 && rope.scalar_type() == at::kFloat && rope.is_contiguous(), "rope");
+  const int mt = check_out(out, T, H * V, 0, packed, "out");
+  MP_CHECK(blk.dim() == 2 && blk.size(0) == 3, "blk int32 [3, nblk]");
+  const int64_t nb = blk.size(1);
+  check_launch(mp_latent_wide(q.data_ptr(), q.stride(0), kv.data_ptr(), kv.stride(0), lat.data_ptr(),
+                              f32_vec(sink, H, "sink"), rope.data_ptr<float>(), i32_vec(q_ctx, T, "q_ctx"), out.data_ptr(),
+                              H, D, R, V, C, (float)scale, i32_vec(blk, 3 * nb, "blk"), nb, (int)waves, mt, cur_stream()),
+               "latent_wide");
+}
+
 }  // namespace
 
 TORCH_LIBRARY_FRAGMENT(mpamd, m) {
@@ -320,6 +361,11 @@ TORCH_LIBRARY_FRAGMENT(mpamd, m) {
       "latent_attention(Tensor q, Tensor uk, Tensor uv, Tensor sink, Tensor rope, Tensor cache, Tensor bt, Tensor q_seq, "
       "Tensor q_ctx, Tensor(a!) out, float scale, int form, Tensor(b!)? u, Tensor(c!)? oc, Tensor? rows, Tensor? blk, "
       "int part_size, int parts, Tensor(d!)? ws, int packed) -> ()");
+  m.def("latent_wide_ok(int D, int R, int V, int C) -> bool", &latent_wide_ok);
+  m.def("latent_gather(Tensor cache, Tensor idx, Tensor(a!) out) -> ()");
+  m.def(
+      "latent_wide(Tensor q, Tensor kv, Tensor lat, Tensor sink, Tensor rope, Tensor q_ctx, Tensor(a!) out, int D, int V, "
+      "float scale, Tensor blk, int waves, int packed) -> ()");
 }
 
 TORCH_LIBRARY_IMPL(mpamd, CUDA, m) {
@@ -331,4 +377,6 @@ TORCH_LIBRARY_IMPL(mpamd, CUDA, m) {
   m.impl("linear_chunk", &linear_chunk);
   m.impl("latent_prep", &latent_prep);
   m.impl("latent_attention", &latent_attention);
+  m.impl("latent_gather", &latent_gather);
+  m.impl("latent_wide", &latent_wide);
 }

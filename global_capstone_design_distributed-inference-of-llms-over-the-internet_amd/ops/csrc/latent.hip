@@ -13,6 +13,9 @@
 //   latent_query_kernel   u, by MFMA: 16 rows of a head at a time
 //   latent_attn_kernel    the core on MFMA: rows = (token, head) against 64-key tiles of the cache, split contexts
 //   latent_value_kernel   merges the splits, applies the sink, W_h by MFMA
+//   latent_gather_kernel, latent_wide_kernel   long portions of prompts: the context's latents in one piece (a library
+//                         GEMM makes every head's keys and values of them), then attention over those, whose scores
+//                         have D + R terms where the shared row's have C + R
 #include "common.h"
 #include "act_io.h"
 
@@ -461,6 +464,222 @@ static int latent_geometry(int H, int D, int R, int V, int C, int page_log2, int
   return 0;
 }
 
+// out[i] = cache row idx[i], 16-B chunks
+__global__ __launch_bounds__(256) void latent_gather_kernel(const bf16_t* __restrict__ cache,
+                                                            const int64_t* __restrict__ idx, bf16_t* __restrict__ out,
+                                                            int64_t n, int KW) {
+  const int cpr = KW >> 3;
+  const int64_t total = n * cpr;
+  for (int64_t i = blockIdx.x * (int64_t)256 + threadIdx.x; i < total; i += (int64_t)gridDim.x * 256) {
+    const int64_t r = i / cpr;
+    const int c = (int)(i - r * cpr) * 8;
+    *reinterpret_cast<u16x8*>(out + r * KW + c) = *reinterpret_cast<const u16x8*>(cache + idx[r] * KW + c);
+  }
+}
+
+// LDS image of a tile of 32 NS columns (16-B chunks ch): 8-row x 32-column subtiles of 512 B, the chunk XOR-swizzled by
+// the row, so that row reads and transposed reads are both free of bank conflicts
+template <int NS>
+__device__ __forceinline__ int lw_off(int row, int ch) {
+  return 512 * NS * (row >> 3) + 512 * (ch >> 2) + 64 * (row & 7) + 16 * ((ch & 3) ^ ((row >> 2) & 3));
+}
+__device__ __forceinline__ f32x16 mfma_lw(const u16x8& a, const u16x8& b, const f32x16& c) {
+  return __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_l, a), __builtin_bit_cast(bf16x8_l, b), c, 0,
+                                                 0, 0);
+}
+__device__ __forceinline__ u16x4 lw_tr(const unsigned char* p) { return lds_tr(reinterpret_cast<const bf16_t*>(p)); }
+
+struct WideArgs {
+  const bf16_t* kv;       // [N, kvs] every context row's keys and values, head by head [D | V]
+  int64_t kvs;
+  const bf16_t* lat;      // [N, C + R] gathered cache rows (the rotated key part lies behind C)
+  const int32_t* blk;     // [3, nblk] first token, tokens, first context row of the sequence
+  int nblk;
+};
+
+// One workgroup: 32 NW query tokens of one head and sequence against 64-key tiles, double-buffered in LDS.
+// S^T = K q^T and O^T += V^T P^T on 32x32x16 MFMA: a lane owns one query row, the softmax is lane-local plus one
+// exchange, the weights go as hi + lo bf16 straight from the accumulators.  DF, RF, VF: 32-column slices of D, R, V.
+// A long query block and its short mirror are taken by one workgroup, so all stream about the same context.
+template <int DF, int RF, int VF, int NW>
+__global__ __launch_bounds__(NW * 64) void latent_wide_kernel(LatentArgs a, WideArgs b) {
+  constexpr int NSK = DF + RF, KT = 64 * 64 * NSK, VT = 64 * 64 * VF, NT = NW * 64;  // tile bytes
+  constexpr int KCH = 64 * 4 * NSK / NT, VCH = 64 * 4 * VF / NT;
+  static_assert(64 * 4 * NSK % NT == 0 && 64 * 4 * VF % NT == 0, "tile chunks split evenly over the threads");
+  extern __shared__ __attribute__((aligned(16))) unsigned char lw[];
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int H = a.H, D = a.D, R = a.R, V = a.V, C = a.C, KW = C + R;
+  const int NBP = (b.nblk + 1) / 2, G = gridDim.x;
+  int lin = blockIdx.x;
+  if ((G & 7) == 0) lin = (lin & 7) * (G >> 3) + (lin >> 3);  // a head's query blocks share an XCD's L2
+  const int h = lin / NBP, jb = lin - h * NBP;
+  const int r = lane & 31, hh = lane >> 5;
+  const float sl2 = a.scale * LOG2E_F;
+  const int npass = b.nblk - 1 - jb != jb ? 2 : 1;
+  for (int pass = 0; pass < npass; ++pass) {
+    const int bx = pass == 0 ? b.nblk - 1 - jb : jb;
+    const int tok0 = b.blk[bx], ntok = b.blk[b.nblk + bx];
+    const int64_t row0 = b.blk[2 * b.nblk + bx];
+    const int end = a.q_ctx[tok0 + ntok - 1];
+    const int wt = 32 * w;
+    const bool wave_rows = wt < ntok;
+    const int wave_ctx = wave_rows ? a.q_ctx[tok0 + min(wt + 31, ntok - 1)] : 0;
+    const int wave_lim0 = wave_rows ? a.q_ctx[tok0 + wt] : 0;  // smallest limit of its rows
+    const bool row_ok = wt + r < ntok;
+    const int tok = tok0 + min(wt + r, ntok - 1);
+    const int lim = row_ok ? a.q_ctx[tok] : 0;
+
+    u16x8 qf[2 * NSK];
+    {
+      const bf16_t* q = (const bf16_t*)a.q + (int64_t)tok * a.qs + (int64_t)h * (D + R);
+#pragma unroll
+      for (int s = 0; s < 2 * DF; ++s) {
+        const int d = 16 * s + 8 * hh;
+        const u16x8 x = *reinterpret_cast<const u16x8*>(q + min(d, D - 8));
+        qf[s] = row_ok && d < D ? x : (u16x8)(0);
+      }
+      const int half = R >> 1;
+      const float* cs = a.rope + (int64_t)(max(a.q_ctx[tok], 1) - 1) * R;
+#pragma unroll
+      for (int s = 0; s < 2 * RF; ++s) {
+        const int d = min(16 * s + 8 * hh, R - 8), e = d < half ? d + half : d - half, f = d < half ? d : e;
+        const u16x8 x = *reinterpret_cast<const u16x8*>(q + D + d), y = *reinterpret_cast<const u16x8*>(q + D + e);
+        u16x8 z;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+          const float c = cs[f + j], sn = d < half ? -cs[half + f + j] : cs[half + f + j];
+          z[j] = f2bf(bf2f(x[j]) * c + bf2f(y[j]) * sn);
+        }
+        qf[2 * DF + s] = row_ok && 16 * s + 8 * hh < R ? z : (u16x8)(0);
+      }
+    }
+    f32x16 o[VF];
+#pragma unroll
+    for (int t = 0; t < VF; ++t) o[t] = (f32x16)(0.f);
+    float m = -INFINITY, l = 0.f;
+
+    u16x8 kreg[KCH], vreg[VCH];
+    auto fetch = [&](int s0) {
+#pragma unroll
+      for (int j = 0; j < KCH; ++j) {
+        const int c = tid + NT * j, row = c / (4 * NSK), ch = c - row * (4 * NSK);
+        const int64_t cr = row0 + min(s0 + row, end - 1);
+        const bf16_t* p = ch < 4 * DF ? b.kv + cr * b.kvs + h * (D + V) + min(ch * 8, D - 8)
+                                      : b.lat + cr * KW + C + min((ch - 4 * DF) * 8, R - 8);
+        kreg[j] = *reinterpret_cast<const u16x8*>(p);
+      }
+#pragma unroll
+      for (int j = 0; j < VCH; ++j) {
+        const int c = tid + NT * j, row = c / (4 * VF), ch = c - row * (4 * VF);
+        vreg[j] = *reinterpret_cast<const u16x8*>(b.kv + (row0 + min(s0 + row, end - 1)) * b.kvs + h * (D + V) + D +
+                                                  min(ch * 8, V - 8));
+      }
+    };
+    // (columns past D and R meet a 0 in q, columns past V are not stored, rows past the context repeat the last one
+    // and meet a weight of 0)
+    auto stash = [&](int buf) {
+      unsigned char* kb = lw + buf * (KT + VT);
+#pragma unroll
+      for (int j = 0; j < KCH; ++j) {
+        const int c = tid + NT * j, row = c / (4 * NSK), ch = c - row * (4 * NSK);
+        *reinterpret_cast<u16x8*>(kb + lw_off<NSK>(row, ch)) = kreg[j];
+      }
+#pragma unroll
+      for (int j = 0; j < VCH; ++j) {
+        const int c = tid + NT * j, row = c / (4 * VF), ch = c - row * (4 * VF);
+        *reinterpret_cast<u16x8*>(kb + KT + lw_off<VF>(row, ch)) = vreg[j];
+      }
+    };
+    const int grp = lane >> 4, gi = lane & 15, tq = gi >> 2, tp = gi & 3;
+    const int kb0 = lw_off<NSK>(r, hh), kb1 = lw_off<NSK>(r, 2 + hh);
+    const int trc = 2 * (grp & 1) + (tp >> 1);
+    const int vb0 = KT + lw_off<VF>(4 * hh + tq, trc) + 8 * (tp & 1), vb1 = KT + lw_off<VF>(8 + 4 * hh + tq, trc) + 8 * (tp & 1);
+
+    fetch(0);
+    stash(0);
+    __syncthreads();
+    int cur = 0;
+    for (int s0 = 0; s0 < end; s0 += 64, cur ^= 1) {
+      const bool more = s0 + 64 < end;
+      if (more) fetch(s0 + 64);
+      if (s0 < wave_ctx) {
+        const unsigned char* tb = lw + cur * (KT + VT);
+        f32x16 st[2];
+        st[0] = st[1] = (f32x16)(0.f);
+#pragma unroll
+        for (int s = 0; s < 2 * NSK; ++s)
+#pragma unroll
+          for (int sub = 0; sub < 2; ++sub)
+            st[sub] = mfma_lw(*reinterpret_cast<const u16x8*>(tb + ((s & 1) ? kb1 : kb0) + 2048 * NSK * sub + 512 * (s >> 1)),
+                              qf[s], st[sub]);
+        if (s0 + 64 > wave_lim0) {  // diagonal and last tiles
+#pragma unroll
+          for (int sub = 0; sub < 2; ++sub)
+#pragma unroll
+            for (int j = 0; j < 16; ++j)
+              st[sub][j] = s0 + 32 * sub + 4 * hh + (j & 3) + 8 * (j >> 2) < lim ? st[sub][j] : -INFINITY;
+        }
+        float lm = -INFINITY;
+#pragma unroll
+        for (int sub = 0; sub < 2; ++sub)
+#pragma unroll
+          for (int j = 0; j < 16; ++j) lm = fmaxf(lm, st[sub][j]);
+        lm = fmaxf(lm, __shfl_xor(lm, 32, 64)) * sl2;
+        if (!__all(lm <= m + LT_GROW)) {
+          const float mn = fmaxf(m, lm), al = mn == -INFINITY ? 1.f : __builtin_amdgcn_exp2f(m - mn);
+          l *= al;
+#pragma unroll
+          for (int t = 0; t < VF; ++t) o[t] *= al;
+          m = mn;
+        }
+        const float mu = m == -INFINITY ? 0.f : m;
+#pragma unroll
+        for (int sub = 0; sub < 2; ++sub)
+#pragma unroll
+          for (int s2 = 0; s2 < 2; ++s2) {
+            u16x8 ph, pl;
+#pragma unroll
+            for (int j = 0; j < 8; ++j) {
+              const float x = __builtin_amdgcn_exp2f(__builtin_fmaf(st[sub][8 * s2 + j], sl2, -mu));
+              l += x;
+              ph[j] = f2bf(x);
+              pl[j] = f2bf(x - bf2f(ph[j]));
+            }
+#pragma unroll
+            for (int t = 0; t < VF; ++t) {
+              const int imm = 2048 * VF * sub + 1024 * VF * s2 + 512 * t;
+              const u16x4 v0 = lw_tr(tb + vb0 + imm), v1 = lw_tr(tb + vb1 + imm);
+              const u16x8 va = {v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
+              o[t] = mfma_lw(va, ph, o[t]);
+              o[t] = mfma_lw(va, pl, o[t]);
+            }
+          }
+      }
+      if (more) stash(cur ^ 1);
+      __syncthreads();
+    }
+    l += __shfl_xor(l, 32, 64);
+    if (!row_ok) continue;  // (every tile ended in a barrier: the LDS is free)
+    const float sk = fmaxf(a.sink[h] * LOG2E_F, -1e30f), mf = fmaxf(m, sk);
+    const float f = __builtin_amdgcn_exp2f(m - mf), inv = f / (l * f + __builtin_amdgcn_exp2f(sk - mf));
+#pragma unroll
+    for (int t = 0; t < VF; ++t)
+#pragma unroll
+      for (int gq = 0; gq < 4; ++gq) {
+        const int v = 32 * t + 8 * gq + 4 * hh;
+        if (v >= V) continue;
+        const float y[4] = {o[t][4 * gq] * inv, o[t][4 * gq + 1] * inv, o[t][4 * gq + 2] * inv, o[t][4 * gq + 3] * inv};
+        st_act_vec<4>((bf16_t*)a.out, tok, h * V + v, H * V, a.packed_mt, y);
+      }
+  }
+}
+
+static int latent_wide_form(int D, int R, int V) {
+  if (D % 8 || R % 16 || V % 8) return 0;
+  return D <= 64 && R <= 32 && V <= 64 ? 1 : D <= 128 && R <= 64 && V <= 128 ? 2 : 0;
+}
+
 }  // namespace mp
 
 extern "C" int mp_latent_prep(const void* z, int64_t zs, const float* qw, const float* cw, void* cq, void* cache,
@@ -542,5 +761,51 @@ extern "C" int mp_latent_attention(int form, const void* q, int64_t qs, const vo
   rc = (int)hipGetLastError();
   if (rc) return rc;
   hipLaunchKernelGGL(latent_value_kernel, dim3(nb16, H, zv), dim3(256), 16 * (C + 8) * 2, stream, a, n, pp, NP);
+  return (int)hipGetLastError();
+}
+
+// Query tokens of a block of the wide form per wave (0: it does not cover the shape)
+extern "C" int mp_latent_wide_ok(int D, int R, int V, int C) { return C % 8 == 0 && mp::latent_wide_form(D, R, V) != 0; }
+
+extern "C" int mp_latent_gather(const void* cache, const int64_t* idx, void* out, int64_t n, int KW, hipStream_t stream) {
+  using namespace mp;
+  (void)hipGetLastError();
+  if (n == 0) return 0;
+  if (KW % 8) return -1;
+  int64_t g = (n * (KW / 8) + 255) / 256;
+  if (g > 16384) g = 16384;
+  hipLaunchKernelGGL(latent_gather_kernel, dim3((unsigned)g), dim3(256), 0, stream, (const bf16_t*)cache, idx, (bf16_t*)out,
+                     n, KW);
+  return (int)hipGetLastError();
+}
+
+// blk [3, nblk]: first token, tokens (<= 32 nw) and first context row of every query block
+extern "C" int mp_latent_wide(const void* q, int64_t qs, const void* kv, int64_t kvs, const void* lat, const float* sink,
+                              const float* rope, const int32_t* q_ctx, void* out, int H, int D, int R, int V, int C,
+                              float scale, const int32_t* blk, int nblk, int nw, int packed_mt, hipStream_t stream) {
+  using namespace mp;
+  (void)hipGetLastError();
+  if (nblk == 0) return 0;
+  const int form = latent_wide_form(D, R, V);
+  if (form == 0 || C % 8 || qs % 8 || kvs % 8 || (nw != 4 && nw != 8)) return -1;
+  LatentArgs a{};
+  a.q = q, a.qs = qs, a.sink = sink, a.rope = rope, a.q_ctx = q_ctx, a.out = out;
+  a.H = H, a.D = D, a.R = R, a.V = V, a.C = C, a.packed_mt = packed_mt, a.scale = scale;
+  const WideArgs b{(const bf16_t*)kv, kvs, (const bf16_t*)lat, blk, nblk};
+  const dim3 grid(H * ((nblk + 1) / 2));
+#define MP_LW(DF_, RF_, VF_, NW_)                                                                                      \
+  {                                                                                                                    \
+    constexpr int lds = 2 * 64 * 64 * (DF_ + RF_ + VF_);                                                               \
+    if (lds > 65536)                                                                                                   \
+      (void)hipFuncSetAttribute((const void*)latent_wide_kernel<DF_, RF_, VF_, NW_>,                                   \
+                                hipFuncAttributeMaxDynamicSharedMemorySize, lds);                                      \
+    hipLaunchKernelGGL((latent_wide_kernel<DF_, RF_, VF_, NW_>), grid, dim3(NW_ * 64), lds, stream, a, b);              \
+  }
+  if (form == 1) {
+    if (nw == 4) MP_LW(2, 1, 2, 4) else { return -1; }
+  } else {
+    if (nw == 4) MP_LW(4, 2, 4, 4) else MP_LW(4, 2, 4, 8)
+  }
+#undef MP_LW
   return (int)hipGetLastError();
 }

@@ -224,7 +224,7 @@ struct ChunkLds {
 };
 
 template <int KIND, int DF, int VT, bool STATE>
-__global__ __launch_bounds__(256, DF * VT > 16 ? 1 : 2) void linear_chunk_kernel(LinArgs a, const int32_t* __restrict__ seg,
+__global__ __launch_bounds__(256, DF * VT <= 4 || (DF == 4 && VT == 2) ? 2 : 1) void linear_chunk_kernel(LinArgs a, const int32_t* __restrict__ seg,
                                                                                  int nseg, float* __restrict__ ws) {
   typedef ChunkLds<KIND, DF, VT, STATE> L;
   constexpr int NI = DF > 4 ? DF / 4 : 1;  // pair items of a thread

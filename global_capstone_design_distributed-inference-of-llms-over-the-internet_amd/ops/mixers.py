@@ -138,3 +138,46 @@ def latent_attention(q, uk, uv, sink, rope, cache, table, q_seq, q_ctx, out, sca
                                      0 if u is None else 1, u, oc, rows, blocks, int(parts[0]), int(parts[1]), ws,
                                      int(packed))
     return out
+
+
+# a portion of a prompt of this many tokens or more has its context's keys and values made for every head
+LATENT_WIDE_TOKENS = 64
+
+
+def latent_wide_ok(D: int, R: int, V: int, C: int) -> bool:
+    """Does the form with every head's own keys and values cover the shape?"""
+    return bool(torch.ops.mpamd.latent_wide_ok(int(D), int(R), int(V), int(C)))
+
+
+def latent_wide_plan(ntoks, starts, heads: int, dim: int, n_cu: int = 256, max_rows: int = 1 << 62):
+    """Sequences of a ragged step that take the wide form: (sequence numbers, int32 ``blk`` [3, nblk], waves), None when
+    there is none.  ``max_rows``: context rows at most; sequences past it keep the other form."""
+    pick, rows, base = [], 0, []
+    for i, (n, s) in enumerate(zip(np.asarray(ntoks).tolist(), np.asarray(starts).tolist())):
+        if n >= LATENT_WIDE_TOKENS and rows + n + s <= max_rows:
+            pick.append(i)
+            base.append(rows)
+            rows += n + s
+    if not pick:
+        return None
+    off = np.concatenate([[0], np.cumsum(ntoks)[:-1]])
+    for waves in (8, 4):
+        tb = 32 * waves
+        blk = [(off[i] + k, min(tb, ntoks[i] - k), b) for i, b in zip(pick, base) for k in range(0, int(ntoks[i]), tb)]
+        if dim > 64 and heads * len(blk) > 2 * n_cu:  # (the small form has four waves)
+            break
+    return pick, np.ascontiguousarray(np.asarray(blk, dtype=np.int32).reshape(-1, 3).T), waves
+
+
+def latent_gather(cache, idx, out):
+    """out[i] = cache row idx[i] (slots)."""
+    torch.ops.mpamd.latent_gather(cache, idx, out)
+    return out
+
+
+def latent_wide(q, kv, lat, sink, rope, q_ctx, out, D, V, scale, blk, waves, packed=False):
+    """The wide form of ``latent_attention`` for the tokens of ``blk``: ``kv`` [N, H (D + V)] keys and values of the
+    context rows ``lat`` [N, C + R]."""
+    torch.ops.mpamd.latent_wide(q, kv, lat, sink, rope, q_ctx, out, int(D), int(V), float(scale), blk, int(waves),
+                                int(packed))
+    return out

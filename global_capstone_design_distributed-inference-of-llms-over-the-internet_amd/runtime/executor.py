@@ -394,7 +394,7 @@ class StageExecutor:
                 d32 = h32[: 2 * T + S].clone()
             return d64, d32
 
-        hp = self._hybrid.plan(ntoks, st) if self._hybrid is not None and not is_decode else None
+        hp = self._hybrid.plan(ntoks, st, rows) if self._hybrid is not None and not is_decode else None
         qb = sb = fb = None
         fa_waves = 4
         if self.device.type == "cuda" and not is_decode and self._attn_fa:

@@ -27,6 +27,8 @@ from ..ops import mixers as mops
 
 # most bytes of fp32 partial sums of a latent attention step whose contexts are split
 LATENT_WS_BYTES = 256 << 20
+# most bytes of the keys and values that long portions of prompts make of their contexts' latents, per step
+LATENT_KV_BYTES = 4 << 30
 
 
 class HybridStage:
@@ -163,13 +165,23 @@ class HybridStage:
         cq = self._act(e, "cq", T, sp.q_rank, pkq)
         mops.latent_prep(z, lay.q_norm, lay.c_norm, cq, kv, m["slots"], m["q_ctx"], rope, self.eps, packed=pkq)
         q = self._mm(cq, lay.w_uq, lay.w_uq_p, T, pkq, e(f"q{sp.q_rows}", (T, sp.q_rows)))
-        kw = {}
         key = self._latent_key(sp)
+        lp = plan["latent"][key] if plan is not None and self.latent_block.get(key, 0) else None
+        if lp is not None and lp["wide"] is not None:  # long portions: every head's own keys and values
+            wd = lp["wide"]
+            lat = mops.latent_gather(kv, wd["idx"], e("lat_rows", (wd["idx"].numel(), kv.shape[3])))
+            own = e("lat_kv", (lat.shape[0], lay.w_ukv.shape[0]))
+            torch.mm(lat[:, :sp.kv_rank], lay.w_ukv.t(), out=own)
+            mops.latent_wide(q, own, lat, lay.sink, rope, m["q_ctx"], o, sp.dim, sp.vdim, sp.scale, wd["blk"],
+                             wd["waves"], packed=pko)
+            if lp["blocks"] is None:
+                return
+        kw = {}
         if self.latent_block.get(key, 0):
             H, C, R = sp.heads, sp.kv_rank, sp.rot_dim
             kw = dict(u=e("lat_u", (T, H, C + R)), oc=e("lat_oc", (T, H, C)))
-            if plan is not None:
-                kw.update(plan["latent"][key])
+            if lp is not None:
+                kw.update(blocks=lp["blocks"], rows=lp["rows"], parts=lp["parts"])
             else:
                 kw["parts"] = mops.latent_parts(T * -(-H // 32), m["span"], ex._n_cu)
             if kw["parts"][1] > 1:
@@ -272,9 +284,9 @@ class HybridStage:
         return logits[:, :V]
 
     # ------------------------------------------------------------------ plans
-    def plan(self, ntoks, starts) -> dict:
+    def plan(self, ntoks, starts, rows) -> dict:
         """Device description of a ragged step (not one token per session): ``ntoks`` tokens per session after the
-        ``starts`` it already holds."""
+        ``starts`` it already holds; ``rows``: the sessions' rows of the block table."""
         if self.ex.device.type != "cuda":
             return {}
         up = lambda a: torch.from_numpy(a).to(self.ex.device, non_blocking=True)  # noqa: E731
@@ -287,18 +299,38 @@ class HybridStage:
             h = mops.linear_plan(ntoks, self.lin_heads, self.ex._n_cu)
             p["linear"] = {"seqs": up(h["seqs"]), "seg": up(h["seg"]), "slots": h["slots"],
                            "multi": up(h["multi"]) if h["slots"] else None}
-        p["latent"] = {}
-        T, span = int(np.sum(ntoks)), int(np.max(np.asarray(ntoks) + np.asarray(starts)))
-        for key, tb in self.latent_block.items():
-            if not tb:
-                continue
-            H, C = key[0], key[4]
-            blk = hops.talk_blocks(ntoks, tb)
-            ps, n = mops.latent_parts(blk.shape[1] * -(-H // 32), span, self.ex._n_cu)
-            if n * T * H * (C + 2) * 4 > LATENT_WS_BYTES:
-                ps, n = 0, 1
-            p["latent"][key] = {"blocks": up(blk), "parts": (ps, n)}
+        p["latent"] = {key: self._latent_plan(key, tb, ntoks, starts, rows, up)
+                       for key, tb in self.latent_block.items() if tb}
         return p
+
+    def _latent_plan(self, key, tb, ntoks, starts, rows, up) -> dict:
+        """Which sessions' tokens go which way: long portions on the wide form, the rest in query blocks of the other."""
+        H, D, R, V, C = key
+        ntoks, starts = np.asarray(ntoks), np.asarray(starts)
+        off = np.concatenate([[0], np.cumsum(ntoks)[:-1]])
+        wide = mops.latent_wide_plan(ntoks, starts, H, D, self.ex._n_cu, LATENT_KV_BYTES // (2 * H * (D + V))) \
+            if mops.latent_wide_ok(D, R, V, C) else None
+        out = {"wide": None, "blocks": None, "rows": None, "parts": (0, 1)}
+        rest = np.arange(len(ntoks))
+        if wide is not None:
+            pick, blk, waves = wide
+            ps, table = self.ex.cache.page_size, self.ex.sessions.table
+            idx = np.concatenate([(table[rows[i], np.arange(n) // ps].astype(np.int64) * ps + np.arange(n) % ps)
+                                  for i in pick for n in [int(starts[i] + ntoks[i])]])
+            out["wide"] = {"idx": up(idx), "blk": up(blk), "waves": waves}
+            rest = np.setdiff1d(rest, pick)
+        rest = rest[ntoks[rest] > 0]
+        if not rest.size:
+            return out
+        blk = np.concatenate([hops.talk_blocks(ntoks[i:i + 1], tb) + [[off[i]], [0]] for i in rest], 1).astype(np.int32)
+        if wide is not None:
+            out["rows"] = up(np.concatenate([np.arange(off[i], off[i] + ntoks[i]) for i in rest]).astype(np.int32))
+        n, T = int((starts + ntoks)[rest].max()), int(ntoks.sum())
+        parts = mops.latent_parts(blk.shape[1] * -(-H // 32), n, self.ex._n_cu)
+        if parts[1] > 1 and parts[1] * T * H * (C + 2) * 4 <= LATENT_WS_BYTES:
+            out["parts"] = parts
+        out["blocks"] = up(np.ascontiguousarray(blk))
+        return out
 
     def span(self, max_ctx: int) -> int:
         """Most keys a decode query of context <= max_ctx can see."""

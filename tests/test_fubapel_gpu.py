@@ -329,3 +329,71 @@ def test_latent_decode(H, D, R, V, C, splits, page):
     close(run_lat(a, (D + R) ** -0.5, "rows", splits), want, TOL["bf16"])
     if (H * V) % 32 == 0:
         close(run_lat(a, (D + R) ** -0.5, "rows", splits, packed=True), want, TOL["bf16"])
+
+
+def run_wide(a, scale, waves, packed=False):
+    """The form that makes every head's own keys and values of the gathered contexts."""
+    H, D, R, V, C = (a[k] for k in "HDRVC")
+    T, page = a["q"].shape[0], a["page"]
+    ctx = [n + s for n, s in zip(a["ntoks"], a["starts"])]
+    table = a["table"].cpu().long()
+    idx = torch.cat([table[i + 1][torch.arange(n) // page] * page + torch.arange(n) % page for i, n in enumerate(ctx)])
+    lat = mops.latent_gather(a["cache"], idx.to(DEV), torch.empty(len(idx), C + R, dtype=torch.bfloat16, device=DEV))
+    assert torch.equal(lat, a["cache"].view(-1, C + R)[idx.to(DEV)])
+    w = torch.cat([a["uk"], a["uv"]], 1).reshape(H * (D + V), C).to(DEV)
+    kv = lat[:, :C] @ w.t()
+    blk, off, base, tb = [], 0, 0, 32 * waves
+    for n, c in zip(a["ntoks"], ctx):
+        blk += [(off + k, min(tb, n - k), base) for k in range(0, n, tb)]
+        off, base = off + n, base + c
+    out = torch.zeros(ops.packed_numel(T, H * V) if packed else T * H * V, dtype=torch.bfloat16, device=DEV)
+    mops.latent_wide(a["q"], kv, lat, a["sink"].to(DEV), a["rope"], a["q_ctx"], out, D, V, scale,
+                     torch.tensor(blk, dtype=torch.int32).t().contiguous().to(DEV), waves, packed)
+    return ops.unpack_act(out, T, H * V) if packed else out.view(T, H * V)
+
+
+@pytest.mark.parametrize("H,D,R,V,C", [(4, 64, 16, 64, 128), (1, 8, 16, 8, 32), (3, 40, 32, 24, 96), (8, 128, 64, 128, 512),
+                                       (5, 72, 48, 104, 64), (2, 128, 16, 32, 256)])
+@pytest.mark.parametrize("waves", [4, 8])
+def test_latent_wide(H, D, R, V, C, waves):
+    if waves == 8 and D <= 64:
+        pytest.skip("the small form has four waves")
+    a = lat_case([70, 2, 1, 300, 33, 129], [0, 30, 63, 64, 100, 0], H, D, R, V, C, "bf16")
+    want, _ = lat_oracle(a, (D + R) ** -0.5)
+    assert mops.latent_wide_ok(D, R, V, C)
+    close(run_wide(a, (D + R) ** -0.5, waves), want, TOL["bf16"])
+    if (H * V) % 32 == 0:
+        close(run_wide(a, (D + R) ** -0.5, waves, packed=True), want, TOL["bf16"])
+
+
+@pytest.mark.parametrize("form", ["any", "blocks", "rows", "wide"])
+@pytest.mark.parametrize("i,j", [(299, 0), (299, 63), (299, 64), (128, 127), (128, 128), (64, 63), (191, 64), (255, 191)])
+def test_a_far_key_stands_out(form, i, j):
+    """One key among hundreds is what the query asks for: it is found, in a prompt and decoded, wherever its page is;
+    and a key after the query is not seen."""
+    H, D, R, V, C = 4, 64, 16, 64, 128
+    ntoks, starts = ([1], [i]) if form == "rows" else ([i + 1], [0])
+    res = []
+    for q_at, sign in ((i, 1), (i, -1)):
+        a = lat_case(ntoks, starts, H, D, R, V, C, "bf16", spike=(0, q_at, j))
+        if sign < 0:
+            pg, off = int(a["table"][1, j // 64]), j % 64
+            a["cache"][pg, 0, off, :C] *= -1
+            a["seqs"][0][j, a["Q"]:a["Q"] + C] *= -1
+        got = (run_wide(a, 0.3, 4) if form == "wide" else run_lat(a, 0.3, form))[-1]
+        close(got, lat_oracle(a, 0.3)[0][-1], TOL["bf16"])
+        res.append(got.float())
+    assert (res[0] - res[1]).abs().max() > 0.3
+
+
+@pytest.mark.parametrize("form", ["any", "blocks", "rows", "wide"])
+@pytest.mark.parametrize("sink", [-30.0, 0.0, 4.0, 40.0])
+def test_the_sink_counts_once(form, sink):
+    """Among the first keys a sink decides how much is left for them; a towering one leaves nothing."""
+    H, D, R, V, C = 4, 64, 16, 64, 128
+    ntoks, starts = ([1, 1, 1], [0, 1, 130]) if form == "rows" else ([1, 3, 140], [0, 0, 0])
+    a = lat_case(ntoks, starts, H, D, R, V, C, "bf16", sink=torch.full((H,), sink))
+    for splits in (1, 2) if form in ("blocks", "rows") else (1,):
+        got = run_wide(a, 0.2, 4) if form == "wide" else run_lat(a, 0.2, form, splits)
+        close(got, lat_oracle(a, 0.2)[0], TOL["bf16"])
+    assert (got.abs().max() < 1e-3) == (sink == 40.0)
