@@ -47,31 +47,40 @@ struct LatentArgs {
 
 constexpr float LOG2E_F = 1.44269504088896340736f;
 
-template <typename T>
-__global__ __launch_bounds__(256) void latent_prep_kernel(LatentArgs a) {
+// VEC columns a thread and step; NT threads (decode rows are few: more threads, one round of loads)
+template <typename T, int VEC, int NT>
+__global__ __launch_bounds__(NT) void latent_prep_kernel(LatentArgs a) {
   __shared__ float red[16];
-  const int t = blockIdx.x, tid = threadIdx.x;
+  const int t = blockIdx.x, tid = threadIdx.x, Q = a.Q, QC = a.Q + a.C;
   const int64_t slot = a.slots[t];
   if (slot < 0) return;
   const T* z = (const T*)a.z + (int64_t)t * a.zs;
   float sq = 0.f, sc = 0.f;
-  for (int i = tid; i < a.Q; i += 256) {
-    const float x = to_f(z[i]);
-    sq += x * x;
+  for (int i = tid * VEC; i < QC; i += NT * VEC) {
+    float x[VEC], s = 0.f;
+    ld_vec<VEC>(z + i, x);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) s += x[j] * x[j];
+    if (i < Q) sq += s;
+    else sc += s;
   }
-  for (int i = tid; i < a.C; i += 256) {
-    const float x = to_f(z[a.Q + i]);
-    sc += x * x;
-  }
-  sq = 1.f / sqrtf(block_sum(sq, red) / (float)a.Q + a.eps);
+  sq = 1.f / sqrtf(block_sum(sq, red) / (float)Q + a.eps);
   sc = 1.f / sqrtf(block_sum(sc, red) / (float)a.C + a.eps);
-  for (int i = tid; i < a.Q; i += 256) st_act((T*)a.cq, t, i, a.Q, a.packed_q, to_f(z[i]) * sq * a.qw[i]);
   T* row = (T*)a.cache + slot * (a.C + a.R);
-  for (int i = tid; i < a.C; i += 256) from_f(to_f(z[a.Q + i]) * sc * a.cw[i], row[i]);
+  for (int i = tid * VEC; i < QC; i += NT * VEC) {
+    float x[VEC], g[VEC];
+    ld_vec<VEC>(z + i, x);
+    ld_vec<VEC>(i < Q ? a.qw + i : a.cw + i - Q, g);
+    const float s = i < Q ? sq : sc;
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) x[j] *= s * g[j];
+    if (i < Q) st_act_vec<VEC>((T*)a.cq, t, i, Q, a.packed_q, x);
+    else st_vec<VEC>(row + i - Q, x);
+  }
   const float* cs = a.rope + (int64_t)(a.q_ctx[t] - 1) * a.R;
   const int half = a.R >> 1;
-  const T* zr = z + a.Q + a.C;
-  for (int i = tid; i < half; i += 256) {
+  const T* zr = z + QC;
+  for (int i = tid; i < half; i += NT) {
     const float x = to_f(zr[i]), y = to_f(zr[i + half]), c = cs[i], s = cs[half + i];
     from_f(x * c - y * s, row[a.C + i]);
     from_f(y * c + x * s, row[a.C + half + i]);
@@ -196,17 +205,21 @@ __global__ __launch_bounds__(256) void latent_query_kernel(LatentArgs a, int n) 
 constexpr int LT_KEYS = 64, LT_PS = LT_KEYS + 8;
 constexpr float LT_GROW = 8.f;  // log2 units a row's maximum may grow before its sums are rescaled
 
-// A workgroup owns up to 16 RT query rows (token-major x heads) of one sequence.  Per 64-key tile wave w makes the
-// scores of keys 16 w .. + 15 for all rows (S^T = rows u^T: a lane owns one query row), the row maxima meet in LDS,
-// the weights go to LDS as hi + lo bf16 (32-bit in effect), and wave w adds them into its 16 CW of the C value
-// columns (O^T += c^T P^T, c^T by transposed reads of the same tile).  The next tile is in flight in registers.
-template <int RT, int CW>
-__global__ __launch_bounds__(256) void latent_attn_kernel(LatentArgs a, const int32_t* __restrict__ blk, int nblk, int PS,
-                                                          float* __restrict__ part) {
-  constexpr int KPT = 2 * CW + 2;  // 16-B chunks of a tile per thread: C + R <= 64 CW + 64
+// A workgroup of NW waves owns up to 16 RT query rows (token-major x heads) of one sequence.  Per 64-key tile wave w
+// makes the scores of keys 16 (w % 4) .. + 15 for RW of the row tiles (S^T = rows u^T: a lane owns one query row), the
+// row maxima meet in LDS, the weights go to LDS as hi + lo bf16 (32-bit in effect), and wave w adds them into its
+// 16 CW of the C value columns (O^T += c^T P^T, c^T by transposed reads of the same tile).  The next tile is in flight
+// in registers.
+template <int RT, int CW, int NW>
+__global__ __launch_bounds__(NW * 64) void latent_attn_kernel(LatentArgs a, const int32_t* __restrict__ blk, int nblk,
+                                                              int PS, float* __restrict__ part) {
+  constexpr int NT = NW * 64, KPT = 2 * CW + 8 / NW;  // 16-B chunks of a tile per thread: C + R <= 16 CW NW + 64
+  constexpr int RG = NW / 4, RW = RT / RG;
+  static_assert(RT % RG == 0, "row tiles split evenly over the waves");
   extern __shared__ __attribute__((aligned(16))) bf16_t ls[];
   const int tid = threadIdx.x, lane = tid & 63, c16 = lane & 15, g4 = lane >> 4;
   const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int ws = w & 3, rg = w >> 2;
   const int H = a.H, C = a.C, KW = C + a.R, KF = (KW + 31) >> 5, STR = 32 * KF + 8;
   bf16_t *kt = ls, *qt = kt + LT_KEYS * STR, *ph = qt + 16 * RT * STR, *pl = ph + 16 * RT * LT_PS;
   float* wred = (float*)(pl + 16 * RT * LT_PS);  // [4][16 RT]
@@ -223,7 +236,7 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(LatentArgs a, const in
   const float rcp = 1.f / (float)cpr, sl2 = a.scale * LOG2E_F;
 
   // query rows, zero past the row count and past KW; the tile's own columns past KW
-  for (int x = tid; x < 16 * RT * 4 * KF; x += 256) {
+  for (int x = tid; x < 16 * RT * 4 * KF; x += NT) {
     const int r = x / (4 * KF), col = (x - r * 4 * KF) * 8;
     const int rr = min(r, nrow - 1);
     const bf16_t* src = (const bf16_t*)a.u + ((int64_t)(tok0 + rr / hg) * H + h0 + rr % hg) * KW;
@@ -231,35 +244,38 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(LatentArgs a, const in
     *reinterpret_cast<u16x8*>(qt + r * STR + col) = r < nrow && col < KW ? v : (u16x8)(0);
   }
   if (KW & 31)
-    for (int x = tid; x < LT_KEYS * (4 * KF - cpr); x += 256) {
+    for (int x = tid; x < LT_KEYS * (4 * KF - cpr); x += NT) {
       const int r = x / (4 * KF - cpr), col = KW + (x - r * (4 * KF - cpr)) * 8;
       *reinterpret_cast<u16x8*>(kt + r * STR + col) = (u16x8)(0);
     }
 
-  int khi[RT];
   float m[RT], l[RT];
   f32x4 o[RT][CW];
 #pragma unroll
   for (int r = 0; r < RT; ++r) {
-    const int row = 16 * r + c16;
-    khi[r] = row < nrow ? min(a.q_ctx[tok0 + row / hg], s_hi) : 0;
     m[r] = -INFINITY;
     l[r] = 0.f;
 #pragma unroll
     for (int t = 0; t < CW; ++t) o[r][t] = (f32x4)(0.f);
   }
 
+  int khi[RW];
+#pragma unroll
+  for (int r = 0; r < RW; ++r) {
+    const int row = 16 * (rg * RW + r) + c16;
+    khi[r] = row < nrow ? min(a.q_ctx[tok0 + row / hg], s_hi) : 0;
+  }
   u16x8 kreg[KPT];
   auto fetch = [&](int s0) {  // a tile's rows are consecutive in the page; past the context the last row repeats
     const bf16_t* base = (const bf16_t*)a.cache + (((int64_t)bt[s0 >> a.page_log2] << a.page_log2) + (s0 & pmask)) * KW;
     const int lastc = min(LT_KEYS, s_hi - s0) * cpr - 1;
 #pragma unroll
-    for (int k = 0; k < KPT; ++k) kreg[k] = *reinterpret_cast<const u16x8*>(base + min(tid + 256 * k, lastc) * 8);
+    for (int k = 0; k < KPT; ++k) kreg[k] = *reinterpret_cast<const u16x8*>(base + min(tid + NT * k, lastc) * 8);
   };
   auto stash = [&]() {
 #pragma unroll
     for (int k = 0; k < KPT; ++k) {
-      const int x = tid + 256 * k, key = (int)(((float)x + 0.5f) * rcp);
+      const int x = tid + NT * k, key = (int)(((float)x + 0.5f) * rcp);
       if (key < LT_KEYS) *reinterpret_cast<u16x8*>(kt + key * STR + (x - key * cpr) * 8) = kreg[k];
     }
   };
@@ -269,27 +285,28 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(LatentArgs a, const in
     stash();
     if (s0 + LT_KEYS < s_hi) fetch(s0 + LT_KEYS);
     __syncthreads();
-    f32x4 st[RT];
+    f32x4 st[RW];
 #pragma unroll
-    for (int r = 0; r < RT; ++r) st[r] = (f32x4)(0.f);
-    const bf16_t *kp = kt + (16 * w + c16) * STR + 8 * g4, *qp = qt + c16 * STR + 8 * g4;
-#pragma unroll 2
+    for (int r = 0; r < RW; ++r) st[r] = (f32x4)(0.f);
+    const bf16_t *kp = kt + (16 * ws + c16) * STR + 8 * g4, *qp = qt + (16 * rg * RW + c16) * STR + 8 * g4;
+#pragma unroll 3
     for (int f = 0; f < KF; ++f) {
       const u16x8 ka = *reinterpret_cast<const u16x8*>(kp + 32 * f);
 #pragma unroll
-      for (int r = 0; r < RT; ++r) st[r] = mfma_l(ka, *reinterpret_cast<const u16x8*>(qp + 16 * r * STR + 32 * f), st[r]);
+      for (int r = 0; r < RW; ++r) st[r] = mfma_l(ka, *reinterpret_cast<const u16x8*>(qp + 16 * r * STR + 32 * f), st[r]);
     }
 #pragma unroll
-    for (int r = 0; r < RT; ++r) {
+    for (int r = 0; r < RW; ++r) {
+      const int row = 16 * (rg * RW + r) + c16;
       float lm = -INFINITY;
 #pragma unroll
       for (int k = 0; k < 4; ++k) {
-        st[r][k] = s0 + 16 * w + 4 * g4 + k < khi[r] ? st[r][k] * sl2 : -INFINITY;
+        st[r][k] = s0 + 16 * ws + 4 * g4 + k < khi[r] ? st[r][k] * sl2 : -INFINITY;
         lm = fmaxf(lm, st[r][k]);
       }
       lm = fmaxf(lm, __shfl_xor(lm, 16, 64));
       lm = fmaxf(lm, __shfl_xor(lm, 32, 64));
-      if (g4 == 0) wred[w * 16 * RT + 16 * r + c16] = lm;
+      if (g4 == 0) wred[ws * 16 * RT + row] = lm;
     }
     __syncthreads();
 #pragma unroll
@@ -304,15 +321,16 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(LatentArgs a, const in
         for (int t = 0; t < CW; ++t) o[r][t] *= al;
         m[r] = mn;
       }
+      if (r / RW != rg) continue;  // (uniform over the wave: this wave's scores)
       const float mu = m[r] == -INFINITY ? 0.f : m[r];
       float x[4];
 #pragma unroll
       for (int k = 0; k < 4; ++k) {
-        x[k] = __builtin_amdgcn_exp2f(st[r][k] - mu);
+        x[k] = __builtin_amdgcn_exp2f(st[r % RW][k] - mu);
         l[r] += x[k];
       }
       const u16x4 xh = pack4(x[0], x[1], x[2], x[3]);
-      const int off = (16 * r + c16) * LT_PS + 16 * w + 4 * g4;
+      const int off = (16 * r + c16) * LT_PS + 16 * ws + 4 * g4;
       *reinterpret_cast<u16x4*>(ph + off) = xh;
       *reinterpret_cast<u16x4*>(pl + off) =
           pack4(x[0] - bf2f(xh[0]), x[1] - bf2f(xh[1]), x[2] - bf2f(xh[2]), x[3] - bf2f(xh[3]));
@@ -348,7 +366,7 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(LatentArgs a, const in
     float x = l[r];
     x += __shfl_xor(x, 16, 64);
     x += __shfl_xor(x, 32, 64);
-    if (g4 == 0) wred[w * 16 * RT + 16 * r + c16] = x;
+    if (g4 == 0 && r / RW == rg) wred[ws * 16 * RT + 16 * r + c16] = x;
   }
   __syncthreads();
 #pragma unroll
@@ -385,51 +403,87 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(LatentArgs a, const in
 }
 
 // values of head blockIdx.y for 16 token rows: the latent sums go to LDS (merged over NP splits when part is given),
-// then each wave makes 16-column tiles of V
+// then each wave makes 16-column tiles of V.  CF: 32-column slices of C the kernel is built for; the first tile's
+// weights are in flight during the merge
+constexpr int LV_NP = 64;  // splits whose factors fit in LDS (the host gives no more)
+template <int CF>
 __global__ __launch_bounds__(256) void latent_value_kernel(LatentArgs a, int n, const float* __restrict__ part, int NP) {
-  extern __shared__ __attribute__((aligned(16))) bf16_t ls[];  // [16][C + 8]
+  constexpr int STR = 32 * CF + 8;
+  __shared__ __attribute__((aligned(16))) bf16_t ls[16 * STR];
+  __shared__ float fac[16][LV_NP + 1];
   const int tid = threadIdx.x, lane = tid & 63, c16 = lane & 15, g4 = lane >> 4;
   const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int h = blockIdx.y, H = a.H, C = a.C, V = a.V, STR = C + 8;
+  const int h = blockIdx.y, H = a.H, C = a.C, V = a.V;
+  u16x8 wf[CF];
+  auto weights = [&](int vt) {  // (slices past C repeat the last one and meet zeros)
+    const bf16_t* wv = (const bf16_t*)a.uv + ((int64_t)h * V + min(vt * 16 + c16, V - 1)) * C + 8 * g4;
+#pragma unroll
+    for (int f = 0; f < CF; ++f) wf[f] = *reinterpret_cast<const u16x8*>(wv + min(32 * f, C - 32));
+  };
+  weights(blockIdx.z * 4 + w);
   {
-    const int r = tid >> 4, i = blockIdx.x * 16 + r;  // 16 threads a row
+    const int r = tid >> 4, k0 = tid & 15, i = blockIdx.x * 16 + r;  // 16 threads a row
     const int t = i < n ? (a.rows ? a.rows[i] : i) : -1;
     const bool live = t >= 0 && a.q_ctx[max(t, 0)] > 0;
     const int64_t TH = (int64_t)a.T * H, th = (int64_t)max(t, 0) * H + h;
     if (part == nullptr) {
-      for (int c = (tid & 15) * 8; c < C; c += 128) {
-        const u16x8 x = *reinterpret_cast<const u16x8*>((const bf16_t*)a.oc + th * C + c);
-        *reinterpret_cast<u16x8*>(ls + r * STR + c) = live ? x : (u16x8)(0);
+#pragma unroll
+      for (int k = 0; k < CF; k += 4) {
+        const int c = 32 * k + k0 * 8;
+        const u16x8 x = *reinterpret_cast<const u16x8*>((const bf16_t*)a.oc + th * C + min(c, C - 8));
+        if (c < 32 * CF) *reinterpret_cast<u16x8*>(ls + r * STR + c) = live && c < C ? x : (u16x8)(0);
       }
     } else {
       const float* ml = part + (int64_t)NP * TH * C + th * 2;
       const float sk = fmaxf(a.sink[h] * LOG2E_F, -1e30f);
-      float m = sk;
-      if (live)
-        for (int p = 0; p < NP; ++p) m = fmaxf(m, ml[p * TH * 2]);
-      float l = __builtin_amdgcn_exp2f(sk - m);
-      if (live)
-        for (int p = 0; p < NP; ++p) l += ml[p * TH * 2 + 1] * __builtin_amdgcn_exp2f(ml[p * TH * 2] - m);
+      float pm[LV_NP / 16], plv[LV_NP / 16], m = sk;
+#pragma unroll
+      for (int k = 0; k < LV_NP / 16; ++k) {  // thread k0 has the splits k0, k0 + 16, ..
+        const int p = k0 + 16 * k;
+        const bool ok = live && p < NP;
+        pm[k] = ok ? ml[min(p, NP - 1) * TH * 2] : -INFINITY;
+        plv[k] = ok ? ml[min(p, NP - 1) * TH * 2 + 1] : 0.f;
+        m = fmaxf(m, pm[k]);
+      }
+#pragma unroll
+      for (int s = 1; s < 16; s <<= 1) m = fmaxf(m, __shfl_xor(m, s, 64));
+      float l = k0 == 0 ? __builtin_amdgcn_exp2f(sk - m) : 0.f;
+#pragma unroll
+      for (int k = 0; k < LV_NP / 16; ++k) {
+        pm[k] = __builtin_amdgcn_exp2f(pm[k] - m);
+        l += plv[k] * pm[k];
+      }
+#pragma unroll
+      for (int s = 1; s < 16; s <<= 1) l += __shfl_xor(l, s, 64);
       const float inv = 1.f / l;
-      for (int c = (tid & 15) * 8; c < C; c += 128) {
-        float x[8];
 #pragma unroll
-        for (int k = 0; k < 8; ++k) x[k] = 0.f;
-        if (live)
-          for (int p0 = 0; p0 < NP; p0 += 4) {  // four splits' loads in flight
-            float y[4][8], f[4];
+      for (int k = 0; k < LV_NP / 16; ++k) fac[r][k0 + 16 * k] = pm[k] * inv;
+      __syncthreads();
+      float x[CF / 4][8];
 #pragma unroll
-            for (int k = 0; k < 4; ++k) {
-              const int p = min(p0 + k, NP - 1);
-              ld_vec<8>(part + ((int64_t)p * TH + th) * C + c, y[k]);
-              f[k] = p0 + k < NP ? __builtin_amdgcn_exp2f(ml[p * TH * 2] - m) * inv : 0.f;
-            }
+      for (int k = 0; k < CF / 4; ++k)
 #pragma unroll
-            for (int k = 0; k < 4; ++k)
+        for (int e = 0; e < 8; ++e) x[k][e] = 0.f;
+      for (int p = 0; p < NP; p += 2) {  // two splits' rows in flight
+        float y[2][CF / 4][8];
 #pragma unroll
-              for (int e = 0; e < 8; ++e) x[e] += f[k] * y[k][e];
-          }
-        st_vec<8>(ls + r * STR + c, x);
+        for (int q = 0; q < 2; ++q)
+#pragma unroll
+          for (int k = 0; k < CF / 4; ++k)
+            ld_vec<8>(part + ((int64_t)min(p + q, NP - 1) * TH + th) * C + min(128 * k + k0 * 8, C - 8), y[q][k]);
+        const float f0 = fac[r][p], f1 = p + 1 < NP ? fac[r][p + 1] : 0.f;
+#pragma unroll
+        for (int k = 0; k < CF / 4; ++k)
+#pragma unroll
+          for (int e = 0; e < 8; ++e) x[k][e] += f0 * y[0][k][e] + f1 * y[1][k][e];
+      }
+#pragma unroll
+      for (int k = 0; k < CF / 4; ++k) {
+        const int c = 128 * k + k0 * 8;
+        if (!live || c >= C)
+#pragma unroll
+          for (int e = 0; e < 8; ++e) x[k][e] = 0.f;
+        st_vec<8>(ls + r * STR + c, x[k]);
       }
     }
   }
@@ -437,25 +491,25 @@ __global__ __launch_bounds__(256) void latent_value_kernel(LatentArgs a, int n, 
   const int i = blockIdx.x * 16 + c16;
   const int t = i < n ? (a.rows ? a.rows[i] : i) : -1;
   for (int vt = blockIdx.z * 4 + w; vt * 16 < V; vt += 4 * gridDim.z) {
-    const bf16_t* wv = (const bf16_t*)a.uv + ((int64_t)h * V + min(vt * 16 + c16, V - 1)) * C + 8 * g4;
     f32x4 x = (f32x4)(0.f);
-#pragma unroll 4
-    for (int f = 0; f < C >> 5; ++f)
-      x = mfma_l(*reinterpret_cast<const u16x8*>(wv + 32 * f),
-                 *reinterpret_cast<const u16x8*>(ls + c16 * STR + 32 * f + 8 * g4), x);
+#pragma unroll
+    for (int f = 0; f < CF; ++f)
+      x = mfma_l(wf[f], *reinterpret_cast<const u16x8*>(ls + c16 * STR + 32 * f + 8 * g4), x);
     const int v = vt * 16 + 4 * g4;
     if (t >= 0 && v < V) {
       const float y[4] = {x[0], x[1], x[2], x[3]};
       st_act_vec<4>((bf16_t*)a.out, t, h * V + v, H * V, a.packed_mt, y);
     }
+    if ((vt + 4 * gridDim.z) * 16 < V) weights(vt + 4 * gridDim.z);
   }
 }
 
-// row tiles of a workgroup (0: the MFMA forms do not cover the shape) and its LDS; rows: query rows that there are
+// row tiles of a workgroup (0: the MFMA forms do not cover the shape), the value columns the kernels are built for, and
+// the LDS; rows: query rows that there are
 static int latent_geometry(int H, int D, int R, int V, int C, int page_log2, int rows, int& cw, size_t& lds) {
   if (page_log2 < 6 || D % 8 || R % 8 || V % 4 || C % 32 || C > 512 || D > 256) return 0;
-  cw = C <= 128 ? 2 : C <= 256 ? 4 : 8;
-  if (C + R > 64 * cw + 64) return 0;
+  cw = C <= 128 ? 128 : C <= 256 ? 256 : 512;
+  if (C + R > cw + 64) return 0;
   const int str = (C + R + 31) / 32 * 32 + 8;
   for (int rt = rows > 32 ? 4 : rows > 16 ? 2 : 1; rt; rt >>= 1) {
     lds = (size_t)(LT_KEYS + 16 * rt) * str * 2 + 2 * 16 * rt * LT_PS * 2 + 4 * 16 * rt * 4;
@@ -691,8 +745,11 @@ extern "C" int mp_latent_prep(const void* z, int64_t zs, const float* qw, const 
   LatentArgs a{};
   a.z = z, a.zs = zs, a.qw = qw, a.cw = cw, a.cq = cq, a.cache = cache, a.slots = slots, a.q_ctx = q_ctx, a.rope = rope;
   a.Q = Q, a.C = C, a.R = R, a.eps = eps, a.packed_q = packed_q;
-  if (f32) hipLaunchKernelGGL(latent_prep_kernel<float>, dim3(n), dim3(256), 0, stream, a);
-  else hipLaunchKernelGGL(latent_prep_kernel<bf16_t>, dim3(n), dim3(256), 0, stream, a);
+  const bool vec = Q % 8 == 0 && C % 8 == 0 && R % 8 == 0 && zs % 8 == 0;
+  if (f32 && vec) hipLaunchKernelGGL((latent_prep_kernel<float, 8, 256>), dim3(n), dim3(256), 0, stream, a);
+  else if (f32) hipLaunchKernelGGL((latent_prep_kernel<float, 1, 256>), dim3(n), dim3(256), 0, stream, a);
+  else if (vec) hipLaunchKernelGGL((latent_prep_kernel<bf16_t, 8, 256>), dim3(n), dim3(256), 0, stream, a);
+  else hipLaunchKernelGGL((latent_prep_kernel<bf16_t, 1, 256>), dim3(n), dim3(256), 0, stream, a);
   return (int)hipGetLastError();
 }
 
@@ -732,7 +789,7 @@ extern "C" int mp_latent_attention(int form, const void* q, int64_t qs, const vo
   const int tb = blk ? mp_latent_block(H, D, R, V, C, page_log2) : 1;
   const int rt = f32 ? 0 : latent_geometry(H, D, R, V, C, page_log2, tb * H, cw, lds);
   if (rt == 0 || qs % 8) return -1;
-  if (NP < 1 || NP > 65535 || (NP > 1 && (PS <= 0 || PS % LT_KEYS || part == nullptr))) return -2;
+  if (NP < 1 || NP > LV_NP || (NP > 1 && (PS <= 0 || PS % LT_KEYS || part == nullptr))) return -2;
   const int nb16 = (n + 15) / 16;
   const int ctiles = (C / 16 + 3) / 4, vtiles = ((V + 15) / 16 + 3) / 4;
   const int zq = nb16 * H >= 1024 ? 1 : ctiles, zv = nb16 * H >= 1024 ? 1 : vtiles;
@@ -744,23 +801,26 @@ extern "C" int mp_latent_attention(int form, const void* q, int64_t qs, const vo
   const dim3 grid(blk ? nblk : T, (H + 16 * rt - 1) / (16 * rt), NP);
   float* pp = NP > 1 ? part : nullptr;
   const int ps = NP > 1 ? PS : 0;
-#define MP_LA(RT_, CW_)                                                                                               \
-  {                                                                                                                   \
-    if (lds > 65536)                                                                                                  \
-      (void)hipFuncSetAttribute((const void*)latent_attn_kernel<RT_, CW_>, hipFuncAttributeMaxDynamicSharedMemorySize, \
-                                (int)lds);                                                                            \
-    hipLaunchKernelGGL((latent_attn_kernel<RT_, CW_>), grid, dim3(256), lds, stream, a, blk, nblk, ps, pp);            \
+#define MP_LA(RT_, CW_, NW_)                                                                                           \
+  {                                                                                                                    \
+    if (lds > 65536)                                                                                                   \
+      (void)hipFuncSetAttribute((const void*)latent_attn_kernel<RT_, CW_, NW_>,                                        \
+                                hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);                                 \
+    hipLaunchKernelGGL((latent_attn_kernel<RT_, CW_, NW_>), grid, dim3(NW_ * 64), lds, stream, a, blk, nblk, ps, pp);   \
   }
-#define MP_LAC(CW_)            \
-  if (rt == 1) MP_LA(1, CW_)   \
-  else if (rt == 2) MP_LA(2, CW_) \
-  else MP_LA(4, CW_)
-  if (cw == 2) { MP_LAC(2) } else if (cw == 4) { MP_LAC(4) } else { MP_LAC(8) }
+#define MP_LAC(C_)                       \
+  if (rt == 1) MP_LA(1, C_ / 64, 4)      \
+  else if (rt == 2) MP_LA(2, C_ / 128, 8) \
+  else MP_LA(4, C_ / 128, 8)
+  if (cw == 128) { MP_LAC(128) } else if (cw == 256) { MP_LAC(256) } else { MP_LAC(512) }
 #undef MP_LAC
 #undef MP_LA
   rc = (int)hipGetLastError();
   if (rc) return rc;
-  hipLaunchKernelGGL(latent_value_kernel, dim3(nb16, H, zv), dim3(256), 16 * (C + 8) * 2, stream, a, n, pp, NP);
+  const dim3 gv(nb16, H, zv);
+  if (cw == 128) hipLaunchKernelGGL(latent_value_kernel<4>, gv, dim3(256), 0, stream, a, n, pp, NP);
+  else if (cw == 256) hipLaunchKernelGGL(latent_value_kernel<8>, gv, dim3(256), 0, stream, a, n, pp, NP);
+  else hipLaunchKernelGGL(latent_value_kernel<16>, gv, dim3(256), 0, stream, a, n, pp, NP);
   return (int)hipGetLastError();
 }
 

@@ -101,6 +101,7 @@ def _linear(kind, z, rope, decay, bias, norm_w, state, aux, q_seq, q_ctx, out, c
 
 # ------------------------------------------------------------------ latent attention
 LATENT_KEYS = 64  # keys of a tile: splits of a context are multiples of it
+LATENT_SPLITS = 64  # most splits of a context
 
 
 def latent_prep(z, qw, cw, cq, cache, slots, q_ctx, rope, eps, packed=False):
@@ -121,7 +122,7 @@ def latent_parts(groups: int, span: int, n_cu: int = 256):
     """(keys per split, splits) for ``groups`` workgroups whose queries see at most ``span`` keys: about one workgroup
     per CU, no split under two tiles."""
     span = max(1, int(span))
-    n = max(1, min(n_cu // max(1, groups), span // (2 * LATENT_KEYS)))
+    n = max(1, min(n_cu // max(1, groups), span // (2 * LATENT_KEYS), LATENT_SPLITS))
     ps = LATENT_KEYS * -(-span // (LATENT_KEYS * n))
     return ps, -(-span // ps)
 
@@ -142,6 +143,7 @@ def latent_attention(q, uk, uv, sink, rope, cache, table, q_seq, q_ctx, out, sca
 
 # a portion of a prompt of this many tokens or more has its context's keys and values made for every head
 LATENT_WIDE_TOKENS = 64
+WIDE_WAVES = 0  # waves of a workgroup of that form (0: by the portions' length)
 
 
 def latent_wide_ok(D: int, R: int, V: int, C: int) -> bool:
@@ -161,11 +163,9 @@ def latent_wide_plan(ntoks, starts, heads: int, dim: int, n_cu: int = 256, max_r
     if not pick:
         return None
     off = np.concatenate([[0], np.cumsum(ntoks)[:-1]])
-    for waves in (8, 4):
-        tb = 32 * waves
-        blk = [(off[i] + k, min(tb, ntoks[i] - k), b) for i, b in zip(pick, base) for k in range(0, int(ntoks[i]), tb)]
-        if dim > 64 and heads * len(blk) > 2 * n_cu:  # (the small form has four waves)
-            break
+    waves = WIDE_WAVES or (8 if dim > 64 and max(int(ntoks[i]) for i in pick) >= 2048 else 4)
+    tb = 32 * waves
+    blk = [(off[i] + k, min(tb, ntoks[i] - k), b) for i, b in zip(pick, base) for k in range(0, int(ntoks[i]), tb)]
     return pick, np.ascontiguousarray(np.asarray(blk, dtype=np.int32).reshape(-1, 3).T), waves
 
 
