@@ -208,8 +208,8 @@ constexpr float LT_GROW = 8.f;  // log2 units a row's maximum may grow before it
 // A workgroup of NW waves owns up to 16 RT query rows (token-major x heads) of one sequence.  Per 64-key tile wave w
 // makes the scores of keys 16 (w % 4) .. + 15 for RW of the row tiles (S^T = rows u^T: a lane owns one query row), the
 // row maxima meet in LDS, the weights go to LDS as hi + lo bf16 (32-bit in effect), and wave w adds them into its
-// 16 CW of the C value columns (O^T += c^T P^T, c^T by transposed reads of the same tile).  The next tile is in flight
-// in registers.
+// 16 CW of the C value columns (O^T += c^T P^T, c^T by transposed reads of the same tile).  The next two tiles are in
+// flight in registers.
 template <int RT, int CW, int NW>
 __global__ __launch_bounds__(NW * 64) void latent_attn_kernel(LatentArgs a, const int32_t* __restrict__ blk, int nblk,
                                                               int PS, float* __restrict__ part) {
@@ -235,20 +235,6 @@ __global__ __launch_bounds__(NW * 64) void latent_attn_kernel(LatentArgs a, cons
   const int cpr = KW >> 3;  // chunks per cache row
   const float rcp = 1.f / (float)cpr, sl2 = a.scale * LOG2E_F;
 
-  // query rows, zero past the row count and past KW; the tile's own columns past KW
-  for (int x = tid; x < 16 * RT * 4 * KF; x += NT) {
-    const int r = x / (4 * KF), col = (x - r * 4 * KF) * 8;
-    const int rr = min(r, nrow - 1);
-    const bf16_t* src = (const bf16_t*)a.u + ((int64_t)(tok0 + rr / hg) * H + h0 + rr % hg) * KW;
-    const u16x8 v = *reinterpret_cast<const u16x8*>(src + min(col, KW - 8));
-    *reinterpret_cast<u16x8*>(qt + r * STR + col) = r < nrow && col < KW ? v : (u16x8)(0);
-  }
-  if (KW & 31)
-    for (int x = tid; x < LT_KEYS * (4 * KF - cpr); x += NT) {
-      const int r = x / (4 * KF - cpr), col = KW + (x - r * (4 * KF - cpr)) * 8;
-      *reinterpret_cast<u16x8*>(kt + r * STR + col) = (u16x8)(0);
-    }
-
   float m[RT], l[RT];
   f32x4 o[RT][CW];
 #pragma unroll
@@ -265,14 +251,14 @@ __global__ __launch_bounds__(NW * 64) void latent_attn_kernel(LatentArgs a, cons
     const int row = 16 * (rg * RW + r) + c16;
     khi[r] = row < nrow ? min(a.q_ctx[tok0 + row / hg], s_hi) : 0;
   }
-  u16x8 kreg[KPT];
-  auto fetch = [&](int s0) {  // a tile's rows are consecutive in the page; past the context the last row repeats
+  u16x8 ka_reg[KPT], kb_reg[KPT];  // the next two tiles, in flight
+  auto fetch = [&](u16x8 (&kreg)[KPT], int s0) {  // a tile's rows are consecutive in the page; past the context the last row repeats
     const bf16_t* base = (const bf16_t*)a.cache + (((int64_t)bt[s0 >> a.page_log2] << a.page_log2) + (s0 & pmask)) * KW;
     const int lastc = min(LT_KEYS, s_hi - s0) * cpr - 1;
 #pragma unroll
     for (int k = 0; k < KPT; ++k) kreg[k] = *reinterpret_cast<const u16x8*>(base + min(tid + NT * k, lastc) * 8);
   };
-  auto stash = [&]() {
+  auto stash = [&](const u16x8 (&kreg)[KPT]) {
 #pragma unroll
     for (int k = 0; k < KPT; ++k) {
       const int x = tid + NT * k, key = (int)(((float)x + 0.5f) * rcp);
@@ -280,16 +266,15 @@ __global__ __launch_bounds__(NW * 64) void latent_attn_kernel(LatentArgs a, cons
     }
   };
 
-  if (s_lo < s_hi) fetch(s_lo);
-  for (int s0 = s_lo; s0 < s_hi; s0 += LT_KEYS) {
-    stash();
-    if (s0 + LT_KEYS < s_hi) fetch(s0 + LT_KEYS);
+  auto tile = [&](u16x8 (&kreg)[KPT], int s0) {
+    stash(kreg);
+    if (s0 + 2 * LT_KEYS < s_hi) fetch(kreg, s0 + 2 * LT_KEYS);
     __syncthreads();
     f32x4 st[RW];
 #pragma unroll
     for (int r = 0; r < RW; ++r) st[r] = (f32x4)(0.f);
     const bf16_t *kp = kt + (16 * ws + c16) * STR + 8 * g4, *qp = qt + (16 * rg * RW + c16) * STR + 8 * g4;
-#pragma unroll 3
+#pragma unroll 6
     for (int f = 0; f < KF; ++f) {
       const u16x8 ka = *reinterpret_cast<const u16x8*>(kp + 32 * f);
 #pragma unroll
@@ -360,6 +345,25 @@ __global__ __launch_bounds__(NW * 64) void latent_attn_kernel(LatentArgs a, cons
       }
     }
     __syncthreads();
+  };
+  if (s_lo < s_hi) fetch(ka_reg, s_lo);
+  if (s_lo + LT_KEYS < s_hi) fetch(kb_reg, s_lo + LT_KEYS);
+  // query rows, zero past the row count and past KW; the tile's own columns past KW
+  for (int x = tid; x < 16 * RT * 4 * KF; x += NT) {
+    const int r = x / (4 * KF), col = (x - r * 4 * KF) * 8;
+    const int rr = min(r, nrow - 1);
+    const bf16_t* src = (const bf16_t*)a.u + ((int64_t)(tok0 + rr / hg) * H + h0 + rr % hg) * KW;
+    const u16x8 v = *reinterpret_cast<const u16x8*>(src + min(col, KW - 8));
+    *reinterpret_cast<u16x8*>(qt + r * STR + col) = r < nrow && col < KW ? v : (u16x8)(0);
+  }
+  if (KW & 31)
+    for (int x = tid; x < LT_KEYS * (4 * KF - cpr); x += NT) {
+      const int r = x / (4 * KF - cpr), col = KW + (x - r * (4 * KF - cpr)) * 8;
+      *reinterpret_cast<u16x8*>(kt + r * STR + col) = (u16x8)(0);
+    }
+  for (int s0 = s_lo; s0 < s_hi; s0 += 2 * LT_KEYS) {
+    tile(ka_reg, s0);
+    if (s0 + LT_KEYS < s_hi) tile(kb_reg, s0 + LT_KEYS);
   }
 #pragma unroll
   for (int r = 0; r < RT; ++r) {
@@ -599,12 +603,13 @@ __global__ __launch_bounds__(NW * 64) void latent_wide_kernel(LatentArgs a, Wide
       for (int s = 0; s < 2 * RF; ++s) {
         const int d = min(16 * s + 8 * hh, R - 8), e = d < half ? d + half : d - half, f = d < half ? d : e;
         const u16x8 x = *reinterpret_cast<const u16x8*>(q + D + d), y = *reinterpret_cast<const u16x8*>(q + D + e);
+        float c[8], sn[8];
+        ld_vec<8>(cs + f, c);
+        ld_vec<8>(cs + half + f, sn);
+        const float sg = d < half ? -1.f : 1.f;
         u16x8 z;
 #pragma unroll
-        for (int j = 0; j < 8; ++j) {
-          const float c = cs[f + j], sn = d < half ? -cs[half + f + j] : cs[half + f + j];
-          z[j] = f2bf(bf2f(x[j]) * c + bf2f(y[j]) * sn);
-        }
+        for (int j = 0; j < 8; ++j) z[j] = f2bf(bf2f(x[j]) * c[j] + sg * bf2f(y[j]) * sn[j]);
         qf[2 * DF + s] = row_ok && 16 * s + 8 * hh < R ? z : (u16x8)(0);
       }
     }

@@ -163,7 +163,7 @@ def latent_wide_plan(ntoks, starts, heads: int, dim: int, n_cu: int = 256, max_r
     if not pick:
         return None
     off = np.concatenate([[0], np.cumsum(ntoks)[:-1]])
-    waves = WIDE_WAVES or (8 if dim > 64 and max(int(ntoks[i]) for i in pick) >= 2048 else 4)
+    waves = WIDE_WAVES or (8 if dim > 64 and max(int(ntoks[i]) for i in pick) > 128 else 4)
     tb = 32 * waves
     blk = [(off[i] + k, min(tb, ntoks[i] - k), b) for i, b in zip(pick, base) for k in range(0, int(ntoks[i]), tb)]
     return pick, np.ascontiguousarray(np.asarray(blk, dtype=np.int32).reshape(-1, 3).T), waves

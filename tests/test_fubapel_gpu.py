@@ -142,7 +142,7 @@ def run_lin(c, dt, plan, packed=False):
         mops.mlstm(z, c["bias"].to(DEV), c["cap"], c["norm"].to(DEV), st, aux, q_seq, q_ctx, out, c["eps"], plan=plan,
                    packed=packed)
     else:
-        rope = mops.rope_table(3000.0, c["rot"], 600, DEV)
+        rope = mops.rope_table(3000.0, c["rot"], 800, DEV)
         mops.retention(z, rope, torch.log2(c["decay"]).float().to(DEV), st, q_seq, q_ctx, out, c["eps"], plan=plan,
                        packed=packed)
     return (ops.unpack_act(out, T, HV) if packed else out.view(T, HV)), st, aux
@@ -397,3 +397,119 @@ def test_the_sink_counts_once(form, sink):
         got = run_wide(a, 0.2, 4) if form == "wide" else run_lat(a, 0.2, form, splits)
         close(got, lat_oracle(a, 0.2)[0], TOL["bf16"])
     assert (got.abs().max() < 1e-3) == (sink == 40.0)
+
+
+# ------------------------------------------------------------------ executor
+@pytest.fixture(scope="module", params=sorted(U.MODELS) + ["packed"])
+def model(request, tmp_path_factory):
+    if request.param == "packed":  # every GEMM has a decode form, the recurrences and attention fill their tiles
+        cfg = U.config([U.ret(4, 64, 64), U.mla(8, 64, 64, 32, 128, 128, ff=384), U.mem(2, 128, 128),
+                        U.mla(5, 32, 64, 16, 256, 160, ff=128), U.ret(2, 128, 128, 64), U.mem(4, 64, 48, ff=256)], vocab=333,
+                       width=256, loop={"start": 1, "stop": 3, "times": 2})
+    else:
+        cfg = U.MODELS[request.param]
+    w = U.tensors(cfg, seed=3)
+    return cfg, w, U.write(tmp_path_factory.mktemp(request.param), cfg, w), request.param
+
+
+def check(got, want, dt, name, scale):
+    if dt == "fp32":
+        return torch.testing.assert_close(got.float().cpu(), want, atol=1e-3, rtol=1e-3)
+    err = (got.float().cpu() - want).pow(2).mean(-1).sqrt() / scale
+    # (heads of one value are normed to their sign, which rounding can flip)
+    assert err.quantile(0.9 if name == "ones" else 1.0) < 0.06, err
+
+
+@pytest.mark.parametrize("dt", sorted(DTYPES))
+def test_prompts_decoding_portions_and_batches(model, dt):
+    cfg, w, d, name = model
+    n = 230
+    toks = {k: U.ids(n, cfg["vocab"], s) for s, k in enumerate("abc")}
+    want = {k: O.forward(cfg, w, t).float() for k, t in toks.items()}
+    scale = want["a"].std()
+    ex = U.executor(d, DEV, dt, max_sessions=4)
+    check(ex.forward([("w", n)], toks["a"].to(DEV), logit_rows=range(n)), want["a"], dt, name, scale)
+    ex.sessions.close("w")
+    # one token at a time (graph replays), three sessions of different lengths together
+    got = {k: [] for k in toks}
+    at = {"a": 5, "b": 2, "c": 64}
+    ex.forward(list(at.items()), torch.cat([toks[k][:m] for k, m in at.items()]).to(DEV))
+    for _ in range(70):
+        x = torch.cat([toks[k][at[k]:at[k] + 1] for k in toks]).to(DEV)
+        y = ex.forward([(k, 1) for k in toks], x)
+        assert ex.last_graphed
+        for r, k in enumerate(toks):
+            got[k].append(y[r].float().cpu())
+            at[k] += 1
+    for k, lo in (("a", 5), ("b", 2), ("c", 64)):
+        check(torch.stack(got[k]), want[k][lo:lo + 70], dt, name, scale)
+    # portions, short and long, beside decoded tokens
+    for step in ({"a": 2, "b": 1}, {"b": 30, "c": 1, "a": 1}, {"a": 17, "b": 3}, {"c": 2, "a": 70, "b": 1},
+                 {"b": 64, "a": 2, "c": 65}):
+        x = torch.cat([toks[k][at[k]:at[k] + m] for k, m in step.items()]).to(DEV)
+        y = ex.forward(list(step.items()), x, logit_rows=range(x.numel())).cpu()
+        off = 0
+        for k, m in step.items():
+            check(y[off:off + m], want[k][at[k]:at[k] + m], dt, name, scale)
+            off += m
+            at[k] += m
+    # everything given back and used again, whatever it holds
+    for k in toks:
+        ex.sessions.close(k)
+    for s in ([] if ex.state is None else ex.state.states) + ex.cache.rows + ex.cache.rk:
+        s.fill_(1e4)
+    check(ex.forward([("z", n)], toks["b"].to(DEV), logit_rows=range(n)), want["b"], dt, name, scale)
+
+
+def test_long_contexts_of_whole_and_cut_prompts(model):
+    """1100 tokens: segments of the recurrences, split contexts, both forms of latent attention."""
+    cfg, w, d, name = model
+    if name != "packed":
+        pytest.skip("one model is enough")
+    n = 1100
+    t = U.ids(n, cfg["vocab"], 7)
+    want = O.forward(cfg, w, t, torch.float32).float()
+    ex = U.executor(d, DEV, "bf16", max_seq_len=1280, max_tokens_per_step=2048)
+    check(ex.forward([("w", n)], t.to(DEV), logit_rows=range(n)), want, "bf16", name, want.std())
+    at = 0
+    for m in (700, 2, 63, 64, 1, 200, 3, 33, 1, 33):
+        y = ex.forward([("c", m)], t[at:at + m].to(DEV), logit_rows=range(m))
+        check(y, want[at:at + m], "bf16", name, want.std())
+        at += m
+    assert at == n
+
+
+def test_long_contexts_of_the_recurrences_alone():
+    """Segments of a session that already has a state."""
+    for kind in KINDS:
+        ntoks, starts = [700, 3, 513], [40, 0, 0]
+        c = lin_case(kind, ntoks, 2, 64, 64, "bf16", starts, 32)
+        plan = lin_plan(ntoks, 2, 128)
+        assert plan["slots"] > 4
+        out, st, _ = run_lin(c, "bf16", plan)
+        close(out, c["want"], LIN_TOL["bf16"])
+        close(st[1:], c["states"][1:], dict(atol=2e-3, rtol=1e-3))
+
+
+def test_wide_decode_batches(model):
+    """65 and more rows take other GEMM forms."""
+    cfg, w, d, name = model
+    ex = U.executor(d, DEV, "bf16", max_sessions=80, max_seq_len=64, kv_cache_bytes=512 << 20)
+    t = U.ids(80 * 6, cfg["vocab"], 5).view(80, 6)
+    ex.forward([(f"s{i}", 5) for i in range(80)], t[:, :5].reshape(-1).to(DEV))
+    y = ex.forward([(f"s{i}", 1) for i in range(80)], t[:, 5].to(DEV)).float().cpu()
+    want = torch.stack([O.forward(cfg, w, t[i])[-1].float() for i in range(80)])
+    check(y, want, "bf16", name, want.std())
+
+
+def test_greedy_generation_through_the_scheduler(model):
+    from tests.test_kafunex import serve
+
+    cfg, w, d, name = model
+    reqs = [(U.ids(n, cfg["vocab"], n).tolist(), 6 + n % 3) for n in (1, 2, 9, 40, 71)]
+    want = [O.greedy(cfg, w, torch.tensor(p), n) for p, n in reqs]
+    ex = U.executor(d, DEV, "fp32")
+    assert serve(ex, reqs, batch=3, n_slots=2) == want
+    assert serve(ex, reqs, batch=5, prefill_chunk=4, max_step_tokens=11) == want
+    out = serve(U.executor(d, DEV, "bf16"), reqs, batch=4)  # bf16 may part from it at a near tie
+    assert all(len(a) == len(b) for a, b in zip(out, want))
