@@ -296,8 +296,9 @@ class ModelConfig:
 
 def hybrid_config(model_type: str, vocab: int, width: int, eps: float, layers, name: str,
                   max_positions: int = 32768, **stream) -> ModelConfig:
-    """A hybrid decoder's ModelConfig; ``stream``: its residual stream's fields.  The uniform fields (heads, kv heads, head size, ff) describe its
-    first attention layer, else its first layer: estimates and announcements read them, kernels do not."""
+    """A hybrid decoder's ModelConfig; ``stream``: its residual stream's fields.  The uniform fields (heads, kv heads,
+    head size, ff) describe its first attention layer, else its first layer: estimates and announcements read them,
+    kernels do not."""
     layers = tuple(layers)
     ref = next((sp for sp in layers if not sp.recurrent), layers[0])
     return ModelConfig(model_type=model_type, vocab_size=vocab, hidden_size=width, intermediate_size=ref.ff,
