@@ -20,10 +20,33 @@ import math
 import os
 from typing import Callable, Dict, Optional, Tuple
 
-SUPPORTED_TYPES = ("llama", "mistral", "mixtral", "gpt2", "kafunex", "fubapel")
-MIXERS = ("attention", "hgrn2", "latent_attention", "mlstm", "retention")
+SUPPORTED_TYPES = ("llama", "mistral", "mixtral", "gpt2", "kafunex", "fubapel", "nuvorax")
+MIXERS = ("attention", "hgrn2", "latent_attention", "mlstm", "retention", "mixed_attention")
 RECURRENT = ("hgrn2", "mlstm", "retention")
-FEED_FORWARDS = ("relu2", "clamped_glu")
+FEED_FORWARDS = ("relu2", "clamped_glu", "gelu")
+MAX_EXPERTS = 512
+
+
+@dataclasses.dataclass(frozen=True)
+class MoESpec:
+    """Routed experts of a layer: ``top`` of ``experts`` clamped gated feed-forwards of width ``ff`` per token, chosen by
+    softmax scores among the ``keep`` best of ``groups`` equal groups of neighbouring experts (a group counts as its
+    best expert); the chosen scores are divided by their sum and multiplied by ``scale``."""
+    experts: int
+    top: int
+    ff: int
+    limit: float
+    groups: int = 1
+    keep: int = 1
+    scale: float = 1.0
+
+    def validate(self) -> None:
+        if not 1 <= self.experts <= MAX_EXPERTS or self.ff < 1 or not self.limit > 0:
+            raise ValueError(f"bad experts: {self}")
+        if self.groups < 1 or self.experts % self.groups or not 1 <= self.keep <= self.groups:
+            raise ValueError("experts must form equal groups, of which 1 .. groups.count are kept")
+        if not 1 <= self.top <= self.keep * (self.experts // self.groups):
+            raise ValueError("top must be at most the number of experts in the kept groups")
 
 
 @dataclasses.dataclass(frozen=True)
@@ -34,7 +57,12 @@ class LayerSpec:
     ``attention``: chunked talking-heads attention whose values are the projected keys; ``hgrn2``: the
     gated linear recurrence (no kv heads, no mask, no scale); ``latent_attention``: keys and values are made from
     one cached latent per token, plus a rotated key part that all heads share; ``mlstm``: matrix memory with
-    exponential gates; ``retention``: linear attention with a fixed decay per head."""
+    exponential gates; ``retention``: linear attention with a fixed decay per head; ``mixed_attention``: grouped-query
+    attention over rotated keys and rotated values, soft-capped scores, a sink of score 0 in the softmax, the heads'
+    weights mixed after the softmax, one output gate per head.
+
+    ``parallel``: mixer and feed-forward read one norm and are added together.  ``moe``: routed experts; the layer's own
+    feed-forward (``ff``, ``ffn``) is then the shared expert, added times a gate per token."""
     mixer: str
     heads: int
     dim: int
@@ -43,7 +71,7 @@ class LayerSpec:
     kv_heads: int = 0
     chunk: int = 0
     scale: float = 1.0
-    ffn: str = "relu2"                      # feed-forward: squared relu, or the clamped gated form
+    ffn: str = "relu2"                      # feed-forward: squared relu, the clamped gated form, or the exact gelu
     limit: float = 0.0                      # clamped_glu: bound of its two inputs
     q_rank: int = 0                         # latent_attention: size of the queries' latent
     kv_rank: int = 0                        # latent_attention: size of the keys' and values' latent
@@ -52,6 +80,10 @@ class LayerSpec:
     rot_base: float = 10000.0
     decay: Tuple[float, ...] = ()           # retention: one factor per head
     gate_cap: float = 0.0                   # mlstm: soft cap of the gates' inputs
+    softcap: float = 0.0                    # mixed_attention: bound of the scores
+    rot_scaling: Optional[Tuple[float, float, float, float]] = None  # rotary: (factor, low, high, original)
+    moe: Optional[MoESpec] = None
+    parallel: bool = False
     source: Optional[int] = None            # checkpoint layer whose weights these are (None: its own place)
 
     @property
@@ -59,9 +91,9 @@ class LayerSpec:
         return self.mixer in RECURRENT
 
     @property
-    def in_rows(self) -> int:
-        """Rows of the fused input projection: [q | f | v], [q | k | gate], [q latent | kv latent | rotated key],
-        [q | k | v | gate] or that and the two log gates, filled up to a whole GEMM tile."""
+    def mix_rows(self) -> int:
+        """Rows of the mixer's fused input projection: [q | f | v], [q | k | gate], [q latent | kv latent | rotated
+        key], [q | k | v | gate] or that and the two log gates, filled up to a whole GEMM tile."""
         if self.mixer == "hgrn2":
             return self.heads * (2 * self.dim + self.vdim)
         if self.mixer == "latent_attention":
@@ -70,11 +102,34 @@ class LayerSpec:
             return 2 * self.heads * (self.dim + self.vdim)
         if self.mixer == "mlstm":
             return 16 * -(-2 * self.heads * (self.dim + self.vdim + 1) // 16)
+        if self.mixer == "mixed_attention":
+            return 16 * -(-(self.heads * (self.dim + 1) + self.kv_heads * (self.dim + self.vdim)) // 16)
         return (2 * self.heads + self.kv_heads) * self.dim
+
+    @property
+    def glu(self) -> bool:
+        return self.ffn == "clamped_glu"
+
+    @property
+    def ff_rows(self) -> int:
+        """Rows of the feed-forward's input projection: [up], [gate and up], a shared expert's with its gate after
+        them; where it is fused to the mixer's or has such a gate, filled up to a whole GEMM tile."""
+        n = (2 if self.glu else 1) * self.ff + (1 if self.ff and self.moe else 0)
+        return 16 * -(-n // 16) if self.parallel or self.moe else n
+
+    @property
+    def in_rows(self) -> int:
+        """Rows of the GEMM that reads the layer's (first) norm."""
+        return self.mix_rows + (self.ff_rows if self.parallel else 0)
 
     @property
     def out_cols(self) -> int:
         return self.heads * self.vdim
+
+    @property
+    def o_cols(self) -> int:
+        """Columns of the mixer's output projection; in a parallel layer the feed-forward's follow them."""
+        return self.out_cols + (self.ff if self.parallel else 0)
 
     @property
     def q_rows(self) -> int:
@@ -88,6 +143,8 @@ class LayerSpec:
             return None
         if self.mixer == "latent_attention":
             return 1, self.kv_rank + self.rot_dim, False
+        if self.mixer == "mixed_attention":  # (key rows and value columns of a page side by side)
+            return self.kv_heads, self.dim + self.vdim, False
         return self.kv_heads, self.dim, True
 
     @property
@@ -111,8 +168,12 @@ class LayerSpec:
         return sum(math.prod(s) for s in self.state_shapes)
 
     def param_count(self, width: int) -> int:
-        n = width * (self.in_rows + self.out_cols + (3 if self.ffn == "clamped_glu" else 2) * self.ff) + 2 * width
+        n = width * (self.mix_rows + self.out_cols + (3 if self.glu else 2) * self.ff) + 2 * width
+        if self.moe:
+            n += width * self.moe.experts * (1 + 3 * self.moe.ff)
         H, D, V = self.heads, self.dim, self.vdim
+        if self.mixer == "mixed_attention":
+            return n + 2 * D + H * H
         if self.mixer == "hgrn2":
             return n + 2 * H * D + V
         if self.mixer == "latent_attention":
@@ -130,7 +191,13 @@ class LayerSpec:
             raise ValueError(f"unsupported feed-forward {self.ffn!r}; supported: {FEED_FORWARDS}")
         if min(self.heads, self.dim, self.vdim) < 1 or self.ff < 0:
             raise ValueError(f"bad layer sizes: {self}")
-        if self.ff and self.ffn == "clamped_glu" and not self.limit > 0:
+        if self.moe is not None:
+            self.moe.validate()
+            if not self.glu:
+                raise ValueError("a shared expert has the experts' gated form")
+        if self.parallel and self.mixer != "mixed_attention":
+            raise ValueError(f"{self.mixer} has no parallel form")
+        if self.ff and self.glu and not self.limit > 0:
             raise ValueError("the clamped feed-forward needs a limit > 0")
         if self.mixer == "attention":
             if self.kv_heads < 1 or self.heads % self.kv_heads:
@@ -150,7 +217,15 @@ class LayerSpec:
             raise ValueError("retention needs decays >= 0")
         if self.mixer == "mlstm" and not self.gate_cap > 0:
             raise ValueError("mlstm needs a gate_cap > 0")
-        if self.mixer in ("latent_attention", "retention"):
+        if self.mixer == "mixed_attention":
+            if self.kv_heads < 1 or self.heads % self.kv_heads:
+                raise ValueError("attention heads must be a multiple of kv_heads")
+            if self.vdim % 2:
+                raise ValueError("rotated values need an even vdim")
+            if self.softcap < 0 or (self.rot_scaling is not None and not (
+                    min(self.rot_scaling) > 0 and self.rot_scaling[1] < self.rot_scaling[2])):
+                raise ValueError(f"bad softcap or rot.scaling: {self}")
+        if self.mixer in ("latent_attention", "retention", "mixed_attention"):
             whole = self.rot_dim if self.mixer == "latent_attention" else self.dim
             if self.rot_dims % 2 or not 0 <= self.rot_dims <= whole:
                 raise ValueError(f"rot.dims must be even and at most {whole}")
@@ -188,6 +263,8 @@ class ModelConfig:
     norm: str = "rms"
     residual_mult: float = 1.0
     embed_positions: bool = True
+    embed_scale: float = 1.0
+    logit_scale: float = 1.0
 
     @property
     def hybrid(self) -> bool:
@@ -243,6 +320,8 @@ class ModelConfig:
                 raise ValueError(f"unsupported residual stream: {self.stream!r}, {self.norm!r}")
             for sp in self.layers:
                 sp.validate()
+                if self.stream == "post" and (sp.parallel or sp.moe is not None):
+                    raise ValueError("parallel layers and routed experts need a pre-norm stream")
             return
         if self.num_attention_heads % self.num_key_value_heads:
             raise ValueError("num_attention_heads must be a multiple of num_key_value_heads")
@@ -362,9 +441,43 @@ def _fubapel_config(d: dict, name: str) -> ModelConfig:
                          residual_mult=float(d["residual_mult"]), embed_positions=False)
 
 
+def _nuvorax_config(d: dict, name: str) -> ModelConfig:
+    layers = []
+    for i, e in enumerate(d["layers"]):
+        m, mlp = e["mixer"], e.get("mlp")
+        if e["type"] != "attention":
+            raise ValueError(f"layer {i}: unsupported mixer {e['type']!r}")
+        rot, kw = m["rot"], {"ffn": "gelu"}
+        kind = "dense" if mlp is None else mlp.get("kind", "dense")
+        if mlp is not None and kind == "dense":
+            kw.update(ff=int(mlp["ff"]))
+        elif kind == "moe":
+            r, x, sh = mlp["router"], mlp["expert"], mlp.get("shared")
+            gr = r.get("groups") or {"count": 1, "keep": 1}
+            kw.update(ffn="clamped_glu", moe=MoESpec(int(r["experts"]), int(r["top"]), int(x["ff"]), float(x["limit"]),
+                                                     int(gr["count"]), int(gr["keep"]), float(r.get("scale", 1.0))))
+            if sh is not None:
+                kw.update(ff=int(sh["ff"]), limit=float(sh["limit"]))
+        elif mlp is not None:
+            raise ValueError(f"layer {i}: unsupported feed-forward kind {kind!r}")
+        sc = rot.get("scaling")
+        if sc is not None:
+            kw.update(rot_scaling=tuple(float(sc[k]) for k in ("factor", "low", "high", "original")))
+        layers.append(LayerSpec("mixed_attention", int(m["heads"]), int(m["dim"]), int(m["vdim"]),
+                                kv_heads=int(m["kv_heads"]), scale=float(m["scale"]), softcap=float(m.get("softcap") or 0),
+                                rot_dims=int(rot["dims"]), rot_base=float(rot["base"]), parallel=True, **kw))
+    return hybrid_config("nuvorax", int(d["vocab"]), int(d["width"]), float(d["norm"]["eps"]), layers, name,
+                         embed_scale=float((d.get("embedding") or {}).get("scale", 1.0)),
+                         logit_scale=float(d.get("logit_scale", 1.0)), **PARALLEL_STREAM)
+
+
+# the residual stream of a decoder whose sublayers share one layer norm
+PARALLEL_STREAM = dict(stream="pre", norm="layer", embed_positions=False)
+
 # config.json "architecture" -> reader (the other families are told apart by Hugging Face's "model_type")
 ARCHITECTURES: Dict[str, Callable[[dict, str], ModelConfig]] = {"Kafunex": _kafunex_config,
-                                                                     "Fubapel": _fubapel_config}
+                                                                     "Fubapel": _fubapel_config,
+                                                                     "Nuvorax": _nuvorax_config}
 
 
 def _kafunex_preset(name, vocab, width, ff, groups, rec, att) -> ModelConfig:
@@ -392,6 +505,18 @@ def _mlstm(heads, dim, vdim, cap=15.0) -> LayerSpec:
     return LayerSpec("mlstm", heads, dim, vdim, ffn="clamped_glu", gate_cap=cap)
 
 
+def _mixed(heads, kv_heads, dim, vdim, rot, moe=None, ff=0, limit=0.0, cap=50.0) -> LayerSpec:
+    return LayerSpec("mixed_attention", heads, dim, vdim, ff, kv_heads, scale=dim ** -0.5, softcap=cap, rot_dims=rot,
+                     rot_base=5e5, rot_scaling=(8.0, 1.0, 4.0, 8192.0), ffn="clamped_glu" if moe else "gelu",
+                     limit=limit, moe=moe, parallel=True)
+
+
+def _nuvorax_preset(name, vocab, width, dense, moe, n) -> ModelConfig:
+    """One dense layer, then ``n`` with experts."""
+    return hybrid_config("nuvorax", vocab, width, 1e-6, (dense,) + (moe,) * n, name, embed_scale=width ** 0.5,
+                         logit_scale=0.5, **PARALLEL_STREAM)
+
+
 PRESETS = {
     # hybrid decoders: a small one for tests, and one with a 7B-class model's layer sizes
     "tiny-kafunex": _kafunex_preset("tiny-kafunex", 640, 128, 256, 1, LayerSpec("hgrn2", 2, 32, 48, 256),
@@ -403,6 +528,10 @@ PRESETS = {
     "fubapel-7b": _fubapel_preset("fubapel-7b", 32000, 4096, 14336, {"start": 4, "stop": 8, "times": 2},
                                   _latent(32, 128, 128, 64, 1536, 512, 14336), _mlstm(16, 256, 256),
                                   _retention(32, 128, 128), 8),
+    "tiny-nuvorax": _nuvorax_preset("tiny-nuvorax", 640, 128, _mixed(4, 2, 32, 48, 16, ff=256),
+                                    _mixed(4, 2, 32, 48, 16, MoESpec(8, 3, 64, 5.0, 4, 2, 1.5), 96, 7.0), 2),
+    "nuvorax-7b": _nuvorax_preset("nuvorax-7b", 32000, 2048, _mixed(16, 4, 128, 128, 64, ff=10752),
+                                  _mixed(16, 4, 128, 128, 64, MoESpec(32, 4, 1408, 7.0, 4, 2, 2.0), 1408, 7.0), 23),
     "llama2-7b": ModelConfig(name="llama2-7b"),
     "llama3-8b": ModelConfig(vocab_size=128256, intermediate_size=14336, num_key_value_heads=8,
                              rope_theta=500000.0, max_position_embeddings=8192, bos_token_id=128000,

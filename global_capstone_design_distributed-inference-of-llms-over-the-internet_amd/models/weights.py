@@ -129,7 +129,9 @@ class GPT2Layer:
 class HybridLayer:
     """A layer of a hybrid decoder.  GEMM weights have the stage's dtype; norms, gates and mixing matrices
     are fp32.  ``w_in`` fuses the mixer's input projections (``LayerSpec.in_rows``); ``*_p`` are the
-    fragment-native copies for the decode GEMM where the shape allows one."""
+    fragment-native copies for the decode GEMM where the shape allows one.  In a parallel layer the feed-forward's
+    projections are part of ``w_in`` (rows from ``mix_rows`` on) and ``w_o`` (columns from ``out_cols`` on).  Expert
+    weights are held in one form: packed (``w_eu_p``, ``w_ed_p``) where the MFMA kernels cover the shape."""
     spec: LayerSpec
     w_in: torch.Tensor                       # [in_rows, W]
     w_o: torch.Tensor                        # [W, heads * vdim]
@@ -152,6 +154,14 @@ class HybridLayer:
     sink: Optional[torch.Tensor] = None      # latent_attention [heads]
     log_decay: Optional[torch.Tensor] = None  # retention [heads]: log2 of the decay
     gate_bias: Optional[torch.Tensor] = None  # mlstm [2, heads]: input and forget gate
+    q_gain: Optional[torch.Tensor] = None    # mixed_attention [dim]
+    k_gain: Optional[torch.Tensor] = None    # mixed_attention [dim]
+    w_r: Optional[torch.Tensor] = None       # experts: router [experts, W]
+    w_eu: Optional[torch.Tensor] = None      # experts [experts, 2 ff, W]: gate and up rows in blocks of ``expert_block``
+    w_ed: Optional[torch.Tensor] = None      # experts [experts, W, ff]
+    expert_block: int = 0
+    w_eu_p: Optional[torch.Tensor] = None    # [experts, 2 ff / 16, W / 32, 64, 8]
+    w_ed_p: Optional[torch.Tensor] = None    # [experts, W / 16, ff / 32, 64, 8]
     ffn_block: int = 0                       # gated feed-forward: rows of a gate / up block of ``w_up``
     w_in_p: Optional[torch.Tensor] = None
     w_o_p: Optional[torch.Tensor] = None
@@ -209,6 +219,10 @@ class StageWeights:
                     if w is not None and w.dtype == torch.bfloat16 and w.shape[0] % 16 == 0 and w.shape[1] % 128 == 0 \
                             and getattr(lay, name + "_p") is None:
                         setattr(lay, name + "_p", ops.pack_weight(w))
+                if lay.w_eu is not None and ops.expert_mfma_ok(lay.spec.moe.ff, self.cfg.hidden_size, lay.w_eu.dtype):
+                    lay.w_eu_p = torch.stack([ops.pack_weight(w) for w in lay.w_eu])
+                    lay.w_ed_p = torch.stack([ops.pack_weight(w) for w in lay.w_ed])
+                    lay.w_eu = lay.w_ed = None
             if isinstance(lay, LlamaLayer) and lay.qkv_p is None and lay.qkv is not None:
                 if fold_norms and not lay.moe:
                     lay.qkv_p = ops.pack_weight((lay.qkv.float() * lay.input_norm.float()[None, :])
@@ -353,6 +367,10 @@ def _random_gpt2_layer(cfg: ModelConfig, idx: int, device, dtype, seed: int) -> 
 
 
 # ------------------------------------------------------------------ hybrid decoders
+def _ffn_prefix(spec: LayerSpec) -> str:
+    return "mlp.shared." if spec.moe else "mlp."
+
+
 def _hybrid_names(spec: LayerSpec, cfg: ModelConfig) -> Dict[str, tuple]:
     """Checkpoint tensors of one layer (after its 'l<i>.' prefix) -> shape."""
     width = cfg.hidden_size
@@ -373,14 +391,28 @@ def _hybrid_names(spec: LayerSpec, cfg: ModelConfig) -> Dict[str, tuple]:
                   "mix.o": (width, H * V)})
         if spec.mixer == "mlstm":
             n.update({"mix.norm": (H * V,), "mix.i": (H, width), "mix.i.b": (H,), "mix.f": (H, width), "mix.f.b": (H,)})
+    elif spec.mixer == "mixed_attention":
+        G = spec.kv_heads
+        n.update({"mix.q": (H * D, width), "mix.k": (G * D, width), "mix.v": (G * V, width), "mix.q.norm": (D,),
+                  "mix.k.norm": (D,), "mix.talk": (H, H), "mix.g": (H, width), "mix.o": (width, H * V)})
     else:
         KD = spec.kv_heads * D
         n.update({"mix.q": (H * D, width), "mix.k": (KD, width), "mix.q.norm": (H * D,), "mix.k.norm": (KD,),
                   "mix.talk": (H, H), "mix.g": (H * D, width), "mix.o": (width, H * D)})
     if spec.ff:
-        n.update({"mlp.up": (spec.ff, width), "mlp.down": (width, spec.ff), "norm2": norm})
-        if spec.ffn == "clamped_glu":
-            n["mlp.gate"] = (spec.ff, width)
+        p = _ffn_prefix(spec)
+        n.update({p + "up": (spec.ff, width), p + "down": (width, spec.ff)})
+        if spec.glu:
+            n[p + "gate"] = (spec.ff, width)
+        if spec.moe:
+            n[p + "sg"] = (1, width)
+    if spec.moe:
+        n["mlp.router"] = (spec.moe.experts, width)
+        for e in range(spec.moe.experts):
+            n.update({f"mlp.e{e}.gate": (spec.moe.ff, width), f"mlp.e{e}.up": (spec.moe.ff, width),
+                      f"mlp.e{e}.down": (width, spec.moe.ff)})
+    if (spec.ff or spec.moe) and not spec.parallel:
+        n["norm2"] = norm
     if scaled:
         n["ls1"] = (width,)
         if spec.ff:
@@ -390,7 +422,20 @@ def _hybrid_names(spec: LayerSpec, cfg: ModelConfig) -> Dict[str, tuple]:
 
 # a mixer's input projections in the order in which ``w_in`` fuses them
 _IN_PARTS = {"hgrn2": ("q", "f", "v"), "attention": ("q", "k", "g"), "latent_attention": ("dq", "dkv"),
-             "retention": ("q", "k", "v", "g"), "mlstm": ("q", "k", "v", "g", "i", "f")}
+             "retention": ("q", "k", "v", "g"), "mlstm": ("q", "k", "v", "g", "i", "f"),
+             "mixed_attention": ("q", "k", "v", "g")}
+
+
+def _stacked_gate_up(gate: torch.Tensor, up: torch.Tensor):
+    """Gate and up rows in alternating blocks, and the block: one kernel tile where the width has whole ones."""
+    F = gate.shape[0]
+    if F % GU_BLOCK == 0:
+        return interleave_gate_up(gate, up), GU_BLOCK
+    return torch.cat([gate, up], 0), F
+
+
+def _fill_rows(w: torch.Tensor, rows: int) -> torch.Tensor:
+    return w if w.shape[0] == rows else torch.cat([w, w.new_zeros(rows - w.shape[0], w.shape[1])], 0)
 
 
 def _hybrid_layer(spec: LayerSpec, cfg: ModelConfig, get, device, dtype) -> HybridLayer:
@@ -407,16 +452,29 @@ def _hybrid_layer(spec: LayerSpec, cfg: ModelConfig, get, device, dtype) -> Hybr
     g = lambda n: raw[n].to(dtype).contiguous()  # noqa: E731
     gain = lambda n, ls: f32(n) * f32(ls) if ls in raw else f32(n)  # noqa: E731
     w_in = torch.cat([raw["mix." + p].to(dtype) for p in _IN_PARTS[spec.mixer]], 0)
-    pad = spec.in_rows - w_in.shape[0]
-    if pad:
-        w_in = torch.cat([w_in, w_in.new_zeros(pad, w_in.shape[1])], 0)
-    lay = HybridLayer(spec, w_in.contiguous(), g("mix.o"), gain("norm1", "ls1"))
+    lay = HybridLayer(spec, _fill_rows(w_in, spec.mix_rows).contiguous(), g("mix.o"), gain("norm1", "ls1"))
     if spec.ff:
-        lay.w_up, lay.w_down, lay.n2 = g("mlp.up"), g("mlp.down"), gain("norm2", "ls2")
-        if spec.ffn == "clamped_glu":
-            lay.ffn_block = GU_BLOCK if spec.ff % GU_BLOCK == 0 else spec.ff
-            gate = g("mlp.gate")
-            lay.w_up = interleave_gate_up(gate, lay.w_up) if lay.ffn_block == GU_BLOCK else torch.cat([gate, lay.w_up], 0)
+        p = _ffn_prefix(spec)
+        lay.w_up, lay.w_down = g(p + "up"), g(p + "down")
+        if spec.glu:
+            lay.w_up, lay.ffn_block = _stacked_gate_up(g(p + "gate"), lay.w_up)
+        if spec.moe:
+            lay.w_up = torch.cat([lay.w_up, g(p + "sg")], 0)
+        lay.w_up = _fill_rows(lay.w_up, spec.ff_rows).contiguous()
+        if spec.parallel:
+            lay.w_in, lay.w_o = torch.cat([lay.w_in, lay.w_up], 0), torch.cat([lay.w_o, lay.w_down], 1).contiguous()
+            lay.w_up = lay.w_down = None
+    if spec.moe:
+        E, F, W = spec.moe.experts, spec.moe.ff, cfg.hidden_size
+        lay.w_r = g("mlp.router")
+        lay.w_eu = torch.empty(E, 2 * F, W, dtype=dtype, device=device)
+        lay.w_ed = torch.empty(E, W, F, dtype=dtype, device=device)
+        for e in range(E):
+            up, lay.expert_block = _stacked_gate_up(raw[f"mlp.e{e}.gate"], raw[f"mlp.e{e}.up"])
+            lay.w_eu[e].copy_(up)
+            lay.w_ed[e].copy_(raw[f"mlp.e{e}.down"])
+    if "norm2" in raw:
+        lay.n2 = gain("norm2", "ls2")
     H, D, V = spec.heads, spec.dim, spec.vdim
     if spec.mixer == "hgrn2":
         lay.f_bias, lay.f_lower, lay.o_norm = f32("mix.f.b"), f32("mix.lower"), f32("mix.norm")
@@ -430,6 +488,8 @@ def _hybrid_layer(spec: LayerSpec, cfg: ModelConfig, get, device, dtype) -> Hybr
         lay.log_decay = torch.log2(torch.tensor(spec.decay, dtype=torch.float64)).clamp(min=-1e30).float().to(device)
     elif spec.mixer == "mlstm":
         lay.o_norm, lay.gate_bias = f32("mix.norm"), torch.stack([f32("mix.i.b"), f32("mix.f.b")])
+    elif spec.mixer == "mixed_attention":
+        lay.q_gain, lay.k_gain, lay.talk = f32("mix.q.norm"), f32("mix.k.norm"), f32("mix.talk")
     else:
         kn = f32("mix.k.norm").view(spec.kv_heads, 1, spec.dim)
         kn = kn.expand(spec.kv_heads, spec.heads // spec.kv_heads, spec.dim).reshape(-1)
@@ -515,6 +575,8 @@ def random_stage_weights(cfg: ModelConfig, start: int, end: int, *, has_embed: b
             sw.lm_head = emb
     if has_head:
         sw.final_norm = torch.ones(H, dtype=torch.float32 if cfg.hybrid else dtype, device=device)
+        if cfg.hybrid:
+            sw.final_norm *= cfg.logit_scale
         if cfg.model_type == "gpt2":
             sw.final_norm_b = torch.zeros(H, dtype=dtype, device=device)
         if sw.lm_head is None:
@@ -613,7 +675,7 @@ def load_stage_weights(cfg: ModelConfig, path: str, start: int, end: int, *, has
             sw.embed = t("embed").contiguous()
         if has_head:
             fn = ck.get("final.norm").to(dev).float().reshape(-1)
-            sw.final_norm = fn.expand(W).contiguous()  # (one gain for all, or one each)
+            sw.final_norm = (fn * cfg.logit_scale).expand(W).contiguous()  # (one gain for all, or one each)
             sw.lm_head = _pad_rows(t("head"), 16).contiguous()
         return sw
     if cfg.model_type == "gpt2":

@@ -1471,3 +1471,4 @@ def autotune_w8(shapes, device, ms=(4, 16, 32, 48, 64), iters: int = 12, rounds:
 
 # the hybrid decoders' ops (imported last: they dispatch through this module)
 from . import hybrid, mixers  # noqa: E402,F401
+from .moe import expert_mfma_ok  # noqa: E402,F401

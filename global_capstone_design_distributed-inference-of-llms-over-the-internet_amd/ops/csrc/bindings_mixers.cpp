@@ -6,7 +6,8 @@
 extern "C" {
 int mp_stream_norm(int src, const void* y, int64_t ys, const float* part, int S, int64_t slab, const int64_t* ids,
                    int64_t vocab, const int32_t* rows, float* res, const float* w, void* x, int n, int W, float mult,
-                   float eps, int center, int packed_mt, int f32, hipStream_t stream);
+                   float eps, int center, int packed_mt, int f32, const void* ye, int ye_f32, const int32_t* eslot,
+                   const float* ew, int top, hipStream_t stream);
 int mp_clamped_glu(const void* x, int64_t xs, void* out, int64_t M, int F, int B, float limit, int packed_mt, int f32,
                    hipStream_t stream);
 int mp_linear_scan(int kind, const void* z, int64_t zs, const float* rope, int rot, const float* decay,
@@ -45,9 +46,10 @@ void check_res(const at::Tensor& res, int64_t n, int64_t W) {
   MP_CHECK(res.scalar_type() == at::kFloat && res.is_contiguous(), "res: fp32 contiguous");
 }
 
-// res += mult * y, x = norm(res) * w.  y: [n, W] rows, fp32 [S, n, W] slabs, or none
+// res += mult * (y + routed experts' rows), x = norm(res) * w.  y: [n, W] rows, fp32 [S, n, W] slabs, or none;
+// ye [slots, W] with eslot, ew [n, top]
 void add_norm(const opt_tensor& y, at::Tensor& res, const opt_tensor& w, const opt_tensor& x, double mult, double eps,
-              int64_t center, int64_t packed) {
+              int64_t center, int64_t packed, const opt_tensor& ye, const opt_tensor& eslot, const opt_tensor& ew) {
   const int64_t n = res.size(0), W = res.size(1);
   check_res(res, n, W);
   int f32 = 0, mt = 0;
@@ -76,13 +78,26 @@ void add_norm(const opt_tensor& y, at::Tensor& res, const opt_tensor& w, const o
     check_rows(*y, n, W, "y");
     src = 0, yp = y->data_ptr(), ys = y->stride(0);
   }
+  const void* ep = nullptr;
+  const int32_t* sp = nullptr;
+  const float* gp = nullptr;
+  int top = 0, ef = 0;
+  if (ye.has_value()) {
+    MP_CHECK(eslot.has_value() && ew.has_value() && eslot->dim() == 2 && eslot->size(0) == n, "experts: eslot, ew [n, top]");
+    top = eslot->size(1);
+    ef = act_type(*ye, "ye");
+    MP_CHECK(ef || !f32, "ye: fp32, or the activations' type");
+    check_rows(*ye, n * top, W, "ye");
+    MP_CHECK(ye->is_contiguous() && top >= 1, "ye: contiguous rows");
+    ep = ye->data_ptr(), sp = i32_vec(*eslot, n * top, "eslot"), gp = f32_vec(*ew, n * top, "ew");
+  }
   check_launch(mp_stream_norm(src, yp, ys, part, S, n * W, nullptr, 0, nullptr, res.data_ptr<float>(), wp, xp, n, W,
-                              (float)mult, (float)eps, (int)center, mt, f32, cur_stream()),
+                              (float)mult, (float)eps, (int)center, mt, f32, ep, ef, sp, gp, top, cur_stream()),
                "add_norm");
 }
 
 void embed_norm(const at::Tensor& ids, const at::Tensor& table, at::Tensor& res, const at::Tensor& w, at::Tensor& x,
-                double eps, int64_t center, int64_t packed) {
+                double eps, int64_t center, int64_t packed, double scale) {
   const int f32 = act_type(table, "table");
   const int64_t n = ids.numel(), W = table.size(1);
   MP_CHECK(table.dim() == 2 && table.is_contiguous(), "table [vocab, W]");
@@ -90,8 +105,8 @@ void embed_norm(const at::Tensor& ids, const at::Tensor& table, at::Tensor& res,
   check_res(res, n, W);
   const int mt = check_out(x, n, W, f32, packed, "x");
   check_launch(mp_stream_norm(3, table.data_ptr(), W, nullptr, 0, 0, i64_vec(ids, n, "ids"), table.size(0), nullptr,
-                              res.data_ptr<float>(), f32_vec(w, W, "w"), x.data_ptr(), n, W, 1.f, (float)eps,
-                              (int)center, mt, f32, cur_stream()),
+                              res.data_ptr<float>(), f32_vec(w, W, "w"), x.data_ptr(), n, W, (float)scale,
+                              (float)eps, (int)center, mt, f32, nullptr, 0, nullptr, nullptr, 0, cur_stream()),
                "embed_norm");
 }
 
@@ -104,7 +119,7 @@ void rows_stream_norm(const at::Tensor& res, const at::Tensor& rows, const at::T
   const int mt = check_out(out, n, W, f32, packed, "out");
   check_launch(mp_stream_norm(2, nullptr, W, nullptr, 0, 0, nullptr, 0, i32_vec(rows, n, "rows"), res.data_ptr<float>(),
                               f32_vec(w, W, "w"), out.data_ptr(), n, W, 0.f, (float)eps, (int)center, mt, f32,
-                              cur_stream()),
+                              nullptr, 0, nullptr, nullptr, 0, cur_stream()),
                "rows_stream_norm");
 }
 
@@ -335,11 +350,11 @@ void latent_wide(const at::Tensor& q, const at::Tensor& kv, const at::Tensor& la
 
 TORCH_LIBRARY_FRAGMENT(mpamd, m) {
   m.def(
-      "add_norm(Tensor? y, Tensor(a!) res, Tensor? w, Tensor(b!)? x, float mult, float eps, int center, int packed) -> "
-      "()");
+      "add_norm(Tensor? y, Tensor(a!) res, Tensor? w, Tensor(b!)? x, float mult, float eps, int center, int packed, "
+      "Tensor? ye=None, Tensor? eslot=None, Tensor? ew=None) -> ()");
   m.def(
-      "embed_norm(Tensor ids, Tensor table, Tensor(a!) res, Tensor w, Tensor(b!) x, float eps, int center, int packed) "
-      "-> ()");
+      "embed_norm(Tensor ids, Tensor table, Tensor(a!) res, Tensor w, Tensor(b!) x, float eps, int center, int packed, "
+      "float scale=1.0) -> ()");
   m.def(
       "rows_stream_norm(Tensor res, Tensor rows, Tensor w, Tensor(a!) out, float eps, int center, int packed) -> ()");
   m.def("clamped_glu(Tensor x, Tensor(a!) out, int block, float limit, int packed) -> ()");

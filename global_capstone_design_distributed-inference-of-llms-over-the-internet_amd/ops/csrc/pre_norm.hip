@@ -2,7 +2,8 @@
 //
 //   stream_norm   res[t] += mult * y[t], then x[t] = norm(res[t]) * w for the next sublayer
 //                 y: activation rows, the S fp32 split-K slabs of the projection that made it, rows of the
-//                 embedding table (res[t] = table[id]), or none
+//                 embedding table (res[t] = mult * table[id]), or none; routed experts' rows may come on top:
+//                 res[t] += mult * sum_k ew[t, k] ye[eslot[t, k]]
 //                 norm: centred (layer norm: mean and variance) or not (root mean square); w == null: no x
 //   clamped_glu   out = g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit)
 //
@@ -26,7 +27,38 @@ struct StreamArgs {
   void* x;
   int W, packed_mt, center;
   float mult, eps;
+  const void* ye;         // [slots, W] rows of the routed experts (fp32, or the activations' type), or null
+  const int32_t* eslot;   // [n, top] row of ye, -1: none
+  const float* ew;        // [n, top]
+  int top, ye_f32;
 };
+
+// v += mult * sum_k ew[k] ye[eslot[k]][c ..], four rows' loads in flight
+template <typename T, int VEC>
+__device__ __forceinline__ void add_experts(const StreamArgs& a, int row, int c, float (&v)[VEC]) {
+  const int32_t* sl = a.eslot + (int64_t)row * a.top;
+  const float* ew = a.ew + (int64_t)row * a.top;
+  float y[VEC];
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) y[j] = 0.f;
+  for (int k = 0; k < a.top; k += 4) {
+    float p[4][VEC], w[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int kk = min(k + i, a.top - 1), r = sl[kk];
+      w[i] = k + i < a.top && r >= 0 ? ew[kk] : 0.f;
+      const int64_t at = (int64_t)max(r, 0) * a.W + c;
+      if (a.ye_f32) ld_vec<VEC>((const float*)a.ye + at, p[i]);
+      else ld_vec<VEC>((const T*)a.ye + at, p[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) y[j] += w[i] != 0.f ? w[i] * p[i][j] : 0.f;
+  }
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) v[j] += a.mult * y[j];
+}
 
 enum { SRC_ROWS = 0, SRC_SLABS = 1, SRC_NONE = 2, SRC_TABLE = 3 };
 
@@ -50,6 +82,8 @@ __global__ __launch_bounds__(NT) void stream_norm_kernel(StreamArgs a) {
     if (a.w != nullptr) ld_vec<VEC>(a.w + c, g[k]);
     if constexpr (SRC == SRC_TABLE) {
       ld_vec<VEC>((const T*)a.y + id * W + c, v[k]);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) v[k][j] *= a.mult;
     } else {
       ld_vec<VEC>(a.res + (int64_t)row * W + c, v[k]);
       if constexpr (SRC == SRC_ROWS) {
@@ -75,9 +109,10 @@ __global__ __launch_bounds__(NT) void stream_norm_kernel(StreamArgs a) {
 #pragma unroll
         for (int j = 0; j < VEC; ++j) v[k][j] += a.mult * y[j];
       }
+      if (a.ye != nullptr) add_experts<T, VEC>(a, row, c, v[k]);
     }
     if (ch < nch) {
-      if constexpr (SRC != SRC_NONE) st_vec<VEC>(a.res + (int64_t)row * W + c, v[k]);
+      if (SRC != SRC_NONE || a.ye != nullptr) st_vec<VEC>(a.res + (int64_t)row * W + c, v[k]);
 #pragma unroll
       for (int j = 0; j < VEC; ++j) sum += v[k][j];
     }
@@ -159,11 +194,13 @@ __global__ __launch_bounds__(256) void clamped_glu_kernel(const T* __restrict__ 
 extern "C" int mp_stream_norm(int src, const void* y, int64_t ys, const float* part, int S, int64_t slab,
                               const int64_t* ids, int64_t vocab, const int32_t* rows, float* res, const float* w,
                               void* x, int n, int W, float mult, float eps, int center, int packed_mt, int f32,
+                              const void* ye, int ye_f32, const int32_t* eslot, const float* ew, int top,
                               hipStream_t stream) {
   using namespace mp;
   (void)hipGetLastError();
   if (n == 0) return 0;
-  const StreamArgs a{y, ys, part, S, slab, ids, vocab, rows, res, w, x, W, packed_mt, center, mult, eps};
+  const StreamArgs a{y,   ys,        part,   S,    slab, ids, vocab,  rows, res, w, x,
+                     W,   packed_mt, center, mult, eps,  ye,  eslot, ew,   top, ye_f32};
   switch (src) {
     case SRC_ROWS: return f32 ? launch_stream_norm<float, 0>(a, n, stream) : launch_stream_norm<bf16_t, 0>(a, n, stream);
     case SRC_SLABS: return f32 ? -2 : launch_stream_norm<bf16_t, 1>(a, n, stream);

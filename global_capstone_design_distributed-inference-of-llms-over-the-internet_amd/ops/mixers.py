@@ -14,31 +14,44 @@ from . import reference_mixers as rm
 from .hybrid import _native, _put
 
 
-def rope_table(base: float, dims: int, positions: int, device) -> torch.Tensor:
-    """fp32 [positions, dims]: cosines, then sines, of position * base^(-2i / dims) (angles made in fp64)."""
+def rope_table(base: float, dims: int, positions: int, device, scaling=None) -> torch.Tensor:
+    """fp32 [positions, dims]: cosines, then sines, of position * f_i, f_i = base^(-2i / dims) (angles made in fp64).
+    ``scaling`` (factor, low, high, original): frequencies whose wavelength is above original / low are divided by the
+    factor, those below original / high are kept, and between them the two are blended linearly in 1 / wavelength."""
     i = torch.arange(dims // 2, dtype=torch.float64)
-    a = torch.arange(positions, dtype=torch.float64)[:, None] * torch.pow(float(base), -2.0 * i / max(dims, 1))[None]
+    f = torch.pow(float(base), -2.0 * i / max(dims, 1))
+    if scaling is not None:
+        factor, low, high, original = (float(x) for x in scaling)
+        keep = ((original * f / (2.0 * torch.pi) - low) / (high - low)).clamp(0.0, 1.0)
+        f = keep * f + (1.0 - keep) * f / factor
+    a = torch.arange(positions, dtype=torch.float64)[:, None] * f[None]
     return torch.cat([torch.cos(a), torch.sin(a)], 1).float().to(device)
 
 
 # ------------------------------------------------------------------ residual stream
-def embed_norm(ids, table, res, w, eps, x, center=False, packed=False):
-    """res[t] = table[ids[t]] (fp32), x = norm(res) * w; ``center``: layer norm, else root mean square."""
+def embed_norm(ids, table, res, w, eps, x, center=False, packed=False, scale=1.0):
+    """res[t] = scale * table[ids[t]] (fp32), x = norm(res) * w; ``center``: layer norm, else root mean square."""
     if not _native(table):
-        res.copy_(table[ids.long()].float())
+        res.copy_(table[ids.long()].float() * scale)
         return _put(x, rm.norm(res, w, eps, center), packed)
-    torch.ops.mpamd.embed_norm(ids, table, res, w, x, float(eps), int(center), int(packed))
+    torch.ops.mpamd.embed_norm(ids, table, res, w, x, float(eps), int(center), int(packed), float(scale))
     return x
 
 
-def add_norm(y, res, mult, w, eps, x, center=False, packed=False):
+def add_norm(y, res, mult, w, eps, x, center=False, packed=False, experts=None):
     """res += mult * y, then x = norm(res) * w.  ``y``: [n, W], fp32 split-K slabs [S, n, W], or None; ``w`` None:
-    the sum alone."""
+    the sum alone.  ``experts``: routed experts' outputs that belong to y, (rows, row of every choice [n, top] with -1
+    for none, weights [n, top])."""
     if not _native(res):
         if y is not None:
             res.add_((y.sum(0) if y.dim() == 3 else y).float() * mult)
+        if experts is not None:
+            ye, slot, ew = experts
+            pick = torch.where((slot >= 0)[..., None], ye[slot.clamp(min=0).long()].float(), 0.0)
+            res.add_((pick * ew[..., None]).sum(1) * mult)
         return _put(x, rm.norm(res, w, eps, center), packed) if w is not None else None
-    torch.ops.mpamd.add_norm(y, res, w, x, float(mult), float(eps), int(center), int(packed))
+    torch.ops.mpamd.add_norm(y, res, w, x, float(mult), float(eps), int(center), int(packed),
+                             *(experts if experts is not None else ()))
     return x
 
 

@@ -7,7 +7,12 @@ The residual stream is fp32 and lives in one buffer; a sublayer f reads an activ
 
 One kernel closes a sublayer: it adds the output projection (rows, or the fp32 split-K slabs of a decode GEMM) to the
 stream and writes the next sublayer's ``xb``.  A mixer is one fused input projection z = xb W_in^T, its own ops, and
-an output projection; the feed-forward is squared relu or the clamped gated form.
+an output projection; the feed-forward is squared relu, gelu or the clamped gated form, with or without routed experts.
+
+    parallel layers     xb = norm(res) gain ; res += mult * (f(xb) + g(xb))
+
+run as one sublayer: z has the feed-forward's columns too, its activation lies beside the mixer's in the input of one
+output projection, and the kernel that closes the layer adds the routed experts' rows.
 
 Activations feeding a decode-sized GEMM stay in the packed MFMA-fragment layout where the shape has a native
 GEMM (``ops.native_gemm_ok``); other shapes, prompts and fp32 run the library GEMM on row-major activations.
@@ -23,7 +28,9 @@ import torch
 
 from .. import ops
 from ..ops import hybrid as hops
+from ..ops import mixed as xops
 from ..ops import mixers as mops
+from ..ops import moe as eops
 
 # most bytes of fp32 partial sums of a latent attention step whose contexts are split
 LATENT_WS_BYTES = 256 << 20
@@ -50,9 +57,10 @@ class HybridStage:
                 self.index.append(na)
                 na += 1
         specs = [lay.spec for lay in ex.w.layers]
-        self.rope = {(sp.rot_base, sp.rot_dims): None for sp in specs if sp.mixer in ("retention", "latent_attention")}
-        for base, dims in self.rope:
-            self.rope[(base, dims)] = mops.rope_table(base, dims, ex.max_seq_len, ex.device)
+        # angle tables: (base, dimensions, frequency scaling)
+        keys = {self._rope_key(sp) for sp in specs if sp.mixer in ("retention", "latent_attention", "mixed_attention")}
+        keys |= {(sp.rot_base, sp.vdim, None) for sp in specs if sp.mixer == "mixed_attention"}
+        self.rope = {k: mops.rope_table(k[0], k[1], ex.max_seq_len, ex.device, k[2]) for k in keys}
         # query-block tokens of each attention shape's MFMA form (0: the any-shape form)
         self.talk_block, self.latent_block = {}, {}
         for sp in specs if ex.device.type == "cuda" else ():
@@ -66,8 +74,12 @@ class HybridStage:
                 self.latent_block[key] = mops.latent_block(*key, ex.cache.page_size) if bf16 else 0
         self.rec_heads = min([sp.heads for sp in specs if sp.mixer == "hgrn2"], default=0)
         self.lin_heads = min([sp.heads for sp in specs if sp.mixer in ("retention", "mlstm")], default=0)
-        self.max_chunk = max([sp.chunk if sp.mixer == "attention" else 1 << 30 for sp in specs if not sp.recurrent],
+        self.max_chunk = max([sp.chunk or 1 << 30 for sp in specs if not sp.recurrent],
                              default=1)
+
+    @staticmethod
+    def _rope_key(sp):
+        return sp.rot_base, sp.rot_dims, sp.rot_scaling
 
     @staticmethod
     def _latent_key(sp):
@@ -77,8 +89,9 @@ class HybridStage:
         """Decode-GEMM kernel choices for this stage's shapes (none while tuning is off)."""
         if ops.autotune_mode() == "off":
             return
-        up = {"relu2": 4, "clamped_glu": 1}
-        shapes = {(getattr(lay, n).shape[0], getattr(lay, n).shape[1], up[lay.spec.ffn] if n == "w_up" else 0)
+        up = {"relu2": 4, "clamped_glu": 1, "gelu": 0}
+        shapes = {(getattr(lay, n).shape[0], getattr(lay, n).shape[1],
+                   up[lay.spec.ffn] if n == "w_up" and not lay.spec.moe else 0)
                   for lay in self.ex.w.layers for n in lay.GEMMS if getattr(lay, n + "_p") is not None}
         if self.ex.w.lm_head_p is not None:
             shapes.add((self.ex.w.lm_head.shape[0], self.W, 0))
@@ -101,17 +114,20 @@ class HybridStage:
             return ops.linear(x, None, wp=wp, a_rows=T, out=out)
         return ops.linear(x, w, out=out)
 
-    def _add(self, y_in, w, wp, packed: bool, T: int, res, gain, nxt, xb, xb_packed: bool, e):
+    def _add(self, y_in, w, wp, packed: bool, T: int, res, gain, nxt, xb, xb_packed: bool, e, experts=None):
         """Close a sublayer: add y = y_in w^T to the stream and write the next sublayer's ``xb``.  ``gain``: the
         sublayer's own norm gain, ``nxt``: the next one's (None after the last).  A packed projection with a split-K
-        form hands its fp32 slabs straight to the kernel (no reduce launch, no rounding of y)."""
-        if packed and ops.rwk_split(T, w.shape[0], w.shape[1]) > 0:
+        form hands its fp32 slabs straight to the kernel (no reduce launch, no rounding of y).  ``experts``: routed
+        experts' rows that belong to y (``y_in`` None: the only ones)."""
+        if y_in is None:
+            y = None
+        elif packed and ops.rwk_split(T, w.shape[0], w.shape[1]) > 0:
             y = ops.linear_partials(y_in, T, wp=wp, out=e("y", (T, self.W)))
         else:
             y = self._mm(y_in, w, wp, T, packed, e("y", (T, self.W)))
         if self.pre:
             mops.add_norm(y, res, self.mult, nxt, self.eps, xb if nxt is not None else None, self.center,
-                          packed=xb_packed)
+                          packed=xb_packed, experts=experts)
         else:
             hops.residual_norm(y, res, gain, self.eps, xb, packed=xb_packed)
 
@@ -133,7 +149,7 @@ class HybridStage:
 
     def _retention(self, i, lay, z, o, pko, m, e):
         sp = lay.spec
-        mops.retention(z, self.rope[(sp.rot_base, sp.rot_dims)], lay.log_decay, self.ex.state.layer(self.index[i])[0],
+        mops.retention(z, self.rope[self._rope_key(sp)], lay.log_decay, self.ex.state.layer(self.index[i])[0],
                        m["q_seq"], m["q_ctx"], o, self.eps, plan=m["linear"], packed=pko)
 
     def _mlstm(self, i, lay, z, o, pko, m, e):
@@ -160,7 +176,7 @@ class HybridStage:
     def _latent(self, i, lay, z, o, pko, m, e):
         ex, sp, T, plan = self.ex, lay.spec, m["T"], m["plan"]
         kv, _ = ex.cache.layer(self.index[i])
-        rope = self.rope[(sp.rot_base, sp.rot_dims)]
+        rope = self.rope[self._rope_key(sp)]
         pkq = self._packed(T, lay.w_uq, lay.w_uq_p)
         cq = self._act(e, "cq", T, sp.q_rank, pkq)
         mops.latent_prep(z, lay.q_norm, lay.c_norm, cq, kv, m["slots"], m["q_ctx"], rope, self.eps, packed=pkq)
@@ -189,16 +205,43 @@ class HybridStage:
         mops.latent_attention(q, lay.w_uk, lay.w_uv, lay.sink, rope, kv, m["table"], m["q_seq"], m["q_ctx"], o, sp.scale,
                               packed=pko, **kw)
 
+    def _mixed(self, i, lay, z, o, pko, m, e):
+        ex, sp, T = self.ex, lay.spec, m["T"]
+        kv, _ = ex.cache.layer(self.index[i])
+        rope, vrope = self.rope[self._rope_key(sp)], self.rope[(sp.rot_base, sp.vdim, None)]
+        qn = e(f"qn{sp.heads * sp.dim}", (T, sp.heads * sp.dim))
+        ff = (self._ff_kind(sp), sp.ff, lay.ffn_block or 1, sp.mix_rows, sp.limit) if sp.parallel and sp.ff else None
+        xops.mixed_prep(z, lay.q_gain, lay.k_gain, qn, kv, m["slots"], m["q_ctx"], rope, vrope, o, sp.o_cols, self.eps,
+                        ff=ff, packed=pko)
+        xops.mixed_attention(z, qn, lay.talk, kv, m["table"], m["q_seq"], m["q_ctx"], vrope, o, sp.o_cols, sp.scale,
+                             sp.softcap, packed=pko)
+
     MIX = {"hgrn2": _hgrn2, "retention": _retention, "mlstm": _mlstm, "attention": _attention,
-           "latent_attention": _latent}
+           "latent_attention": _latent, "mixed_attention": _mixed}
+
+    @staticmethod
+    def _ff_kind(sp):
+        """Activation of a feed-forward that the decode GEMM's epilogues do not cover."""
+        return "gated_glu" if sp.moe else sp.ffn
+
+    def _experts(self, lay, x, packed: bool, m, e):
+        """Routed experts of the rows ``x``: (rows, row of every choice, weights)."""
+        c = eops.choose(x, lay.w_r, m["q_ctx"], lay.spec.moe, e, packed=packed)
+        y = eops.experts(x, c, lay.w_eu, lay.w_ed, lay.w_eu_p, lay.w_ed_p, lay.expert_block, e, packed=packed)
+        return y, c.slot, c.weights
 
     def _ffn(self, lay, xu, pku: bool, T: int, e):
         """Feed-forward activation (what ``w_down`` reads) and whether it is packed."""
         sp = lay.spec
+        if lay.w_down is None:  # routed experts alone
+            return None, False
         pkd = self._packed(T, lay.w_down, lay.w_down_p)
         a = self._act(e, "act", T, sp.ff, pkd)
         rows = lay.w_up.shape[0]
-        glu = sp.ffn == "clamped_glu"
+        if sp.moe or sp.ffn == "gelu":
+            u = self._mm(xu, lay.w_up, lay.w_up_p, T, pku, e(f"u{rows}", (T, rows)))
+            return xops.ffn_act(u, a, self._ff_kind(sp), sp.ff, lay.ffn_block or 1, sp.limit, packed=pkd), pkd
+        glu = sp.glu
         fused = dict(epilogue=1, glu_limit=sp.limit) if glu else dict(epilogue=4)
         if pku and (not glu or lay.ffn_block == ops.GU_BLOCK) and \
                 ops.native_gemm_ok(T, rows, self.W, fused["epilogue"], pkd):
@@ -244,9 +287,9 @@ class HybridStage:
         elif not self.pre:
             hops.embed_pos(x, ex.w.embed, positions, self.inv, res, xb, packed=pk)
         elif layers:
-            mops.embed_norm(x, ex.w.embed, res, first_gain(0), eps, xb, self.center, packed=pk)
+            mops.embed_norm(x, ex.w.embed, res, first_gain(0), eps, xb, self.center, packed=pk, scale=ex.cfg.embed_scale)
         else:
-            res.copy_(ex.w.embed[x.long()])
+            res.copy_(ex.w.embed[x.long()].float() * ex.cfg.embed_scale)
         m = {"T": T, "slots": slots, "q_seq": q_seq, "q_ctx": q_ctx, "plan": plan, "span": span,
              "linear": plan.get("linear") if plan else None, "table": ex.sessions.table_dev}
         for i, lay in enumerate(layers):
@@ -256,18 +299,20 @@ class HybridStage:
                 self._enter(res, first_gain(i), xb, pk)
             z = self._mm(xb, lay.w_in, lay.w_in_p, T, pk, e(f"z{sp.in_rows}", (T, sp.in_rows)))
             pko = self._packed(T, lay.w_o, lay.w_o_p)
-            o = self._act(e, "o", T, sp.out_cols, pko)
+            o = self._act(e, "o", T, sp.o_cols, pko)
             self.MIX[sp.mixer](self, i, lay, z, o, pko, m, e)
-            if sp.ff:
-                pku = self._packed(T, lay.w_up, lay.w_up_p)
+            if (sp.ff or sp.moe) and not sp.parallel:
+                pku = lay.w_up is not None and self._packed(T, lay.w_up, lay.w_up_p)
                 xu = self._act(e, "xb", T, W, pku)
                 self._add(o, lay.w_o, lay.w_o_p, pko, T, res, lay.n1, lay.n2, xu, pku, e)
                 a, pkd = self._ffn(lay, xu, pku, T, e)
+                rows = self._experts(lay, xu, pku, m, e) if sp.moe else None
                 pk, xb = entry(i + 1)
-                self._add(a, lay.w_down, lay.w_down_p, pkd, T, res, lay.n2, first_gain(i + 1), xb, pk, e)
+                self._add(a, lay.w_down, lay.w_down_p, pkd, T, res, lay.n2, first_gain(i + 1), xb, pk, e, rows)
             else:
+                rows = self._experts(lay, xb, pk, m, e) if sp.moe else None
                 pk, xb = entry(i + 1)
-                self._add(o, lay.w_o, lay.w_o_p, pko, T, res, lay.n1, first_gain(i + 1), xb, pk, e)
+                self._add(o, lay.w_o, lay.w_o_p, pko, T, res, lay.n1, first_gain(i + 1), xb, pk, e, rows)
         if not ex.is_last:
             return res
         S, V = last_rows.numel(), ex.cfg.vocab_size
