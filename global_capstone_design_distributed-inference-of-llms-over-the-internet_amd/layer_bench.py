@@ -1,22 +1,25 @@
 """Prefill and decode throughput of a hybrid decoder's layers beside the closest other families at equal size.
 
-``python bench.py --layer-bench [--layer-model kafunex|fubapel]`` (one GPU): for every width an 8-layer stage of the
+``python bench.py --layer-bench [--layer-model kafunex|fubapel|nuvorax]`` (one GPU): for every width an 8-layer stage of the
 model and of its like, of the same width, query heads, head size and feed-forward parameters, all bf16 with random
 weights, run in turn on the same executor code: prompts of several shapes, then decode steps (hipGraph replays) at
 several batch sizes, at contexts that end inside a 1024-token attention chunk (a query then sees as many keys on all
 sides).  One JSON line.
 
 * ``kafunex``: (three recurrent layers, one attention layer) x 2, beside Llama;
-* ``fubapel``: (retention, latent attention, mLSTM, latent attention) x 2, beside Kafunex and Llama.
+* ``fubapel``: (retention, latent attention, mLSTM, latent attention) x 2, beside Kafunex and Llama;
+* ``nuvorax``: (dense, experts, experts, experts) x 2, 20 routed experts of which a token uses 4 and a shared one, beside
+  Mixtral (8 experts, 2 used: as many expert weights, as many of them used), Kafunex and Llama.
 """
 from __future__ import annotations
 
+import dataclasses
 import json
 import statistics
 
 import torch
 
-from .models.config import LayerSpec, ModelConfig, hybrid_config
+from .models.config import LayerSpec, ModelConfig, MoESpec, PARALLEL_STREAM, hybrid_config
 from .models.weights import random_stage_weights
 from .runtime.executor import StageExecutor
 
@@ -40,6 +43,18 @@ def configs(width: int, layers: int, model: str = "kafunex"):
                       name=f"llama-w{width}")
     if model == "kafunex":
         return hyb, uni
+    if model == "nuvorax":
+        F = 128 * round(ff_glu / 5 / 128)
+        mix = dict(kv_heads=G, scale=128 ** -0.5, softcap=50.0, rot_dims=64, rot_base=5e5, rot_scaling=(8.0, 1.0, 4.0, 8192.0),
+                   parallel=True)
+        dense = LayerSpec("mixed_attention", H, 128, 128, ff, ffn="gelu", **mix)
+        moe = LayerSpec("mixed_attention", H, 128, 128, F, ffn="clamped_glu", limit=7.0,
+                        moe=MoESpec(20, 4, F, 7.0, 4, 2, 1.0), **mix)
+        nuv = hybrid_config("nuvorax", VOCAB, width, 1e-6, [moe if i % 4 else dense for i in range(layers)],
+                            f"nuvorax-w{width}", embed_scale=width ** 0.5, logit_scale=0.5, **PARALLEL_STREAM)
+        mxt = dataclasses.replace(uni, model_type="mixtral", intermediate_size=ff_glu // 2, num_local_experts=8,
+                                  num_experts_per_tok=2, name=f"mixtral-w{width}")
+        return nuv, mxt, hyb, uni
     glu = dict(ff=ff_glu, ffn="clamped_glu", limit=7.0)
     ret = LayerSpec("retention", H, 128, 128, rot_dims=128, decay=tuple(1 - 2.0 ** (-5 - h % 8) for h in range(H)), **glu)
     mem = LayerSpec("mlstm", H, 128, 128, gate_cap=15.0, **glu)

@@ -15,41 +15,15 @@
 //   mixed_prep_kernel   projected row [q (H D) | k (G D) | v (G V) | gate (H)] -> q', cache; and the feed-forward's
 //                       activation where its projection lies in the same row
 //   mixed_any_kernel    any shape and both element types: one workgroup per query token
-#include "common.h"
-#include "act_io.h"
+#include "attn_mixed.h"
 
 namespace mp {
-
-struct MixedArgs {
-  const void* z;         // [T, zs] projected rows
-  int64_t zs;
-  void* qn;              // [T, H D] q'
-  const float *qg, *kg;  // [D] gains
-  const float* talk;     // [H, H]
-  const float* rope;     // [positions, rot] cosines, then sines
-  const float* vrope;    // [positions, V]
-  void* cache;           // [pages, G, page (D + V)]
-  const int64_t* slots;
-  const int32_t* bt;
-  int bt_stride;
-  const int32_t *q_seq, *q_ctx;
-  void* out;             // row-major [T, os] or packed
-  int64_t os;
-  int H, G, D, V, rot, page_log2, packed_mt;
-  float scale, cap, eps;
-};
 
 struct FfArgs {          // feed-forward activation of the row's columns from ``col`` on
   int kind;              // 0: none, 1: gelu, 2: clamped gated form, 3: the same times a gate per token
   int F, block, col, out_col;
   float limit;
 };
-
-// element offset of value column v of key ``off`` of a page, after the page's key rows
-__device__ __forceinline__ int64_t val_at(int off, int v, int V, int blk_log2) {
-  return ((int64_t)(off >> blk_log2) * V + v) * (1 << blk_log2) + (off & ((1 << blk_log2) - 1));
-}
-__device__ __forceinline__ int val_block_log2(int page_log2) { return min(page_log2, 5); }
 
 constexpr int MIX_HEAD = 512;  // largest head size of the prep kernel
 constexpr float MIX_GLU_ALPHA = 1.702f;

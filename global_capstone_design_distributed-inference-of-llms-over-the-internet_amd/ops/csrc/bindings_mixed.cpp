@@ -14,6 +14,15 @@ int mp_mixed_any(const void* z, int64_t zs, const void* qn, const float* talk, c
                  int bt_stride, const int32_t* q_seq, const int32_t* q_ctx, const float* vrope, void* out, int64_t os,
                  int packed_mt, int n, int H, int G, int D, int V, int page_log2, float scale, float cap, int f32,
                  hipStream_t stream);
+int mp_mixed_mfma_ok(int H, int G, int D, int V, int page_log2, float cap);
+int mp_mixed_prompt(const void* z, int64_t zs, const void* qn, const float* talk, const void* cache, const int32_t* bt,
+                    int bt_stride, const int32_t* q_seq, const int32_t* q_ctx, const float* vrope, void* out, int64_t os,
+                    int packed_mt, int n, int H, int G, int D, int V, int page_log2, float scale, float cap,
+                    const int32_t* blk, int nblk, int PS, int NP, float* sums, float* part, hipStream_t stream);
+int mp_mixed_decode(const void* z, int64_t zs, const void* qn, const float* talk, const void* cache, const int32_t* bt,
+                    int bt_stride, const int32_t* q_seq, const int32_t* q_ctx, const float* vrope, void* out, int64_t os,
+                    int packed_mt, int n, int H, int G, int D, int V, int page_log2, float scale, float cap, int PS, int NP,
+                    float* sums, float* part, hipStream_t stream);
 int64_t mp_moe_lists(int E);
 int mp_moe_router_splits(int T, int W, int E, int f32);
 int mp_moe_route(const void* x, int64_t xs, int mt, const void* w, const int32_t* ctx, float* part, int S, float* ew,
@@ -104,9 +113,19 @@ void ffn_act(const at::Tensor& z, at::Tensor& out, int64_t kind, int64_t F, int6
                "ffn_act");
 }
 
+int64_t mixed_mfma_ok(int64_t H, int64_t G, int64_t D, int64_t V, int64_t page, double cap) {
+  int l = 0;
+  while ((1ll << l) < page) ++l;
+  return (1ll << l) == page ? mp_mixed_mfma_ok((int)H, (int)G, (int)D, (int)V, l, (float)cap) : 0;
+}
+
+// form 0: any shape; 1: prompts, blk [2, nblk] (first token, tokens <= 16); 2: decode.  The keys in ``parts`` splits of
+// ``part_size``; sums fp32 [parts T H], part fp32 [parts T H V] (prompts, parts > 1) or [parts T G H V] (decode)
 void mixed_attention(const at::Tensor& z, const at::Tensor& qn, const at::Tensor& talk, const at::Tensor& cache,
                      const at::Tensor& bt, const at::Tensor& q_seq, const at::Tensor& q_ctx, const at::Tensor& vrope,
-                     at::Tensor& out, int64_t K, double scale, double cap, int64_t packed) {
+                     at::Tensor& out, int64_t K, double scale, double cap, int64_t packed, int64_t form,
+                     const opt_tensor& blk, int64_t part_size, int64_t parts, const opt_tensor& sums,
+                     const opt_tensor& part) {
   MP_CHECK(talk.dim() == 2 && talk.size(0) == talk.size(1), "talk [H, H]");
   const MixShape s = check_mixed(z, cache, vrope, talk.size(0));
   check_act(qn, s.f32, "qn");
@@ -115,6 +134,34 @@ void mixed_attention(const at::Tensor& z, const at::Tensor& qn, const at::Tensor
   MP_CHECK(bt.is_cuda() && bt.dim() == 2 && bt.scalar_type() == at::kInt && bt.stride(1) == 1, "block table int32");
   MP_CHECK(K >= s.H * s.V, "out columns");
   const int mt = check_out(out, s.T, K, s.f32, packed, "out");
+  if (form) {
+    MP_CHECK(!s.f32 && parts >= 1, "the MFMA forms are bf16");
+    MP_CHECK(K % 2 == 0, "out columns");
+    auto ws = [&](const opt_tensor& t, int64_t n, const char* name) {
+      MP_CHECK(t.has_value() && t->is_cuda() && t->scalar_type() == at::kFloat && t->is_contiguous() && t->numel() >= n &&
+                   reinterpret_cast<uintptr_t>(t->data_ptr()) % 16 == 0, std::string(name) + ": fp32 scratch");
+      return t->data_ptr<float>();
+    };
+    float* sp = ws(sums, parts * s.T * s.H, "sums");
+    if (form == 2) {
+      check_launch(mp_mixed_decode(z.data_ptr(), z.stride(0), qn.data_ptr(), f32_vec(talk, s.H * s.H, "talk"),
+                                   cache.data_ptr(), bt.data_ptr<int32_t>(), bt.stride(0), i32_vec(q_seq, s.T, "q_seq"),
+                                   i32_vec(q_ctx, s.T, "q_ctx"), vrope.data_ptr<float>(), out.data_ptr(), K, mt, s.T, s.H,
+                                   s.G, s.D, s.V, s.pl2, (float)scale, (float)cap, part_size, parts, sp,
+                                   ws(part, parts * s.T * s.G * s.H * s.V, "part"), cur_stream()),
+                   "mixed_decode");
+      return;
+    }
+    MP_CHECK(blk.has_value() && blk->dim() == 2 && blk->size(0) == 2, "blk int32 [2, nblk]");
+    const int64_t nb = blk->size(1);
+    check_launch(mp_mixed_prompt(z.data_ptr(), z.stride(0), qn.data_ptr(), f32_vec(talk, s.H * s.H, "talk"), cache.data_ptr(),
+                                 bt.data_ptr<int32_t>(), bt.stride(0), i32_vec(q_seq, s.T, "q_seq"),
+                                 i32_vec(q_ctx, s.T, "q_ctx"), vrope.data_ptr<float>(), out.data_ptr(), K, mt, s.T, s.H, s.G,
+                                 s.D, s.V, s.pl2, (float)scale, (float)cap, i32_vec(*blk, 2 * nb, "blk"), nb, part_size,
+                                 parts, sp, parts > 1 ? ws(part, parts * s.T * s.H * s.V, "part") : nullptr, cur_stream()),
+                 "mixed_prompt");
+    return;
+  }
   check_launch(mp_mixed_any(z.data_ptr(), z.stride(0), qn.data_ptr(), f32_vec(talk, s.H * s.H, "talk"), cache.data_ptr(),
                             bt.data_ptr<int32_t>(), bt.stride(0), i32_vec(q_seq, s.T, "q_seq"),
                             i32_vec(q_ctx, s.T, "q_ctx"), vrope.data_ptr<float>(), out.data_ptr(), K, mt, s.T, s.H, s.G,
@@ -202,7 +249,9 @@ TORCH_LIBRARY_FRAGMENT(mpamd, m) {
   m.def("ffn_act(Tensor z, Tensor(a!) out, int kind, int F, int block, float limit, int packed) -> ()");
   m.def(
       "mixed_attention(Tensor z, Tensor qn, Tensor talk, Tensor cache, Tensor bt, Tensor q_seq, Tensor q_ctx, Tensor "
-      "vrope, Tensor(a!) out, int K, float scale, float cap, int packed) -> ()");
+      "vrope, Tensor(a!) out, int K, float scale, float cap, int packed, int form=0, Tensor? blk=None, int part_size=0, int "
+      "parts=1, Tensor(b!)? sums=None, Tensor(c!)? part=None) -> ()");
+  m.def("mixed_mfma_ok(int H, int G, int D, int V, int page, float cap) -> int", &mixed_mfma_ok);
   m.def("moe_lists(int E) -> int", &moe_lists);
   m.def("moe_router_splits(int T, int W, int E, bool f32) -> int", &moe_router_splits);
   m.def(

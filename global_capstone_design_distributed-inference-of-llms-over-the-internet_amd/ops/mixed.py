@@ -39,11 +39,33 @@ def mixed_prep(z, q_gain, k_gain, qn, cache, slots, q_ctx, rope, vrope, out, K, 
                                int(F), int(block), int(col), float(limit), float(eps), int(packed))
 
 
-def mixed_attention(z, qn, talk, cache, table, q_seq, q_ctx, vrope, out, K, scale, cap, packed=False):
-    """Causal attention over the cache, into columns [0, H V) of ``out`` [T, K]; the head gates come from ``z``."""
+KEYS = 32  # keys of a tile: splits of a context are multiples of it
+BLOCK = 16  # tokens of a prompt's query block
+
+
+def mfma_ok(H, G, D, V, page, cap) -> int:
+    """Bit 0: the prompt form on MFMA covers the shape, bit 1: the decode form."""
+    return int(torch.ops.mpamd.mixed_mfma_ok(int(H), int(G), int(D), int(V), int(page), float(cap)))
+
+
+def mixed_parts(groups: int, span: int, n_cu: int = 256, least: int = 2 * KEYS):
+    """(keys per split, splits) of ``groups`` workgroups whose queries see at most ``span`` keys: about one workgroup per
+    CU, no split under ``least`` keys."""
+    span = max(1, int(span))
+    n = max(1, min(n_cu // max(1, int(groups)), span // least))
+    ps = KEYS * -(-span // (KEYS * n))
+    return ps, -(-span // ps)
+
+
+def mixed_attention(z, qn, talk, cache, table, q_seq, q_ctx, vrope, out, K, scale, cap, packed=False, form=0, blocks=None,
+                    parts=(0, 1), sums=None, part=None):
+    """Causal attention over the cache, into columns [0, H V) of ``out`` [T, K]; the head gates come from ``z``.
+    On the GPU ``form`` 1 (prompts: ``blocks`` [2, n] first token and tokens of every query block) and 2 (decode: every
+    row one token) run on MFMA, with the context in ``parts`` (keys per split, splits) and fp32 scratch ``sums``
+    [splits T H] and ``part`` [splits T H V] (prompts of several splits) or [splits T G H V]; 0 takes any shape."""
     if not _native(z):
         y = rx.mixed_attention(z, qn, talk, cache, table, q_seq, q_ctx, vrope, scale, cap)
         return rx.put_columns(out, y, 0, K, packed)
     torch.ops.mpamd.mixed_attention(z, qn, talk, cache, table, q_seq, q_ctx, vrope, out, int(K), float(scale), float(cap),
-                                    int(packed))
+                                    int(packed), int(form), blocks, int(parts[0]), int(parts[1]), sums, part)
     return out

@@ -34,6 +34,8 @@ from ..ops import moe as eops
 
 # most bytes of fp32 partial sums of a latent attention step whose contexts are split
 LATENT_WS_BYTES = 256 << 20
+# most bytes of fp32 partial sums of a head-mixing attention prompt whose contexts are split
+MIXED_WS_BYTES = 256 << 20
 # most bytes of the keys and values that long portions of prompts make of their contexts' latents, per step
 LATENT_KV_BYTES = 4 << 30
 
@@ -62,7 +64,7 @@ class HybridStage:
         keys |= {(sp.rot_base, sp.vdim, None) for sp in specs if sp.mixer == "mixed_attention"}
         self.rope = {k: mops.rope_table(k[0], k[1], ex.max_seq_len, ex.device, k[2]) for k in keys}
         # query-block tokens of each attention shape's MFMA form (0: the any-shape form)
-        self.talk_block, self.latent_block = {}, {}
+        self.talk_block, self.latent_block, self.mixed_ok = {}, {}, {}
         for sp in specs if ex.device.type == "cuda" else ():
             bf16 = ex.dtype == torch.bfloat16
             if sp.mixer == "attention":
@@ -72,6 +74,9 @@ class HybridStage:
             elif sp.mixer == "latent_attention":
                 key = self._latent_key(sp)
                 self.latent_block[key] = mops.latent_block(*key, ex.cache.page_size) if bf16 else 0
+            elif sp.mixer == "mixed_attention":
+                key = self._mixed_key(sp)
+                self.mixed_ok[key] = xops.mfma_ok(*key[:4], ex.cache.page_size, key[4]) if bf16 else 0
         self.rec_heads = min([sp.heads for sp in specs if sp.mixer == "hgrn2"], default=0)
         self.lin_heads = min([sp.heads for sp in specs if sp.mixer in ("retention", "mlstm")], default=0)
         self.max_chunk = max([sp.chunk or 1 << 30 for sp in specs if not sp.recurrent],
@@ -80,6 +85,10 @@ class HybridStage:
     @staticmethod
     def _rope_key(sp):
         return sp.rot_base, sp.rot_dims, sp.rot_scaling
+
+    @staticmethod
+    def _mixed_key(sp):
+        return sp.heads, sp.kv_heads, sp.dim, sp.vdim, sp.softcap
 
     @staticmethod
     def _latent_key(sp):
@@ -213,8 +222,20 @@ class HybridStage:
         ff = (self._ff_kind(sp), sp.ff, lay.ffn_block or 1, sp.mix_rows, sp.limit) if sp.parallel and sp.ff else None
         xops.mixed_prep(z, lay.q_gain, lay.k_gain, qn, kv, m["slots"], m["q_ctx"], rope, vrope, o, sp.o_cols, self.eps,
                         ff=ff, packed=pko)
+        kw, ok, plan, f32 = {}, self.mixed_ok.get(self._mixed_key(sp), 0), m["plan"], torch.float32
+        H, V = sp.heads, sp.vdim
+        if plan is not None and ok & 1:
+            mp = plan["mixed"]
+            parts = mp["parts"] if mp["parts"][1] * T * H * V * 4 <= MIXED_WS_BYTES else (0, 1)
+            kw = dict(form=1, blocks=mp["blocks"], parts=parts, sums=e("mix_sums", (parts[1] * T * H,), f32))
+            if parts[1] > 1:
+                kw["part"] = e("mix_part", (parts[1] * T * H * V,), f32)
+        elif plan is None and ok & 2:
+            parts = xops.mixed_parts(T, m["span"], ex._n_cu)
+            kw = dict(form=2, parts=parts, sums=e("mix_sums", (parts[1] * T * H,), f32),
+                      part=e("mix_part", (parts[1] * T * sp.kv_heads * H * V,), f32))
         xops.mixed_attention(z, qn, lay.talk, kv, m["table"], m["q_seq"], m["q_ctx"], vrope, o, sp.o_cols, sp.scale,
-                             sp.softcap, packed=pko)
+                             sp.softcap, packed=pko, **kw)
 
     MIX = {"hgrn2": _hgrn2, "retention": _retention, "mlstm": _mlstm, "attention": _attention,
            "latent_attention": _latent, "mixed_attention": _mixed}
@@ -344,6 +365,10 @@ class HybridStage:
             h = mops.linear_plan(ntoks, self.lin_heads, self.ex._n_cu)
             p["linear"] = {"seqs": up(h["seqs"]), "seg": up(h["seg"]), "slots": h["slots"],
                            "multi": up(h["multi"]) if h["slots"] else None}
+        if any(self.mixed_ok.values()):
+            blk = hops.talk_blocks(ntoks, xops.BLOCK)
+            span = int((np.asarray(starts) + np.asarray(ntoks)).max())
+            p["mixed"] = {"blocks": up(blk), "parts": xops.mixed_parts(blk.shape[1], span, self.ex._n_cu, 256)}
         p["latent"] = {key: self._latent_plan(key, tb, ntoks, starts, rows, up)
                        for key, tb in self.latent_block.items() if tb}
         return p
