@@ -14,6 +14,7 @@
 //
 //   mixed_prep_kernel   projected row [q (H D) | k (G D) | v (G V) | gate (H)] -> q', cache; and the feed-forward's
 //                       activation where its projection lies in the same row
+//   mixed_prep_vec_kernel  the same for whole 8-column vectors
 //   mixed_any_kernel    any shape and both element types: one workgroup per query token
 #include "attn_mixed.h"
 
@@ -109,6 +110,81 @@ __global__ __launch_bounds__(256) void mixed_prep_kernel(MixedArgs a, FfArgs f, 
     if (job < H) from_f(y, ((T*)a.qn)[((int64_t)t * H + job) * D + i]);
     else if (!val) from_f(y, pb[off * D + i]);
     else from_f(y, pb[page * D + val_at((int)off, i < half ? 2 * i : 2 * (i - half) + 1, V, val_block_log2(a.page_log2))]);
+  }
+}
+
+// The same for whole 8-column vectors: a workgroup of blockIdx.y 0 takes all of a row's heads.  Pass 1 brings the row to LDS
+// with a sum of squares per vector; pass 2 makes a vector from it and its rotation partner, half the turned entries away.
+constexpr int PREP_VECS = 2048;  // vectors of a row at most (LDS: 20 bytes each)
+
+__global__ __launch_bounds__(256) void mixed_prep_vec_kernel(MixedArgs a, FfArgs f) {
+  extern __shared__ __attribute__((aligned(16))) bf16_t row[];
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const bf16_t* z = (const bf16_t*)a.z + (int64_t)t * a.zs;
+  if (blockIdx.y > 0) {
+    ff_columns<bf16_t, 8>(z, f, (bf16_t*)a.out, t, a.os, a.packed_mt, ((int)blockIdx.y - 1) * 256 + tid,
+                          ((int)gridDim.y - 1) * 256);
+    return;
+  }
+  const int64_t slot = a.slots[t];
+  if (slot < 0) return;  // (uniform: a padding row)
+  const int H = a.H, G = a.G, D = a.D, V = a.V, dv = D >> 3, vv = V >> 3, nk = (H + G) * dv, n = nk + G * vv;
+  float* sq = reinterpret_cast<float*>(row + n * 8);
+  for (int i = tid; i < n; i += 256) {
+    const u16x8 x = *reinterpret_cast<const u16x8*>(z + i * 8);
+    *reinterpret_cast<u16x8*>(row + i * 8) = x;
+    float s = 0.f;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) s += bf2f(x[j]) * bf2f(x[j]);
+    sq[i] = s;
+  }
+  __syncthreads();
+  const int pos = a.q_ctx[t] - 1, bl = val_block_log2(a.page_log2);
+  const int64_t pg = slot >> a.page_log2, page = 1 << a.page_log2;
+  const int off = (int)(slot & (page - 1));
+  for (int i = tid; i < n; i += 256) {
+    const bool val = i >= nk;
+    const int head = val ? (i - nk) / vv : i / dv, c = val ? (i - nk) - head * vv : i - head * dv;
+    const int half = (val ? V : a.rot) >> 1, base = i - c, e0 = 8 * c;  // (whole vectors: half is a multiple of 8)
+    float x[8], p[8];
+    ld_vec<8>(row + i * 8, x);
+    const bool turn = e0 < 2 * half;
+    const bool up = e0 >= half;  // the pair's second entry
+    const float* cs = (val ? a.vrope + (int64_t)pos * V : a.rope + (int64_t)pos * a.rot) + (turn ? e0 - (up ? half : 0) : 0);
+    if (turn) ld_vec<8>(row + (base + ((up ? e0 - half : e0 + half) >> 3)) * 8, p);
+    if (!val) {
+      float ss = 0.f;
+      for (int k = 0; k < dv; ++k) ss += sq[base + k];
+      const float r = 1.f / sqrtf(ss / (float)D + a.eps);
+      const float* g = head < H ? a.qg : a.kg;
+      float gx[8], gp[8];
+      ld_vec<8>(g + e0, gx);
+      if (turn) ld_vec<8>(g + (up ? e0 - half : e0 + half), gp);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        x[j] *= r * gx[j];
+        if (turn) p[j] *= r * gp[j];
+      }
+    }
+    if (turn) {
+      float c8[8], s8[8];
+      ld_vec<8>(cs, c8);
+      ld_vec<8>(cs + half, s8);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[j] = up ? x[j] * c8[j] + p[j] * s8[j] : x[j] * c8[j] - p[j] * s8[j];
+    }
+    if (!val && head < H) {
+      st_vec<8>((bf16_t*)a.qn + (int64_t)t * H * D + i * 8, x);
+      continue;
+    }
+    bf16_t* pb = (bf16_t*)a.cache + (pg * G + (val ? head : head - H)) * page * (D + V);
+    if (!val) {
+      st_vec<8>(pb + (int64_t)off * D + e0, x);
+    } else {
+      pb += page * D + val_at(off, 2 * (up ? e0 - half : e0) + up, V, bl);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) pb[(int64_t)j << (bl + 1)] = f2bf(x[j]);
+    }
   }
 }
 
@@ -235,9 +311,17 @@ static int launch_mixed_any(const MixedArgs& a, int n, hipStream_t stream) {
 template <typename T>
 static int launch_prep(const MixedArgs& a, const FfArgs& f, int n, hipStream_t stream) {
   const int nh = (a.H + 2 * a.G + 3) / 4;
-  const bool vec = f.F % 8 == 0 && f.block % 8 == 0 && f.col % 8 == 0 && f.out_col % 8 == 0 && a.zs % 8 == 0 && a.os % 8 == 0;
+  const bool vec = f.F % 8 == 0 && (f.kind < 2 || f.block % 8 == 0) && f.col % 8 == 0 && f.out_col % 8 == 0 &&
+                   a.zs % 8 == 0 && a.os % 8 == 0;
   int nf = f.kind ? (f.F + 256 * (vec ? 8 : 1) - 1) / (256 * (vec ? 8 : 1)) : 0;
   if (nf > 64) nf = 64;
+  if constexpr (sizeof(T) == 2) {
+    const int vecs = ((a.H + a.G) * a.D + a.G * a.V) / 8;
+    if (vec && a.D % 8 == 0 && a.V % 16 == 0 && a.rot % 16 == 0 && vecs <= PREP_VECS) {
+      hipLaunchKernelGGL(mixed_prep_vec_kernel, dim3(n, 1 + nf), dim3(256), vecs * 20, stream, a, f);
+      return (int)hipGetLastError();
+    }
+  }
   if (vec) hipLaunchKernelGGL((mixed_prep_kernel<T, 8>), dim3(n, nh + nf), dim3(256), 0, stream, a, f, nh);
   else hipLaunchKernelGGL((mixed_prep_kernel<T, 1>), dim3(n, nh + nf), dim3(256), 0, stream, a, f, nh);
   return (int)hipGetLastError();
@@ -245,7 +329,7 @@ static int launch_prep(const MixedArgs& a, const FfArgs& f, int n, hipStream_t s
 
 template <typename T>
 static int launch_ffn(const T* z, int64_t zs, T* out, int64_t os, int mt, const FfArgs& f, int n, hipStream_t stream) {
-  const bool vec = f.F % 8 == 0 && f.block % 8 == 0 && zs % 8 == 0 && os % 8 == 0;
+  const bool vec = f.F % 8 == 0 && (f.kind < 2 || f.block % 8 == 0) && zs % 8 == 0 && os % 8 == 0;
   int nf = (f.F + 256 * (vec ? 8 : 1) - 1) / (256 * (vec ? 8 : 1));
   if (nf > 64) nf = 64;
   if (vec) hipLaunchKernelGGL((ffn_act_kernel<T, 8>), dim3(n, nf), dim3(256), 0, stream, z, zs, out, os, mt, f);

@@ -7,12 +7,14 @@
 //   mixed_core_kernel  the scores again, p = exp(s) / (1 + sum); p goes to LDS as hi + lo bf16 (16 bits of mantissa), one
 //                      MFMA with T mixes the heads of a (key, token), the mixed weights return through LDS to the waves
 //                      that own the heads, where they are the B operand of O^T += V^T A^T
-// A workgroup owns 16 tokens (the columns of all products) and all heads; a wave owns up to UPW heads.  K and V^T are
-// read from the cache as A operands.  Two barriers per 32 keys.
+// A workgroup owns 16 or 8 tokens and all heads; a wave owns UPW units of 16 columns, a unit being HPU heads of 16 / HPU
+// tokens.  K and V^T are read from the cache as A operands, a tile ahead.  Two barriers per 32 keys.
 //
 // Decode: a token's value product has all heads' weights as columns, so mixing after it costs no MFMA work:
 //   mixed_decode_kernel  per (token, split of the keys): O_{g, c} = sum_j exp(s_g) v_c(j) for all heads g and kv heads c
 //   mixed_merge_kernel   adds the splits, o_h = sum_g T[h, g] / (1 + sum_g) O_{g, c(h)}, turns back, applies the gate
+#include <type_traits>
+
 #include "attn_mixed.h"
 
 namespace mp {
@@ -23,13 +25,14 @@ __device__ __forceinline__ f32x4 mfma_bf(const u16x8& a, const u16x8& b, const f
                                                  0, 0);
 }
 
-constexpr int MX_KEYS = 32, MX_TOK = 16, MX_NW = 8, MX_HEADS = 32, MX_PITCH = 40;
+constexpr int MX_KEYS = 32, MX_NW = 8, MX_HEADS = 32, MX_PITCH = 40;
 constexpr float MX_LOG2E = 1.44269504088896340736f;
 
-// exp(cap tanh(scale s / cap)) = 2^(c - 2 c / (2^(b s) + 1)),  b = 2 scale log2(e) / cap, c = cap log2(e)
-__device__ __forceinline__ float cap_exp(float s, float b, float c) {
+// exp(cap tanh(scale s / cap)) = 2^(c - 2 c / (2^(b s) + 1)),  b = 2 scale log2(e) / cap, c = cap log2(e); c0 in place of
+// the first c: times 2^(c0 - c)
+__device__ __forceinline__ float cap_exp(float s, float b, float c, float c0) {
   const float r = __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s * b) + 1.f);
-  return __builtin_amdgcn_exp2f(__builtin_fmaf(-2.f * c, r, c));
+  return __builtin_amdgcn_exp2f(__builtin_fmaf(-2.f * c, r, c0));
 }
 
 // A query head's B operand: columns = tokens of the block, zero past the head and the block
@@ -61,8 +64,9 @@ struct BlockRange {
   int tok0, ntok, lo, hi;  // tokens, keys of this split
 };
 __device__ __forceinline__ BlockRange block_range(const MixedArgs& a, const int32_t* blk, int nblk, int PS) {
-  const int bx = nblk - 1 - (int)blockIdx.x;  // (later tokens see more keys: first)
+  const int bx = blockIdx.x;
   BlockRange r{blk[bx], blk[nblk + bx], 0, 0};
+  if (r.ntok <= 0) return r;  // (a filler)
   r.hi = a.q_ctx[r.tok0 + r.ntok - 1];
   if (PS > 0) {
     r.lo = blockIdx.z * PS;
@@ -71,39 +75,54 @@ __device__ __forceinline__ BlockRange block_range(const MixedArgs& a, const int3
   return r;
 }
 
+// What a lane owns of a wave's units: one token, heads head(u)
+template <int UPW, int HPU>
+struct Owner {
+  int tok, h0, hh, khi;
+  bool ok;
+  __device__ __forceinline__ Owner(const MixedArgs& a, const BlockRange& br, int w, int c16) {
+    constexpr int TB = 16 / HPU;
+    const int t = c16 % TB;
+    ok = t < br.ntok;
+    tok = br.tok0 + min(t, br.ntok - 1);
+    hh = c16 / TB;
+    h0 = w * UPW * HPU;
+    khi = ok ? a.q_ctx[tok] : 0;
+  }
+  __device__ __forceinline__ int head(int u) const { return h0 + hh * UPW + u; }
+};
+
 // sums [splits][T][H] of exp(s)
-template <int DH, int UPW, bool SHARE>
+template <int DH, int UPW, int HPU, bool SHARE>
 __global__ __launch_bounds__(MX_NW * 64) void mixed_sum_kernel(MixedArgs a, const int32_t* __restrict__ blk, int nblk, int PS,
                                                                float* __restrict__ sums, int T) {
   const int lane = threadIdx.x & 63, c16 = lane & 15, g4 = lane >> 4;
-  const int w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), h0 = w * UPW, rep = a.H / a.G;
+  const int w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), rep = a.H / a.G;
   const BlockRange br = block_range(a, blk, nblk, PS);
-  if (br.lo >= br.hi || h0 >= a.H) return;
+  if (br.lo >= br.hi || w * UPW * HPU >= a.H) return;
+  const Owner<UPW, HPU> own(a, br, w, c16);
   const int32_t* bt = a.bt + (int64_t)a.q_seq[br.tok0] * a.bt_stride;
   const int pmask = (1 << a.page_log2) - 1;
   const int64_t prow = (int64_t)(a.D + a.V) << a.page_log2;
   const float sb = 2.f * a.scale * MX_LOG2E / a.cap, sc = a.cap * MX_LOG2E;
-  const bool ok = c16 < br.ntok;
-  const int tok = br.tok0 + min(c16, br.ntok - 1), khi = ok ? a.q_ctx[tok] : 0, first = a.q_ctx[br.tok0];
+  const int first = a.q_ctx[br.tok0];
   u16x8 q[UPW][DH];
   float l[UPW];
 #pragma unroll
   for (int u = 0; u < UPW; ++u) {
-    load_q<DH>(a, tok, ok, min(h0 + u, a.H - 1), g4, q[u]);
+    load_q<DH>(a, own.tok, own.ok && own.head(u) < a.H, min(own.head(u), a.H - 1), g4, q[u]);
     l[u] = 0.f;
   }
-  auto kbase = [&](int s0, int u) {
-    return (const bf16_t*)a.cache + ((int64_t)bt[s0 >> a.page_log2] * a.G + min(h0 + u, a.H - 1) / rep) * prow;
-  };
   u16x8 kf[2][DH];
   auto fetch = [&](int s0, int u) {
-    const bf16_t* kp = kbase(s0, u);
-    const int off = s0 & pmask, last = off + min(MX_KEYS, br.hi - s0) - 1;
+    const bf16_t* kp = (const bf16_t*)a.cache + ((int64_t)bt[s0 >> a.page_log2] * a.G + min(own.h0 + u, a.H - 1) / rep) * prow;
+    const int off = s0 & pmask, last = off + br.hi - 1 - s0;
 #pragma unroll
     for (int sub = 0; sub < 2; ++sub) load_k<DH>(a, kp, off + 16 * sub, last, c16, g4, kf[sub]);
   };
   fetch(br.lo, 0);
-  for (int s0 = br.lo; s0 < br.hi; s0 += MX_KEYS) {
+  auto tile = [&](int s0, auto masked) {
+    constexpr bool MASK = decltype(masked)::value;
     f32x4 st[2][UPW];
 #pragma unroll
     for (int u = 0; u < UPW; ++u) {
@@ -116,25 +135,25 @@ __global__ __launch_bounds__(MX_NW * 64) void mixed_sum_kernel(MixedArgs a, cons
       }
     }
     if (s0 + MX_KEYS < br.hi) fetch(s0 + MX_KEYS, 0);
-    const bool all = s0 + MX_KEYS <= min(first, br.hi);  // (uniform: every token sees the whole tile)
+    const int see = min(own.khi, br.hi) - s0 - 4 * g4;
 #pragma unroll
     for (int sub = 0; sub < 2; ++sub)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int j = s0 + 16 * sub + 4 * g4 + r;
-        const bool see = all || (j < khi && j < br.hi);
+      for (int r = 0; r < 4; ++r)
 #pragma unroll
         for (int u = 0; u < UPW; ++u) {
-          const float p = cap_exp(st[sub][u][r], sb, sc);
-          l[u] += see ? p : 0.f;
+          const float p = cap_exp(st[sub][u][r], sb, sc, sc);
+          l[u] += !MASK || 16 * sub + r < see ? p : 0.f;
         }
-      }
-  }
+  };
+  int s0 = br.lo;  // (tiles that every token sees whole, then those with an edge)
+  for (; s0 + MX_KEYS <= min(first, br.hi); s0 += MX_KEYS) tile(s0, std::false_type{});
+  for (; s0 < br.hi; s0 += MX_KEYS) tile(s0, std::true_type{});
 #pragma unroll
   for (int u = 0; u < UPW; ++u) {
     l[u] += __shfl_xor(l[u], 16, 64);
     l[u] += __shfl_xor(l[u], 32, 64);
-    if (ok && g4 == 0 && h0 + u < a.H) sums[((int64_t)blockIdx.z * T + tok) * a.H + h0 + u] = l[u];
+    if (own.ok && g4 == 0 && own.head(u) < a.H) sums[((int64_t)blockIdx.z * T + own.tok) * a.H + own.head(u)] = l[u];
   }
 }
 
@@ -159,38 +178,38 @@ __device__ __forceinline__ float head_gate(const MixedArgs& a, int t, int h) {
   return 1.f / (1.f + __expf(-z));
 }
 
-constexpr int MX_PBYTES = MX_KEYS * MX_TOK * MX_PITCH * 2;  // one of p's two terms, [key][token][head]
-constexpr int MX_WBYTES = MX_HEADS * MX_TOK * MX_PITCH * 2;  // mixed weights [head][token][key]
+// LDS: p's two terms [key][token][head], mixed weights [head][token][key]
+constexpr int mx_lds(int tb) { return (2 * MX_KEYS + MX_HEADS) * tb * MX_PITCH * 2; }
 
-template <int DH, int VT, int UPW, bool SHARE>
-__global__ __launch_bounds__(MX_NW * 64) void mixed_core_kernel(MixedArgs a, const int32_t* __restrict__ blk, int nblk, int PS,
+template <int DH, int VT, int UPW, int HPU, bool SHARE>
+__global__ __launch_bounds__(MX_NW * 64) void mixed_core_kernel(MixedArgs a, const int32_t* __restrict__ blk, int nblk, int PS, int SPS,
                                                                 const float* __restrict__ sums, float* __restrict__ part,
                                                                 int T) {
-  constexpr int HB = UPW > 2 ? 2 : 1;
-  extern __shared__ __attribute__((aligned(16))) char smem[];
-  bf16_t* ph = reinterpret_cast<bf16_t*>(smem);
-  bf16_t* pl = ph + MX_PBYTES / 2;
-  bf16_t* wt = pl + MX_PBYTES / 2;
+  constexpr int HB = UPW * HPU > 2 ? 2 : 1, TB = 16 / HPU, NK = 4 / HPU, PTERM = MX_KEYS * TB * MX_PITCH;
+  extern __shared__ __attribute__((aligned(16))) bf16_t ph[];
+  bf16_t* wt = ph + 2 * PTERM;
   const int tid = threadIdx.x, lane = tid & 63, c16 = lane & 15, g4 = lane >> 4;
-  const int w = __builtin_amdgcn_readfirstlane(tid >> 6), h0 = w * UPW, H = a.H, rep = a.H / a.G;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6), H = a.H, rep = a.H / a.G;
   const BlockRange br = block_range(a, blk, nblk, PS);
   if (br.lo >= br.hi) return;
+  const Owner<UPW, HPU> own(a, br, w, c16);
   const int32_t* bt = a.bt + (int64_t)a.q_seq[br.tok0] * a.bt_stride;
   const int pmask = (1 << a.page_log2) - 1;
   const int64_t prow = (int64_t)(a.D + a.V) << a.page_log2, voff = (int64_t)a.D << a.page_log2;
   const float sb = 2.f * a.scale * MX_LOG2E / a.cap, sc = a.cap * MX_LOG2E;
-  const bool ok = c16 < br.ntok, mine = h0 < H;
-  const int tok = br.tok0 + min(c16, br.ntok - 1), khi = ok ? a.q_ctx[tok] : 0, first = a.q_ctx[br.tok0];
-  for (int i = tid; i < 2 * MX_PBYTES / 16; i += MX_NW * 64) reinterpret_cast<u16x8*>(smem)[i] = (u16x8)(0);
+  const bool mine = own.h0 < H;
+  const int first = a.q_ctx[br.tok0];
+  for (int i = tid; i < 2 * PTERM / 8; i += MX_NW * 64) reinterpret_cast<u16x8*>(ph)[i] = (u16x8)(0);
   u16x8 q[UPW][DH];
   f32x4 o[UPW][VT];
-  float inv[UPW];
+  float c0[UPW];  // the score's constant with the row's denominator in it
 #pragma unroll
   for (int u = 0; u < UPW; ++u) {
-    load_q<DH>(a, tok, ok && mine, min(h0 + u, H - 1), g4, q[u]);
+    const int h = min(own.head(u), H - 1);
+    load_q<DH>(a, own.tok, own.ok && own.head(u) < H, h, g4, q[u]);
     float l = 1.f;  // the sink
-    for (int p = 0; p == 0 || (PS > 0 && p * PS < khi); ++p) l += sums[((int64_t)p * T + tok) * H + min(h0 + u, H - 1)];
-    inv[u] = 1.f / l;
+    for (int p = 0; p * SPS < max(own.khi, 1); ++p) l += sums[((int64_t)p * T + own.tok) * H + h];
+    c0[u] = sc - __log2f(l);
 #pragma unroll
     for (int t = 0; t < VT; ++t) o[u][t] = (f32x4)(0.f);
   }
@@ -204,63 +223,73 @@ __global__ __launch_bounds__(MX_NW * 64) void mixed_core_kernel(MixedArgs a, con
       tf[hb][j] = h < H && g < H ? f2bf(t) : (bf16_t)0;
     }
   auto page = [&](int s0, int u) {
-    return (const bf16_t*)a.cache + ((int64_t)bt[s0 >> a.page_log2] * a.G + min(h0 + u, H - 1) / rep) * prow;
+    return (const bf16_t*)a.cache + ((int64_t)bt[s0 >> a.page_log2] * a.G + min(own.h0 + u, H - 1) / rep) * prow;
   };
-  u16x8 kf[2][DH];
+  u16x8 kf[2][DH], vf[VT];
   auto fetch = [&](int s0, int u) {
     const bf16_t* kp = page(s0, u);
-    const int off = s0 & pmask, last = off + min(MX_KEYS, br.hi - s0) - 1;
+    const int off = s0 & pmask, last = off + br.hi - 1 - s0;
 #pragma unroll
     for (int sub = 0; sub < 2; ++sub) load_k<DH>(a, kp, off + 16 * sub, last, c16, g4, kf[sub]);
   };
+  auto fetch_v = [&](int s0, int u) {
+    const bf16_t* vp = page(s0, u) + voff + (int64_t)((s0 & pmask) >> 5) * a.V * 32 + 8 * g4;
+#pragma unroll
+    for (int t = 0; t < VT; ++t) vf[t] = *reinterpret_cast<const u16x8*>(vp + min(16 * t + c16, a.V - 1) * 32);
+  };
+  const int pw = (4 * g4 * TB + c16 % TB) * MX_PITCH + own.head(0);             // p: this lane's first place to write
+  const int pr = ((4 * w + NK * own.hh) * TB + c16 % TB) * MX_PITCH + 8 * g4;   // and to read
+  const int ww = (4 * g4 * TB + c16 % TB) * MX_PITCH + 4 * w + NK * own.hh;     // mixed weights
   if (mine) fetch(br.lo, 0);
   __syncthreads();
-  for (int s0 = br.lo; s0 < br.hi; s0 += MX_KEYS) {
-    const bool all = s0 + MX_KEYS <= min(first, br.hi);
+  auto tile = [&](int s0, auto masked) {
+    constexpr bool MASK = decltype(masked)::value;
     if (mine) {
+      if (SHARE) fetch_v(s0, 0);
+      f32x4 st[2][UPW];
 #pragma unroll
-      for (int sub = 0; sub < 2; ++sub) {
-        f32x4 st[UPW];
+      for (int u = 0; u < UPW; ++u) {
+        if (!SHARE && u > 0) fetch(s0, u);
 #pragma unroll
-        for (int u = 0; u < UPW; ++u) {
-          if (!SHARE && (u > 0 || sub > 0))
-            load_k<DH>(a, page(s0, u), (s0 & pmask) + 16 * sub, (s0 & pmask) + min(MX_KEYS, br.hi - s0) - 1, c16, g4, kf[sub]);
-          st[u] = (f32x4)(0.f);
+        for (int sub = 0; sub < 2; ++sub) {
+          st[sub][u] = (f32x4)(0.f);
 #pragma unroll
-          for (int f = 0; f < DH; ++f) st[u] = mfma_bf(kf[sub][f], q[u][f], st[u]);
+          for (int f = 0; f < DH; ++f) st[sub][u] = mfma_bf(kf[sub][f], q[u][f], st[sub][u]);
         }
+      }
+      if (s0 + MX_KEYS < br.hi) fetch(s0 + MX_KEYS, 0);
+      const int see = min(own.khi, br.hi) - s0 - 4 * g4;
+#pragma unroll
+      for (int sub = 0; sub < 2; ++sub)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const int kk = 16 * sub + 4 * g4 + r, j = s0 + kk;
-          const bool see = all || (j < khi && j < br.hi);
           bf16_t hi[4], lo[4];
 #pragma unroll
           for (int u = 0; u < UPW; ++u) {
-            const float p = see ? cap_exp(st[u][r], sb, sc) * inv[u] : 0.f;
+            const float p = !MASK || 16 * sub + r < see ? cap_exp(st[sub][u][r], sb, sc, c0[u]) : 0.f;
             hi[u] = f2bf(p);
             lo[u] = f2bf(p - bf2f(hi[u]));
           }
-          const int at = (kk * MX_TOK + c16) * MX_PITCH + h0;
+          bf16_t* at = ph + pw + (16 * sub + r) * TB * MX_PITCH;
           if constexpr (UPW == 4) {
-            *reinterpret_cast<u16x4*>(ph + at) = (u16x4){hi[0], hi[1], hi[2], hi[3]};
-            *reinterpret_cast<u16x4*>(pl + at) = (u16x4){lo[0], lo[1], lo[2], lo[3]};
+            *reinterpret_cast<u16x4*>(at) = (u16x4){hi[0], hi[1], hi[2], hi[3]};
+            *reinterpret_cast<u16x4*>(at + PTERM) = (u16x4){lo[0], lo[1], lo[2], lo[3]};
           } else if constexpr (UPW == 2) {
-            *reinterpret_cast<u16x2*>(ph + at) = (u16x2){hi[0], hi[1]};
-            *reinterpret_cast<u16x2*>(pl + at) = (u16x2){lo[0], lo[1]};
+            *reinterpret_cast<u16x2*>(at) = (u16x2){hi[0], hi[1]};
+            *reinterpret_cast<u16x2*>(at + PTERM) = (u16x2){lo[0], lo[1]};
           } else {
-            ph[at] = hi[0];
-            pl[at] = lo[0];
+            at[0] = hi[0];
+            at[PTERM] = lo[0];
           }
         }
-      }
     }
     lds_wait_barrier();
     {  // mix: wave w takes keys 4 w .. 4 w + 3
-      f32x4 y[4][HB];
+      f32x4 y[NK][HB];
 #pragma unroll
-      for (int k = 0; k < 4; ++k) {
-        const int at = ((4 * w + k) * MX_TOK + c16) * MX_PITCH + 8 * g4;
-        const u16x8 bh = *reinterpret_cast<const u16x8*>(ph + at), bl = *reinterpret_cast<const u16x8*>(pl + at);
+      for (int k = 0; k < NK; ++k) {
+        const bf16_t* at = ph + pr + k * TB * MX_PITCH;
+        const u16x8 bh = *reinterpret_cast<const u16x8*>(at), bl = *reinterpret_cast<const u16x8*>(at + PTERM);
 #pragma unroll
         for (int hb = 0; hb < HB; ++hb) {
           y[k][hb] = mfma_bf(tf[hb], bl, (f32x4)(0.f));
@@ -270,58 +299,52 @@ __global__ __launch_bounds__(MX_NW * 64) void mixed_core_kernel(MixedArgs a, con
 #pragma unroll
       for (int hb = 0; hb < HB; ++hb)
 #pragma unroll
-        for (int r = 0; r < 4; ++r)
-          *reinterpret_cast<u16x4*>(wt + ((16 * hb + 4 * g4 + r) * MX_TOK + c16) * MX_PITCH + 4 * w) =
-              (u16x4){f2bf(y[0][hb][r]), f2bf(y[1][hb][r]), f2bf(y[2][hb][r]), f2bf(y[3][hb][r])};
+        for (int r = 0; r < 4; ++r) {
+          bf16_t* at = wt + ww + (16 * hb + r) * TB * MX_PITCH;
+          if constexpr (NK == 4)
+            *reinterpret_cast<u16x4*>(at) = (u16x4){f2bf(y[0][hb][r]), f2bf(y[1][hb][r]), f2bf(y[2][hb][r]), f2bf(y[NK - 1][hb][r])};
+          else
+            *reinterpret_cast<u16x2*>(at) = (u16x2){f2bf(y[0][hb][r]), f2bf(y[1][hb][r])};
+        }
     }
-    if (mine && s0 + MX_KEYS < br.hi) fetch(s0 + MX_KEYS, 0);
     lds_wait_barrier();
     if (mine) {
-      const int left = br.hi - s0;
       u16x8 wf[UPW];
 #pragma unroll
       for (int u = 0; u < UPW; ++u)
-        wf[u] = *reinterpret_cast<const u16x8*>(wt + (min(h0 + u, H - 1) * MX_TOK + c16) * MX_PITCH + 8 * g4);
-      const int64_t vb = (int64_t)((s0 & pmask) >> 5) * a.V * 32 + 8 * g4;
+        wf[u] = *reinterpret_cast<const u16x8*>(wt + (min(own.head(u), H - 1) * TB + c16 % TB) * MX_PITCH + 8 * g4);
 #pragma unroll
-      for (int t = 0; t < VT; ++t) {
-        const int64_t vc = vb + (int64_t)min(16 * t + c16, a.V - 1) * 32;
+      for (int v = 0; v < (SHARE ? 1 : UPW); ++v) {
+        if (!SHARE) fetch_v(s0, v);
 #pragma unroll
-        for (int u = 0; u < UPW; ++u) {
-          u16x8 vf;
-          if (SHARE ? u == 0 : true) {
-            vf = *reinterpret_cast<const u16x8*>(page(s0, u) + voff + vc);
-            if (left < MX_KEYS) clear_tail(vf, left, g4);
-          }
-          if constexpr (SHARE) {
-            if (u == 0) {
+        for (int t = 0; t < VT; ++t) {
+          if constexpr (MASK) clear_tail(vf[t], br.hi - s0, g4);
 #pragma unroll
-              for (int x = 0; x < UPW; ++x) o[x][t] = mfma_bf(vf, wf[x], o[x][t]);
-            }
-          } else {
-            o[u][t] = mfma_bf(vf, wf[u], o[u][t]);
-          }
+          for (int u = SHARE ? 0 : v; u < (SHARE ? UPW : v + 1); ++u) o[u][t] = mfma_bf(vf[t], wf[u], o[u][t]);
         }
       }
     }
-  }
-  if (!mine || !ok) return;
+  };
+  int s0 = br.lo;  // (tiles that every token sees whole, then those with an edge)
+  for (; s0 + MX_KEYS <= min(first, br.hi); s0 += MX_KEYS) tile(s0, std::false_type{});
+  for (; s0 < br.hi; s0 += MX_KEYS) tile(s0, std::true_type{});
+  if (!mine || !own.ok) return;
 #pragma unroll
   for (int u = 0; u < UPW; ++u) {
-    const int h = h0 + u;
+    const int h = own.head(u);
     if (h >= H) continue;
     if (part != nullptr) {  // [splits][T][H][V]
-      float* pp = part + (((int64_t)blockIdx.z * T + tok) * H + h) * a.V + 4 * g4;
+      float* pp = part + (((int64_t)blockIdx.z * T + own.tok) * H + h) * a.V + 4 * g4;
 #pragma unroll
       for (int t = 0; t < VT; ++t)
         if (16 * t < a.V) *reinterpret_cast<f32x4*>(pp + 16 * t) = o[u][t];
       continue;
     }
-    const float gate = head_gate(a, tok, h);
-    const float* cs = a.vrope + (int64_t)(khi - 1) * a.V;
+    const float gate = head_gate(a, own.tok, h);
+    const float* cs = a.vrope + (int64_t)(own.khi - 1) * a.V;
 #pragma unroll
     for (int t = 0; t < VT; ++t)
-      if (16 * t < a.V) store_out(a, tok, h, 16 * t + 4 * g4, cs, gate, o[u][t]);
+      if (16 * t < a.V) store_out(a, own.tok, h, 16 * t + 4 * g4, cs, gate, o[u][t]);
   }
 }
 
@@ -388,7 +411,8 @@ __global__ __launch_bounds__(MX_NW * 64, 2) void mixed_decode_kernel(MixedArgs a
   fetch(pg, lo);
   __syncthreads();
   int cur = 0;
-  for (int s0 = lo; s0 < hi; s0 += MX_KEYS, cur ^= 1) {
+  auto tile = [&](int s0, auto partial) {
+    constexpr bool TAIL = decltype(partial)::value;
     const int left = hi - s0;
     u16x8 vf[NT];
     const bf16_t* vb = pg + voff + (int64_t)((s0 & pmask) >> 5) * a.V * 32 + 8 * g4;
@@ -415,8 +439,8 @@ __global__ __launch_bounds__(MX_NW * 64, 2) void mixed_decode_kernel(MixedArgs a
       u16x4 h4, l4;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const bool see = 16 * us[i] + 4 * g4 + r < left;
-        const float p = see ? cap_exp(st[i][r], sb, sc) : 0.f;
+        const bool see = !TAIL || 16 * us[i] + 4 * g4 + r < left;
+        const float p = see ? cap_exp(st[i][r], sb, sc, sc) : 0.f;
         l[i] += p;
         h4[r] = f2bf(p);
         l4[r] = f2bf(p - bf2f(h4[r]));
@@ -435,7 +459,7 @@ __global__ __launch_bounds__(MX_NW * 64, 2) void mixed_decode_kernel(MixedArgs a
     }
 #pragma unroll
     for (int k = 0; k < NT; ++k) {
-      if (left < MX_KEYS) clear_tail(vf[k], left, g4);
+      if constexpr (TAIL) clear_tail(vf[k], left, g4);
 #pragma unroll
       for (int hb = 0; hb < 2; ++hb)
         if (16 * hb < H) {  // (uniform)
@@ -443,7 +467,11 @@ __global__ __launch_bounds__(MX_NW * 64, 2) void mixed_decode_kernel(MixedArgs a
           o[k][hb] = mfma_bf(vf[k], bh[hb], o[k][hb]);
         }
     }
-  }
+    cur ^= 1;
+  };
+  int s0 = lo;
+  for (; s0 + MX_KEYS <= hi; s0 += MX_KEYS) tile(s0, std::false_type{});
+  if (s0 < hi) tile(s0, std::true_type{});
 #pragma unroll
   for (int i = 0; i < UN; ++i) {
     l[i] += __shfl_xor(l[i], 16, 64);
@@ -504,15 +532,17 @@ __global__ __launch_bounds__(256) void mixed_merge_kernel(MixedArgs a, const flo
 }
 
 struct MixGeom {
-  int dh, vt, upw, share, un, nt;
+  int dh, vt, upw, hpu, share, un, nt;
 };
 static bool mixed_geometry(int H, int G, int D, int V, MixGeom& m) {
   if (H > MX_HEADS || G < 1 || H % G || D % 8 || D < 8 || D > 128 || V % 16 || V > 128) return false;
   const int rep = H / G;
   m.dh = D <= 64 ? 2 : 4;
   m.vt = V <= 64 ? 4 : 8;
-  m.upw = H <= 8 ? 1 : H <= 16 ? 2 : 4;
-  m.share = rep % m.upw == 0;
+  // many heads: a wave's four share a kv head, or they take a wave's registers to the last
+  m.hpu = H > 16 && rep % 4 == 0 ? 2 : 1;
+  m.upw = H <= 8 ? 1 : H <= 16 || m.hpu == 2 ? 2 : 4;
+  m.share = rep % (m.upw * m.hpu) == 0;
   const int units = (2 * G * ((rep + 15) / 16) + MX_NW - 1) / MX_NW, tiles = (G * V / 16 + MX_NW - 1) / MX_NW;
   m.un = units <= 2 ? 2 : units <= 4 ? 4 : 0;
   m.nt = tiles <= 4 ? 4 : tiles <= 8 ? 8 : tiles <= 16 ? 16 : 0;
@@ -521,53 +551,54 @@ static bool mixed_geometry(int H, int G, int D, int V, MixGeom& m) {
 
 }  // namespace mp
 
-// bit 0: the prompt kernels cover the shape, bit 1: the decode kernels
+// bit 0: the prompt kernels cover the shape, bit 1: the decode kernels; from bit 8 on: tokens of a prompt's block
 extern "C" int mp_mixed_mfma_ok(int H, int G, int D, int V, int page_log2, float cap) {
   using namespace mp;
   MixGeom m;
   if (page_log2 < 5 || !(cap > 0.f && cap <= 64.f) || !mixed_geometry(H, G, D, V, m)) return 0;
-  return 1 | (m.un && m.nt ? 2 : 0);
+  return 1 | (m.un && m.nt ? 2 : 0) | (16 / m.hpu) << 8;
 }
 
-// blk [2, nblk] (first token, tokens <= 16).  NP splits of PS keys; sums NP T H floats, part NP T H V floats when NP > 1
+// blk [2, nblk] (first token, tokens <= a block's; no tokens: a filler).  The denominators in SNP splits of SPS keys
+// (sums: SNP T H floats), the values in NP splits of PS keys (part: NP T H V floats when NP > 1)
 extern "C" int mp_mixed_prompt(const void* z, int64_t zs, const void* qn, const float* talk, const void* cache,
                                const int32_t* bt, int bt_stride, const int32_t* q_seq, const int32_t* q_ctx,
                                const float* vrope, void* out, int64_t os, int packed_mt, int n, int H, int G, int D, int V,
                                int page_log2, float scale, float cap, const int32_t* blk, int nblk, int PS, int NP,
-                               float* sums, float* part, hipStream_t stream) {
+                               int SPS, int SNP, float* sums, float* part, hipStream_t stream) {
   using namespace mp;
   (void)hipGetLastError();
   if (n == 0 || nblk == 0) return 0;
   MixGeom m;
   if (!(mp_mixed_mfma_ok(H, G, D, V, page_log2, cap) & 1) || !mixed_geometry(H, G, D, V, m)) return -1;
-  if (NP < 1 || NP > 65535 || sums == nullptr || (NP > 1 && (PS <= 0 || PS % MX_KEYS || part == nullptr))) return -2;
+  if (NP < 1 || NP > 65535 || (NP > 1 && (PS <= 0 || PS % MX_KEYS || part == nullptr))) return -2;
+  if (SNP < 1 || SNP > 65535 || SPS <= 0 || SPS % MX_KEYS || sums == nullptr) return -2;
   MixedArgs a{};
   a.z = z, a.zs = zs, a.qn = (void*)qn, a.talk = talk, a.cache = (void*)cache, a.bt = bt, a.bt_stride = bt_stride;
   a.q_seq = q_seq, a.q_ctx = q_ctx, a.vrope = vrope, a.out = out, a.os = os, a.packed_mt = packed_mt;
   a.H = H, a.G = G, a.D = D, a.V = V, a.page_log2 = page_log2, a.scale = scale, a.cap = cap;
   const int ps = NP > 1 ? PS : 0;
   float* pp = NP > 1 ? part : nullptr;
-  const dim3 grid(nblk, 1, NP), nt(MX_NW * 64);
-  constexpr size_t lds = 2 * MX_PBYTES + MX_WBYTES;
-#define MP_MC(DH_, VT_, UPW_, SH_)                                                                                 \
-  {                                                                                                                \
-    (void)hipFuncSetAttribute((const void*)mixed_core_kernel<DH_, VT_, UPW_, SH_>,                                 \
-                              hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);                               \
-    hipLaunchKernelGGL((mixed_core_kernel<DH_, VT_, UPW_, SH_>), grid, nt, lds, stream, a, blk, nblk, ps, sums, pp, n); \
+  const dim3 grid(nblk, 1, NP), sgrid(nblk, 1, SNP), nt(MX_NW * 64);
+#define MP_MC(DH_, VT_, UPW_, HPU_, SH_)                                                                                \
+  {                                                                                                                     \
+    constexpr int lds = mx_lds(16 / HPU_);                                                                              \
+    (void)hipFuncSetAttribute((const void*)mixed_core_kernel<DH_, VT_, UPW_, HPU_, SH_>,                                \
+                              hipFuncAttributeMaxDynamicSharedMemorySize, lds);                                         \
+    hipLaunchKernelGGL((mixed_core_kernel<DH_, VT_, UPW_, HPU_, SH_>), grid, nt, lds, stream, a, blk, nblk, ps, SPS, sums, pp, n); \
   }
-#define MP_MS(DH_, UPW_, SH_)                                                                                \
-  {                                                                                                          \
-    hipLaunchKernelGGL((mixed_sum_kernel<DH_, UPW_, SH_>), grid, nt, 0, stream, a, blk, nblk, ps, sums, n);  \
-    if (m.vt == 4) MP_MC(DH_, 4, UPW_, SH_) else MP_MC(DH_, 8, UPW_, SH_)                                    \
+#define MP_MS(DH_, UPW_, HPU_, SH_)                                                                               \
+  {                                                                                                               \
+    hipLaunchKernelGGL((mixed_sum_kernel<DH_, UPW_, HPU_, SH_>), sgrid, nt, 0, stream, a, blk, nblk, SPS, sums, n); \
+    if (m.vt == 4) MP_MC(DH_, 4, UPW_, HPU_, SH_) else MP_MC(DH_, 8, UPW_, HPU_, SH_)                             \
   }
-#define MP_MD(DH_)                                                    \
-  {                                                                   \
-    if (m.upw == 1) MP_MS(DH_, 1, true)                               \
-    else if (m.upw == 2) {                                            \
-      if (m.share) MP_MS(DH_, 2, true) else MP_MS(DH_, 2, false)      \
-    } else {                                                          \
-      if (m.share) MP_MS(DH_, 4, true) else MP_MS(DH_, 4, false)      \
-    }                                                                 \
+#define MP_MD(DH_)                              \
+  {                                             \
+    if (m.hpu == 2) MP_MS(DH_, 2, 2, true)      \
+    else if (m.upw == 4) MP_MS(DH_, 4, 1, false) \
+    else if (m.upw == 1) MP_MS(DH_, 1, 1, true) \
+    else if (m.share) MP_MS(DH_, 2, 1, true)    \
+    else MP_MS(DH_, 2, 1, false)                \
   }
   if (m.dh == 2) MP_MD(2) else MP_MD(4)
 #undef MP_MD

@@ -18,7 +18,7 @@ int mp_mixed_mfma_ok(int H, int G, int D, int V, int page_log2, float cap);
 int mp_mixed_prompt(const void* z, int64_t zs, const void* qn, const float* talk, const void* cache, const int32_t* bt,
                     int bt_stride, const int32_t* q_seq, const int32_t* q_ctx, const float* vrope, void* out, int64_t os,
                     int packed_mt, int n, int H, int G, int D, int V, int page_log2, float scale, float cap,
-                    const int32_t* blk, int nblk, int PS, int NP, float* sums, float* part, hipStream_t stream);
+                    const int32_t* blk, int nblk, int PS, int NP, int SPS, int SNP, float* sums, float* part, hipStream_t stream);
 int mp_mixed_decode(const void* z, int64_t zs, const void* qn, const float* talk, const void* cache, const int32_t* bt,
                     int bt_stride, const int32_t* q_seq, const int32_t* q_ctx, const float* vrope, void* out, int64_t os,
                     int packed_mt, int n, int H, int G, int D, int V, int page_log2, float scale, float cap, int PS, int NP,
@@ -120,12 +120,12 @@ int64_t mixed_mfma_ok(int64_t H, int64_t G, int64_t D, int64_t V, int64_t page, 
 }
 
 // form 0: any shape; 1: prompts, blk [2, nblk] (first token, tokens <= 16); 2: decode.  The keys in ``parts`` splits of
-// ``part_size``; sums fp32 [parts T H], part fp32 [parts T H V] (prompts, parts > 1) or [parts T G H V] (decode)
+// ``part_size`` (a prompt's denominators in ``sum_parts`` of ``sum_size``); sums fp32 [parts (sum_parts) T H], part fp32 [parts T H V] (prompts, parts > 1) or [parts T G H V] (decode)
 void mixed_attention(const at::Tensor& z, const at::Tensor& qn, const at::Tensor& talk, const at::Tensor& cache,
                      const at::Tensor& bt, const at::Tensor& q_seq, const at::Tensor& q_ctx, const at::Tensor& vrope,
                      at::Tensor& out, int64_t K, double scale, double cap, int64_t packed, int64_t form,
                      const opt_tensor& blk, int64_t part_size, int64_t parts, const opt_tensor& sums,
-                     const opt_tensor& part) {
+                     const opt_tensor& part, int64_t sum_size, int64_t sum_parts) {
   MP_CHECK(talk.dim() == 2 && talk.size(0) == talk.size(1), "talk [H, H]");
   const MixShape s = check_mixed(z, cache, vrope, talk.size(0));
   check_act(qn, s.f32, "qn");
@@ -142,7 +142,7 @@ void mixed_attention(const at::Tensor& z, const at::Tensor& qn, const at::Tensor
                    reinterpret_cast<uintptr_t>(t->data_ptr()) % 16 == 0, std::string(name) + ": fp32 scratch");
       return t->data_ptr<float>();
     };
-    float* sp = ws(sums, parts * s.T * s.H, "sums");
+    float* sp = ws(sums, (form == 2 ? parts : sum_parts) * s.T * s.H, "sums");
     if (form == 2) {
       check_launch(mp_mixed_decode(z.data_ptr(), z.stride(0), qn.data_ptr(), f32_vec(talk, s.H * s.H, "talk"),
                                    cache.data_ptr(), bt.data_ptr<int32_t>(), bt.stride(0), i32_vec(q_seq, s.T, "q_seq"),
@@ -158,7 +158,7 @@ void mixed_attention(const at::Tensor& z, const at::Tensor& qn, const at::Tensor
                                  bt.data_ptr<int32_t>(), bt.stride(0), i32_vec(q_seq, s.T, "q_seq"),
                                  i32_vec(q_ctx, s.T, "q_ctx"), vrope.data_ptr<float>(), out.data_ptr(), K, mt, s.T, s.H, s.G,
                                  s.D, s.V, s.pl2, (float)scale, (float)cap, i32_vec(*blk, 2 * nb, "blk"), nb, part_size,
-                                 parts, sp, parts > 1 ? ws(part, parts * s.T * s.H * s.V, "part") : nullptr, cur_stream()),
+                                 parts, sum_size, sum_parts, sp, parts > 1 ? ws(part, parts * s.T * s.H * s.V, "part") : nullptr, cur_stream()),
                  "mixed_prompt");
     return;
   }
@@ -212,7 +212,7 @@ void moe_route(const at::Tensor& x, const at::Tensor& w, const at::Tensor& ctx, 
                "moe_route");
 }
 
-// form 0: w [E, N, K]; 1, 2: w in fragment order [E, N / 16, K / 32, 64, 8].  ``glu``: N gate / up rows, out [rows, N / 2]
+// form 0: w [E, N, K]; 1, 2, 3: w in fragment order [E, N / 16, K / 32, 64, 8].  ``glu``: N gate / up rows, out [rows, N / 2]
 void moe_gemm(int64_t form, const at::Tensor& x, const opt_tensor& tok, const at::Tensor& lists, const at::Tensor& w,
               at::Tensor& out, int64_t rows, int64_t tokens, int64_t glu, int64_t block, double limit, int64_t packed) {
   const int f32 = act_type(w, "w");
@@ -250,7 +250,7 @@ TORCH_LIBRARY_FRAGMENT(mpamd, m) {
   m.def(
       "mixed_attention(Tensor z, Tensor qn, Tensor talk, Tensor cache, Tensor bt, Tensor q_seq, Tensor q_ctx, Tensor "
       "vrope, Tensor(a!) out, int K, float scale, float cap, int packed, int form=0, Tensor? blk=None, int part_size=0, int "
-      "parts=1, Tensor(b!)? sums=None, Tensor(c!)? part=None) -> ()");
+      "parts=1, Tensor(b!)? sums=None, Tensor(c!)? part=None, int sum_size=0, int sum_parts=1) -> ()");
   m.def("mixed_mfma_ok(int H, int G, int D, int V, int page, float cap) -> int", &mixed_mfma_ok);
   m.def("moe_lists(int E) -> int", &moe_lists);
   m.def("moe_router_splits(int T, int W, int E, bool f32) -> int", &moe_router_splits);

@@ -7,7 +7,7 @@
 //   moe_place        rows sorted by expert: first row of every expert, the token of every row, the row of every choice
 //   moe_gemm_any     any shape and both element types
 //   moe_gemm_rows    bf16, few rows per expert: weights stream once through registers in fragment order
-//   moe_gemm_tile    bf16, many rows per expert: 128 x 128 tiles through LDS
+//   moe_gemm_tile    bf16, many rows per expert: 128 x 128 or 256 x 256 tiles through LDS
 //
 // The products come in two kinds: gathered rows x gate/up weights with the clamped gated form as epilogue
 // (GLU: out = g sigmoid(1.702 g) (u + 1), g <= limit, |u| <= limit), and sorted rows x down weights.
@@ -165,7 +165,13 @@ __global__ __launch_bounds__(CH_WAVES * 64) void moe_choose_kernel(ChooseArgs a,
         v[j] = -INFINITY;
         if (e < E) {
           float x = 0.f;
-          for (int s = 0; s < a.S; ++s) x += a.part[((int64_t)s * a.T + t) * E + e];
+          for (int s = 0; s < a.S; s += 8) {  // eight slices' loads in flight, added in order
+            float p[8];
+#pragma unroll
+            for (int i = 0; i < 8; ++i) p[i] = a.part[((int64_t)min(s + i, a.S - 1) * a.T + t) * E + e];
+#pragma unroll
+            for (int i = 0; i < 8; ++i) x += s + i < a.S ? p[i] : 0.f;
+          }
           v[j] = fmaxf(x, -3e38f);  // (not a number: last, so that every rank is taken once)
           z[e] = v[j];
           mx = fmaxf(mx, v[j]);
@@ -413,22 +419,28 @@ __global__ __launch_bounds__(256) void moe_gemm_rows_kernel(MoeGemm a) {
   }
 }
 
-// Many rows per expert: 128 rows x 128 weight rows a workgroup, 64 columns a stage.  Both operands arrive in LDS in
-// fragment order (global_load_lds, 1 KiB a wave: packed weights as they lie, rows gathered by lane), two slots; a wave
-// makes 64 x 64.
-constexpr int MG_BM = 128, MG_BN = 128, MG_SLOT = 32 * 1024;
+// Many rows per expert: WM x WN waves of MW x NW fragment tiles (rows x weight rows), 32 columns a stage.  Both operands
+// arrive in LDS in fragment order (global_load_lds, 1 KiB a wave: packed weights as they lie, rows gathered by lane)
+// through a ring of MG_P slots, MG_P - 1 of them in flight.
+constexpr int MG_P = 4;
 
-template <bool GLU, typename TO>
-__global__ __launch_bounds__(256, 2) void moe_gemm_tile_kernel(MoeGemm a) {
+__device__ __forceinline__ int moe_tile_count(const MoeLists& l, int E, int i, int lane, int bm) {
+  return i + lane < E ? (l.cnt[i + lane] + bm - 1) / bm : 0;
+}
+
+template <bool GLU, typename TO, int MW, int NW, int WM, int WN>
+__global__ __launch_bounds__(WM * WN * 64) void moe_gemm_tile_kernel(MoeGemm a) {
+  constexpr int BM = 16 * MW * WM, BN = 16 * NW * WN, FX = BM / 16, J = (BM + BN) / 16 / (WM * WN), SLOT = (BM + BN) * 64;
+  static_assert((BM + BN) / 16 % (WM * WN) == 0, "whole fragments a wave");
   extern __shared__ __attribute__((aligned(1024))) char smem[];
   __shared__ int pick[4];
   const MoeLists l = moe_lists(const_cast<int32_t*>(a.lists), a.E);
   const int tid = threadIdx.x, lane = tid & 63, c16 = lane & 15, g4 = lane >> 4;
   const int wv = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int ntn = (a.N + MG_BN - 1) / MG_BN;
+  const int ntn = (a.N + BN - 1) / BN;
   if (wv == 0) {  // which tile: experts' row tiles in order, an expert's tiles by weight rows, then rows
     int total = 0;
-    for (int i = 0; i < a.E; i += 64) total += i + lane < a.E ? (l.cnt[i + lane] + MG_BM - 1) / MG_BM : 0;
+    for (int i = 0; i < a.E; i += 64) total += moe_tile_count(l, a.E, i, lane, BM);
 #pragma unroll
     for (int d = 32; d > 0; d >>= 1) total += __shfl_xor(total, d, 64);
     const int all = total * ntn, per = (all + 7) / 8;  // a contiguous run of tiles per XCD
@@ -437,7 +449,7 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_tile_kernel(MoeGemm a) {
     if (lane == 0) pick[0] = -1;
     int base = 0;
     for (int i = 0; i < a.E && on; i += 64) {
-      const int c = i + lane < a.E ? (l.cnt[i + lane] + MG_BM - 1) / MG_BM : 0;
+      const int c = moe_tile_count(l, a.E, i, lane, BM);
       int x = c;
 #pragma unroll
       for (int d = 1; d < 64; d <<= 1) {
@@ -456,64 +468,62 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_tile_kernel(MoeGemm a) {
   __syncthreads();
   const int e = pick[0];
   if (e < 0) return;
-  const int n0 = pick[1] * MG_BN, m0 = pick[2] * MG_BM, r0 = l.off[e], n = l.cnt[e], nt = a.N / 16, ks = a.K / 32;
+  const int n0 = pick[1] * BN, m0 = pick[2] * BM, r0 = l.off[e], n = l.cnt[e], nt = a.N / 16, ks = a.K / 32;
   const bf16_t* w = (const bf16_t*)a.w + (int64_t)e * a.N * a.K;
-  // this wave's fragments of a stage: row tiles 2 wv, 2 wv + 1 and weight tiles 2 wv, 2 wv + 1, both steps
-  const bf16_t *xp[2], *wp[2];
+  const bf16_t* fp[J];  // this wave's fragments of a stage, and their step to the next one
+  int fs[J];
 #pragma unroll
-  for (int i = 0; i < 2; ++i) {
-    const int m = r0 + min(m0 + 16 * (2 * wv + i) + c16, n - 1), row = a.tok ? a.tok[m] : m;
-    xp[i] = (const bf16_t*)a.x + (int64_t)row * a.xs + 8 * g4;
-    wp[i] = w + (int64_t)min(n0 / 16 + 2 * wv + i, nt - 1) * a.K * 16 + lane * 8;
+  for (int j = 0; j < J; ++j) {
+    const int f = wv * J + j;
+    if (f < FX) {
+      const int m = r0 + min(m0 + 16 * f + c16, n - 1), row = a.tok ? a.tok[m] : m;
+      fp[j] = (const bf16_t*)a.x + (int64_t)row * a.xs + 8 * g4;
+      fs[j] = 32;
+    } else {
+      fp[j] = w + (int64_t)min(n0 / 16 + f - FX, nt - 1) * a.K * 16 + lane * 8;
+      fs[j] = 512;
+    }
   }
   typedef __attribute__((address_space(3))) void* lptr_t;
   typedef __attribute__((address_space(1))) const void* gptr_t;
-  auto issue = [&](int slot, int st) {
+  auto issue = [&](int st) {
+    char* b = smem + (st & (MG_P - 1)) * SLOT + wv * J * 1024;
+    const int k = min(st, ks - 1);  // (past the end: a slot that is not read)
 #pragma unroll
-    for (int i = 0; i < 2; ++i)
-#pragma unroll
-      for (int h = 0; h < 2; ++h) {
-        const int64_t k = min(2 * st + h, ks - 1);
-        char* b = smem + slot * MG_SLOT + ((2 * wv + i) * 2 + h) * 1024;
-        __builtin_amdgcn_global_load_lds((gptr_t)(xp[i] + k * 32), (lptr_t)b, 16, 0, 0);
-        __builtin_amdgcn_global_load_lds((gptr_t)(wp[i] + k * 512), (lptr_t)(b + 16 * 1024), 16, 0, 0);
-      }
+    for (int j = 0; j < J; ++j)
+      __builtin_amdgcn_global_load_lds((gptr_t)(fp[j] + (int64_t)k * fs[j]), (lptr_t)(b + j * 1024), 16, 0, 0);
   };
-  const int wm = wv & 1, wn = wv >> 1;  // 64 rows, 64 weight rows of this wave
-  f32x4 acc[4][4];                      // [weight tile][row tile]
+  const int wm = wv % WM, wn = wv / WM;
+  f32x4 acc[NW][MW];
 #pragma unroll
-  for (int i = 0; i < 4; ++i)
+  for (int i = 0; i < NW; ++i)
 #pragma unroll
-    for (int j = 0; j < 4; ++j) acc[i][j] = (f32x4)(0.f);
-  const int ns = (ks + 1) / 2;
-  issue(0, 0);
-  for (int st = 0; st < ns; ++st) {
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    __syncthreads();
-    if (st + 1 < ns) issue((st + 1) & 1, st + 1);
-    const char* b = smem + (st & 1) * MG_SLOT;
+    for (int j = 0; j < MW; ++j) acc[i][j] = (f32x4)(0.f);
 #pragma unroll
-    for (int h = 0; h < 2; ++h) {
-      if (2 * st + h >= ks) break;  // (uniform)
-      u16x8 xf[4], wf[4];
+  for (int p = 0; p < MG_P - 1; ++p) issue(p);
+  for (int st = 0; st < ks; ++st) {
+    asm volatile("s_waitcnt vmcnt(%0)" ::"n"(J * (MG_P - 2)) : "memory");
+    lds_wait_barrier();  // stage st has landed for all waves, and all have read stage st - 1
+    issue(st + MG_P - 1);
+    const char* b = smem + (st & (MG_P - 1)) * SLOT + lane * 16;
+    u16x8 xf[MW], wf[NW];
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        xf[j] = *reinterpret_cast<const u16x8*>(b + ((4 * wm + j) * 2 + h) * 1024 + lane * 16);
-        wf[j] = *reinterpret_cast<const u16x8*>(b + 16 * 1024 + ((4 * wn + j) * 2 + h) * 1024 + lane * 16);
-      }
+    for (int j = 0; j < MW; ++j) xf[j] = *reinterpret_cast<const u16x8*>(b + (MW * wm + j) * 1024);
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
+    for (int i = 0; i < NW; ++i) wf[i] = *reinterpret_cast<const u16x8*>(b + (FX + NW * wn + i) * 1024);
 #pragma unroll
-        for (int j = 0; j < 4; ++j) acc[i][j] = mfma_bf(wf[i], xf[j], acc[i][j]);
-    }
+    for (int i = 0; i < NW; ++i)
+#pragma unroll
+      for (int j = 0; j < MW; ++j) acc[i][j] = mfma_bf(wf[i], xf[j], acc[i][j]);
   }
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // (the ring's last loads end before the workgroup does)
 #pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    const int m = m0 + 16 * (4 * wm + j) + c16;
+  for (int j = 0; j < MW; ++j) {
+    const int m = m0 + 16 * (MW * wm + j) + c16;
     if (m >= n) continue;
 #pragma unroll
-    for (int i = 0; i < 4; i += GLU ? 2 : 1) {
-      const int o = n0 + 16 * (4 * wn + i);
+    for (int i = 0; i < NW; i += GLU ? 2 : 1) {
+      const int o = n0 + 16 * (NW * wn + i);
       if (o >= a.N) continue;
       float y[4];
 #pragma unroll
@@ -521,6 +531,18 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_tile_kernel(MoeGemm a) {
       st_vec<4>((TO*)a.out + (int64_t)(r0 + m) * (GLU ? a.N / 2 : a.N) + (GLU ? o / 2 : o) + 4 * g4, y);
     }
   }
+}
+
+template <bool GLU, typename TO, int MW, int NW, int WM, int WN>
+static int launch_moe_tile(const MoeGemm& a, int rows, int act, hipStream_t stream) {
+  constexpr int BM = 16 * MW * WM, BN = 16 * NW * WN, LDS = MG_P * (BM + BN) * 64;
+  // (row tiles: at most one more than full ones per expert that has rows)
+  const int tiles = (rows / BM + act) * ((a.N + BN - 1) / BN);
+  (void)hipFuncSetAttribute((const void*)moe_gemm_tile_kernel<GLU, TO, MW, NW, WM, WN>,
+                            hipFuncAttributeMaxDynamicSharedMemorySize, LDS);
+  hipLaunchKernelGGL((moe_gemm_tile_kernel<GLU, TO, MW, NW, WM, WN>), dim3((tiles + 7) / 8 * 8), dim3(WM * WN * 64), LDS,
+                     stream, a);
+  return (int)hipGetLastError();
 }
 
 }  // namespace mp
@@ -568,7 +590,7 @@ extern "C" int mp_moe_route(const void* x, int64_t xs, int mt, const void* w, co
   return (int)hipGetLastError();
 }
 
-// form 0: any shape, 1: few rows per expert, 2: many
+// form 0: any shape, 1: few rows per expert, 2: many, 3: very many
 extern "C" int mp_moe_gemm(int form, int glu, const void* x, int64_t xs, int mt, const int32_t* tok,
                            const int32_t* lists, const void* w, void* out, int out_f32, int rows, int E, int N, int K,
                            int block, float limit, int f32, hipStream_t stream) {
@@ -588,20 +610,15 @@ extern "C" int mp_moe_gemm(int form, int glu, const void* x, int64_t xs, int mt,
       return (int)hipGetLastError();
     }
     if (mt > 0) return -1;
-    // (row tiles: at most one more than full ones per expert that has rows)
-    const int tiles = (rows / MG_BM + act) * ((N + MG_BN - 1) / MG_BN);
-    const dim3 g((tiles + 7) / 8 * 8);
-#define MP_MT(GLU_, TO_)                                                                                          \
-  {                                                                                                               \
-    (void)hipFuncSetAttribute((const void*)moe_gemm_tile_kernel<GLU_, TO_>, hipFuncAttributeMaxDynamicSharedMemorySize, \
-                              2 * MG_SLOT);                                                                       \
-    hipLaunchKernelGGL((moe_gemm_tile_kernel<GLU_, TO_>), g, dim3(256), 2 * MG_SLOT, stream, a);                  \
-  }
+    // 256 x 256 tiles where an expert's rows fill them, else 128 x 128
+    const bool big = form == 3;
+#define MP_MT(GLU_, TO_)                                                       \
+  return big ? launch_moe_tile<GLU_, TO_, 4, 8, 4, 2>(a, rows, act, stream) \
+             : launch_moe_tile<GLU_, TO_, 4, 4, 2, 2>(a, rows, act, stream);
     if (glu) MP_MT(true, bf16_t)
-    else if (out_f32) MP_MT(false, float)
-    else MP_MT(false, bf16_t)
+    if (out_f32) MP_MT(false, float)
+    MP_MT(false, bf16_t)
 #undef MP_MT
-    return (int)hipGetLastError();
   }
   if (!glu && !out_f32) return -1;
   if (f32) {

@@ -6,6 +6,7 @@ layer's output projection; ``packed`` writes it in the packed decode-GEMM layout
 """
 from __future__ import annotations
 
+import numpy as np
 import torch
 
 from . import reference_mixed as rx
@@ -40,12 +41,53 @@ def mixed_prep(z, q_gain, k_gain, qn, cache, slots, q_ctx, rope, vrope, out, K, 
 
 
 KEYS = 32  # keys of a tile: splits of a context are multiples of it
-BLOCK = 16  # tokens of a prompt's query block
+XCDS = 8
 
 
-def mfma_ok(H, G, D, V, page, cap) -> int:
-    """Bit 0: the prompt form on MFMA covers the shape, bit 1: the decode form."""
-    return int(torch.ops.mpamd.mixed_mfma_ok(int(H), int(G), int(D), int(V), int(page), float(cap)))
+def mfma_ok(H, G, D, V, page, cap):
+    """(tokens of a query block of the MFMA form for prompts, 0: not covered; does the decode form cover the shape)."""
+    r = int(torch.ops.mpamd.mixed_mfma_ok(int(H), int(G), int(D), int(V), int(page), float(cap)))
+    return (r >> 8 if r & 1 else 0), bool(r & 2)
+
+
+def sum_splits(blocks: int, span: int, n_cu: int = 256):
+    """(keys per split, splits) of a prompt's denominators: as many as even out the triangle of a causal mask."""
+    span = max(1, int(span))
+    n = max(1, min(-(-4 * n_cu // max(1, int(blocks))), span // 256, 16))
+    ps = KEYS * -(-span // (KEYS * n))
+    return ps, -(-span // ps)
+
+
+def mixed_blocks(ntoks, starts, tokens: int):
+    """Query blocks of a ragged step: int32 [2, n] (first flat token, tokens; 0: a filler).  Workgroup i runs on XCD
+    i % 8, and every XCD has an L2 of its own: a sequence's blocks stay on one XCD unless it is more than an XCD's share
+    of the keys to read.  Blocks with long contexts come first."""
+    seqs, off = [], 0
+    for n, s in zip(np.asarray(ntoks).tolist(), np.asarray(starts).tolist()):
+        b = [(s + min(k + tokens, n), off + k, min(tokens, n - k)) for k in range(0, n, tokens)]
+        if b:
+            seqs.append((sum(x[0] for x in b), b))
+        off += n
+    seqs.sort(key=lambda x: -x[0])
+    total = sum(w for w, _ in seqs)
+    bins, load = [[] for _ in range(XCDS)], [0] * XCDS
+    for w, b in seqs:
+        if w * XCDS > total * 1.05:
+            for x in b:
+                i = load.index(min(load))
+                bins[i].append(x)
+                load[i] += x[0]
+        else:
+            i = load.index(min(load))
+            bins[i] += b
+            load[i] += w
+    depth = max((len(b) for b in bins), default=0)
+    out = np.zeros((2, depth, XCDS), dtype=np.int32)
+    for i, b in enumerate(bins):
+        b.sort(key=lambda x: -x[0])
+        for k, (_, t, n) in enumerate(b):
+            out[:, k, i] = t, n
+    return np.ascontiguousarray(out.reshape(2, -1))
 
 
 def mixed_parts(groups: int, span: int, n_cu: int = 256, least: int = 2 * KEYS):
@@ -58,14 +100,16 @@ def mixed_parts(groups: int, span: int, n_cu: int = 256, least: int = 2 * KEYS):
 
 
 def mixed_attention(z, qn, talk, cache, table, q_seq, q_ctx, vrope, out, K, scale, cap, packed=False, form=0, blocks=None,
-                    parts=(0, 1), sums=None, part=None):
+                    parts=(0, 1), sums=None, part=None, sum_parts=(0, 1)):
     """Causal attention over the cache, into columns [0, H V) of ``out`` [T, K]; the head gates come from ``z``.
     On the GPU ``form`` 1 (prompts: ``blocks`` [2, n] first token and tokens of every query block) and 2 (decode: every
     row one token) run on MFMA, with the context in ``parts`` (keys per split, splits) and fp32 scratch ``sums``
-    [splits T H] and ``part`` [splits T H V] (prompts of several splits) or [splits T G H V]; 0 takes any shape."""
+    [splits T H] and ``part`` [splits T H V] (prompts of several splits) or [splits T G H V]; a prompt's denominators
+    have splits of their own (``sum_parts``, ``sums``).  0 takes any shape."""
     if not _native(z):
         y = rx.mixed_attention(z, qn, talk, cache, table, q_seq, q_ctx, vrope, scale, cap)
         return rx.put_columns(out, y, 0, K, packed)
     torch.ops.mpamd.mixed_attention(z, qn, talk, cache, table, q_seq, q_ctx, vrope, out, int(K), float(scale), float(cap),
-                                    int(packed), int(form), blocks, int(parts[0]), int(parts[1]), sums, part)
+                                    int(packed), int(form), blocks, int(parts[0]), int(parts[1]), sums, part, int(sum_parts[0]),
+                                    int(sum_parts[1]))
     return out

@@ -165,17 +165,17 @@ def experts(x, c: Choice, up, down, up_p, down_p, block, e, packed=False):
             at += n
         return y
     form = 0 if up_p is None else expert_form(R, m.experts, packed)
-    y = e("moe_y", (R, W), dt if form == 2 else torch.float32)
+    y = e("moe_y", (R, W), dt if form > 1 else torch.float32)
     torch.ops.mpamd.moe_gemm(form, x, c.tok, c.lists, up_p if form else up, act, R, c.tokens, 1, block, float(m.limit),
                              int(packed))
     torch.ops.mpamd.moe_gemm(form, act, None, c.lists, down_p if form else down, y, R, c.tokens, 0, 1, 0.0, 0)
     return y
 
 
-# mean rows per expert from which the tiled product runs instead of the weight-streaming one
-TILE_ROWS = 48
+# mean rows per expert from which the tiled products (128 and 256 rows a tile) run instead of the weight-streaming one
+TILE_ROWS, BIG_TILE_ROWS = 48, 384
 
 
 def expert_form(rows: int, experts: int, packed: bool) -> int:
-    """Product of ``rows`` choices: 1 few rows per expert, 2 many."""
-    return 1 if packed or rows < TILE_ROWS * experts else 2
+    """Product of ``rows`` choices: 1 few rows per expert, 2 many, 3 very many."""
+    return 1 if packed or rows < TILE_ROWS * experts else 2 if rows < BIG_TILE_ROWS * experts else 3

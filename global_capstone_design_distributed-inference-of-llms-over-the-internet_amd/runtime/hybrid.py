@@ -76,7 +76,7 @@ class HybridStage:
                 self.latent_block[key] = mops.latent_block(*key, ex.cache.page_size) if bf16 else 0
             elif sp.mixer == "mixed_attention":
                 key = self._mixed_key(sp)
-                self.mixed_ok[key] = xops.mfma_ok(*key[:4], ex.cache.page_size, key[4]) if bf16 else 0
+                self.mixed_ok[key] = xops.mfma_ok(*key[:4], ex.cache.page_size, key[4]) if bf16 else (0, False)
         self.rec_heads = min([sp.heads for sp in specs if sp.mixer == "hgrn2"], default=0)
         self.lin_heads = min([sp.heads for sp in specs if sp.mixer in ("retention", "mlstm")], default=0)
         self.max_chunk = max([sp.chunk or 1 << 30 for sp in specs if not sp.recurrent],
@@ -222,15 +222,16 @@ class HybridStage:
         ff = (self._ff_kind(sp), sp.ff, lay.ffn_block or 1, sp.mix_rows, sp.limit) if sp.parallel and sp.ff else None
         xops.mixed_prep(z, lay.q_gain, lay.k_gain, qn, kv, m["slots"], m["q_ctx"], rope, vrope, o, sp.o_cols, self.eps,
                         ff=ff, packed=pko)
-        kw, ok, plan, f32 = {}, self.mixed_ok.get(self._mixed_key(sp), 0), m["plan"], torch.float32
+        (tb, dec), kw, plan, f32 = self.mixed_ok.get(self._mixed_key(sp), (0, False)), {}, m["plan"], torch.float32
         H, V = sp.heads, sp.vdim
-        if plan is not None and ok & 1:
-            mp = plan["mixed"]
+        if plan is not None and tb:
+            mp = plan["mixed"][tb]
             parts = mp["parts"] if mp["parts"][1] * T * H * V * 4 <= MIXED_WS_BYTES else (0, 1)
-            kw = dict(form=1, blocks=mp["blocks"], parts=parts, sums=e("mix_sums", (parts[1] * T * H,), f32))
+            kw = dict(form=1, blocks=mp["blocks"], parts=parts, sum_parts=mp["sums"],
+                      sums=e("mix_sums", (mp["sums"][1] * T * H,), f32))
             if parts[1] > 1:
                 kw["part"] = e("mix_part", (parts[1] * T * H * V,), f32)
-        elif plan is None and ok & 2:
+        elif plan is None and dec:
             parts = xops.mixed_parts(T, m["span"], ex._n_cu)
             kw = dict(form=2, parts=parts, sums=e("mix_sums", (parts[1] * T * H,), f32),
                       part=e("mix_part", (parts[1] * T * sp.kv_heads * H * V,), f32))
@@ -365,10 +366,12 @@ class HybridStage:
             h = mops.linear_plan(ntoks, self.lin_heads, self.ex._n_cu)
             p["linear"] = {"seqs": up(h["seqs"]), "seg": up(h["seg"]), "slots": h["slots"],
                            "multi": up(h["multi"]) if h["slots"] else None}
-        if any(self.mixed_ok.values()):
-            blk = hops.talk_blocks(ntoks, xops.BLOCK)
+        p["mixed"] = {}
+        for tb in {t for t, _ in self.mixed_ok.values() if t}:
+            blk = xops.mixed_blocks(ntoks, starts, tb)
             span = int((np.asarray(starts) + np.asarray(ntoks)).max())
-            p["mixed"] = {"blocks": up(blk), "parts": xops.mixed_parts(blk.shape[1], span, self.ex._n_cu, 256)}
+            p["mixed"][tb] = {"blocks": up(blk), "sums": xops.sum_splits(blk.shape[1], span, self.ex._n_cu),
+                              "parts": xops.mixed_parts(blk.shape[1], span, self.ex._n_cu, 256)}
         p["latent"] = {key: self._latent_plan(key, tb, ntoks, starts, rows, up)
                        for key, tb in self.latent_block.items() if tb}
         return p
