@@ -21,6 +21,7 @@ every layer run has its own, also where a loop runs the same weights again.
 """
 from __future__ import annotations
 
+import os
 from typing import Optional
 
 import numpy as np
@@ -34,6 +35,8 @@ from ..ops import moe as eops
 
 # most bytes of fp32 partial sums of a latent attention step whose contexts are split
 LATENT_WS_BYTES = 256 << 20
+# decode steps of parallel layers run the routed experts beside the mixer
+PARALLEL_EXPERTS = os.environ.get("MPAMD_PARALLEL_EXPERTS", "1") != "0"
 # most bytes of fp32 partial sums of a head-mixing attention prompt whose contexts are split
 MIXED_WS_BYTES = 256 << 20
 # most bytes of the keys and values that long portions of prompts make of their contexts' latents, per step
@@ -77,6 +80,8 @@ class HybridStage:
             elif sp.mixer == "mixed_attention":
                 key = self._mixed_key(sp)
                 self.mixed_ok[key] = xops.mfma_ok(*key[:4], ex.cache.page_size, key[4]) if bf16 else (0, False)
+        self.side = torch.cuda.Stream(ex.device) if ex.device.type == "cuda" and PARALLEL_EXPERTS and \
+            any(sp.parallel and sp.moe for sp in specs) else None
         self.rec_heads = min([sp.heads for sp in specs if sp.mixer == "hgrn2"], default=0)
         self.lin_heads = min([sp.heads for sp in specs if sp.mixer in ("retention", "mlstm")], default=0)
         self.max_chunk = max([sp.chunk or 1 << 30 for sp in specs if not sp.recurrent],
@@ -123,17 +128,20 @@ class HybridStage:
             return ops.linear(x, None, wp=wp, a_rows=T, out=out)
         return ops.linear(x, w, out=out)
 
-    def _add(self, y_in, w, wp, packed: bool, T: int, res, gain, nxt, xb, xb_packed: bool, e, experts=None):
+    def _add(self, y_in, w, wp, packed: bool, T: int, res, gain, nxt, xb, xb_packed: bool, e, experts=None,
+             join=None):
         """Close a sublayer: add y = y_in w^T to the stream and write the next sublayer's ``xb``.  ``gain``: the
         sublayer's own norm gain, ``nxt``: the next one's (None after the last).  A packed projection with a split-K
         form hands its fp32 slabs straight to the kernel (no reduce launch, no rounding of y).  ``experts``: routed
-        experts' rows that belong to y (``y_in`` None: the only ones)."""
+        experts' rows that belong to y (``y_in`` None: the only ones); ``join``: the stream that waits for them."""
         if y_in is None:
             y = None
         elif packed and ops.rwk_split(T, w.shape[0], w.shape[1]) > 0:
             y = ops.linear_partials(y_in, T, wp=wp, out=e("y", (T, self.W)))
         else:
             y = self._mm(y_in, w, wp, T, packed, e("y", (T, self.W)))
+        if join is not None:
+            join.wait_stream(self.side)
         if self.pre:
             mops.add_norm(y, res, self.mult, nxt, self.eps, xb if nxt is not None else None, self.center,
                           packed=xb_packed, experts=experts)
@@ -246,6 +254,16 @@ class HybridStage:
         """Activation of a feed-forward that the decode GEMM's epilogues do not cover."""
         return "gated_glu" if sp.moe else sp.ffn
 
+    def _fork(self, lay, x, packed: bool, m, e):
+        """``_experts`` of a parallel layer beside its mixer: decode steps run them on a stream of their own (both paths
+        are chains of short launches), joined before the layer closes."""
+        if self.side is None or m["plan"] is not None:
+            return self._experts(lay, x, packed, m, e), None
+        cur = torch.cuda.current_stream()
+        self.side.wait_stream(cur)
+        with torch.cuda.stream(self.side):
+            return self._experts(lay, x, packed, m, e), cur
+
     def _experts(self, lay, x, packed: bool, m, e):
         """Routed experts of the rows ``x``: (rows, row of every choice, weights)."""
         c = eops.choose(x, lay.w_r, m["q_ctx"], lay.spec.moe, e, packed=packed)
@@ -319,6 +337,7 @@ class HybridStage:
             if prompt is not None:  # deep prompt: the block input += prompt[i]
                 res.index_add_(0, prompt[0], prompt[1][i].float())
                 self._enter(res, first_gain(i), xb, pk)
+            rows, join = self._fork(lay, xb, pk, m, e) if sp.moe and sp.parallel else (None, None)
             z = self._mm(xb, lay.w_in, lay.w_in_p, T, pk, e(f"z{sp.in_rows}", (T, sp.in_rows)))
             pko = self._packed(T, lay.w_o, lay.w_o_p)
             o = self._act(e, "o", T, sp.o_cols, pko)
@@ -332,9 +351,8 @@ class HybridStage:
                 pk, xb = entry(i + 1)
                 self._add(a, lay.w_down, lay.w_down_p, pkd, T, res, lay.n2, first_gain(i + 1), xb, pk, e, rows)
             else:
-                rows = self._experts(lay, xb, pk, m, e) if sp.moe else None
                 pk, xb = entry(i + 1)
-                self._add(o, lay.w_o, lay.w_o_p, pko, T, res, lay.n1, first_gain(i + 1), xb, pk, e, rows)
+                self._add(o, lay.w_o, lay.w_o_p, pko, T, res, lay.n1, first_gain(i + 1), xb, pk, e, rows, join)
         if not ex.is_last:
             return res
         S, V = last_rows.numel(), ex.cfg.vocab_size
