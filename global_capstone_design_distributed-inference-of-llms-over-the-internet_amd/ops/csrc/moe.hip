@@ -152,9 +152,33 @@ __global__ __launch_bounds__(CH_WAVES * 64) void moe_choose_kernel(ChooseArgs a,
   for (int e = tid; e < E; e += blockDim.x) hist[e] = 0;
   __syncthreads();
   const int t0 = (blockIdx.x * nw + wv) * per;
+  // the next token's logits are on their way while this one's experts are ranked
+  float nx[CH_PER];
+  auto fetch = [&](int t) {
+#pragma unroll
+    for (int j = 0; j < CH_PER; ++j) {
+      const int e = lane + 64 * j;
+      nx[j] = 0.f;
+      if (64 * j < E) {  // (uniform)
+        for (int s = 0; s < a.S; s += 8) {  // eight slices' loads in flight, added in order
+          float p[8];
+#pragma unroll
+          for (int i = 0; i < 8; ++i)
+            p[i] = a.part[((int64_t)min(s + i, a.S - 1) * a.T + min(t, a.T - 1)) * E + min(e, E - 1)];
+#pragma unroll
+          for (int i = 0; i < 8; ++i) nx[j] += s + i < a.S ? p[i] : 0.f;
+        }
+      }
+    }
+  };
+  fetch(t0);
   for (int i = 0; i < per; ++i) {
     const int t = t0 + i;
     const bool live = t < a.T && a.ctx[t] > 0;
+    float cur[CH_PER];
+#pragma unroll
+    for (int j = 0; j < CH_PER; ++j) cur[j] = nx[j];
+    if (i + 1 < per) fetch(t + 1);
     if (t < a.T && !live)
       for (int k = lane; k < a.top; k += 64) a.idx[t * a.top + k] = a.slot[t * a.top + k] = -1, a.ew[t * a.top + k] = 0.f;
     if (live) {
@@ -164,15 +188,7 @@ __global__ __launch_bounds__(CH_WAVES * 64) void moe_choose_kernel(ChooseArgs a,
         const int e = lane + 64 * j;
         v[j] = -INFINITY;
         if (e < E) {
-          float x = 0.f;
-          for (int s = 0; s < a.S; s += 8) {  // eight slices' loads in flight, added in order
-            float p[8];
-#pragma unroll
-            for (int i = 0; i < 8; ++i) p[i] = a.part[((int64_t)min(s + i, a.S - 1) * a.T + t) * E + e];
-#pragma unroll
-            for (int i = 0; i < 8; ++i) x += s + i < a.S ? p[i] : 0.f;
-          }
-          v[j] = fmaxf(x, -3e38f);  // (not a number: last, so that every rank is taken once)
+          v[j] = fmaxf(cur[j], -3e38f);  // (not a number: last, so that every rank is taken once)
           z[e] = v[j];
           mx = fmaxf(mx, v[j]);
         }
@@ -186,6 +202,7 @@ __global__ __launch_bounds__(CH_WAVES * 64) void moe_choose_kernel(ChooseArgs a,
       __builtin_amdgcn_wave_barrier();
       for (int g = lane; g < a.groups; g += 64) {
         float b = z[g * gs];
+#pragma unroll 8
         for (int j = 1; j < gs; ++j) b = fmaxf(b, z[g * gs + j]);
         gz[g] = b;
       }
@@ -198,6 +215,7 @@ __global__ __launch_bounds__(CH_WAVES * 64) void moe_choose_kernel(ChooseArgs a,
         const int e = lane + 64 * j, g = min(e, E - 1) / gs;
         int better = 0;
         if (e < E)
+#pragma unroll 8
           for (int q = 0; q < a.groups; ++q) better += gz[q] > gz[g] || (gz[q] == gz[g] && q < g);
         in[j] = e < E && better < a.keep;
       }
@@ -216,6 +234,7 @@ __global__ __launch_bounds__(CH_WAVES * 64) void moe_choose_kernel(ChooseArgs a,
         s[j] = 0.f;
         if (in[j]) {
           int better = 0;
+#pragma unroll 8
           for (int q = 0; q < E; ++q) better += z[q] > v[j] || (z[q] == v[j] && q < e);
           rank[j] = better;
           if (better < a.top) s[j] = expf(v[j] - mx) / sum;
@@ -584,7 +603,8 @@ extern "C" int mp_moe_route(const void* x, int64_t xs, int mt, const void* w, co
   const ChooseArgs a{part, ctx, S, T, E, top, groups, keep, scale, ew, idx, slot, lists, tok};
   const int nw = E <= 256 ? CH_WAVES : CH_WAVES / 2;  // (LDS: 8 E bytes a wave)
   const size_t lds = (2 * E + 1 + nw * 2 * E) * sizeof(float);
-  const int per = T <= 256 ? (T + nw - 1) / nw : 4, nb = T <= 256 ? 1 : (T + nw * per - 1) / (nw * per);
+  // one token a wave as long as that fills no more than the chip; a single workgroup also places the rows
+  const int per = (T + 256 * nw - 1) / (256 * nw), nb = (T + nw * per - 1) / (nw * per);
   hipLaunchKernelGGL(moe_choose_kernel, dim3(nb), dim3(nw * 64), lds, stream, a, per);
   if (nb > 1) hipLaunchKernelGGL(moe_place_kernel, dim3((T * top + 255) / 256), dim3(256), 0, stream, a);
   return (int)hipGetLastError();
