@@ -62,34 +62,45 @@ __global__ __launch_bounds__(256) void moe_router_any_kernel(const T* __restrict
   if (lane == 0) part[((int64_t)s * T_ + t) * E + e] = a;
 }
 
-// 16 tokens x 64 experts a workgroup; the slice's 32-column steps go round the waves
+// 16 tokens x 16 NT experts a workgroup; the slice's 32-column steps go round the waves, U of them in flight
+template <int NT, int U>
 __global__ __launch_bounds__(256) void moe_router_mfma_kernel(const bf16_t* __restrict__ x, int64_t xs, int mt,
                                                               const bf16_t* __restrict__ w, float* __restrict__ part,
                                                               int T, int E, int W, int ks, int32_t* __restrict__ cnt) {
-  __shared__ float red[4][64 * 17];
+  __shared__ float red[4][16 * NT * 17];
   const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, c16 = lane & 15, g4 = lane >> 4;
-  const int t0 = blockIdx.x * 16, e0 = blockIdx.y * 64, s = blockIdx.z;
-  if (blockIdx.x == 0 && s == 0 && tid < 64 && e0 + tid < E) cnt[e0 + tid] = 0;
+  const int t0 = blockIdx.x * 16, e0 = blockIdx.y * 16 * NT, s = blockIdx.z;
+  if (blockIdx.x == 0 && s == 0 && tid < 16 * NT && e0 + tid < E) cnt[e0 + tid] = 0;
   const int row = min(t0 + c16, T - 1), k1 = min(W, (s + 1) * ks);
-  f32x4 acc[4];
+  f32x4 acc[NT];
+  const bf16_t* wp[NT];
 #pragma unroll
-  for (int n = 0; n < 4; ++n) acc[n] = (f32x4)(0.f);
-  for (int k = s * ks + 32 * wv; k < k1; k += 128) {
-    const u16x8 b = *reinterpret_cast<const u16x8*>(x + act_at(row, k + 8 * g4, xs, mt));
+  for (int n = 0; n < NT; ++n) {
+    acc[n] = (f32x4)(0.f);
+    wp[n] = w + (int64_t)min(e0 + 16 * n + c16, E - 1) * W + 8 * g4;
+  }
+  for (int k = s * ks + 32 * wv; k < k1; k += 128 * U) {
+    u16x8 b[U], a[U][NT];
 #pragma unroll
-    for (int n = 0; n < 4; ++n) {
-      const int e = min(e0 + 16 * n + c16, E - 1);
-      const u16x8 a = *reinterpret_cast<const u16x8*>(w + (int64_t)e * W + k + 8 * g4);
-      acc[n] = mfma_bf(a, b, acc[n]);  // rows: experts, columns: tokens
+    for (int u = 0; u < U; ++u) {
+      const int kk = min(k + 128 * u, W - 32);  // (past the slice: loaded, not used)
+      b[u] = *reinterpret_cast<const u16x8*>(x + act_at(row, kk + 8 * g4, xs, mt));
+#pragma unroll
+      for (int n = 0; n < NT; ++n) a[u][n] = *reinterpret_cast<const u16x8*>(wp[n] + kk);
     }
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+      if (k + 128 * u < k1)  // (uniform)
+#pragma unroll
+        for (int n = 0; n < NT; ++n) acc[n] = mfma_bf(a[u][n], b[u], acc[n]);  // rows: experts, columns: tokens
   }
 #pragma unroll
-  for (int n = 0; n < 4; ++n)
+  for (int n = 0; n < NT; ++n)
 #pragma unroll
     for (int r = 0; r < 4; ++r) red[wv][(16 * n + 4 * g4 + r) * 17 + c16] = acc[n][r];
   __syncthreads();
-  for (int i = tid; i < 1024; i += 256) {
-    const int t = i >> 6, e = i & 63, at = e * 17 + t;
+  for (int i = tid; i < 256 * NT; i += 256) {
+    const int t = i / (16 * NT), e = i % (16 * NT), at = e * 17 + t;
     if (t0 + t < T && e0 + e < E)
       part[((int64_t)s * T + t0 + t) * E + e0 + e] = red[0][at] + red[1][at] + red[2][at] + red[3][at];
   }
@@ -589,8 +600,13 @@ extern "C" int mp_moe_route(const void* x, int64_t xs, int mt, const void* w, co
   int ks = (W + S - 1) / S;
   ks = (ks + 31) / 32 * 32;
   if (!f32 && W % 32 == 0 && (mt > 0 || xs % 8 == 0)) {
-    hipLaunchKernelGGL(moe_router_mfma_kernel, dim3((T + 15) / 16, (E + 63) / 64, S), dim3(256), 0, stream,
-                       (const bf16_t*)x, xs, mt, (const bf16_t*)w, part, T, E, W, ks, l.cnt);
+#define MP_RT(NT_, U_)                                                                                                  \
+  hipLaunchKernelGGL((moe_router_mfma_kernel<NT_, U_>), dim3((T + 15) / 16, (E + 16 * NT_ - 1) / (16 * NT_), S),        \
+                     dim3(256), 0, stream, (const bf16_t*)x, xs, mt, (const bf16_t*)w, part, T, E, W, ks, l.cnt)
+    if (E <= 16) MP_RT(1, 8);
+    else if (E <= 32) MP_RT(2, 8);
+    else MP_RT(4, 4);
+#undef MP_RT
   } else {
     const dim3 grid(T, (E + 3) / 4, S);
     if (f32)
